@@ -39,7 +39,7 @@
 extern "C" {
 #endif
 
-#define TAH_DUO_ABI_VERSION 7
+#define TAH_DUO_ABI_VERSION 8
 
 enum {
     TAH_OK = 0,
@@ -459,7 +459,8 @@ int tah_silu_mul_normed(const void* gate_up, void* out, int32_t rows, int32_t in
  * act_fn(gate) * up, down_proj + residual add.  Products accumulate in float32 in a fixed order (results do not
  * vary from run to run) and are rounded to bf16 where the eager modules round. */
 enum { TAH_LINEAR_PLAIN = 0, TAH_LINEAR_GATE_UP = 1 };
-enum { TAH_ACT_NONE = 0, TAH_ACT_RELU = 1, TAH_ACT_GELU = 2 };      /* GELU: x Phi(x), nn.GELU's default */
+enum { TAH_ACT_NONE = 0, TAH_ACT_RELU = 1, TAH_ACT_GELU = 2,        /* GELU: x Phi(x), nn.GELU's default */
+       TAH_ACT_GELU_TANH = 3 };                                     /* its tanh form */
 enum { TAH_NORM_NONE = 0, TAH_NORM_RMS = 1, TAH_NORM_LAYER = 2 };
 
 /* w bf16 [n, k] row-major (nn.Linear weight), or [2 n, k] = [gate; up] stacked for TAH_LINEAR_GATE_UP; k % 32 == 0,
@@ -489,8 +490,17 @@ typedef struct tah_linear_rows_args {
     float norm_eps;
     const void* bias;         /* TAH_LINEAR_PLAIN: bf16 [n] added to the product (after its rounding to bf16, before the
                                * residual), or NULL */
-    int32_t activation;       /* TAH_LINEAR_PLAIN: TAH_ACT_RELU / TAH_ACT_GELU applied last (a small MLP's first layer) */
+    int32_t activation;       /* TAH_LINEAR_PLAIN: TAH_ACT_* applied last (an MLP's first layer) */
     const float* ln_colsum;   /* TAH_NORM_LAYER: float32 [n], sum over k of the bf16 weight row as packed; else ignored */
+    /* Several products of these sizes in one launch (per-head products of latent attention, the experts of a mixture):
+     * product i (i < batch; 0 or 1: one product) uses operands and results i * stride elements further on (strides
+     * % 8 == 0; an operand shared by all has stride 0).  No residual, bias or input norm with batch > 1. */
+    int32_t batch;
+    int32_t out_packed_col_step; /* != 0: result i goes to columns i * step ... of one packed rows buffer (step >= n,
+                                  * step % 8 == 0), so that the results lie side by side as one operand */
+    int64_t w_batch_stride, x_batch_stride, out_batch_stride, out_packed_batch_stride;
+    const int32_t* batch_select; /* int32 [n_select], or NULL: only products whose index is listed run */
+    int32_t n_select;
 } tah_linear_rows_args;
 int tah_linear_rows(const tah_linear_rows_args* args, tah_stream_t stream);
 

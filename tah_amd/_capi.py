@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import ctypes as C
 
-ABI_VERSION = 7
+ABI_VERSION = 8
 
 c_void_p, c_int32, c_int64, c_float = C.c_void_p, C.c_int32, C.c_int64, C.c_float
 
@@ -118,6 +118,9 @@ class LinearRowsArgs(C.Structure):
         ("residual_row_stride", c_int64), ("out_row_stride", c_int64),
         ("rows", c_int32), ("n", c_int32), ("k", c_int32), ("kind", c_int32), ("input_norm", c_int32), ("norm_eps", c_float),
         ("bias", c_void_p), ("activation", c_int32), ("ln_colsum", c_void_p),
+        ("batch", c_int32), ("out_packed_col_step", c_int32),
+        ("w_batch_stride", c_int64), ("x_batch_stride", c_int64), ("out_batch_stride", c_int64), ("out_packed_batch_stride", c_int64),
+        ("batch_select", c_void_p), ("n_select", c_int32),
     ]
 
 
@@ -246,6 +249,66 @@ class QkPrepBwdArgs(C.Structure):
     ]
 
 
+class EmbedRowsArgs(C.Structure):
+    """``tah_embed_rows_args``"""
+
+    _fields_ = [
+        ("tok", c_void_p), ("pos", c_void_p), ("finished", c_void_p), ("embed", c_void_p), ("x", c_void_p), ("xe", c_void_p),
+        ("x_packed", c_void_p), ("slot", c_void_p), ("q_pos", c_void_p), ("active", c_void_p),
+        ("rows", c_int32), ("vocab", c_int32), ("cols", c_int32), ("dtype", c_int32), ("slot_base", c_int32),
+    ]
+
+
+class ResidualNormArgs(C.Structure):
+    """``tah_residual_norm_args``"""
+
+    _fields_ = [
+        ("y", c_void_p), ("y_scale", c_void_p), ("experts", c_void_p), ("index", c_void_p), ("weight", c_void_p), ("coef", c_void_p),
+        ("final_coef", c_void_p), ("x", c_void_p), ("xe", c_void_p), ("x_packed", c_void_p), ("normed", c_void_p),
+        ("normed_packed", c_void_p), ("y_row_stride", c_int64), ("experts_row_stride", c_int64),
+        ("rows", c_int32), ("width", c_int32), ("cols", c_int32), ("top", c_int32), ("index_scale", c_int32), ("index_row", c_int32), ("dtype", c_int32),
+        ("eps", c_float),
+    ]
+
+
+class DeltaLayer(C.Structure):
+    """``tah_delta_layer``"""
+
+    _fields_ = [
+        ("proj", c_void_p), ("proj_row_stride", c_int64),
+        ("q_col", c_int32), ("k_col", c_int32), ("v_col", c_int32), ("gate_col", c_int32), ("b_col", c_int32), ("a_col", c_int32),
+        ("conv", c_void_p), ("a_log", c_void_p), ("dt_bias", c_void_p), ("norm", c_void_p), ("conv_state", c_void_p), ("state", c_void_p),
+        ("heads", c_int32), ("kv_heads", c_int32), ("dim", c_int32), ("vdim", c_int32), ("taps", c_int32), ("nslots", c_int32),
+        ("dtype", c_int32), ("eps", c_float),
+    ]
+
+
+class Portions(C.Structure):
+    """``tah_portions``"""
+
+    _fields_ = [("cu", c_void_p), ("slot", c_void_p), ("pos0", c_void_p), ("row_seq", c_void_p), ("nseq", c_int32), ("rows", c_int32)]
+
+
+class LatentLayer(C.Structure):
+    """``tah_latent_layer``"""
+
+    _fields_ = [
+        ("ring", c_void_p), ("heads", c_int32), ("dim_pad", c_int32), ("rot_dim", c_int32), ("rot_pad", c_int32), ("rank", c_int32),
+        ("rank_pad", c_int32), ("vdim_pad", c_int32), ("capacity", c_int32), ("nslots", c_int32), ("dtype", c_int32),
+        ("window", c_int32), ("scale", c_float),
+    ]
+
+
+class LatentPrepArgs(C.Structure):
+    """``tah_latent_prep_args``"""
+
+    _fields_ = [
+        ("proj", c_void_p), ("proj_row_stride", c_int64), ("q_col", c_int32), ("dkv_col", c_int32), ("norm", c_void_p),
+        ("cos", c_void_p), ("sin", c_void_p), ("pos", c_void_p), ("slot", c_void_p), ("rows_out", c_void_p), ("q_packed", c_void_p),
+        ("q_rows", c_void_p), ("rows", c_int32), ("table_rows", c_int32), ("eps", c_float),
+    ]
+
+
 PROTOTYPES = {
     "tah_duo_abi_version": (C.c_int, []),
     "tah_duo_error_string": (C.c_char_p, [C.c_int]),
@@ -280,6 +343,27 @@ PROTOTYPES = {
     "tah_pad_rows_build": (C.c_int, [c_void_p, c_void_p, c_int32, c_void_p, c_int32, c_void_p, c_void_p, c_void_p]),
     "tah_rows_copy": (C.c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_int64,
                                 c_int64, c_void_p]),
+    # include/tah_mixers.h
+    "tah_embed_rows": (C.c_int, [C.POINTER(EmbedRowsArgs), c_void_p]),
+    "tah_residual_norm": (C.c_int, [C.POINTER(ResidualNormArgs), c_void_p]),
+    "tah_activate_rows": (C.c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int32, c_int32, c_int32, c_int32, c_void_p]),
+    "tah_delta_step": (C.c_int, [C.POINTER(DeltaLayer), c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int32, c_void_p]),
+    "tah_delta_prepare": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 6),
+    "tah_delta_scan": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 7),
+    "tah_delta_finish": (C.c_int, [C.POINTER(DeltaLayer), c_void_p, c_int32, c_void_p, c_int64, c_int32, c_void_p]),
+    "tah_latent_prep": (C.c_int, [C.POINTER(LatentLayer), C.POINTER(LatentPrepArgs), c_void_p]),
+    "tah_latent_context": (C.c_int, [C.POINTER(LatentLayer), C.POINTER(Portions), c_void_p, c_int32, c_void_p, c_void_p, c_void_p]),
+    "tah_latent_attend": (C.c_int, [C.POINTER(LatentLayer), C.POINTER(Portions), c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int64,
+                                    c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p]),
+    "tah_latent_decode_workspace": (C.c_size_t, [C.POINTER(LatentLayer), c_int32]),
+    "tah_latent_decode": (C.c_int, [C.POINTER(LatentLayer), c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+                                    c_void_p, c_void_p, C.c_size_t, c_void_p]),
+    "tah_moe_route": (C.c_int, [c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_int32, c_int32, c_void_p, c_void_p, c_void_p, c_int32,
+                                c_void_p]),
+    "tah_moe_places": (c_int32, [c_int32, c_int32, c_int32]),
+    "tah_moe_plan": (C.c_int, [c_void_p, c_int32, c_int32, c_int32, c_void_p, c_void_p, c_void_p, c_void_p]),
+    "tah_moe_linear": (C.c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_int32, c_int32, c_void_p, c_int64,
+                                 c_int32, c_void_p]),
 }
 
 

@@ -1,0 +1,542 @@
+// Gated delta rule, gfx950.  Per head and token, with a float32 state S [dim, vdim] per sequence:
+//     S = g S;   u = beta (v - S^T k);   S = S + k u^T;   o = S^T q.
+// Both the step and the scan use  o = g S_old^T q + (k . q) u  for the read-out: S_old^T k and S_old^T q are then
+// independent reductions of one pass over the state, and the write follows in a second pass over registers.
+//
+//  * delta_step_kernel: one token per row.  One workgroup per (row, head) holds the head's state in registers between
+//    its load and its store -- the state crosses HBM once in each direction, which is all the step costs (64 KB each
+//    way at 128 x 128) -- and does everything around it: short convolution on the projections, unit norms, decay,
+//    output norm and gate.
+//  * delta_prepare_kernel / delta_scan_kernel / delta_finish_kernel: portions of many tokens.  Columns of the state do
+//    not interact, so a head is split over workgroups of 16 columns: a wave owns 4 columns, 16 lanes share a column's
+//    rows and reduce over them with DPP row rotations; k and q of the next 16 tokens are fetched while the current 16
+//    run.  State and inputs are float32 throughout (no reduced-precision matrix instruction touches the recurrence).
+//
+// The convolution's inputs of the last `taps` tokens are kept as a ring (token p at p % taps): a step writes the entry
+// that no row of the step reads, so workgroups that share channels need no order among themselves.
+#include <hip/hip_runtime.h>
+
+#include "mixer_device.h"
+
+namespace tah {
+namespace {
+
+constexpr int kDeltaThreads = 256;
+constexpr float kUnitEps = 1e-6f;
+
+__device__ __forceinline__ int proj_col(const tah_delta_layer& L, int ch) {
+    const int qk = L.kv_heads * L.dim;
+    return ch < qk ? L.q_col + ch : (ch < 2 * qk ? L.k_col + ch - qk : L.v_col + ch - 2 * qk);
+}
+__device__ __forceinline__ float decay_log(const tah_delta_layer& L, float a, int h) {
+    return -expf(L.a_log[h]) * softplus_exact(a + L.dt_bias[h]);
+}
+
+// LDS floats of delta_step_kernel
+inline int step_lds(int dim, int vdim, int vec) { return 2 * dim + 2 * vdim + 2 * kDeltaThreads * vec + 16; }
+
+// VEC: state columns per thread (4 or 1); NR: state rows per thread kept in registers, 0: any number, read twice.
+template <class E, int VEC, int NR>
+__global__ __launch_bounds__(kDeltaThreads) void delta_step_kernel(const tah_delta_layer L, const int32_t* slots, const int32_t* poss,
+                                                                   E* out, int64_t out_rs, __bf16* out_packed, int out_cols) {
+    HIP_DYNAMIC_SHARED(float, sm)
+    float* const sq_ = sm;                     // q [dim]
+    float* const sk_ = sq_ + L.dim;            // k [dim]
+    float* const sv_ = sk_ + L.dim;            // v [vdim]
+    float* const su_ = sv_ + L.vdim;           // u [vdim]
+    float* const part = su_ + L.vdim;          // [2][row groups][columns]
+    float* const red = part + 2 * kDeltaThreads * VEC;
+    const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
+    const int slot = slots[row], pos = poss[row];
+    const int group = L.heads / L.kv_heads, kh = h / group;
+    const int ct = (L.vdim + VEC - 1) / VEC;   // threads across the columns
+    const int rg = kDeltaThreads / ct;         // row groups
+    const bool dead = slot < 0 || slot >= L.nslots || pos < 0;
+    const E* pr = static_cast<const E*>(L.proj) + (int64_t)row * L.proj_row_stride;
+    if (dead) {  // a dropped row: zeros (uniform per workgroup)
+        for (int v = tid; v < L.vdim; v += kDeltaThreads) {
+            if (out) out[row * out_rs + h * L.vdim + v] = (E)0.f;
+            if (out_packed) out_packed[rows_form_elem(row, h * L.vdim + v)] = (__bf16)0.f;
+        }
+    } else {
+        const int c0 = (tid % ct) * VEC, r0 = tid / ct;
+        const bool holder = r0 < rg;
+        float* const S = L.state + (((int64_t)slot * L.heads + h) * L.dim) * L.vdim + c0;
+        const bool fresh = pos == 0;
+        float s[NR > 0 ? NR : 1][VEC];
+        if constexpr (NR > 0) {
+#pragma unroll
+            for (int n = 0; n < NR; ++n) {
+                const int i = r0 + rg * n;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) s[n][e] = 0.f;
+                if (holder && i < L.dim && !fresh) {
+                    if constexpr (VEC == 4) {
+                        const f32x4 x = *reinterpret_cast<const f32x4*>(S + (int64_t)i * L.vdim);
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) s[n][e] = x[e];
+                    } else s[n][0] = S[(int64_t)i * L.vdim];
+                }
+            }
+        }
+        // short convolution of this head's q, k and v channels
+        const int qk = L.kv_heads * L.dim, nch = 2 * qk + L.heads * L.vdim;
+        E* const cs = static_cast<E*>(L.conv_state) + (int64_t)slot * L.taps * nch;
+        for (int i = tid; i < 2 * L.dim + L.vdim; i += kDeltaThreads) {
+            const int ch = i < L.dim ? kh * L.dim + i : (i < 2 * L.dim ? qk + kh * L.dim + i - L.dim : 2 * qk + h * L.vdim + i - 2 * L.dim);
+            const E cur = pr[proj_col(L, ch)];
+            const float* w = L.conv + (int64_t)ch * L.taps;
+            float y = w[L.taps - 1] * (float)cur;
+            for (int d = 1; d < L.taps; ++d)
+                if (pos - d >= 0) y += w[L.taps - 1 - d] * (float)cs[(int64_t)((pos - d) % L.taps) * nch + ch];
+            if (i >= 2 * L.dim || h % group == 0) cs[(int64_t)(pos % L.taps) * nch + ch] = cur;
+            sq_[i] = silu_exact(y);  // q, k and v lie one after another
+        }
+        const float g = expf(decay_log(L, (float)pr[L.a_col + h], h));
+        const float beta = sigmoid_exact((float)pr[L.b_col + h]);
+        __syncthreads();
+        float qq = 0.f, kk = 0.f, kq = 0.f;
+        for (int i = tid; i < L.dim; i += kDeltaThreads) {
+            const float q = sq_[i], k = sk_[i];
+            qq += q * q;
+            kk += k * k;
+            kq += k * q;
+        }
+        qq = wave_sum(qq);
+        kk = wave_sum(kk);
+        kq = wave_sum(kq);
+        if (tid % kWave == 0) {
+            red[tid / kWave] = qq;
+            red[4 + tid / kWave] = kk;
+            red[8 + tid / kWave] = kq;
+        }
+        // S_old^T k and S_old^T q over this thread's rows (k and q not yet unit vectors: a factor, applied below)
+        float ak[VEC], aq[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ak[e] = aq[e] = 0.f;
+        auto accumulate = [&](const float* x, int i) __attribute__((always_inline)) {
+            const float k = sk_[i], q = sq_[i];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                ak[e] += x[e] * k;
+                aq[e] += x[e] * q;
+            }
+        };
+        auto fetch = [&](int i, float* x) __attribute__((always_inline)) {
+            if constexpr (VEC == 4) {
+                const f32x4 y = *reinterpret_cast<const f32x4*>(S + (int64_t)i * L.vdim);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[e] = y[e];
+            } else x[0] = S[(int64_t)i * L.vdim];
+        };
+        if constexpr (NR > 0) {
+#pragma unroll
+            for (int n = 0; n < NR; ++n) {
+                const int i = r0 + rg * n;
+                if (i < L.dim) accumulate(s[n], i);
+            }
+        } else if (holder && !fresh) {
+            for (int i = r0; i < L.dim; i += rg) {
+                float x[VEC];
+                fetch(i, x);
+                accumulate(x, i);
+            }
+        }
+        if (holder) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                part[r0 * ct * VEC + c0 + e] = ak[e];
+                part[kDeltaThreads * VEC + r0 * ct * VEC + c0 + e] = aq[e];
+            }
+        }
+        __syncthreads();
+        qq = (red[0] + red[1]) + (red[2] + red[3]);
+        kk = (red[4] + red[5]) + (red[6] + red[7]);
+        kq = (red[8] + red[9]) + (red[10] + red[11]);
+        const float rq = 1.0f / sqrtf((float)L.dim) / sqrtf(qq + kUnitEps), rk = 1.0f / sqrtf(kk + kUnitEps);
+        kq *= rq * rk;
+        float oo = 0.f;
+        for (int v = tid; v < L.vdim; v += kDeltaThreads) {
+            float xk = 0.f, xq = 0.f;
+            for (int r = 0; r < rg; ++r) {
+                xk += part[r * ct * VEC + v];
+                xq += part[kDeltaThreads * VEC + r * ct * VEC + v];
+            }
+            const float u = beta * (sv_[v] - g * (xk * rk));
+            const float o = g * (xq * rq) + kq * u;
+            su_[v] = u;
+            sv_[v] = o;  // (each entry is read and rewritten by one thread)
+            oo += o * o;
+        }
+        __syncthreads();
+        oo = block_sum<kDeltaThreads / kWave>(oo, red);
+        auto write = [&](const float* x, int i) __attribute__((always_inline)) {
+            const float k = sk_[i] * rk;
+            float y[VEC];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) y[e] = g * x[e] + k * su_[c0 + e];
+            if constexpr (VEC == 4) *reinterpret_cast<f32x4*>(S + (int64_t)i * L.vdim) = f32x4{y[0], y[1], y[2], y[3]};
+            else S[(int64_t)i * L.vdim] = y[0];
+        };
+        if constexpr (NR > 0) {
+#pragma unroll
+            for (int n = 0; n < NR; ++n) {
+                const int i = r0 + rg * n;
+                if (holder && i < L.dim) write(s[n], i);
+            }
+        } else if (holder) {
+            for (int i = r0; i < L.dim; i += rg) {
+                float x[VEC];
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) x[e] = 0.f;
+                if (!fresh) fetch(i, x);
+                write(x, i);
+            }
+        }
+        const float r = 1.0f / sqrtf(oo / (float)L.vdim + L.eps);
+        for (int v = tid; v < L.vdim; v += kDeltaThreads) {
+            const float y = sv_[v] * r * L.norm[v] * silu_exact((float)pr[L.gate_col + h * L.vdim + v]);
+            if (out) out[row * out_rs + h * L.vdim + v] = (E)y;
+            if (out_packed) out_packed[rows_form_elem(row, h * L.vdim + v)] = (__bf16)y;
+        }
+    }
+    if (h == L.heads - 1) {
+        for (int c = L.heads * L.vdim + tid; c < out_cols; c += kDeltaThreads) {
+            if (out) out[row * out_rs + c] = (E)0.f;
+            if (out_packed) out_packed[rows_form_elem(row, c)] = (__bf16)0.f;
+        }
+    }
+}
+
+// ---- portions ------------------------------------------------------------------------------------------------
+constexpr int kPrepTokens = 16;  // tokens per wave
+
+// blockIdx.y: q heads, k heads, v heads, then one for the gates.  NCH: 64-channel pieces of a head.
+template <class E, int NCH>
+__global__ __launch_bounds__(kDeltaThreads) void delta_prepare_kernel(const tah_delta_layer L, const tah_portions P, float* q, float* k, float* v,
+                                                                      float* lg, float* beta) {
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, hs = blockIdx.y;
+    const int t0 = (blockIdx.x * (kDeltaThreads / kWave) + wave) * kPrepTokens;
+    const E* proj = static_cast<const E*>(L.proj);
+    const int qk = L.kv_heads * L.dim, nch = 2 * qk + L.heads * L.vdim;
+    if (hs == 2 * L.kv_heads + L.heads) {
+        for (int t = t0; t < t0 + kPrepTokens && t < P.rows; ++t) {
+            const E* pr = proj + (int64_t)t * L.proj_row_stride;
+            for (int h = lane; h < L.heads; h += kWave) {
+                lg[(int64_t)t * L.heads + h] = decay_log(L, (float)pr[L.a_col + h], h);
+                beta[(int64_t)t * L.heads + h] = sigmoid_exact((float)pr[L.b_col + h]);
+            }
+        }
+        return;
+    }
+    const bool is_q = hs < L.kv_heads, is_v = hs >= 2 * L.kv_heads;
+    const int d = is_v ? L.vdim : L.dim;
+    const int head = is_q ? hs : (is_v ? hs - 2 * L.kv_heads : hs - L.kv_heads);
+    const int ch0 = is_q ? head * L.dim : (is_v ? 2 * qk + head * L.vdim : qk + head * L.dim);
+    const int col0 = (is_q ? L.q_col : (is_v ? L.v_col : L.k_col)) + head * d;
+    float* const dst = is_q ? q : (is_v ? v : k);
+    const int nheads = is_v ? L.heads : L.kv_heads;
+    const float out_scale = is_q ? 1.0f / sqrtf((float)L.dim) : 1.0f;
+    for (int t = t0; t < t0 + kPrepTokens && t < P.rows; ++t) {
+        const int b = P.row_seq[t];
+        const int first = P.cu[b], pos = P.pos0[b] + t - first, slot = P.slot[b];
+        const E* cs = static_cast<const E*>(L.conv_state) + (int64_t)(slot < 0 ? 0 : slot) * L.taps * nch;
+        float y[NCH], ss = 0.f;
+#pragma unroll
+        for (int n = 0; n < NCH; ++n) {
+            const int c = lane + kWave * n;
+            y[n] = 0.f;
+            if (c < d) {
+                const float* w = L.conv + (int64_t)(ch0 + c) * L.taps;
+                for (int j = 0; j < L.taps; ++j) {
+                    float x = 0.f;
+                    if (t - j >= first) x = (float)proj[(int64_t)(t - j) * L.proj_row_stride + col0 + c];
+                    else if (pos - j >= 0 && slot >= 0) x = (float)cs[(int64_t)((pos - j) % L.taps) * nch + ch0 + c];
+                    y[n] += w[L.taps - 1 - j] * x;
+                }
+                y[n] = silu_exact(y[n]);
+            }
+            ss += y[n] * y[n];
+        }
+        float r = 1.0f;
+        if (!is_v) r = out_scale / sqrtf(wave_sum(ss) + kUnitEps);
+#pragma unroll
+        for (int n = 0; n < NCH; ++n) {
+            const int c = lane + kWave * n;
+            if (c < d) dst[((int64_t)t * nheads + head) * d + c] = y[n] * r;
+        }
+    }
+}
+
+// The convolution's inputs of a portion's last tokens, into the ring.  (After delta_prepare_kernel has read the old ones.)
+template <class E>
+__global__ __launch_bounds__(kDeltaThreads) void conv_tail_kernel(const tah_delta_layer L, const tah_portions P) {
+    const int b = blockIdx.y, slot = P.slot[b];
+    const int nch = 2 * L.kv_heads * L.dim + L.heads * L.vdim, ch = blockIdx.x * kDeltaThreads + threadIdx.x;
+    if (ch >= nch || slot < 0 || slot >= L.nslots) return;
+    const int first = P.cu[b], last = P.cu[b + 1] - 1, pos_last = P.pos0[b] + last - first;
+    E* cs = static_cast<E*>(L.conv_state) + (int64_t)slot * L.taps * nch + ch;
+    const E* src = static_cast<const E*>(L.proj) + proj_col(L, ch);
+    for (int d = 0; d < L.taps && last - d >= first; ++d) cs[(int64_t)((pos_last - d) % L.taps) * nch] = src[(int64_t)(last - d) * L.proj_row_stride];
+}
+
+constexpr int kScanTokens = 16, kScanCols = 16;
+
+// sum over the 16 lanes of a DPP row, in every lane of it
+__device__ __forceinline__ float row16_sum(float x) {
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x124, 0xf, 0xf, false));
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x122, 0xf, 0xf, false));
+    x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x121, 0xf, 0xf, false));
+    return x;
+}
+
+// grid (column blocks of 16, heads, sequences).  NB: 64-row pieces of the state; lane r of 16 holds rows 64 b + 4 r ... + 3.
+template <int NB>
+__global__ __launch_bounds__(kDeltaThreads) void delta_scan_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
+                                                                   const float* v, const float* lg, const float* beta, float* o) {
+    constexpr int kDim = 64 * NB;
+    __shared__ __align__(16) float kb[kScanTokens][kDim], qb[kScanTokens][kDim];
+    __shared__ float vb[kScanTokens][kScanCols], ob[kScanTokens][kScanCols], gb[kScanTokens], bb[kScanTokens], kqb[kScanTokens];
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int h = blockIdx.y, b = blockIdx.z, kh = h / (L.heads / L.kv_heads);
+    const int r = lane % 16, lc = wave * 4 + lane / 16, col = blockIdx.x * kScanCols + lc;
+    const int first = P.cu[b], n = P.cu[b + 1] - first, slot = P.slot[b], pos0 = P.pos0[b];
+    if (n <= 0 || slot < 0 || slot >= L.nslots) return;
+    float* const S = L.state + ((int64_t)slot * L.heads + h) * L.dim * L.vdim;
+    float s[NB][4];
+#pragma unroll
+    for (int x = 0; x < NB; ++x)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int i = 64 * x + 4 * r + e;
+            s[x][e] = (pos0 > 0 && col < L.vdim && i < L.dim) ? S[(int64_t)i * L.vdim + col] : 0.f;
+        }
+    // a thread's share of 16 tokens: NB four-row pieces of k and of q, one v, and (32 threads) a gate
+    f32x4 nk[NB], nq[NB];
+    float nv = 0.f, ng = 0.f;
+    const bool vec = L.dim % 4 == 0;
+    auto fetch = [&](int c0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int x = 0; x < NB; ++x) {
+            const int u = tid + kDeltaThreads * x, t = u / (kDim / 4), i = 4 * (u % (kDim / 4));
+            nk[x] = nq[x] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (c0 + t < n && i < L.dim) {
+                const int64_t at = ((int64_t)(first + c0 + t) * L.kv_heads + kh) * L.dim + i;
+                if (vec) {
+                    nk[x] = *reinterpret_cast<const f32x4*>(k + at);
+                    nq[x] = *reinterpret_cast<const f32x4*>(q + at);
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (i + e < L.dim) {
+                            nk[x][e] = k[at + e];
+                            nq[x][e] = q[at + e];
+                        }
+                }
+            }
+        }
+        const int t = tid / kScanCols, c = blockIdx.x * kScanCols + tid % kScanCols;
+        nv = (c0 + t < n && c < L.vdim) ? v[((int64_t)(first + c0 + t) * L.heads + h) * L.vdim + c] : 0.f;
+        if (tid < 2 * kScanTokens) {
+            const int tt = tid % kScanTokens;
+            ng = c0 + tt < n ? (tid < kScanTokens ? lg : beta)[(int64_t)(first + c0 + tt) * L.heads + h] : 0.f;
+        }
+    };
+    fetch(0);
+    for (int c0 = 0; c0 < n; c0 += kScanTokens) {
+#pragma unroll
+        for (int x = 0; x < NB; ++x) {
+            const int u = tid + kDeltaThreads * x, t = u / (kDim / 4), i = 4 * (u % (kDim / 4));
+            *reinterpret_cast<f32x4*>(&kb[t][i]) = nk[x];
+            *reinterpret_cast<f32x4*>(&qb[t][i]) = nq[x];
+        }
+        vb[tid / kScanCols][tid % kScanCols] = nv;
+        if (tid < kScanTokens) gb[tid] = expf(ng);
+        else if (tid < 2 * kScanTokens) bb[tid - kScanTokens] = ng;
+        __syncthreads();
+        if (c0 + kScanTokens < n) fetch(c0 + kScanTokens);
+        {   // k . q of four tokens per wave, sixteen lanes each
+            const int t = wave * 4 + lane / 16;
+            float x = 0.f;
+#pragma unroll
+            for (int e = 0; e < kDim / 64; ++e) {
+                const f32x4 a = *reinterpret_cast<const f32x4*>(&kb[t][64 * e + 4 * r]), c = *reinterpret_cast<const f32x4*>(&qb[t][64 * e + 4 * r]);
+                x += (a[0] * c[0] + a[1] * c[1]) + (a[2] * c[2] + a[3] * c[3]);
+            }
+            x = row16_sum(x);
+            if (r == 0) kqb[t] = x;
+        }
+        __syncthreads();
+        const int m = n - c0 < kScanTokens ? n - c0 : kScanTokens;
+        for (int t = 0; t < m; ++t) {
+            f32x4 kt[NB];
+            float xk = 0.f, xq = 0.f;
+#pragma unroll
+            for (int x = 0; x < NB; ++x) {
+                kt[x] = *reinterpret_cast<const f32x4*>(&kb[t][64 * x + 4 * r]);
+                const f32x4 qt = *reinterpret_cast<const f32x4*>(&qb[t][64 * x + 4 * r]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    xk += s[x][e] * kt[x][e];
+                    xq += s[x][e] * qt[e];
+                }
+            }
+            xk = row16_sum(xk);
+            xq = row16_sum(xq);
+            const float g = gb[t];
+            const float u = bb[t] * (vb[t][lc] - g * xk);
+            if (r == 0) ob[t][lc] = g * xq + kqb[t] * u;
+#pragma unroll
+            for (int x = 0; x < NB; ++x)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) s[x][e] = g * s[x][e] + kt[x][e] * u;
+        }
+        __syncthreads();
+        {
+            const int t = tid / kScanCols, c = blockIdx.x * kScanCols + tid % kScanCols;
+            if (t < m && c < L.vdim) o[((int64_t)(first + c0 + t) * L.heads + h) * L.vdim + c] = ob[t][tid % kScanCols];
+        }
+    }
+#pragma unroll
+    for (int x = 0; x < NB; ++x)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int i = 64 * x + 4 * r + e;
+            if (col < L.vdim && i < L.dim) S[(int64_t)i * L.vdim + col] = s[x][e];
+        }
+}
+
+// one wave per (row, head)
+template <class E>
+__global__ __launch_bounds__(kDeltaThreads) void delta_finish_kernel(const tah_delta_layer L, const float* o, int64_t items, E* out, int64_t out_rs,
+                                                                     int out_cols) {
+    const int lane = threadIdx.x % kWave;
+    const int64_t it = (int64_t)blockIdx.x * (kDeltaThreads / kWave) + threadIdx.x / kWave;
+    if (it >= items) return;
+    const int64_t row = it / L.heads;
+    const int h = (int)(it % L.heads);
+    const float* x = o + it * L.vdim;
+    float ss = 0.f;
+    for (int v = lane; v < L.vdim; v += kWave) ss += x[v] * x[v];
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)L.vdim + L.eps);
+    const E* gate = static_cast<const E*>(L.proj) + row * L.proj_row_stride + L.gate_col + h * L.vdim;
+    E* y = out + row * out_rs;
+    for (int v = lane; v < L.vdim; v += kWave) y[h * L.vdim + v] = (E)(x[v] * r * L.norm[v] * silu_exact((float)gate[v]));
+    if (h == L.heads - 1)
+        for (int c = L.heads * L.vdim + lane; c < out_cols; c += kWave) y[c] = (E)0.f;
+}
+
+int check_layer(const tah_delta_layer* L) {
+    if (!L) return TAH_E_NULL;
+    if (L->heads <= 0 || L->kv_heads <= 0 || L->heads % L->kv_heads != 0 || L->dim <= 0 || L->vdim <= 0 || L->taps <= 0 || L->nslots <= 0 ||
+        (L->dtype != TAH_DT_BF16 && L->dtype != TAH_DT_F32) || L->heads > 65535)
+        return TAH_E_SHAPE;
+    if (L->dim > 256 || L->vdim > 512) return TAH_E_SHAPE;
+    if (!L->proj || !L->conv || !L->a_log || !L->dt_bias || !L->norm || !L->conv_state || !L->state) return TAH_E_NULL;
+    if (!aligned_16(L->state)) return TAH_E_ALIGN;
+    return TAH_OK;
+}
+int check_portions(const tah_portions* p) {
+    if (!p) return TAH_E_NULL;
+    if (p->nseq < 0 || p->rows < 0 || p->nseq > 65535) return TAH_E_SHAPE;
+    if (p->nseq > 0 && p->rows > 0 && (!p->cu || !p->slot || !p->pos0 || !p->row_seq)) return TAH_E_NULL;
+    return TAH_OK;
+}
+
+template <class E, int VEC, int NR>
+void launch_step(const tah_delta_layer& L, const int32_t* slot, const int32_t* pos, int rows, void* out, int64_t rs, void* packed, int cols,
+                 hipStream_t st) {
+    hipLaunchKernelGGL((delta_step_kernel<E, VEC, NR>), dim3(L.heads, rows), dim3(kDeltaThreads), step_lds(L.dim, L.vdim, VEC) * sizeof(float), st,
+                       L, slot, pos, static_cast<E*>(out), rs, static_cast<__bf16*>(packed), cols);
+}
+template <class E>
+void dispatch_step(const tah_delta_layer& L, const int32_t* slot, const int32_t* pos, int rows, void* out, int64_t rs, void* packed, int cols,
+                   hipStream_t st) {
+    if (L.vdim % 4 == 0) {
+        const int rg = kDeltaThreads / (L.vdim / 4), nr = (L.dim + rg - 1) / rg;
+        if (nr <= 4) launch_step<E, 4, 4>(L, slot, pos, rows, out, rs, packed, cols, st);
+        else if (nr <= 8) launch_step<E, 4, 8>(L, slot, pos, rows, out, rs, packed, cols, st);
+        else if (nr <= 16) launch_step<E, 4, 16>(L, slot, pos, rows, out, rs, packed, cols, st);
+        else launch_step<E, 4, 0>(L, slot, pos, rows, out, rs, packed, cols, st);
+    } else {
+        launch_step<E, 1, 0>(L, slot, pos, rows, out, rs, packed, cols, st);
+    }
+}
+template <class E>
+void launch_prepare(const tah_delta_layer& L, const tah_portions& P, float* q, float* k, float* v, float* lg, float* beta, hipStream_t st) {
+    constexpr int per_block = kPrepTokens * (kDeltaThreads / kWave);
+    const dim3 grid((P.rows + per_block - 1) / per_block, 2 * L.kv_heads + L.heads + 1);
+    const int d = L.dim > L.vdim ? L.dim : L.vdim;
+    if (d <= 64) hipLaunchKernelGGL((delta_prepare_kernel<E, 1>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+    else if (d <= 128) hipLaunchKernelGGL((delta_prepare_kernel<E, 2>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+    else if (d <= 256) hipLaunchKernelGGL((delta_prepare_kernel<E, 4>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+    else hipLaunchKernelGGL((delta_prepare_kernel<E, 8>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+    const int nch = 2 * L.kv_heads * L.dim + L.heads * L.vdim;
+    hipLaunchKernelGGL((conv_tail_kernel<E>), dim3((nch + kDeltaThreads - 1) / kDeltaThreads, P.nseq), dim3(kDeltaThreads), 0, st, L, P);
+}
+
+}  // namespace
+}  // namespace tah
+
+extern "C" int tah_delta_step(const tah_delta_layer* L, const int32_t* slot, const int32_t* pos, int32_t rows, void* out, int64_t out_rs,
+                              void* out_packed, int32_t out_cols, tah_stream_t stream) {
+    using namespace tah;
+    if (const int rc = check_layer(L)) return rc;
+    if (rows < 0 || rows > 65535 || out_cols < L->heads * L->vdim || (out && rows > 1 && out_rs < out_cols)) return TAH_E_SHAPE;
+    if (out_packed && (rows > 32 || out_cols % 32 != 0)) return TAH_E_SHAPE;
+    if (L->vdim % 4 != 0 && L->vdim > kDeltaThreads) return TAH_E_SHAPE;
+    if (rows == 0) return TAH_OK;
+    if (!slot || !pos || (!out && !out_packed)) return TAH_E_NULL;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (L->dtype == TAH_DT_BF16) dispatch_step<__bf16>(*L, slot, pos, rows, out, out_rs, out_packed, out_cols, st);
+    else dispatch_step<float>(*L, slot, pos, rows, out, out_rs, out_packed, out_cols, st);
+    return launch_status();
+}
+
+extern "C" int tah_delta_prepare(const tah_delta_layer* L, const tah_portions* p, float* q, float* k, float* v, float* lg, float* beta,
+                                 tah_stream_t stream) {
+    using namespace tah;
+    if (const int rc = check_layer(L)) return rc;
+    if (const int rc = check_portions(p)) return rc;
+    if (2 * L->kv_heads + L->heads + 1 > 65535) return TAH_E_SHAPE;
+    if (p->rows == 0 || p->nseq == 0) return TAH_OK;
+    if (!q || !k || !v || !lg || !beta) return TAH_E_NULL;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (L->dtype == TAH_DT_BF16) launch_prepare<__bf16>(*L, *p, q, k, v, lg, beta, st);
+    else launch_prepare<float>(*L, *p, q, k, v, lg, beta, st);
+    return launch_status();
+}
+
+extern "C" int tah_delta_scan(const tah_delta_layer* L, const tah_portions* p, const float* q, const float* k, const float* v, const float* lg,
+                              const float* beta, float* o, tah_stream_t stream) {
+    using namespace tah;
+    if (const int rc = check_layer(L)) return rc;
+    if (const int rc = check_portions(p)) return rc;
+    if (p->rows == 0 || p->nseq == 0) return TAH_OK;
+    if (!q || !k || !v || !lg || !beta || !o) return TAH_E_NULL;
+    if (!aligned_16(q) || !aligned_16(k)) return TAH_E_ALIGN;
+    const dim3 grid((L->vdim + kScanCols - 1) / kScanCols, L->heads, p->nseq);
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (L->dim <= 64) hipLaunchKernelGGL((delta_scan_kernel<1>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);
+    else if (L->dim <= 128) hipLaunchKernelGGL((delta_scan_kernel<2>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);
+    else hipLaunchKernelGGL((delta_scan_kernel<4>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);
+    return launch_status();
+}
+
+extern "C" int tah_delta_finish(const tah_delta_layer* L, const float* o, int32_t rows, void* out, int64_t out_rs, int32_t out_cols,
+                                tah_stream_t stream) {
+    using namespace tah;
+    if (const int rc = check_layer(L)) return rc;
+    if (rows < 0 || out_cols < L->heads * L->vdim || (rows > 1 && out_rs < out_cols)) return TAH_E_SHAPE;
+    if (rows == 0) return TAH_OK;
+    if (!o || !out) return TAH_E_NULL;
+    const int64_t items = (int64_t)rows * L->heads;
+    const dim3 grid((unsigned)((items + kDeltaThreads / kWave - 1) / (kDeltaThreads / kWave)));
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (L->dtype == TAH_DT_BF16)
+        hipLaunchKernelGGL((delta_finish_kernel<__bf16>), grid, dim3(kDeltaThreads), 0, st, *L, o, items, static_cast<__bf16*>(out), out_rs, out_cols);
+    else
+        hipLaunchKernelGGL((delta_finish_kernel<float>), grid, dim3(kDeltaThreads), 0, st, *L, o, items, static_cast<float*>(out), out_rs, out_cols);
+    return launch_status();
+}

@@ -59,6 +59,11 @@ struct LinParams {
     float eps;
     int32_t norm;
     int32_t groups;  // column groups (workgroups per row half)
+    // products of the same sizes in one launch (grid.y): operands `batch index * stride` elements further on
+    int64_t w_bs, x_bs, y_bs, yp_bs;
+    int32_t yp_col_step;    // columns a product's packed result is moved by (results side by side in one rows form)
+    const int32_t* select;  // run only products whose index is listed here, or null
+    int32_t n_select;
 };
 
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
@@ -83,6 +88,14 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
     __shared__ float ssum[EPI == kPlainLayerNorm ? kLinWaves : 1][16 * NH];
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
     const int c = lane % 16, kg = lane / 16;
+    const int batch = blockIdx.y;
+    if (p.select) {  // (every wave looks for itself: the answer is the same in all of them)
+        bool hit = false;
+        for (int i = lane; i < p.n_select; i += kWave) hit |= p.select[i] == batch;
+        if (__ballot(hit) == 0) return;
+    }
+    const bf16x8* const pw = p.w + batch * (p.w_bs / 8);
+    const bf16x8* const px = p.x + batch * (p.x_bs / 8);
     int group = blockIdx.x, half = 0;
     if (NH == 1 && (int)gridDim.x == 2 * p.groups) {
         if (p.groups % 8 == 0) {  // workgroups go to the XCDs round robin: i and i + 8 share one
@@ -104,8 +117,8 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
         const int en0 = group * NC * kTileCols + 8 * (writer ? (int)threadIdx.x % kEpiUnits : 0);
         const bool live_row = erow < p.rows;
         // (addresses picked by selects, so that no load sits under a branch)
-        const __bf16* ra = (p.res && live_row) ? p.res + (int64_t)erow * p.res_rs + en0 : reinterpret_cast<const __bf16*>(p.x);
-        const __bf16* ba = p.bias ? p.bias + en0 : reinterpret_cast<const __bf16*>(p.x);
+        const __bf16* ra = (p.res && live_row) ? p.res + (int64_t)erow * p.res_rs + en0 : reinterpret_cast<const __bf16*>(px);
+        const __bf16* ba = p.bias ? p.bias + en0 : reinterpret_cast<const __bf16*>(px);
         res_early = *reinterpret_cast<const bf16x8*>(ra);
         bias_early = *reinterpret_cast<const bf16x8*>(ba);
     }
@@ -116,8 +129,8 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
     const int s0 = nst > 0 ? wave * per_wave : 0;  // a wave without steps still points at valid memory
     const bf16x8* wb[NC];
 #pragma unroll
-    for (int t = 0; t < NC; ++t) wb[t] = p.w + ((int64_t)(group * NC + t) * steps + s0) * 64 + lane;
-    const bf16x8* xb = p.x + (int64_t)s0 * 128 + 64 * half + lane;
+    for (int t = 0; t < NC; ++t) wb[t] = pw + ((int64_t)(group * NC + t) * steps + s0) * 64 + lane;
+    const bf16x8* xb = px + (int64_t)s0 * 128 + 64 * half + lane;
 
     struct Buf {
         bf16x8 w[CH][NC], x[CH][NH];
@@ -325,13 +338,21 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
                     const float v = (float)out[i];
                     out[i] = (__bf16)(0.5f * v * (1.0f + erff(v * 0.70710678118654752f)));
                 }
+            } else if (p.act == TAH_ACT_GELU_TANH) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    const float v = (float)out[i];
+                    out[i] = (__bf16)(0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v))));
+                }
             }
         }
-        if (p.y) *reinterpret_cast<bf16x8*>(p.y + (int64_t)row * p.y_rs + n0) = out;
+        if (p.y) *reinterpret_cast<bf16x8*>(p.y + batch * p.y_bs + (int64_t)row * p.y_rs + n0) = out;
     }
     if (p.yp) {
-        p.yp[packed_rows_unit(row, n0)] = out;  // rows past the last one stay zero for the next layer
-        if (NH == 1 && (int)gridDim.x == p.groups) p.yp[packed_rows_unit(16 + lrow, n0)] = zero8;  // nobody computes the second half
+        bf16x8* const yp = p.yp + batch * (p.yp_bs / 8);
+        const int nc = n0 + batch * p.yp_col_step;
+        yp[packed_rows_unit(row, nc)] = out;  // rows past the last one stay zero for the next layer
+        if (NH == 1 && (int)gridDim.x == p.groups) yp[packed_rows_unit(16 + lrow, nc)] = zero8;  // nobody computes the second half
     }
 }
 
@@ -378,14 +399,14 @@ constexpr int kSplitRowsBelowGroups = 129;
 constexpr int kWideFromCols = 16384;  // plain layers from this many output columns on take 32 columns per workgroup
 
 template <int NC, int CH, int EPI, int PW>
-void launch(LinParams& p, int groups, hipStream_t st) {
+void launch(LinParams& p, int groups, int batch, hipStream_t st) {
     p.groups = groups;
     if (p.rows <= 16)
-        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(groups), dim3(kLinThreads), 0, st, p);
+        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(groups, batch), dim3(kLinThreads), 0, st, p);
     else if (groups < kSplitRowsBelowGroups)
-        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(2 * groups), dim3(kLinThreads), 0, st, p);
+        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(2 * groups, batch), dim3(kLinThreads), 0, st, p);
     else
-        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 2>), dim3(groups), dim3(kLinThreads), 0, st, p);
+        hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 2>), dim3(groups, batch), dim3(kLinThreads), 0, st, p);
 }
 
 }  // namespace
@@ -428,11 +449,19 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
     const bool gate_up = a->kind == TAH_LINEAR_GATE_UP;
     const bool g24 = gate_up && a->n % kGroup24 == 0;
     if (!g24 && a->n % kTileCols != 0) return TAH_E_SHAPE;
-    if (a->activation != TAH_ACT_NONE && a->activation != TAH_ACT_RELU && a->activation != TAH_ACT_GELU) return TAH_E_SHAPE;
+    if (a->activation != TAH_ACT_NONE && a->activation != TAH_ACT_RELU && a->activation != TAH_ACT_GELU &&
+        a->activation != TAH_ACT_GELU_TANH)
+        return TAH_E_SHAPE;
     if (a->input_norm != TAH_NORM_NONE && a->input_norm != TAH_NORM_RMS && a->input_norm != TAH_NORM_LAYER) return TAH_E_SHAPE;
     if (gate_up && (a->residual || a->bias || a->activation != TAH_ACT_NONE || a->input_norm == TAH_NORM_LAYER)) return TAH_E_SHAPE;
     if (a->input_norm == TAH_NORM_LAYER && !a->ln_colsum && a->n > 0 && a->k > 0) return TAH_E_NULL;
-    if (a->out_packed && a->n % kStepK != 0) return TAH_E_SHAPE;  // the packed rows form holds whole steps of 32 columns
+    const int batch = a->batch > 1 ? a->batch : 1;
+    if (a->batch < 0 || a->batch > 65535 || a->n_select < 0) return TAH_E_SHAPE;
+    if (batch > 1 && (a->residual || a->bias || a->input_norm != TAH_NORM_NONE)) return TAH_E_SHAPE;
+    // the packed rows form holds whole steps of 32 columns: a result of its own, or all results side by side
+    if (a->out_packed && (a->out_packed_col_step ? a->out_packed_col_step % 8 != 0 || a->out_packed_col_step < a->n : a->n % kStepK != 0))
+        return TAH_E_SHAPE;
+    if ((a->w_batch_stride | a->x_batch_stride | a->out_batch_stride | a->out_packed_batch_stride) % 8 != 0) return TAH_E_ALIGN;
     if (a->n == 0 || a->k == 0 || (a->rows == 0 && !a->out_packed)) return TAH_OK;
     if (!a->w_packed || !a->x_packed || (!a->out && !a->out_packed)) return TAH_E_NULL;
     if (!aligned16(a->w_packed) || !aligned16(a->x_packed) || !aligned16(a->out) || !aligned16(a->out_packed) || !aligned16(a->residual) ||
@@ -456,6 +485,10 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
     p.k = a->k;
     p.eps = a->norm_eps;
     p.norm = a->input_norm;
+    p.w_bs = a->w_batch_stride; p.x_bs = a->x_batch_stride; p.y_bs = a->out_batch_stride; p.yp_bs = a->out_packed_batch_stride;
+    p.yp_col_step = a->out_packed_col_step;
+    p.select = a->n_select > 0 ? a->batch_select : nullptr;
+    p.n_select = a->n_select;
     hipStream_t st = static_cast<hipStream_t>(stream);
     const int steps = a->k / kStepK;
     const int pw = steps % kLinWaves == 0 ? steps / kLinWaves : 0;  // compile-time K for the sizes of the end-to-end model
@@ -463,30 +496,30 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
         // an output head: two tiles per workgroup, the rows' operand is read half as often
         const int groups = a->n / (2 * kTileCols);
         if (p.norm) {
-            if (pw == 8) launch<2, 2, kPlainNorm, 8>(p, groups, st);
-            else launch<2, 2, kPlainNorm, 0>(p, groups, st);
+            if (pw == 8) launch<2, 2, kPlainNorm, 8>(p, groups, batch, st);
+            else launch<2, 2, kPlainNorm, 0>(p, groups, batch, st);
         } else {
-            if (pw == 8) launch<2, 2, kPlain, 8>(p, groups, st);
-            else launch<2, 2, kPlain, 0>(p, groups, st);
+            if (pw == 8) launch<2, 2, kPlain, 8>(p, groups, batch, st);
+            else launch<2, 2, kPlain, 0>(p, groups, batch, st);
         }
     } else if (!gate_up && a->input_norm == TAH_NORM_LAYER) {
-        launch<1, 4, kPlainLayerNorm, 0>(p, a->n / kTileCols, st);
+        launch<1, 4, kPlainLayerNorm, 0>(p, a->n / kTileCols, batch, st);
     } else if (!gate_up) {
         const int groups = a->n / kTileCols;
         if (p.norm) {
-            if (pw == 8) launch<1, 8, kPlainNorm, 8>(p, groups, st);
-            else launch<1, 4, kPlainNorm, 0>(p, groups, st);
-        } else if (pw == 8) launch<1, 8, kPlain, 8>(p, groups, st);
-        else if (pw == 24) launch<1, 8, kPlain, 24>(p, groups, st);
-        else launch<1, 4, kPlain, 0>(p, groups, st);
+            if (pw == 8) launch<1, 8, kPlainNorm, 8>(p, groups, batch, st);
+            else launch<1, 4, kPlainNorm, 0>(p, groups, batch, st);
+        } else if (pw == 8) launch<1, 8, kPlain, 8>(p, groups, batch, st);
+        else if (pw == 24) launch<1, 8, kPlain, 24>(p, groups, batch, st);
+        else launch<1, 4, kPlain, 0>(p, groups, batch, st);
     } else if (g24) {
         const int groups = a->n / kGroup24;
-        if (pw == 8) launch<3, 4, kGateUp24, 8>(p, groups, st);
-        else launch<3, 2, kGateUp24, 0>(p, groups, st);
+        if (pw == 8) launch<3, 4, kGateUp24, 8>(p, groups, batch, st);
+        else launch<3, 2, kGateUp24, 0>(p, groups, batch, st);
     } else {
         const int groups = a->n / kTileCols;
-        if (pw == 8) launch<2, 4, kGateUp16, 8>(p, groups, st);
-        else launch<2, 2, kGateUp16, 0>(p, groups, st);
+        if (pw == 8) launch<2, 4, kGateUp16, 8>(p, groups, batch, st);
+        else launch<2, 2, kGateUp16, 0>(p, groups, batch, st);
     }
     return hipGetLastError() == hipSuccess ? TAH_OK : TAH_E_LAUNCH;
 }

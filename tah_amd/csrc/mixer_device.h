@@ -1,0 +1,75 @@
+// Device-side helpers of the layer mechanisms in row_norm.hip, delta_rule.hip, latent_attn.hip and moe.hip.
+#pragma once
+#include "duo_device.h"
+#include "tah_mixers.h"
+
+namespace tah {
+
+// Eight elements of a row as float32.
+__device__ __forceinline__ void load8(const __bf16* p, float (&v)[8]) {
+    const bf16x8 x = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = (float)x[i];
+}
+__device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        v[i] = a[i];
+        v[4 + i] = b[i];
+    }
+}
+__device__ __forceinline__ bf16x8 to_bf16x8(const float (&v)[8]) {
+    bf16x8 x;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = (__bf16)v[i];
+    return x;
+}
+__device__ __forceinline__ void store8(__bf16* p, const float (&v)[8]) { *reinterpret_cast<bf16x8*>(p) = to_bf16x8(v); }
+__device__ __forceinline__ void store8(float* p, const float (&v)[8]) {
+    *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+    *reinterpret_cast<f32x4*>(p + 4) = f32x4{v[4], v[5], v[6], v[7]};
+}
+
+// 16-byte unit of the rows form of tah_linear_rows that holds row r, columns c ... c + 7 (c % 8 == 0)
+__device__ __host__ __forceinline__ int64_t rows_form_unit(int r, int c) {
+    return ((int64_t)(c / 32) * 2 + r / 16) * 64 + (r % 16) + 16 * ((c % 32) / 8);
+}
+// element of it
+__device__ __host__ __forceinline__ int64_t rows_form_elem(int r, int c) { return rows_form_unit(r, c) * 8 + c % 8; }
+
+__device__ __forceinline__ float wave_sum(float x) {
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) x += __shfl_xor(x, m);
+    return x;
+}
+__device__ __forceinline__ float wave_max(float x) {
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) x = fmaxf(x, __shfl_xor(x, m));
+    return x;
+}
+// Sum over a workgroup of kWaves waves; `red` is LDS of kWaves floats that nobody else is using.
+template <int kWaves>
+__device__ __forceinline__ float block_sum(float x, float* red) {
+    x = wave_sum(x);
+    if (threadIdx.x % kWave == 0) red[threadIdx.x / kWave] = x;
+    __syncthreads();
+    float s = 0.f;
+#pragma unroll
+    for (int w = 0; w < kWaves; ++w) s += red[w];
+    __syncthreads();
+    return s;
+}
+
+// Accurate forms: what enters a recurrence, a norm or a router is float32 to the last bits.
+__device__ __forceinline__ float sigmoid_exact(float x) { return 1.0f / (1.0f + expf(-x)); }
+__device__ __forceinline__ float silu_exact(float x) { return x / (1.0f + expf(-x)); }
+__device__ __forceinline__ float softplus_exact(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+__device__ __forceinline__ float gelu_tanh_exact(float x) {
+    return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+}
+
+inline bool aligned_16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+inline int launch_status() { return hipGetLastError() == hipSuccess ? TAH_OK : TAH_E_LAUNCH; }
+
+}  // namespace tah

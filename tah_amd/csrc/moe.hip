@@ -1,0 +1,365 @@
+// Mixture of experts, gfx950: router, plan of the rows by expert, and the product of sorted rows with their experts'
+// weights.  (A decode step of at most 32 rows does not sort: its experts run as batched tah_linear_rows calls, every
+// expert that some row chose over all rows.)
+//
+//  * moe_route_kernel: router logits in float32 from the float32 rows, the largest ones and their softmax; RB rows per
+//    workgroup share the router's weights.
+//  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
+//  * moe_tile_kernel: bf16 tiles of 128 places x 128 weight rows on the matrix cores, both operands staged through LDS
+//    by asynchronous copies, two stages; gate and up rows of the same columns share a wave, which applies the gate.
+//  * moe_plain_kernel: the same product in float32 arithmetic (the float32 form of a model).
+#include <hip/hip_runtime.h>
+
+#include "mixer_device.h"
+
+namespace tah {
+namespace {
+
+constexpr int kMoeThreads = 256;
+constexpr int kMoeWaves = kMoeThreads / kWave;
+constexpr int kMaxExperts = 1024;
+constexpr int kMaxTop = 64;
+constexpr int kTile = TAH_MOE_TILE;
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+// LDS: rows [RB][cols] float32, logits [RB][experts + 1]
+template <class E, int RB>
+__global__ __launch_bounds__(kMoeThreads) void moe_route_kernel(const float* x, const E* router, const E* gate_w, int rows, int cols, int experts,
+                                                                int top, int32_t* index, float* weight, float* shared_gate) {
+    HIP_DYNAMIC_SHARED(float, sm)
+    float* const xs = sm;
+    float* const z = sm + RB * cols;
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, row0 = blockIdx.x * RB;
+    const int zs = experts + 1;
+    for (int i = 4 * tid; i < RB * cols; i += 4 * kMoeThreads) {
+        const int r = row0 + i / cols;
+        *reinterpret_cast<f32x4*>(xs + i) = r < rows ? *reinterpret_cast<const f32x4*>(x + (int64_t)r * cols + i % cols) : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    __syncthreads();
+    for (int e = wave; e < experts + (gate_w ? 1 : 0); e += kMoeWaves) {
+        const E* w = e < experts ? router + (int64_t)e * cols : gate_w;
+        float s[RB];
+#pragma unroll
+        for (int r = 0; r < RB; ++r) s[r] = 0.f;
+        for (int c = 8 * lane; c < cols; c += 8 * kWave) {
+            float v[8];
+            load8(w + c, v);
+#pragma unroll
+            for (int r = 0; r < RB; ++r) {
+                float y[8];
+                load8(xs + r * cols + c, y);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) s[r] += v[i] * y[i];
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < RB; ++r) {
+            const float t = wave_sum(s[r]);
+            if (lane == 0) z[r * zs + e] = t;
+        }
+    }
+    __syncthreads();
+    for (int r = wave; r < RB; r += kMoeWaves) {
+        const int row = row0 + r;
+        if (row >= rows) break;
+        float* const zr = z + r * zs;
+        if (gate_w && lane == 0) shared_gate[row] = sigmoid_exact(zr[experts]);
+        // the largest logits one after another, the lower index among equals; a chosen one leaves the race
+        float mine = kNegInf, first = 0.f;
+        int my_index = 0;
+        for (int j = 0; j < top; ++j) {
+            float bv = kNegInf;
+            int bi = 0x7fffffff;
+            for (int e = lane; e < experts; e += kWave) {
+                const float v = zr[e];
+                if (v > bv) { bv = v; bi = e; }
+            }
+#pragma unroll
+            for (int m = 32; m >= 1; m >>= 1) {
+                const float ov = __shfl_xor(bv, m);
+                const int oi = __shfl_xor(bi, m);
+                if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+            }
+            if (bi >= experts) bi = j;  // (only when the logits are not numbers)
+            if (j == 0) first = bv;
+            if (lane == j) { mine = bv; my_index = bi; }
+            if (lane == 0) zr[bi] = kNegInf;
+            TAH_WAVE_LDS_SYNC();
+        }
+        const float p = lane < top ? expf(mine - first) : 0.f;
+        const float sum = wave_sum(p);
+        if (lane < top) {
+            index[(int64_t)row * top + lane] = my_index;
+            weight[(int64_t)row * top + lane] = p / sum;
+        }
+    }
+}
+
+constexpr int kPlanThreads = 1024;
+
+__global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(const int32_t* index, int pairs, int top, int experts, int tiles, int32_t* source,
+                                                                int32_t* tile_expert, int32_t* place) {
+    __shared__ int32_t count[kMaxExperts], cursor[kMaxExperts], scan[2][kPlanThreads];
+    const int tid = threadIdx.x;
+    count[tid] = 0;
+    __syncthreads();
+    for (int i = tid; i < pairs; i += kPlanThreads) atomicAdd(&count[index[i]], 1);
+    __syncthreads();
+    const int n = count[tid], mine = (n + kTile - 1) / kTile;
+    int from = 0;
+    scan[0][tid] = mine;
+    __syncthreads();
+    for (int d = 1; d < kPlanThreads; d <<= 1) {
+        scan[from ^ 1][tid] = scan[from][tid] + (tid >= d ? scan[from][tid - d] : 0);
+        from ^= 1;
+        __syncthreads();
+    }
+    const int t0 = scan[from][tid] - mine, used = scan[from][kPlanThreads - 1];
+    cursor[tid] = t0 * kTile;
+    for (int t = 0; t < mine; ++t) tile_expert[t0 + t] = tid;
+    for (int i = n; i < mine * kTile; ++i) source[t0 * kTile + i] = -1;
+    for (int t = used + tid; t < tiles; t += kPlanThreads) tile_expert[t] = -1;
+    __syncthreads();
+    for (int i = tid; i < pairs; i += kPlanThreads) {
+        const int at = atomicAdd(&cursor[index[i]], 1);
+        source[at] = i / top;
+        place[i] = at;
+    }
+}
+
+struct MoeGemm {
+    const void* x;
+    const void* w;
+    const int32_t *source, *tile_expert;
+    void* out;
+    int64_t x_rs, out_rs;
+    int32_t n, k;
+};
+
+// ---- bf16 tiles ------------------------------------------------------------------------------------------------
+constexpr int kStageK = 64;
+constexpr int kStageBytes = 2 * kTile * kStageK * 2;  // both operands of one stage: 128 x 64 bf16 each
+
+// Four waves, 2 x 2: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
+template <bool GATE>
+__global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) {
+    HIP_DYNAMIC_SHARED(unsigned char, lds)
+    const int expert = p.tile_expert[blockIdx.y];
+    if (expert < 0) return;
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 2, wn = wave % 2;
+    const __bf16* const x = static_cast<const __bf16*>(p.x);
+    const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
+    constexpr int kCols = GATE ? kTile / 2 : kTile;  // output columns of a tile
+    const int n0 = blockIdx.x * kCols;
+    // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
+    // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
+    const __bf16 *ga[4], *gb[4];
+    int chunk[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int r = 8 * (4 * wave + i) + lane / 8;
+        chunk[i] = (lane % 8) ^ ((r >> 1) & 7);
+        int src = GATE ? p.source[blockIdx.y * kTile + r] : blockIdx.y * kTile + r;
+        src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
+        ga[i] = x + (int64_t)src * p.x_rs;
+        int wr;
+        if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
+            int c = n0 + 32 * (r / 64) + r % 32;
+            c = c < p.n ? c : p.n - 1;
+            wr = (r / 32) % 2 ? p.n + c : c;
+        } else {
+            wr = n0 + r < p.n ? n0 + r : p.n - 1;
+        }
+        gb[i] = w + (int64_t)wr * p.k;
+    }
+    auto stage = [&](int s, int k0) __attribute__((always_inline)) {
+        unsigned char* const base = lds + s * kStageBytes;
+        const int valid = (p.k - k0) / 8;  // chunks of this stage inside the rows
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int c = chunk[i] < valid ? chunk[i] : 0;
+            async_copy_16B(ga[i] + k0 + 8 * c, base + (4 * wave + i) * 1024);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int c = chunk[i] < valid ? chunk[i] : 0;
+            async_copy_16B(gb[i] + k0 + 8 * c, base + kTile * kStageK * 2 + (4 * wave + i) * 1024);
+        }
+    };
+    f32x4 acc[4][4];  // [weight tile][place tile]
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int stages = (p.k + kStageK - 1) / kStageK;
+    stage(0, 0);
+    TAH_WAIT_VMEM();
+    __syncthreads();
+    for (int s = 0; s < stages; ++s) {
+        if (s + 1 < stages) stage((s + 1) & 1, (s + 1) * kStageK);
+        const unsigned char* const a = lds + (s & 1) * kStageBytes;
+        const unsigned char* const b = a + kTile * kStageK * 2;
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            if (s * kStageK + 32 * h >= p.k) break;  // (uniform)
+            bf16x8 fx[4], fw[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor64_off(64 * wm + 16 * j + lane % 16, 4 * h + lane / 16));
+                fw[j] = *reinterpret_cast<const bf16x8*>(b + rowmajor64_off(64 * wn + 16 * j + lane % 16, 4 * h + lane / 16));
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
+        }
+        TAH_WAIT_VMEM();
+        __syncthreads();
+    }
+    // accumulator (i, j) register r of lane l: weight row 16 i + 4 (l / 16) + r, place 16 j + l % 16
+    __bf16* const out = static_cast<__bf16*>(p.out);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        __bf16* const row = out + ((int64_t)blockIdx.y * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
+        if constexpr (GATE) {
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
+                bf16x4 y;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
+                if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
+                bf16x4 y;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) y[r] = (__bf16)acc[i][j][r];
+                if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
+            }
+        }
+    }
+}
+
+// ---- float32 ---------------------------------------------------------------------------------------------------
+constexpr int kPlainK = 16, kPlainCols = 32;
+
+// 128 places x 32 columns per workgroup; thread (column tid % 32, places tid / 32 + 8 i)
+template <bool GATE>
+__global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p) {
+    __shared__ float a[kPlainK][kTile + 1], g[kPlainK][kPlainCols + 1], u[GATE ? kPlainK : 1][kPlainCols + 1];
+    const int expert = p.tile_expert[blockIdx.y];
+    if (expert < 0) return;
+    const int tid = threadIdx.x, tc = tid % kPlainCols, tr = tid / kPlainCols, n0 = blockIdx.x * kPlainCols;
+    const float* const x = static_cast<const float*>(p.x);
+    const float* const w = static_cast<const float*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
+    float sg[16], su[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) sg[i] = su[i] = 0.f;
+    for (int k0 = 0; k0 < p.k; k0 += kPlainK) {
+        for (int i = tid; i < kTile * kPlainK; i += kMoeThreads) {
+            const int r = i / kPlainK, c = i % kPlainK;
+            const int src = GATE ? p.source[blockIdx.y * kTile + r] : blockIdx.y * kTile + r;
+            a[c][r] = src >= 0 ? x[(int64_t)src * p.x_rs + k0 + c] : 0.f;
+        }
+        for (int i = tid; i < kPlainCols * kPlainK; i += kMoeThreads) {
+            const int r = i / kPlainK, c = i % kPlainK, wr = n0 + r < p.n ? n0 + r : p.n - 1;
+            g[c][r] = w[(int64_t)wr * p.k + k0 + c];
+            if constexpr (GATE) u[c][r] = w[((int64_t)p.n + wr) * p.k + k0 + c];
+        }
+        __syncthreads();
+#pragma unroll
+        for (int c = 0; c < kPlainK; ++c) {
+            const float wg = g[c][tc], wu = GATE ? u[GATE ? c : 0][tc] : 0.f;
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                const float v = a[c][tr + 8 * i];
+                sg[i] += v * wg;
+                if constexpr (GATE) su[i] += v * wu;
+            }
+        }
+        __syncthreads();
+    }
+    if (n0 + tc >= p.n) return;
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+        static_cast<float*>(p.out)[((int64_t)blockIdx.y * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = GATE ? silu_exact(sg[i]) * su[i] : sg[i];
+}
+
+template <class E>
+void launch_route(const float* x, const void* router, const void* gate_w, int rows, int cols, int experts, int top, int32_t* index, float* weight,
+                  float* shared_gate, hipStream_t st) {
+    const E* const rt = static_cast<const E*>(router);
+    const E* const gw = static_cast<const E*>(gate_w);
+    const auto lds = [&](int rb) { return (size_t)rb * (cols + experts + 1) * sizeof(float); };
+    if (rows > 256 && lds(8) <= 65536)  // many rows: eight share a pass over the router's weights
+        hipLaunchKernelGGL((moe_route_kernel<E, 8>), dim3((rows + 7) / 8), dim3(kMoeThreads), lds(8), st, x, rt, gw, rows, cols, experts, top, index,
+                           weight, shared_gate);
+    else
+        hipLaunchKernelGGL((moe_route_kernel<E, 1>), dim3(rows), dim3(kMoeThreads), lds(1), st, x, rt, gw, rows, cols, experts, top, index, weight,
+                           shared_gate);
+}
+
+int tile_capacity(int64_t pairs, int experts) { return (int)(pairs / kTile + (experts < pairs ? experts : pairs)); }
+
+}  // namespace
+}  // namespace tah
+
+extern "C" int tah_moe_route(const float* x, const void* router, const void* gate_w, int32_t rows, int32_t cols, int32_t experts, int32_t top,
+                             int32_t* index, float* weight, float* shared_gate, int32_t dtype, tah_stream_t stream) {
+    using namespace tah;
+    if (rows < 0 || cols <= 0 || cols % 8 != 0 || experts <= 0 || experts > kMaxExperts || top <= 0 || top > kMaxTop || top > experts ||
+        (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
+        return TAH_E_SHAPE;
+    if ((size_t)(cols + experts + 1) * sizeof(float) > 65536) return TAH_E_SHAPE;
+    if (rows == 0) return TAH_OK;
+    if (!x || !router || !index || !weight || (gate_w && !shared_gate)) return TAH_E_NULL;
+    if (!aligned_16(x) || !aligned_16(router) || !aligned_16(gate_w)) return TAH_E_ALIGN;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (dtype == TAH_DT_BF16) launch_route<__bf16>(x, router, gate_w, rows, cols, experts, top, index, weight, shared_gate, st);
+    else launch_route<float>(x, router, gate_w, rows, cols, experts, top, index, weight, shared_gate, st);
+    return launch_status();
+}
+
+extern "C" int32_t tah_moe_places(int32_t rows, int32_t top, int32_t experts) {
+    return rows <= 0 || top <= 0 || experts <= 0 ? 0 : tah::tile_capacity((int64_t)rows * top, experts) * TAH_MOE_TILE;
+}
+
+extern "C" int tah_moe_plan(const int32_t* index, int32_t rows, int32_t top, int32_t experts, int32_t* source, int32_t* tile_expert, int32_t* place,
+                            tah_stream_t stream) {
+    using namespace tah;
+    if (rows < 0 || top <= 0 || top > kMaxTop || experts <= 0 || experts > kMaxExperts || (int64_t)rows * top > (1 << 30)) return TAH_E_SHAPE;
+    if (rows == 0) return TAH_OK;
+    if (!index || !source || !tile_expert || !place) return TAH_E_NULL;
+    hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(kPlanThreads), 0, static_cast<hipStream_t>(stream), index, (int)(rows * top), (int)top,
+                       (int)experts, tile_capacity((int64_t)rows * top, experts), source, tile_expert, place);
+    return launch_status();
+}
+
+extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const int32_t* source, const int32_t* tile_expert, int32_t tiles, int32_t n,
+                              int32_t k, int32_t kind, void* out, int64_t out_rs, int32_t dtype, tah_stream_t stream) {
+    using namespace tah;
+    if (tiles < 0 || tiles > 65535 || n <= 0 || k <= 0 || n % 4 != 0 || k % 32 != 0 || x_rs < k || out_rs < n || x_rs % 8 != 0 || out_rs % 4 != 0 ||
+        (kind != TAH_LINEAR_PLAIN && kind != TAH_LINEAR_GATE_UP) || (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
+        return TAH_E_SHAPE;
+    if (tiles == 0) return TAH_OK;
+    if (!x || !w || !tile_expert || !out || (kind == TAH_LINEAR_GATE_UP && !source)) return TAH_E_NULL;
+    if (!aligned_16(x) || !aligned_16(w) || !aligned_16(out)) return TAH_E_ALIGN;
+    const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k};
+    const bool gate = kind == TAH_LINEAR_GATE_UP;
+    hipStream_t st = static_cast<hipStream_t>(stream);
+    if (dtype == TAH_DT_BF16) {
+        const int cols = gate ? kTile / 2 : kTile;
+        const dim3 grid((n + cols - 1) / cols, tiles);
+        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
+        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
+    } else {
+        const dim3 grid((n + kPlainCols - 1) / kPlainCols, tiles);
+        if (gate) hipLaunchKernelGGL((moe_plain_kernel<true>), grid, dim3(kMoeThreads), 0, st, p);
+        else hipLaunchKernelGGL((moe_plain_kernel<false>), grid, dim3(kMoeThreads), 0, st, p);
+    }
+    return launch_status();
+}

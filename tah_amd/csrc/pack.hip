@@ -156,18 +156,3 @@ extern "C" int tah_rows_copy(const void* src, const int32_t* src_rows, void* dst
     if (bits % 2 == 0) return launch_copy<uint16_t>(src, src_rows, dst, dst_rows, dst_enable, n, n_dev, row_bytes, src_stride_bytes, dst_stride_bytes, st);
     return launch_copy<uint8_t>(src, src_rows, dst, dst_rows, dst_enable, n, n_dev, row_bytes, src_stride_bytes, dst_stride_bytes, st);
 }
-
-extern "C" int tah_duo_abi_version(void) { return TAH_DUO_ABI_VERSION; }
-
-extern "C" const char* tah_duo_error_string(int code) {
-    switch (code) {
-        case TAH_OK: return "ok";
-        case TAH_E_NULL: return "a required pointer is NULL";
-        case TAH_E_SHAPE: return "unsupported shape (head_dim must be 128, Hq/Hkv in {1,2,4,8}, sizes >= 0)";
-        case TAH_E_ALIGN: return "pointers must be 16-byte aligned and strides multiples of 8 elements";
-        case TAH_E_LAUNCH: return "HIP launch failed";
-        case TAH_E_WORKSPACE: return "workspace too small";
-        case TAH_E_SCRATCH: return "the call needs more split-K scratch than tah_duo_decode_static holds (TAH_DUO_STATIC_SCRATCH_BYTES)";
-        default: return "unknown error";
-    }
-}

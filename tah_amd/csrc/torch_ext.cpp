@@ -5,60 +5,24 @@
 // the entry point on torch's current HIP stream.  Nothing is computed here.  The library itself is opened at
 // run time (load_library), so the same extension serves libtah_duo.so and, in the CPU tests, the host build
 // of the kernels.  There is no fallback: without a loaded library every call throws.
-#include <c10/hip/HIPStream.h>
-#include <dlfcn.h>
-#include <torch/extension.h>
+#include "torch_ext.h"
 
-#include <string>
+#include <dlfcn.h>
+
 #include <tuple>
 
-#include "tah_duo.h"
+namespace tah_ext {
+Api g;
+}
 
 namespace {
 
-using at::Tensor;
-using c10::optional;
+using namespace tah_ext;
 
-struct Api {
-    void* handle = nullptr;
-    bool allow_host = false;
-    decltype(&tah_duo_abi_version) abi_version = nullptr;
-    decltype(&tah_duo_error_string) error_string = nullptr;
-    decltype(&tah_duo_fwd_varlen) fwd_varlen = nullptr;
-    decltype(&tah_duo_bwd_varlen) bwd_varlen = nullptr;
-    decltype(&tah_duo_bwd_workspace_bytes) bwd_workspace_bytes = nullptr;
-    decltype(&tah_duo_schedule_bytes) schedule_bytes = nullptr;
-    decltype(&tah_duo_schedule_build) schedule_build = nullptr;
-    decltype(&tah_greedy_step) greedy_step = nullptr;
-    decltype(&tah_silu_mul_normed) silu_mul_normed = nullptr;
-    decltype(&tah_step_begin) step_begin = nullptr;
-    decltype(&tah_greedy_tick) greedy_tick = nullptr;
-    decltype(&tah_decider_tail) decider_tail = nullptr;
-    decltype(&tah_linear_pack_weight) linear_pack_weight = nullptr;
-    decltype(&tah_linear_pack_rows) linear_pack_rows = nullptr;
-    decltype(&tah_linear_rows) linear_rows = nullptr;
-    decltype(&tah_duo_fwd_masked) fwd_masked = nullptr;
-    decltype(&tah_duo_bwd_masked) bwd_masked = nullptr;
-    decltype(&tah_duo_decode_workspace_bytes) decode_workspace_bytes = nullptr;
-    decltype(&tah_duo_decode) decode = nullptr;
-    decltype(&tah_duo_decode_static) decode_static = nullptr;
-    decltype(&tah_kv_append) kv_append = nullptr;
-    decltype(&tah_qk_prep) qk_prep = nullptr;
-    decltype(&tah_duo_decode_step) decode_step = nullptr;
-    decltype(&tah_duo_decode_step_supported) decode_step_supported = nullptr;
-    decltype(&tah_topk_mix) topk_mix = nullptr;
-    decltype(&tah_qk_prep_bwd) qk_prep_bwd = nullptr;
-    decltype(&tah_sample_rows) sample_rows = nullptr;
-    decltype(&tah_silu_mul) silu_mul = nullptr;
-    decltype(&tah_hard_index_build) hard_index_build = nullptr;
-    decltype(&tah_pad_rows_build) pad_rows_build = nullptr;
-    decltype(&tah_rows_copy) rows_copy = nullptr;
-} g;
-
-template <class F>
-void bind(F& f, const char* name) {
-    f = reinterpret_cast<F>(dlsym(g.handle, name));
-    TORCH_CHECK(f != nullptr, "tah_amd: ", name, " is not exported by the loaded library");
+template <class E>
+void bind(E& e, const char* name) {
+    e.f = reinterpret_cast<decltype(e.f)>(dlsym(g.handle, name));
+    e.name = name;
 }
 
 void load_library(const std::string& path, bool allow_host) {
@@ -93,42 +57,31 @@ void load_library(const std::string& path, bool allow_host) {
     bind(g.decode_step, "tah_duo_decode_step");
     bind(g.decode_step_supported, "tah_duo_decode_step_supported");
     bind(g.topk_mix, "tah_topk_mix");
-    bind(g.sample_rows, "tah_sample_rows");
     bind(g.qk_prep_bwd, "tah_qk_prep_bwd");
+    bind(g.sample_rows, "tah_sample_rows");
     bind(g.silu_mul, "tah_silu_mul");
     bind(g.hard_index_build, "tah_hard_index_build");
     bind(g.pad_rows_build, "tah_pad_rows_build");
     bind(g.rows_copy, "tah_rows_copy");
+    bind(g.embed_rows, "tah_embed_rows");
+    bind(g.residual_norm, "tah_residual_norm");
+    bind(g.activate_rows, "tah_activate_rows");
+    bind(g.delta_step, "tah_delta_step");
+    bind(g.delta_prepare, "tah_delta_prepare");
+    bind(g.delta_scan, "tah_delta_scan");
+    bind(g.delta_finish, "tah_delta_finish");
+    bind(g.latent_prep, "tah_latent_prep");
+    bind(g.latent_context, "tah_latent_context");
+    bind(g.latent_attend, "tah_latent_attend");
+    bind(g.latent_decode_workspace, "tah_latent_decode_workspace");
+    bind(g.latent_decode, "tah_latent_decode");
+    bind(g.moe_route, "tah_moe_route");
+    bind(g.moe_places, "tah_moe_places");
+    bind(g.moe_plan, "tah_moe_plan");
+    bind(g.moe_linear, "tah_moe_linear");
     const int got = g.abi_version();
     TORCH_CHECK(got == TAH_DUO_ABI_VERSION, "tah_amd: library ABI version ", got, ", extension built for ", TAH_DUO_ABI_VERSION);
 }
-
-void need_lib() { TORCH_CHECK(g.handle != nullptr, "tah_amd: no library loaded (tah_amd._lib.lib() loads libtah_duo.so)"); }
-
-void check_rc(int rc, const char* what) {
-    TORCH_CHECK(rc == 0, what, ": ", g.error_string(rc), " (code ", rc, ")");
-}
-
-// One device for all tensors; host tensors only when the loaded library is the host build of the kernels.
-struct Dev {
-    bool set = false;
-    c10::Device dev{c10::kCPU};
-    void see(const Tensor& t) {
-        if (!t.defined()) return;
-        TORCH_CHECK(t.is_cuda() || g.allow_host, "tah_amd ops need CUDA/HIP tensors (no CPU path exists)");
-        if (!set) { dev = t.device(); set = true; }
-        else TORCH_CHECK(t.device() == dev, "tensors on different devices: ", dev, " vs ", t.device());
-    }
-    void see(const optional<Tensor>& t) { if (t.has_value()) see(*t); }
-    tah_stream_t stream() const {
-        if (set && dev.is_cuda()) return static_cast<tah_stream_t>(c10::hip::getCurrentHIPStream(dev.index()).stream());
-        return nullptr;
-    }
-};
-
-const void* ptr(const Tensor& t) { return (!t.defined() || t.numel() == 0) ? nullptr : t.data_ptr(); }
-void* mptr(const Tensor& t) { return (!t.defined() || t.numel() == 0) ? nullptr : t.data_ptr(); }
-const void* ptr(const optional<Tensor>& t) { return t.has_value() ? ptr(*t) : nullptr; }
 
 void thd(const Tensor& t, const char* name) {
     TORCH_CHECK(t.dim() == 3 && t.scalar_type() == at::kBFloat16, name, " must be a bf16 [rows, heads, head_dim] tensor");
@@ -962,38 +915,54 @@ Tensor linear_pack_rows(const Tensor& x, const optional<Tensor>& out) {
 optional<Tensor> linear_rows(const Tensor& w_packed, const Tensor& x_packed, int64_t rows, int64_t n, int64_t k, bool gate_up,
                              const optional<Tensor>& residual, const optional<Tensor>& out, const optional<Tensor>& out_packed,
                              bool want_out, int64_t input_norm, double norm_eps, const optional<Tensor>& bias, int64_t activation,
-                             const optional<Tensor>& ln_colsum) {
+                             const optional<Tensor>& ln_colsum, int64_t batch, bool shared_rows, int64_t packed_col_step,
+                             const optional<Tensor>& select) {
     need_lib();
-    Dev d; d.see(w_packed); d.see(x_packed); d.see(residual); d.see(out); d.see(out_packed); d.see(bias); d.see(ln_colsum);
+    Dev d; d.see(w_packed); d.see(x_packed); d.see(residual); d.see(out); d.see(out_packed); d.see(bias); d.see(ln_colsum); d.see(select);
     if (ln_colsum.has_value())
         TORCH_CHECK(ln_colsum->scalar_type() == at::kFloat && ln_colsum->is_contiguous() && ln_colsum->numel() == n,
                     "linear_rows: ln_colsum must be a contiguous float32 [N] tensor");
     TORCH_CHECK((input_norm == TAH_NORM_LAYER) == ln_colsum.has_value(), "linear_rows: ln_colsum goes with the LayerNorm fold and only with it");
     if (bias.has_value()) TORCH_CHECK(packed_vec(*bias, n), "linear_rows: bias must be a contiguous bf16 [N] tensor");
-    TORCH_CHECK(rows >= 0 && n >= 0 && k >= 0, "linear_rows: negative size");
-    TORCH_CHECK(packed_vec(w_packed, (gate_up ? 2 : 1) * n * k), "linear_rows: w_packed must come from linear_pack_weight for these sizes");
-    TORCH_CHECK(packed_vec(x_packed, 32 * k), "linear_rows: x_packed must be a contiguous bf16 tensor of 32 * K elements");
+    TORCH_CHECK(rows >= 0 && n >= 0 && k >= 0 && batch >= 1, "linear_rows: negative size");
+    const int64_t wn = (gate_up ? 2 : 1) * n * k;
+    TORCH_CHECK(packed_vec(w_packed, batch * wn), "linear_rows: w_packed must come from linear_pack_weight for these sizes");
+    TORCH_CHECK(packed_vec(x_packed, (shared_rows ? 1 : batch) * 32 * k), "linear_rows: x_packed must be a contiguous bf16 tensor of 32 * K elements (per product)");
     optional<Tensor> y = out;
-    if (!y.has_value() && want_out) y = at::empty({rows, n}, x_packed.options());
-    if (y.has_value())
+    if (!y.has_value() && want_out) y = batch > 1 ? at::empty({batch, rows, n}, x_packed.options()) : at::empty({rows, n}, x_packed.options());
+    if (y.has_value() && batch > 1) {
+        TORCH_CHECK(y->dim() == 3 && y->size(0) == batch && y->size(1) == rows && y->size(2) == n && y->scalar_type() == at::kBFloat16 && y->is_contiguous(),
+                    "linear_rows: out must be contiguous bf16 [batch, rows, N]");
+    } else if (y.has_value())
         TORCH_CHECK(y->dim() == 2 && y->size(0) == rows && y->size(1) == n && y->scalar_type() == at::kBFloat16 && (y->numel() == 0 || y->stride(1) == 1),
                     "linear_rows: out must be bf16 [rows, N]");
     if (residual.has_value())
         TORCH_CHECK(residual->dim() == 2 && residual->size(0) == rows && residual->size(1) == n && residual->scalar_type() == at::kBFloat16 &&
                         (residual->numel() == 0 || residual->stride(1) == 1),
                     "linear_rows: residual must be bf16 [rows, N]");
-    if (out_packed.has_value()) TORCH_CHECK(packed_vec(*out_packed, 32 * n), "linear_rows: out_packed must be a contiguous bf16 tensor of 32 * N elements");
+    if (out_packed.has_value() && packed_col_step) {
+        TORCH_CHECK(out_packed->scalar_type() == at::kBFloat16 && out_packed->is_contiguous() && out_packed->numel() % 1024 == 0 &&
+                        out_packed->numel() >= 32 * ((batch - 1) * packed_col_step + n),
+                    "linear_rows: out_packed must be a contiguous bf16 tensor that holds all results side by side");
+    } else if (out_packed.has_value())
+        TORCH_CHECK(packed_vec(*out_packed, batch * 32 * n), "linear_rows: out_packed must be a contiguous bf16 tensor of 32 * N elements (per product)");
+    if (select.has_value()) TORCH_CHECK(select->scalar_type() == at::kInt && select->is_contiguous(), "linear_rows: select must be a contiguous int32 tensor");
     TORCH_CHECK(y.has_value() || out_packed.has_value(), "linear_rows: nothing to write");
     tah_linear_rows_args a{};
     a.w_packed = w_packed.data_ptr(); a.x_packed = x_packed.data_ptr();
     a.residual = ptr(residual); a.residual_row_stride = residual.has_value() ? (rows > 1 ? residual->stride(0) : n) : 0;
-    a.out = y.has_value() ? mptr(*y) : nullptr; a.out_row_stride = y.has_value() ? (rows > 1 ? y->stride(0) : n) : 0;
+    a.out = y.has_value() ? mptr(*y) : nullptr; a.out_row_stride = y.has_value() ? (batch == 1 && rows > 1 ? y->stride(0) : n) : 0;
     a.out_packed = out_packed.has_value() ? out_packed->data_ptr() : nullptr;
     a.rows = (int32_t)rows; a.n = (int32_t)n; a.k = (int32_t)k;
     a.kind = gate_up ? TAH_LINEAR_GATE_UP : TAH_LINEAR_PLAIN;
     a.input_norm = (int32_t)input_norm; a.norm_eps = (float)norm_eps;
     a.bias = bias.has_value() ? bias->data_ptr() : nullptr; a.activation = (int32_t)activation;
     a.ln_colsum = ln_colsum.has_value() ? static_cast<const float*>(ln_colsum->data_ptr()) : nullptr;
+    a.batch = (int32_t)batch; a.out_packed_col_step = (int32_t)packed_col_step;
+    a.w_batch_stride = wn; a.x_batch_stride = shared_rows ? 0 : 32 * k; a.out_batch_stride = rows * n;
+    a.out_packed_batch_stride = packed_col_step ? 0 : 32 * n;
+    a.batch_select = select.has_value() ? static_cast<const int32_t*>(ptr(*select)) : nullptr;
+    a.n_select = select.has_value() ? (int32_t)select->numel() : 0;
     check_rc(g.linear_rows(&a, d.stream()), "tah_linear_rows");
     return y;
 }
@@ -1037,4 +1006,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     m.def("linear_pack_weight", &linear_pack_weight);
     m.def("linear_pack_rows", &linear_pack_rows);
     m.def("linear_rows", &linear_rows);
+    tah_ext::bind_mixers(m);
 }

@@ -57,6 +57,14 @@ class EngineConfig:
     decider_hidden: int = 512
     topk: int = 100
 
+    @staticmethod
+    def from_config(config: dict) -> "EngineConfig":
+        """From a Hugging Face Qwen3 config.json."""
+        heads = config["num_attention_heads"]
+        return EngineConfig(hidden=config["hidden_size"], layers=config["num_hidden_layers"], hq=heads, hkv=config["num_key_value_heads"],
+                            head_dim=config.get("head_dim") or config["hidden_size"] // heads, intermediate=config["intermediate_size"],
+                            vocab=config["vocab_size"], rms_eps=config["rms_norm_eps"], rope_theta=config["rope_theta"])
+
 
 class Weights:
     """Plain tensors of a Qwen3-shaped decoder, the output head and the decider MLP (all bf16)."""
@@ -143,6 +151,22 @@ class Weights:
         return w
 
     @staticmethod
+    def from_tensors(tensors: dict, cfg: EngineConfig, device, dtype=torch.bfloat16) -> "Weights":
+        """From a Qwen3 checkpoint's tensors by name (no decider among them: the engine then needs ``decider=``)."""
+        t = lambda n: tensors[n].to(device=device, dtype=dtype)
+        w = Weights(cfg)
+        w.embed, w.norm = t("model.embed_tokens.weight"), t("model.norm.weight")
+        w.lm_head = t("lm_head.weight") if "lm_head.weight" in tensors else w.embed
+        for i in range(cfg.layers):
+            a, m = f"model.layers.{i}.self_attn.", f"model.layers.{i}.mlp."
+            w.layers.append(dict(
+                ln1=t(f"model.layers.{i}.input_layernorm.weight"),
+                wqkv=torch.cat([t(a + f"{p}_proj.weight") for p in "qkv"], 0), qn=t(a + "q_norm.weight"), kn=t(a + "k_norm.weight"),
+                wo=t(a + "o_proj.weight"), ln2=t(f"model.layers.{i}.post_attention_layernorm.weight"),
+                wgu=torch.cat([t(m + "gate_proj.weight"), t(m + "up_proj.weight")], 0), wdown=t(m + "down_proj.weight")))
+        return w
+
+    @staticmethod
     def from_hf(model, cfg: EngineConfig, device, dtype=torch.bfloat16) -> "Weights":
         """Copies the tensors of a Hugging Face ``Qwen3ForCausalLM`` (q/k/v and gate/up fused row-wise)."""
         w = Weights(cfg)
@@ -169,7 +193,218 @@ def rope_tables(max_len: int, head_dim: int, theta: float, device, dtype=torch.b
     return emb.cos().to(dtype).to(device), emb.sin().to(dtype).to(device)
 
 
-class TaHDecodeEngine:
+class DecodeEngine:
+    """What every model's engine shares: the generation state of a batch of rows (on the device), sampling, the greedy
+    step's bookkeeping, the loop, and its step captured in a HIP graph.  A model's engine provides ``_parts``, one step
+    of all rows, and ``_hold_state``."""
+
+    def _init_generation(self, batch: int, max_len: int, device) -> None:
+        dev = torch.device(device)
+        self.B, self.max_len, self.device = batch, max_len, dev
+        # generation state (all on the device)
+        self.fused_greedy = True  # arg-max + bookkeeping of a greedy step in one launch (tah_greedy_step)
+        self.fused_sampling = True  # draws without a top-k filter in one launch (tah_sample_rows) instead of a sort in torch
+        self.tok = torch.zeros(batch, dtype=torch.long, device=dev)       # token fed to the next step
+        self.pos = torch.zeros(batch, dtype=torch.int32, device=dev)      # its position
+        self.finished = torch.zeros(batch, dtype=torch.bool, device=dev)
+        self.n_hard = torch.zeros((), dtype=torch.long, device=dev)       # tokens that took a second iteration
+        self.n_steps = torch.zeros((), dtype=torch.long, device=dev)      # tokens decoded (active rows x steps)
+        self.step_idx = torch.zeros(1, dtype=torch.long, device=dev)
+        self.out_tokens = torch.zeros(batch, max_len, dtype=torch.long, device=dev)  # generated tokens, column = step
+        self.out_len = torch.zeros(batch, dtype=torch.int32, device=dev)             # tokens of each row before its end
+        self.host_positions = 0  # upper bound on any sequence's length, kept on the host for capacity checks
+        self._graph = None
+
+    def _parts(self):
+        """One step of all rows on the engine's own state: (logits, logits of a second iteration or None, which rows
+        took one or None, active rows)."""
+        raise NotImplementedError
+
+    def _hold_state(self):
+        """Called before a warm-up step; returns a function that undoes what the step changed."""
+        raise NotImplementedError
+
+    def _launch_switches(self):
+        """Every attribute that changes which kernels a captured step launches: part of the graph keys, so that
+        flipping one between two generate() calls on the same prefill captures again instead of replaying a graph
+        of the old path."""
+        return (self.fused_greedy, self.fused_sampling)
+
+    def _state(self):
+        return (self.tok, self.pos, self.finished, self.n_hard, self.n_steps, self.step_idx, self.out_tokens, self.out_len)
+
+    # ── sampling / generation ────────────────────────────────────────────
+    @staticmethod
+    def sample(logits: torch.Tensor, temperature: float = 0.0, *, top_p: float = 1.0, top_k: int = 0, min_p: float = 0.0) -> torch.Tensor:
+        """One token per row, batched on the device: ``sample_next_token`` of the reference
+        (tah/model/utils.py:84-125) -- temperature, softmax, then min_p / top_k / top_p filters with
+        renormalisation, then one draw per row -- with ``temperature <= 0`` meaning ``do_sample=False`` (arg-max).
+        The draw is the exponential-race form of a multinomial draw (arg-max of p / e, e ~ Exp(1)), which can be
+        captured in a graph."""
+        if temperature <= 0.0:
+            return torch.argmax(logits, dim=-1)
+        probs = DecodeEngine.filtered_probs(logits, temperature, top_p=top_p, top_k=top_k, min_p=min_p)
+        return torch.argmax(probs / torch.empty_like(probs).exponential_(), dim=-1)
+
+    @staticmethod
+    def filtered_probs(logits: torch.Tensor, temperature: float, *, top_p: float = 1.0, top_k: int = 0, min_p: float = 0.0) -> torch.Tensor:
+        """The distribution ``sample`` draws from: [rows, V], zero outside the filters."""
+        probs = F.softmax(logits / temperature if temperature != 1.0 else logits, dim=-1)
+        if min_p > 0.0:
+            probs = torch.where(probs >= min_p * probs.max(dim=-1, keepdim=True).values, probs, torch.zeros_like(probs))
+            probs = probs / probs.sum(dim=-1, keepdim=True)
+        if top_k > 0:
+            kth = torch.topk(probs, min(top_k, probs.size(-1)), dim=-1).values[..., -1:]
+            probs = torch.where(probs < kth, torch.zeros_like(probs), probs)
+            probs = probs / probs.sum(dim=-1, keepdim=True)
+        if top_p < 1.0:
+            sp, si = torch.sort(probs, descending=True, dim=-1)
+            remove = torch.cumsum(sp, dim=-1) > top_p
+            remove = torch.cat([torch.zeros_like(remove[..., :1]), remove[..., :-1]], dim=-1)  # keep the one that crosses
+            probs = torch.where(torch.zeros_like(remove).scatter_(-1, si, remove), torch.zeros_like(probs), probs)
+            probs = probs / probs.sum(dim=-1, keepdim=True)
+        return probs
+
+    # With a top-k filter (0 < top_k <= 256) nothing outside the k largest logits can be drawn, and every filter compares
+    # probabilities with each other, never with the softmax's denominator: the whole of ``sample`` can run on the
+    # [rows, k] values that one ``tah_topk_mix`` launch returns (largest first, with their vocabulary indices) instead
+    # of on [rows, V] -- no sort over the vocabulary, about a millisecond less per step at 32 x 151 936.  One
+    # difference: logits equal to the k-th largest beyond the k-th place stay out (the lower indices are taken),
+    # where ``torch.where(probs < kth, 0, probs)`` (utils.py:113) keeps them all.
+    TOPK_SAMPLING_MAX = 256
+
+    @staticmethod
+    def topk_filtered_probs(vals: torch.Tensor, temperature: float, *, top_p: float = 1.0, min_p: float = 0.0) -> torch.Tensor:
+        """``filtered_probs`` on the k largest logits of every row, ``vals`` [rows, k] sorted largest first."""
+        x = vals.float()
+        probs = F.softmax(x / temperature if temperature != 1.0 else x, dim=-1)
+        if min_p > 0.0:
+            probs = torch.where(probs >= min_p * probs[..., :1], probs, torch.zeros_like(probs))
+            probs = probs / probs.sum(dim=-1, keepdim=True)
+        if top_p < 1.0:
+            remove = torch.cumsum(probs, dim=-1) > top_p
+            remove = torch.cat([torch.zeros_like(remove[..., :1]), remove[..., :-1]], dim=-1)  # keep the one that crosses
+            probs = torch.where(remove, torch.zeros_like(probs), probs)
+            probs = probs / probs.sum(dim=-1, keepdim=True)
+        return probs
+
+    @staticmethod
+    def sample_topk(logits: torch.Tensor, temperature: float, *, top_p: float = 1.0, top_k: int, min_p: float = 0.0) -> torch.Tensor:
+        """``sample`` for bf16 logits [rows, V] and 0 < top_k <= TOPK_SAMPLING_MAX."""
+        vals, idx = ops.topk(logits, top_k)
+        probs = DecodeEngine.topk_filtered_probs(vals, temperature, top_p=top_p, min_p=min_p)
+        j = torch.argmax(probs / torch.empty_like(probs).exponential_(), dim=-1, keepdim=True)
+        return torch.gather(idx, 1, j).squeeze(1).to(torch.int64)
+
+    # Without a top-k filter the draw is one ``tah_sample_rows`` launch on the bf16 logits (no sort over the vocabulary);
+    # with one of at most 256 places it runs on the k largest logits; anything else takes the torch formulation.
+    SAMPLE_ROWS_MAX_VOCAB = 155648
+
+    def _draw(self, logits: torch.Tensor, temperature: float, prev: Optional[torch.Tensor] = None,
+              add_prev: Optional[torch.Tensor] = None, **filters) -> torch.Tensor:
+        """One token per row from final logits in bf16.  ``prev`` / ``add_prev`` (int32 [rows]): rows whose entry is not 0
+        draw from ``prev + logits``, summed in bf16 as the step-wise loop forms the final logits of a hard token."""
+        k = int(filters.get("top_k", 0))
+        fits = logits.dtype == torch.bfloat16 and logits.size(-1) <= self.SAMPLE_ROWS_MAX_VOCAB
+        if k == 0 and fits and self.fused_sampling:
+            u = torch.rand(logits.size(0), dtype=torch.float32, device=logits.device)
+            return ops.sample_rows(logits, u, temperature, top_p=float(filters.get("top_p", 1.0)), min_p=float(filters.get("min_p", 0.0)),
+                                   logits_prev=prev, add_prev=add_prev)
+        final = logits if prev is None else torch.where((add_prev != 0)[:, None], prev + logits, logits)
+        if 0 < k <= self.TOPK_SAMPLING_MAX and fits:
+            return self.sample_topk(final, temperature, **filters)
+        return self.sample(final.float(), temperature, **filters)
+
+    def _step_inplace(self, temperature: float, eos: int, **filters):
+        """One generated token for every unfinished row; every state change is an in-place device update."""
+        l0, l1, hard, act = self._parts()
+        if temperature <= 0.0 and self.fused_greedy and l0.dtype == torch.bfloat16 and self.cfg.vocab % 8 == 0:
+            # arg-max of the final logits and the bookkeeping below in one launch; the final logits are not formed
+            ops.greedy_step(l0, l1, hard, eos, self.tok, self.finished, self.pos, self.out_tokens, self.step_idx, self.out_len,
+                            self.n_hard, self.n_steps)
+            self.step_idx += 1
+            return
+        if temperature > 0.0:  # final logits as step_logits forms them: l0, plus l1 for hard tokens (the sum in the logits' dtype)
+            add = {} if l1 is None else dict(prev=l1, add_prev=hard.to(torch.int32))
+            nxt = self._draw(l0, temperature, **add, **filters)
+        else:
+            nxt = self.sample((l0 if l1 is None else torch.where(hard[:, None], l0 + l1, l0)).float(), 0.0)
+        nxt = torch.where(act, nxt, torch.zeros_like(nxt))
+        if eos >= 0:
+            self.finished |= nxt == eos
+        # a row's output ends before its end-of-sequence token (utils.py:241-245); finished rows write zeros
+        keep = ~self.finished
+        self.out_tokens.scatter_(1, self.step_idx.expand(self.B, 1), torch.where(keep, nxt, torch.zeros_like(nxt))[:, None])
+        self.out_len += keep.to(torch.int32)
+        if hard is not None:
+            self.n_hard += hard.sum()
+        self.n_steps += act.sum()
+        self.pos += act.to(torch.int32)
+        self.step_idx += 1
+        self.tok.copy_(nxt)
+
+    def _check_room(self, max_new_tokens: int) -> None:
+        if self.host_positions + max_new_tokens > self.max_len:
+            raise TahDuoError("generation would outgrow the cache: construct the engine with a larger max_len")
+
+    @torch.no_grad()
+    def generate(self, first_logits: torch.Tensor, max_new_tokens: int, *, temperature: float = 0.0, eos: int = -1,
+                 use_graph: bool = True, check_every: int = 64, **filters):
+        """Continues after ``prefill``.  Returns tokens int64 [B, max_new_tokens]; a row's tokens end before its
+        end-of-sequence token and are 0 from there on (``self.out_len`` holds each row's count).  With ``eos`` the
+        loop looks every ``check_every`` steps whether all rows are done (the only host synchronisation)."""
+        self._check_room(max_new_tokens)
+        dev = self.device
+        self.out_tokens.zero_()
+        self.out_len.zero_()
+        self.step_idx.zero_()
+        first = self.sample(first_logits, temperature, **filters)
+        if eos >= 0:
+            self.finished |= first == eos
+        keep = ~self.finished
+        self.out_tokens[:, 0] = torch.where(keep, first, torch.zeros_like(first))
+        self.out_len += keep.to(torch.int32)
+        self.tok.copy_(first)
+        self.step_idx += 1
+        n = max_new_tokens - 1
+        graph = self.capture(temperature, eos, **filters) if (use_graph and dev.type == "cuda" and n > 0) else None
+        done = 0
+        for i in range(n):
+            if graph is not None:
+                graph.replay()
+            else:
+                self._step_inplace(temperature, eos, **filters)
+            done += 1
+            if eos >= 0 and (i + 1) % check_every == 0 and bool(self.finished.all()):
+                break
+        self._advanced(done)
+        return self.out_tokens[:, :max_new_tokens]
+
+    def _advanced(self, steps: int) -> None:
+        self.host_positions += steps
+
+    def capture(self, temperature: float = 0.0, eos: int = -1, **filters):
+        """Captures one generation step in a HIP graph (after a warm-up step run on a side stream whose state
+        changes are undone, so that library workspaces exist before the capture)."""
+        key = (temperature, eos, tuple(sorted(filters.items()))) + self._launch_switches()
+        if self._graph is not None and self._graph_key == key:
+            return self._graph
+        undo = self._hold_state()
+        s = torch.cuda.Stream()
+        s.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(s):
+            self._step_inplace(temperature, eos, **filters)
+        torch.cuda.current_stream().wait_stream(s)
+        torch.cuda.synchronize()
+        undo()
+        g = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(g):
+            self._step_inplace(temperature, eos, **filters)
+        self._graph, self._graph_key = g, key
+        return g
+
+
+class TaHDecodeEngine(DecodeEngine):
     def __init__(self, weights: Weights, batch: int, max_len: int, *, max_hard: Optional[int] = None, device="cuda",
                  fold_norms: bool = True, packed_linear: bool = True, decider=None):
         """``fold_norms``: multiply the layers' input-norm weights into the projections behind them (in place in
@@ -189,8 +424,8 @@ class TaHDecodeEngine:
         self.packed_linear = bool(packed_linear and batch <= ops.LINEAR_MAX_ROWS and weights.can_pack_linear())
         if self.packed_linear:
             weights.pack_linear()
-        self.w, self.cfg, self.B, self.max_len = weights, cfg, batch, max_len
-        self.device = torch.device(device)
+        self.w, self.cfg = weights, cfg
+        self._init_generation(batch, max_len, device)
         self.max_hard = max_hard if max_hard is not None else max_len
         self.cos, self.sin = rope_tables(max_len, cfg.head_dim, cfg.rope_theta, self.device)
         self.slabs0 = [KvSlabs(batch, max_len, cfg.hkv, cfg.head_dim, with_pos=False, device=self.device) for _ in range(cfg.layers)]
@@ -200,22 +435,9 @@ class TaHDecodeEngine:
         self.cu_rows = torch.arange(batch + 1, dtype=torch.int32, device=dev)
         self.minus1 = torch.full((batch,), -1, dtype=torch.int32, device=dev)
         self.zeros_i = torch.zeros(batch, dtype=torch.int32, device=dev)
-        # generation state (all on the device)
-        self.fused_greedy = True  # arg-max + bookkeeping of a greedy step in one launch (tah_greedy_step)
-        self.fused_sampling = True  # draws without a top-k filter in one launch (tah_sample_rows) instead of a sort in torch
         self.use_fused_glue = True  # (tests switch it off to compare with the torch glue)
-        self.tok = torch.zeros(batch, dtype=torch.long, device=dev)       # token fed to the next step
-        self.pos = torch.zeros(batch, dtype=torch.int32, device=dev)      # its position
-        self.finished = torch.zeros(batch, dtype=torch.bool, device=dev)
-        self.n_hard = torch.zeros((), dtype=torch.long, device=dev)       # tokens that took a second iteration
-        self.n_steps = torch.zeros((), dtype=torch.long, device=dev)      # tokens decoded (active rows x steps)
-        self.step_idx = torch.zeros(1, dtype=torch.long, device=dev)
-        self.out_tokens = torch.zeros(batch, max_len, dtype=torch.long, device=dev)  # generated tokens, column = step
-        self.out_len = torch.zeros(batch, dtype=torch.int32, device=dev)             # tokens of each row before its end
         self.scale = float(cfg.head_dim) ** -0.5
-        self.host_positions = 0  # upper bound on any sequence's length, kept on the host for capacity checks
         self.host_hard_rows = 0
-        self._graph = None
         self.static_scratch = self.device.type == "cuda"
         self.measure_without_attention = False
         # depth-1 rows every sequence has cached (what each slabs1[l].len holds), kept once for the fused step kernel
@@ -568,130 +790,29 @@ class TaHDecodeEngine:
         self.finished.zero_()
         return logits_last.float(), hard
 
-    # ── sampling / generation ────────────────────────────────────────────
-    @staticmethod
-    def sample(logits: torch.Tensor, temperature: float = 0.0, *, top_p: float = 1.0, top_k: int = 0, min_p: float = 0.0) -> torch.Tensor:
-        """One token per row, batched on the device: ``sample_next_token`` of the reference
-        (tah/model/utils.py:84-125) -- temperature, softmax, then min_p / top_k / top_p filters with
-        renormalisation, then one draw per row -- with ``temperature <= 0`` meaning ``do_sample=False`` (arg-max).
-        The draw is the exponential-race form of a multinomial draw (arg-max of p / e, e ~ Exp(1)), which can be
-        captured in a graph."""
-        if temperature <= 0.0:
-            return torch.argmax(logits, dim=-1)
-        probs = TaHDecodeEngine.filtered_probs(logits, temperature, top_p=top_p, top_k=top_k, min_p=min_p)
-        return torch.argmax(probs / torch.empty_like(probs).exponential_(), dim=-1)
-
-    @staticmethod
-    def filtered_probs(logits: torch.Tensor, temperature: float, *, top_p: float = 1.0, top_k: int = 0, min_p: float = 0.0) -> torch.Tensor:
-        """The distribution ``sample`` draws from: [rows, V], zero outside the filters."""
-        probs = F.softmax(logits / temperature if temperature != 1.0 else logits, dim=-1)
-        if min_p > 0.0:
-            probs = torch.where(probs >= min_p * probs.max(dim=-1, keepdim=True).values, probs, torch.zeros_like(probs))
-            probs = probs / probs.sum(dim=-1, keepdim=True)
-        if top_k > 0:
-            kth = torch.topk(probs, min(top_k, probs.size(-1)), dim=-1).values[..., -1:]
-            probs = torch.where(probs < kth, torch.zeros_like(probs), probs)
-            probs = probs / probs.sum(dim=-1, keepdim=True)
-        if top_p < 1.0:
-            sp, si = torch.sort(probs, descending=True, dim=-1)
-            remove = torch.cumsum(sp, dim=-1) > top_p
-            remove = torch.cat([torch.zeros_like(remove[..., :1]), remove[..., :-1]], dim=-1)  # keep the one that crosses
-            probs = torch.where(torch.zeros_like(remove).scatter_(-1, si, remove), torch.zeros_like(probs), probs)
-            probs = probs / probs.sum(dim=-1, keepdim=True)
-        return probs
-
-    # With a top-k filter (0 < top_k <= 256) nothing outside the k largest logits can be drawn, and every filter compares
-    # probabilities with each other, never with the softmax's denominator: the whole of ``sample`` can run on the
-    # [rows, k] values that one ``tah_topk_mix`` launch returns (largest first, with their vocabulary indices) instead
-    # of on [rows, V] -- no sort over the vocabulary, about a millisecond less per step at 32 x 151 936.  One
-    # difference: logits equal to the k-th largest beyond the k-th place stay out (the lower indices are taken),
-    # where ``torch.where(probs < kth, 0, probs)`` (utils.py:113) keeps them all.
-    TOPK_SAMPLING_MAX = 256
-
-    @staticmethod
-    def topk_filtered_probs(vals: torch.Tensor, temperature: float, *, top_p: float = 1.0, min_p: float = 0.0) -> torch.Tensor:
-        """``filtered_probs`` on the k largest logits of every row, ``vals`` [rows, k] sorted largest first."""
-        x = vals.float()
-        probs = F.softmax(x / temperature if temperature != 1.0 else x, dim=-1)
-        if min_p > 0.0:
-            probs = torch.where(probs >= min_p * probs[..., :1], probs, torch.zeros_like(probs))
-            probs = probs / probs.sum(dim=-1, keepdim=True)
-        if top_p < 1.0:
-            remove = torch.cumsum(probs, dim=-1) > top_p
-            remove = torch.cat([torch.zeros_like(remove[..., :1]), remove[..., :-1]], dim=-1)  # keep the one that crosses
-            probs = torch.where(remove, torch.zeros_like(probs), probs)
-            probs = probs / probs.sum(dim=-1, keepdim=True)
-        return probs
-
-    @staticmethod
-    def sample_topk(logits: torch.Tensor, temperature: float, *, top_p: float = 1.0, top_k: int, min_p: float = 0.0) -> torch.Tensor:
-        """``sample`` for bf16 logits [rows, V] and 0 < top_k <= TOPK_SAMPLING_MAX."""
-        vals, idx = ops.topk(logits, top_k)
-        probs = TaHDecodeEngine.topk_filtered_probs(vals, temperature, top_p=top_p, min_p=min_p)
-        j = torch.argmax(probs / torch.empty_like(probs).exponential_(), dim=-1, keepdim=True)
-        return torch.gather(idx, 1, j).squeeze(1).to(torch.int64)
-
-    # Without a top-k filter the draw is one ``tah_sample_rows`` launch on the bf16 logits (no sort over the vocabulary);
-    # with one of at most 256 places it runs on the k largest logits; anything else takes the torch formulation.
-    SAMPLE_ROWS_MAX_VOCAB = 155648
-
-    def _draw(self, logits: torch.Tensor, temperature: float, prev: Optional[torch.Tensor] = None,
-              add_prev: Optional[torch.Tensor] = None, **filters) -> torch.Tensor:
-        """One token per row from final logits in bf16.  ``prev`` / ``add_prev`` (int32 [rows]): rows whose entry is not 0
-        draw from ``prev + logits``, summed in bf16 as the step-wise loop forms the final logits of a hard token."""
-        k = int(filters.get("top_k", 0))
-        fits = logits.dtype == torch.bfloat16 and logits.size(-1) <= self.SAMPLE_ROWS_MAX_VOCAB
-        if k == 0 and fits and self.fused_sampling:
-            u = torch.rand(logits.size(0), dtype=torch.float32, device=logits.device)
-            return ops.sample_rows(logits, u, temperature, top_p=float(filters.get("top_p", 1.0)), min_p=float(filters.get("min_p", 0.0)),
-                                   logits_prev=prev, add_prev=add_prev)
-        final = logits if prev is None else torch.where((add_prev != 0)[:, None], prev + logits, logits)
-        if 0 < k <= self.TOPK_SAMPLING_MAX and fits:
-            return self.sample_topk(final, temperature, **filters)
-        return self.sample(final.float(), temperature, **filters)
-
-    def _step_inplace(self, temperature: float, eos: int, **filters):
-        """One generated token for every unfinished row; every state change is an in-place device update."""
-        l0, l1, hard, act = self._parts()
-        if temperature <= 0.0 and self.fused_greedy and self.w.embed.dtype == torch.bfloat16 and self.cfg.vocab % 8 == 0:
-            # arg-max of the final logits and the bookkeeping below in one launch; the final logits are not formed
-            ops.greedy_step(l0, l1, hard, eos, self.tok, self.finished, self.pos, self.out_tokens, self.step_idx, self.out_len,
-                            self.n_hard, self.n_steps)
-            self.step_idx += 1
-            return
-        if temperature > 0.0:  # final logits as step_logits forms them: l0, plus l1 for hard tokens (the sum in the logits' dtype)
-            nxt = self._draw(l0, temperature, prev=l1, add_prev=hard.to(torch.int32), **filters)
-        else:
-            nxt = self.sample(torch.where(hard[:, None], l0 + l1, l0).float(), 0.0)
-        nxt = torch.where(act, nxt, torch.zeros_like(nxt))
-        if eos >= 0:
-            self.finished |= nxt == eos
-        # a row's output ends before its end-of-sequence token (utils.py:241-245); finished rows write zeros
-        keep = ~self.finished
-        self.out_tokens.scatter_(1, self.step_idx.expand(self.B, 1), torch.where(keep, nxt, torch.zeros_like(nxt))[:, None])
-        self.out_len += keep.to(torch.int32)
-        self.n_hard += hard.sum()
-        self.n_steps += act.sum()
-        self.pos += act.to(torch.int32)
-        self.step_idx += 1
-        self.tok.copy_(nxt)
-
+    # ── generation ───────────────────────────────────────────────────────
     def _state(self):
-        return (self.tok, self.pos, self.finished, self.n_hard, self.n_steps, self.step_idx, self.out_tokens, self.out_len,
-                self.hard_len, self.phase)
+        return super()._state() + (self.hard_len, self.phase)
+
+    def _hold_state(self):
+        # state tensors and slab lengths (the rows a warm-up step writes lie beyond the lengths)
+        state = [t.clone() for t in self._state()]
+        lens = [sl.len.clone() for sl in self.slabs0 + self.slabs1]
+
+        def undo():
+            for t, old in zip(self._state(), state):
+                t.copy_(old)
+            for sl, ln in zip(self.slabs0 + self.slabs1, lens):
+                sl.len.copy_(ln)
+        return undo
 
     @torch.no_grad()
     def generate(self, first_logits: torch.Tensor, max_new_tokens: int, *, temperature: float = 0.0, eos: int = -1,
                  use_graph: bool = True, check_every: int = 64, continuous: Optional[bool] = None, **filters):
-        """Continues after :meth:`prefill`.  Returns tokens int64 [B, max_new_tokens]; a row's tokens end before its
-        end-of-sequence token and are 0 from there on (``self.out_len`` holds each row's count).  With ``eos`` the
-        loop looks every ``check_every`` steps whether all rows are done (the only host synchronisation).
-
-        ``continuous`` (default: whenever the engine can): rows do not wait for each other's second latent iterations
+        """As in :class:`DecodeEngine`.  ``continuous`` (default: whenever the engine can): rows do not wait for each other's second latent iterations
         -- see :meth:`_generate_ticks`.  Greedy decoding gives the same tokens per row either way; sampled tokens come from
         the same per-row distributions but from other random draws (a tick draws for every row, a step once per token)."""
-        if self.host_positions + max_new_tokens > self.max_len or self.host_hard_rows + max_new_tokens > self.max_hard:
-            raise TahDuoError("generation would outgrow the KV slabs: construct the engine with a larger max_len / max_hard")
+        self._check_room(max_new_tokens)
         dev = self.device
         greedy_fused = temperature <= 0.0 and self.fused_greedy and self.cfg.vocab % 8 == 0
         can_tick = self.can_run_continuous and self.fused_greedy and self.cfg.vocab % 8 == 0
@@ -703,31 +824,16 @@ class TaHDecodeEngine:
                                   "(at most 32 rows, 256 (row, kv head) pairs, slabs of at most 4096 rows)")
             return self._generate_ticks(first_logits, max_new_tokens, eos, use_graph and dev.type == "cuda",
                                         temperature=temperature, **filters)
-        self.out_tokens.zero_()
-        self.out_len.zero_()
-        self.step_idx.zero_()
-        first = self.sample(first_logits, temperature, **filters)
-        if eos >= 0:
-            self.finished |= first == eos
-        keep = ~self.finished
-        self.out_tokens[:, 0] = torch.where(keep, first, torch.zeros_like(first))
-        self.out_len += keep.to(torch.int32)
-        self.tok.copy_(first)
-        self.step_idx += 1
-        n = max_new_tokens - 1
-        graph = self.capture(temperature, eos, **filters) if (use_graph and dev.type == "cuda" and n > 0) else None
-        done = 0
-        for i in range(n):
-            if graph is not None:
-                graph.replay()
-            else:
-                self._step_inplace(temperature, eos, **filters)
-            done += 1
-            if eos >= 0 and (i + 1) % check_every == 0 and bool(self.finished.all()):
-                break
-        self.host_positions += done
-        self.host_hard_rows += done
-        return self.out_tokens[:, :max_new_tokens]
+        return super().generate(first_logits, max_new_tokens, temperature=temperature, eos=eos, use_graph=use_graph,
+                                check_every=check_every, **filters)
+
+    def _check_room(self, max_new_tokens: int) -> None:
+        if self.host_positions + max_new_tokens > self.max_len or self.host_hard_rows + max_new_tokens > self.max_hard:
+            raise TahDuoError("generation would outgrow the KV slabs: construct the engine with a larger max_len / max_hard")
+
+    def _advanced(self, steps: int) -> None:
+        self.host_positions += steps
+        self.host_hard_rows += steps
 
     # ── rows at different latent iterations in one batch ─────────────────
     def _tick(self, parity: int, eos: int, limit: int, temperature: float = 0.0, **filters):
@@ -758,28 +864,21 @@ class TaHDecodeEngine:
                         hard_len=self.hard_len, n_hard=self.n_hard, n_steps=self.n_steps, chosen=chosen)
 
     def _launch_switches(self):
-        """Every attribute that changes which kernels a captured step launches: part of both graph keys, so that
-        flipping one between two generate() calls on the same prefill captures again instead of replaying a graph
-        of the old path."""
-        return (self.use_fused_glue, self.fused_greedy, self.fused_sampling, self.static_scratch, self.measure_without_attention, id(self.decider))
+        return super()._launch_switches() + (self.use_fused_glue, self.static_scratch, self.measure_without_attention, id(self.decider))
 
     def capture_ticks(self, eos: int, limit: int, temperature: float = 0.0, **filters):
         """The tick as two HIP graphs, one per logits buffer, after a warm-up tick whose state changes are undone."""
         key = (eos, limit, self.w.threshold, temperature, tuple(sorted(filters.items()))) + self._launch_switches()
         if self._tick_graphs is not None and self._tick_key == key:
             return self._tick_graphs
-        state = [t.clone() for t in self._state()]
-        lens = [sl.len.clone() for sl in self.slabs0 + self.slabs1]
+        undo = self._hold_state()
         s = torch.cuda.Stream()
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
             self._tick(0, eos, limit, temperature, **filters)
         torch.cuda.current_stream().wait_stream(s)
         torch.cuda.synchronize()
-        for t, old in zip(self._state(), state):
-            t.copy_(old)
-        for sl, ln in zip(self.slabs0 + self.slabs1, lens):
-            sl.len.copy_(ln)
+        undo()
         graphs = []
         for parity in (0, 1):
             g = torch.cuda.CUDAGraph()
@@ -829,31 +928,6 @@ class TaHDecodeEngine:
         self.host_positions += n_min
         self.host_hard_rows += n_min
         return self.out_tokens[:, :max_new_tokens]
-
-    def capture(self, temperature: float = 0.0, eos: int = -1, **filters):
-        """Captures one generation step in a HIP graph (after a warm-up step run on a side stream whose state
-        changes are undone, so that library workspaces exist before the capture)."""
-        key = (temperature, eos, tuple(sorted(filters.items()))) + self._launch_switches()
-        if self._graph is not None and self._graph_key == key:
-            return self._graph
-        state = [t.clone() for t in self._state()]
-        lens = [sl.len.clone() for sl in self.slabs0 + self.slabs1]
-        s = torch.cuda.Stream()
-        s.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(s):
-            self._step_inplace(temperature, eos, **filters)
-        torch.cuda.current_stream().wait_stream(s)
-        torch.cuda.synchronize()
-        # undo the warm-up step: state tensors and slab lengths (the rows it wrote lie beyond the lengths)
-        for t, old in zip(self._state(), state):
-            t.copy_(old)
-        for sl, ln in zip(self.slabs0 + self.slabs1, lens):
-            sl.len.copy_(ln)
-        g = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(g):
-            self._step_inplace(temperature, eos, **filters)
-        self._graph, self._graph_key = g, key
-        return g
 
 
 def generate(engine: TaHDecodeEngine, tokenizer, model_inputs: dict, *, max_new_tokens: int = 1024, do_sample: bool = True,

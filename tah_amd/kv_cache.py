@@ -190,3 +190,61 @@ def decode(q: torch.Tensor, q_slot: torch.Tensor, q_pos: torch.Tensor, c1: KvSla
     _call("duo_decode", q, o, lse, q_slot, q_pos, q_depth, int(depth), c1.k, c1.v, c1.start, c1.len, *two, ws, float(scale),
           out_packed)
     return (o, lse) if return_lse else o
+
+
+# ── what a sequence carries besides K/V slabs: latent rings, recurrent states, and the slots they belong to ──────────
+class LatentRing:
+    """One latent-attention layer's cache: per slot a ring of ``capacity`` rows, token p at row ``p % capacity``, a row
+    holding the latent (``rank_pad`` elements) and the rotated key part (``rot_pad``).  ``capacity`` is at least the widest
+    window of the layers that read it; nothing older is kept.  There is no length: what a position may see follows
+    from the position, and a sequence that starts over at position 0 sees nothing of the slot's earlier owner."""
+
+    def __init__(self, nslots: int, capacity: int, rank_pad: int, rot_pad: int, *, device, dtype):
+        self.rows = torch.zeros((nslots, capacity, rank_pad + rot_pad), dtype=dtype, device=device)
+
+
+class RecurrentState:
+    """One recurrent layer's state: ``state`` float32 [slots, heads, dim, vdim], and the short convolution's inputs of the
+    last ``taps`` tokens, ``conv`` [slots, taps, channels], token p at ``p % taps``.  Read as zero at position 0."""
+
+    def __init__(self, nslots: int, heads: int, dim: int, vdim: int, taps: int, channels: int, *, device, dtype):
+        self.state = torch.zeros((nslots, heads, dim, vdim), dtype=torch.float32, device=device)
+        self.conv = torch.zeros((nslots, taps, channels), dtype=dtype, device=device)
+
+
+class SlotPool:
+    """The sequence slots of an engine: which are taken, and how many tokens each has (host side)."""
+
+    def __init__(self, nslots: int, capacity: int):
+        self.nslots, self.capacity = nslots, capacity
+        self.length = [0] * nslots
+        self._free = list(range(nslots - 1, -1, -1))
+        self._taken = set()
+
+    def alloc(self) -> int:
+        if not self._free:
+            raise _capi.TahDuoError(f"all {self.nslots} sequence slots are taken")
+        s = self._free.pop()
+        self._taken.add(s)
+        self.length[s] = 0
+        return s
+
+    def release(self, slot: int) -> None:
+        if slot not in self._taken:
+            raise _capi.TahDuoError(f"slot {slot} is not taken")
+        self._taken.remove(slot)
+        self._free.append(slot)
+        self.length[slot] = 0
+
+    def take_all(self) -> None:
+        """Every slot taken and empty: a batch with one row per slot starts."""
+        self._free, self._taken = [], set(range(self.nslots))
+        self.length = [0] * self.nslots
+
+    def grow(self, slot: int, n: int) -> int:
+        """``n`` more tokens for the slot; returns the position of the first."""
+        at = self.length[slot]
+        if at + n > self.capacity:
+            raise _capi.TahDuoError(f"slot {slot}: {at} + {n} tokens exceed the cache capacity of {self.capacity}")
+        self.length[slot] = at + n
+        return at

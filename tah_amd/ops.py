@@ -20,6 +20,9 @@ def _call(name: str, *args):
         raise _capi.TahDuoError(str(e).split("\nException raised from")[0]) from None
 
 
+lib = _lib.lib  # the extension with the library loaded (kernel objects: Portions, DeltaLayer, LatentLayer)
+
+
 MAX_SCHEDULE_SEQS = 4095
 
 
@@ -246,7 +249,8 @@ def linear_rows(w_packed: torch.Tensor, x_packed: torch.Tensor, rows: int, n: in
                 residual: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
                 out_packed: Optional[torch.Tensor] = None, want_out: bool = True, norm_eps: Optional[float] = None,
                 bias: Optional[torch.Tensor] = None, relu: bool = False, gelu: bool = False,
-                ln_colsum: Optional[torch.Tensor] = None):
+                ln_colsum: Optional[torch.Tensor] = None, gelu_tanh: bool = False, batch: int = 1, shared_rows: bool = False,
+                packed_col_step: int = 0, select: Optional[torch.Tensor] = None):
     """A linear layer of a decode step on packed operands (``tah_linear_rows``), bf16, rows <= 32.
 
     ``x @ w.T`` [rows, N], plus ``residual`` [rows, N] when given (``out=residual`` updates it in place); with
@@ -257,14 +261,20 @@ def linear_rows(w_packed: torch.Tensor, x_packed: torch.Tensor, rows: int, n: in
     the weight's rows) ``norm_eps`` is a LayerNorm's: the product becomes ``(x @ w.T - mean(x) * ln_colsum) * rsqrt(var(x) +
     norm_eps)``, a layer behind a LayerNorm whose scale sits in w and whose shift sits in ``bias``.  ``out_packed`` [32 * N] also
     receives the result as the next layer's rows operand; ``want_out=False`` with ``out_packed`` writes only that.
-    Returns the row-major result (None when it was not asked for)."""
-    if relu and gelu:
+    Returns the row-major result (None when it was not asked for).
+
+    ``gelu_tanh``: the tanh form of gelu.  ``batch`` products of the same sizes in one launch: ``w_packed`` holds their weights
+    one after another, ``x_packed`` their rows operands (or one for all, ``shared_rows``), the results are [batch, rows, N] and
+    rows forms one after another -- or, with ``packed_col_step``, side by side in one rows form, ``packed_col_step`` columns
+    apart.  ``select`` (int32): only the products whose index it lists run (the others' results keep what they held)."""
+    if relu + gelu + gelu_tanh > 1:
         raise ValueError("linear_rows: one activation")
     norm = 0 if norm_eps is None else (2 if ln_colsum is not None else 1)
     if ln_colsum is not None and norm_eps is None:
         raise ValueError("linear_rows: ln_colsum needs the LayerNorm's eps")
     return _call("linear_rows", w_packed, x_packed, int(rows), int(n), int(k), bool(gate_up), residual, out, out_packed,
-                 bool(want_out), norm, float(norm_eps or 0.0), bias, 1 if relu else (2 if gelu else 0), ln_colsum)
+                 bool(want_out), norm, float(norm_eps or 0.0), bias, 1 if relu else (2 if gelu else (3 if gelu_tanh else 0)), ln_colsum,
+                 int(batch), bool(shared_rows), int(packed_col_step), select)
 
 
 def greedy_step(logits0, logits1, hard, eos: int, tok, finished, pos, out_tokens, step_idx, out_len, n_hard, n_steps) -> None:

@@ -1,4 +1,4 @@
-"""The C-ABI library loads without a GPU and exports every symbol include/tah_duo.h declares."""
+"""The C-ABI library loads without a GPU and exports every symbol include/tah_duo.h and include/tah_mixers.h declare."""
 import ctypes
 import os
 import re
@@ -7,7 +7,7 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
 def declared_symbols():
-    text = open(os.path.join(ROOT, "include", "tah_duo.h")).read()
+    text = "".join(open(os.path.join(ROOT, "include", n)).read() for n in ("tah_duo.h", "tah_mixers.h"))
     text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
     return sorted(set(re.findall(r"\b(tah_[a-z0-9_]+)\s*\(", text)))
 
@@ -18,7 +18,7 @@ def test_header_symbols_are_exported_and_bound():
     assert "tah_duo_fwd_varlen" in names and "tah_duo_bwd_varlen" in names and "tah_duo_decode" in names
     lib = ctypes.CDLL(_lib.LIB_PATH)
     for n in names:
-        assert hasattr(lib, n), f"{n} declared in include/tah_duo.h but not exported by libtah_duo.so"
+        assert hasattr(lib, n), f"{n} declared in include/ but not exported by libtah_duo.so"
     assert sorted(_capi.PROTOTYPES) == names
     bound = _capi.bind(lib)
     assert bound.tah_duo_abi_version() == _capi.ABI_VERSION
@@ -32,7 +32,8 @@ def test_torch_extension_loads_the_library_and_exposes_every_op():
     ext = _lib.lib()
     assert ext.loaded() and ext.abi_version() == _capi.ABI_VERSION
     for n in ("duo_fwd_varlen", "duo_bwd_varlen", "duo_fwd_masked", "duo_bwd_masked", "duo_decode", "decode_workspace_bytes",
-              "kv_append", "qk_prep", "hard_index_build", "pad_rows_build", "rows_copy", "topk_mix", "sample_rows", "qk_prep_bwd", "silu_mul"):
+              "kv_append", "qk_prep", "hard_index_build", "pad_rows_build", "rows_copy", "topk_mix", "sample_rows", "qk_prep_bwd", "silu_mul",
+              "embed_rows", "residual_norm", "activate_rows", "moe_route", "moe_plan", "moe_linear", "Portions", "DeltaLayer", "LatentLayer"):
         assert callable(getattr(ext, n))
 
 
@@ -49,12 +50,14 @@ def test_struct_sizes_match_c_layout(tmp_path):
              "tah_greedy_step_args": _capi.GreedyStepArgs, "tah_linear_rows_args": _capi.LinearRowsArgs,
              "tah_step_begin_args": _capi.StepBeginArgs, "tah_decider_tail_args": _capi.DeciderTailArgs,
              "tah_greedy_tick_args": _capi.GreedyTickArgs, "tah_sample_rows_args": _capi.SampleRowsArgs,
-             "tah_qk_prep_bwd_args": _capi.QkPrepBwdArgs}
+             "tah_qk_prep_bwd_args": _capi.QkPrepBwdArgs, "tah_embed_rows_args": _capi.EmbedRowsArgs,
+             "tah_residual_norm_args": _capi.ResidualNormArgs, "tah_delta_layer": _capi.DeltaLayer, "tah_portions": _capi.Portions,
+             "tah_latent_layer": _capi.LatentLayer, "tah_latent_prep_args": _capi.LatentPrepArgs}
     assert ctypes.sizeof(_capi.DuoStream) == 9 * 8 + 8 * 8 + 2 * 4
     if shutil.which("gcc") is None:
         return
     src = tmp_path / "sizes.c"
-    src.write_text('#include <stdio.h>\n#include "tah_duo.h"\nint main(void) {\n' +
+    src.write_text('#include <stdio.h>\n#include "tah_mixers.h"\nint main(void) {\n' +
                    "".join(f'  printf("{n} %zu\\n", sizeof({n}));\n' for n in pairs) + "  return 0;\n}\n")
     exe = tmp_path / "sizes"
     subprocess.check_call(["gcc", "-I", os.path.join(ROOT, "include"), str(src), "-o", str(exe)])
