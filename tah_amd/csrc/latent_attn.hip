@@ -7,7 +7,15 @@
 //    the per-head products.
 //  * latent_context_kernel / latent_append_kernel: the rows a batch of portions can see, packed (old ones from the
 //    ring, new ones from the portion), then the new rows into the ring.
-//  * attend_rows_kernel: one workgroup per (query, head), any sizes, either element type.
+//  * attend_tile_kernel (bf16): portions.  128 query rows of one head per workgroup against 64 keys at a time, on the
+//    matrix cores: S^T = K Q^T, so that a query's scores sit in one lane column and the softmax needs two shuffles, and
+//    O^T = V^T P^T with V^T read from the row-major tile by transpose reads.  Keys outside the window are not visited.
+//  * latent_decode_kernel / latent_merge_kernel (bf16): single tokens.  All heads (sixteen at a time) of one row share a
+//    pass over the ring, which is both keys and values; the window is split over workgroups, and the parts are merged.
+//  * attend_rows_kernel: one workgroup per (query, head), any sizes, either element type (the float32 form).
+//
+// Scores, weights and sums are float32.  Where a weight enters a bf16 matrix product it goes in as two bf16 terms
+// (its rounding and what the rounding left), so that it keeps sixteen bits.
 #include <hip/hip_runtime.h>
 
 #include "mixer_device.h"
@@ -198,6 +206,361 @@ __global__ __launch_bounds__(kLatThreads) void attend_rows_kernel(const AttendRo
     }
 }
 
+// ---- bf16 on the matrix cores ------------------------------------------------------------------------------------
+constexpr int kTileKeys = 64, kTileRows = 128;
+constexpr float kNoScore = -1e30f;  // below every score, and finite: differences of it are numbers
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+__device__ __forceinline__ bf16x8 join8(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
+
+// x over the four lane groups that share l % 16
+__device__ __forceinline__ float groups_max(float x) {
+    x = fmaxf(x, __shfl_xor(x, 16));
+    return fmaxf(x, __shfl_xor(x, 32));
+}
+__device__ __forceinline__ float groups_sum(float x) {
+    x += __shfl_xor(x, 16);
+    return x + __shfl_xor(x, 32);
+}
+
+struct AttendTile {
+    const __bf16 *q, *k, *v, *ctx;  // q: head base [dim_pad | rot_pad]; ctx: rotated key part of context row 0
+    int64_t q_rs, k_rs, v_rs, ctx_rs;
+    __bf16* out;
+    int64_t out_rs;
+    const int32_t *cu, *cu_k;
+    int32_t nseq, dim_pad, rot_pad, vdim_pad, window;
+    float scale_log2;
+};
+
+// NQ: 32-wide steps of a query row (at most), NV: 16-wide tiles of a value row (at most).
+template <int NQ, int NV>
+__global__ __launch_bounds__(kLatThreads) void attend_tile_kernel(const AttendTile p) {
+    HIP_DYNAMIC_SHARED(unsigned char, tile_lds)
+    int tile = blockIdx.x, b = 0, row0 = 0, row_end = 0;
+    if (!find_tile(p.cu, p.nseq, kTileRows, tile, b, row0, row_end)) return;
+    const int h = blockIdx.y, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int dq = p.dim_pad + p.rot_pad, nq = dq / 32, nv = p.vdim_pad / 16;
+    const int ks = dq + 8, vs = p.vdim_pad + 8;  // row strides in LDS: rows start in different banks
+    __bf16* const kt = reinterpret_cast<__bf16*>(tile_lds);
+    __bf16* const vt = kt + kTileKeys * ks;
+    const int first = p.cu[b], n = p.cu[b + 1] - first, k0 = p.cu_k[b], lk = p.cu_k[b + 1] - k0;
+    // a query row's own key, as a context row of its sequence: row - first + lk - n
+    const int shift = lk - n - first;
+    const int wrow = row0 + 32 * wave;
+    bf16x8 q[2][NQ];
+    int own[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        int r = wrow + 16 * t + c;
+        r = r < row_end ? r : row_end - 1;  // rows past the end repeat the last one and are not stored
+        own[t] = r + shift;
+#pragma unroll
+        for (int s = 0; s < NQ; ++s)
+            if (s < nq) q[t][s] = *reinterpret_cast<const bf16x8*>(p.q + (int64_t)r * p.q_rs + (int64_t)h * dq + 32 * s + 8 * g);
+    }
+    const int own_lo = (wrow < row_end ? wrow : row_end - 1) + shift;
+    const int own_hi = (wrow + 31 < row_end ? wrow + 31 : row_end - 1) + shift;
+    int j_lo = row0 + shift - p.window + 1;
+    j_lo = j_lo < 0 ? 0 : j_lo;
+    const int j_hi = row_end - 1 + shift;
+    f32x4 acc[NV][2];
+    float m[2] = {kNoScore, kNoScore}, l[2] = {0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+        for (int t = 0; t < 2; ++t) acc[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    // a thread's sixteen-byte units of a tile: NQ of the keys, NV / 2 of the values
+    constexpr int UV = (NV + 1) / 2;
+    const int uk = dq / 8, ukn = p.dim_pad / 8, uv = p.vdim_pad / 8;
+    bf16x8 fk[NQ], fv[UV];
+    auto fetch = [&](int j0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < NQ; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (i < nq) {
+                const int key = u / uk, x = u % uk;
+                int j = j0 + key;
+                j = (j < lk ? j : lk - 1) + k0;
+                fk[i] = *reinterpret_cast<const bf16x8*>(x < ukn ? p.k + j * p.k_rs + (int64_t)h * p.dim_pad + 8 * x : p.ctx + j * p.ctx_rs + 8 * (x - ukn));
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < UV; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (u < kTileKeys * uv) {
+                const int key = u / uv, x = u % uv;
+                int j = j0 + key;
+                j = (j < lk ? j : lk - 1) + k0;
+                fv[i] = *reinterpret_cast<const bf16x8*>(p.v + j * p.v_rs + (int64_t)h * p.vdim_pad + 8 * x);
+            }
+        }
+    };
+    fetch(j_lo);
+    for (int j0 = j_lo; j0 <= j_hi; j0 += kTileKeys) {
+#pragma unroll
+        for (int i = 0; i < NQ; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (i < nq) *reinterpret_cast<bf16x8*>(kt + (u / uk) * ks + 8 * (u % uk)) = fk[i];
+        }
+#pragma unroll
+        for (int i = 0; i < UV; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (u < kTileKeys * uv) *reinterpret_cast<bf16x8*>(vt + (u / uv) * vs + 8 * (u % uv)) = fv[i];
+        }
+        __syncthreads();
+        if (j0 + kTileKeys <= j_hi) fetch(j0 + kTileKeys);
+        // (uniform per wave) does this wave see anything of the tile, and does it see all of it?
+        const bool any = j0 <= own_hi && j0 + kTileKeys - 1 > own_lo - p.window;
+        const bool all = j0 + kTileKeys - 1 <= own_lo && j0 > own_hi - p.window;
+        if (any) {
+            f32x4 sc[4][2];
+#pragma unroll
+            for (int x = 0; x < 4; ++x) {
+#pragma unroll
+                for (int t = 0; t < 2; ++t) sc[x][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < NQ; ++s)
+                    if (s < nq) {
+                        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + (16 * x + c) * ks + 32 * s + 8 * g);
+#pragma unroll
+                        for (int t = 0; t < 2; ++t) sc[x][t] = mfma16(a, q[t][s], sc[x][t]);
+                    }
+            }
+            bf16x8 ph[2][2], pl[2][2];  // [pair of key tiles][query tile]
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                float mx = kNoScore;
+#pragma unroll
+                for (int x = 0; x < 4; ++x)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        float y = sc[x][t][r] * p.scale_log2;
+                        const int j = j0 + 16 * x + 4 * g + r;
+                        if (!all && (j > own[t] || j <= own[t] - p.window)) y = kNegInf;
+                        sc[x][t][r] = y;
+                        mx = fmaxf(mx, y);
+                    }
+                mx = fmaxf(m[t], groups_max(mx));
+                const float a = fast_exp2(m[t] - mx);
+                m[t] = mx;
+                float sum = 0.f;
+#pragma unroll
+                for (int x = 0; x < 4; ++x)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const float w = fast_exp2(sc[x][t][r] - mx);
+                        sum += w;
+                        const __bf16 hi = (__bf16)w;
+                        ph[x / 2][t][4 * (x % 2) + r] = hi;
+                        pl[x / 2][t][4 * (x % 2) + r] = (__bf16)(w - (float)hi);
+                    }
+                l[t] = l[t] * a + sum;
+                if (__ballot(a != 1.0f) != 0) {
+#pragma unroll
+                    for (int i = 0; i < NV; ++i)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) acc[i][t][r] *= a;
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+                if (i < nv) {
+#pragma unroll
+                    for (int x = 0; x < 2; ++x) {
+                        const __bf16* at = vt + (32 * x + 4 * g + c / 4) * vs + 16 * i + 4 * (c % 4);
+                        const bf16x8 a = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
+                                               lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * vs)));
+#pragma unroll
+                        for (int t = 0; t < 2; ++t) {
+                            acc[i][t] = mfma16(a, ph[x][t], acc[i][t]);
+                            acc[i][t] = mfma16(a, pl[x][t], acc[i][t]);
+                        }
+                    }
+                }
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        const float inv = 1.0f / groups_sum(l[t]);
+        const int r = wrow + 16 * t + c;
+        if (r < row_end) {
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+                if (i < nv) {
+                    bf16x4 y;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) y[e] = (__bf16)(acc[i][t][e] * inv);
+                    *reinterpret_cast<bf16x4*>(p.out + (int64_t)r * p.out_rs + (int64_t)h * p.vdim_pad + 16 * i + 4 * g) = y;
+                }
+        }
+    }
+}
+
+struct LatentDecode {
+    const __bf16 *q_latent, *q_rot, *ring;
+    int64_t q_latent_hs, q_rs;
+    const int32_t *slot, *pos;
+    float* part;  // [rows][heads padded to 16][splits]: rank_pad sums, the maximum, the sum of weights
+    int32_t heads, dim_pad, rot_pad, rank_pad, capacity, nslots, window, rows, splits, tiles_per_split;
+    float scale_log2;
+};
+
+// grid (splits, groups of 16 heads, rows).  NT: 16-wide tiles of the latent per wave (at most); NU: 16-byte units of a key
+// tile per thread (at most).
+template <int NT, int NU>
+__global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const LatentDecode p) {
+    HIP_DYNAMIC_SHARED(unsigned char, dec_lds)
+    __shared__ float mx_[kLatWaves][16], sum_[kLatWaves][16];
+    const int row = blockIdx.z, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int lp = p.rank_pad + p.rot_pad, steps = lp / 32, nt = p.rank_pad / 16, ks = lp + 8, ps = kTileKeys + 8;
+    __bf16* const kt = reinterpret_cast<__bf16*>(dec_lds);  // [64 keys][ks]
+    __bf16* const qt = kt + kTileKeys * ks;                 // [16 heads][ks]
+    __bf16* const pt = qt + 16 * ks;                        // [2 terms][16 heads][ps]
+    const int pos = p.pos[row];
+    int slot = p.slot[row];
+    if (slot >= p.nslots) slot = -1;
+    const bool live = slot >= 0 && pos >= 0;
+    const int units = kTileKeys * lp / 8, upk = lp / 8;
+    const __bf16* const ring = p.ring + (int64_t)(slot < 0 ? 0 : slot) * p.capacity * lp;
+    int lo = pos - p.window + 1;
+    lo = lo < 0 ? 0 : lo;
+    const int begin = lo + blockIdx.x * p.tiles_per_split * kTileKeys;
+    int end = begin + p.tiles_per_split * kTileKeys - 1;
+    end = end < pos ? end : pos;
+    if (!live) end = begin - 1;
+    bf16x8 fk[NU];
+    auto fetch = [&](int j0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (u < units) {
+                int j = j0 + u / upk;
+                j = j < end ? j : end;
+                fk[i] = *reinterpret_cast<const bf16x8*>(ring + (int64_t)(j % p.capacity) * lp + 8 * (u % upk));
+            }
+        }
+    };
+    if (begin <= end) fetch(begin);
+    for (int u = tid; u < 16 * upk; u += kLatThreads) {
+        int h = blockIdx.y * 16 + u / upk;
+        h = h < p.heads ? h : p.heads - 1;  // heads past the last one repeat it; nobody reads them
+        const int x = 8 * (u % upk);
+        const __bf16* src = x < p.rank_pad ? p.q_latent + h * p.q_latent_hs + (int64_t)row * p.rank_pad + x
+                                           : p.q_rot + (int64_t)row * p.q_rs + (int64_t)h * (p.dim_pad + p.rot_pad) + x - p.rank_pad;
+        *reinterpret_cast<bf16x8*>(qt + (u / upk) * ks + x) = *reinterpret_cast<const bf16x8*>(src);
+    }
+    f32x4 acc[NT];
+#pragma unroll
+    for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = kNoScore, l = 0.f;
+    for (int j0 = begin; j0 <= end; j0 += kTileKeys) {
+#pragma unroll
+        for (int i = 0; i < NU; ++i) {
+            const int u = tid + kLatThreads * i;
+            if (u < units) *reinterpret_cast<bf16x8*>(kt + (u / upk) * ks + 8 * (u % upk)) = fk[i];
+        }
+        __syncthreads();
+        if (j0 + kTileKeys <= end) fetch(j0 + kTileKeys);
+        // scores of this wave's sixteen keys: register r of lane (c, g) is key 16 wave + 4 g + r, head c
+        f32x4 sc = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < steps; ++s)
+            sc = mfma16(*reinterpret_cast<const bf16x8*>(kt + (16 * wave + c) * ks + 32 * s + 8 * g),
+                        *reinterpret_cast<const bf16x8*>(qt + c * ks + 32 * s + 8 * g), sc);
+        float mw = kNoScore;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            sc[r] = j0 + 16 * wave + 4 * g + r <= end ? sc[r] * p.scale_log2 : kNegInf;
+            mw = fmaxf(mw, sc[r]);
+        }
+        mw = groups_max(mw);
+        if (g == 0) mx_[wave][c] = mw;
+        __syncthreads();
+        const float mn = fmaxf(m, fmaxf(fmaxf(mx_[0][c], mx_[1][c]), fmaxf(mx_[2][c], mx_[3][c])));
+        const float a = fast_exp2(m - mn);
+        m = mn;
+        bf16x4 hi, rest;
+        l *= a;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float w = fast_exp2(sc[r] - mn);
+            l += w;
+            hi[r] = (__bf16)w;
+            rest[r] = (__bf16)(w - (float)hi[r]);
+        }
+        *reinterpret_cast<bf16x4*>(pt + c * ps + 16 * wave + 4 * g) = hi;
+        *reinterpret_cast<bf16x4*>(pt + (16 + c) * ps + 16 * wave + 4 * g) = rest;
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[i][r] *= a;
+        __syncthreads();
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+            const __bf16* pr = pt + c * ps + 32 * x + 4 * g;
+            const bf16x8 ph = join8(*reinterpret_cast<const bf16x4*>(pr), *reinterpret_cast<const bf16x4*>(pr + 16));
+            const bf16x8 pl = join8(*reinterpret_cast<const bf16x4*>(pr + 16 * ps), *reinterpret_cast<const bf16x4*>(pr + 16 * ps + 16));
+#pragma unroll
+            for (int i = 0; i < NT; ++i) {
+                const int t = wave + kLatWaves * i;
+                if (t < nt) {
+                    const __bf16* at = kt + (32 * x + 4 * g + c / 4) * ks + 16 * t + 4 * (c % 4);
+                    const bf16x8 v = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
+                                           lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * ks)));
+                    acc[i] = mfma16(v, ph, acc[i]);
+                    acc[i] = mfma16(v, pl, acc[i]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    l = groups_sum(l);
+    if (g == 0) sum_[wave][c] = l;
+    __syncthreads();
+    const int hp = gridDim.y * 16;
+    float* const out = p.part + (((int64_t)row * hp + blockIdx.y * 16 + c) * p.splits + blockIdx.x) * (p.rank_pad + 2);
+    if (begin <= end) {
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            const int t = wave + kLatWaves * i;
+            if (t < nt) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) out[16 * t + 4 * g + r] = acc[i][r];
+            }
+        }
+    }
+    if (tid < 16) {
+        out[p.rank_pad] = m;
+        out[p.rank_pad + 1] = (sum_[0][c] + sum_[1][c]) + (sum_[2][c] + sum_[3][c]);  // 0: nothing seen, no sums written
+    }
+}
+
+// grid (heads, rows)
+__global__ __launch_bounds__(kLatThreads) void latent_merge_kernel(const float* part, int hp, int splits, int rank_pad, int rows, __bf16* out_packed,
+                                                                   __bf16* out_rows) {
+    const int h = blockIdx.x, row = blockIdx.y;
+    const float* const base = part + ((int64_t)row * hp + h) * splits * (rank_pad + 2);
+    float m = kNoScore, l = 0.f;
+    for (int s = 0; s < splits; ++s)
+        if (base[(int64_t)s * (rank_pad + 2) + rank_pad + 1] > 0.f) m = fmaxf(m, base[(int64_t)s * (rank_pad + 2) + rank_pad]);
+    for (int s = 0; s < splits; ++s) {
+        const float* x = base + (int64_t)s * (rank_pad + 2) + rank_pad;
+        if (x[1] > 0.f) l += x[1] * fast_exp2(x[0] - m);
+    }
+    for (int i = threadIdx.x; i < rank_pad; i += kLatThreads) {
+        float y = 0.f;
+        for (int s = 0; s < splits; ++s) {
+            const float* x = base + (int64_t)s * (rank_pad + 2);
+            if (x[rank_pad + 1] > 0.f) y += x[i] * fast_exp2(x[rank_pad] - m);
+        }
+        y = l > 0.f ? y / l : 0.f;
+        if (out_packed) out_packed[(int64_t)h * 32 * rank_pad + rows_form_elem(row, i)] = (__bf16)y;
+        if (out_rows) out_rows[((int64_t)h * rows + row) * rank_pad + i] = (__bf16)y;
+    }
+}
+
 int check_layer(const tah_latent_layer* L) {
     if (!L) return TAH_E_NULL;
     if (L->heads <= 0 || L->heads > 65535 || L->dim_pad <= 0 || L->dim_pad % 32 != 0 || L->rot_dim < 0 || L->rot_dim % 2 != 0 ||
@@ -221,6 +584,39 @@ void launch_attend_rows(const AttendRows& p, int heads, int dtype, hipStream_t s
     else hipLaunchKernelGGL((attend_rows_kernel<float>), dim3(p.rows, heads), dim3(kLatThreads), lds, st, p);
 }
 size_t elem_bytes(int dtype) { return dtype == TAH_DT_BF16 ? 2 : 4; }
+
+template <int NQ, int NV>
+int launch_attend_tile(const AttendTile& p, int slots, int heads, hipStream_t st) {
+    const size_t lds = (size_t)kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 8) * 2;
+    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                           (int)lds) != hipSuccess)
+        return TAH_E_LAUNCH;
+    hipLaunchKernelGGL((attend_tile_kernel<NQ, NV>), dim3(slots, heads), dim3(kLatThreads), lds, st, p);
+    return launch_status();
+}
+
+// how a decode call splits its window: enough workgroups for the chip, whole tiles of 64 keys each
+constexpr int kDecodeGroups = 512;
+void decode_split(int heads, int rows, int window, int& splits, int& tiles_per_split) {
+    const int tiles = (window + kTileKeys - 1) / kTileKeys, groups = rows * ((heads + 15) / 16);
+    int want = groups > 0 ? kDecodeGroups / groups : 1;
+    want = want < 1 ? 1 : (want > tiles ? tiles : want);
+    tiles_per_split = (tiles + want - 1) / want;
+    splits = (tiles + tiles_per_split - 1) / tiles_per_split;
+}
+size_t decode_lds(int lp) { return ((size_t)(kTileKeys + 16) * (lp + 8) + 2 * 16 * (kTileKeys + 8)) * 2; }
+constexpr size_t kLdsBytes = 160 * 1024 - 1024;  // a compute unit's LDS, less the kernel's static part
+bool decode_on_tiles(const tah_latent_layer* L) { return L->dtype == TAH_DT_BF16 && decode_lds(L->rank_pad + L->rot_pad) <= kLdsBytes; }
+
+template <int NT, int NU>
+int launch_latent_decode(const LatentDecode& p, hipStream_t st) {
+    const size_t lds = decode_lds(p.rank_pad + p.rot_pad);
+    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NT, NU>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                           (int)lds) != hipSuccess)
+        return TAH_E_LAUNCH;
+    hipLaunchKernelGGL((latent_decode_kernel<NT, NU>), dim3(p.splits, (p.heads + 15) / 16, p.rows), dim3(kLatThreads), lds, st, p);
+    return launch_status();
+}
 
 }  // namespace
 }  // namespace tah
@@ -275,6 +671,22 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
     if (p->rows == 0 || p->nseq == 0) return TAH_OK;
     if (!cu_k || !q || !k || !v || !ctx || !out) return TAH_E_NULL;
     if (!aligned_16(q) || !aligned_16(k) || !aligned_16(v) || !aligned_16(ctx) || !aligned_16(out)) return TAH_E_ALIGN;
+    const int nq = (L->dim_pad + L->rot_pad) / 32, nv = (L->vdim_pad + 15) / 16;
+    if (L->dtype == TAH_DT_BF16 && nq <= 10 && nv <= 16) {
+        AttendTile t{};
+        t.q = static_cast<const __bf16*>(q); t.k = static_cast<const __bf16*>(k); t.v = static_cast<const __bf16*>(v);
+        t.ctx = static_cast<const __bf16*>(ctx) + L->rank_pad;
+        t.q_rs = q_rs; t.k_rs = k_rs; t.v_rs = v_rs; t.ctx_rs = L->rank_pad + L->rot_pad;
+        t.out = static_cast<__bf16*>(out); t.out_rs = out_rs;
+        t.cu = p->cu; t.cu_k = cu_k; t.nseq = p->nseq;
+        t.dim_pad = L->dim_pad; t.rot_pad = L->rot_pad; t.vdim_pad = L->vdim_pad; t.window = L->window;
+        t.scale_log2 = L->scale * kLog2e;
+        hipStream_t st = static_cast<hipStream_t>(stream);
+        const int slots = p->rows / kTileRows + p->nseq;
+        if (nq <= 4 && nv <= 4) return launch_attend_tile<4, 4>(t, slots, L->heads, st);
+        if (nq <= 6 && nv <= 8) return launch_attend_tile<6, 8>(t, slots, L->heads, st);
+        return launch_attend_tile<10, 16>(t, slots, L->heads, st);
+    }
     AttendRows a{};
     a.q1 = q; a.q1_rs = q_rs; a.q1_hs = L->dim_pad + L->rot_pad; a.n1 = L->dim_pad;
     a.q2 = static_cast<const char*>(q) + (size_t)L->dim_pad * elem_bytes(L->dtype); a.q2_rs = q_rs; a.q2_hs = a.q1_hs; a.n2 = L->rot_pad;
@@ -289,20 +701,42 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
 }
 
 extern "C" size_t tah_latent_decode_workspace(const tah_latent_layer* L, int32_t rows) {
-    (void)L; (void)rows;
-    return 0;
+    if (tah::check_layer(L) != TAH_OK || rows <= 0 || !tah::decode_on_tiles(L)) return 0;
+    const size_t groups = (size_t)rows * ((L->heads + 15) / 16);
+    return (groups > tah::kDecodeGroups ? groups : (size_t)tah::kDecodeGroups) * 16 * (L->rank_pad + 2) * sizeof(float);  // enough for fewer rows too
 }
 
 extern "C" int tah_latent_decode(const tah_latent_layer* L, const int32_t* slot, const int32_t* pos, int32_t rows, const void* q_latent,
                                  int64_t q_latent_hs, const void* q, int64_t q_rs, void* out_packed, void* out_rows, void* workspace,
                                  size_t workspace_bytes, tah_stream_t stream) {
     using namespace tah;
-    (void)workspace; (void)workspace_bytes;
     if (const int rc = check_layer(L)) return rc;
     if (rows < 0 || (out_packed && rows > 32) || q_rs % 8 != 0 || q_latent_hs % 8 != 0 || L->window > L->capacity) return TAH_E_SHAPE;
     if (rows == 0) return TAH_OK;
     if (!slot || !pos || !q_latent || !q || (!out_packed && !out_rows)) return TAH_E_NULL;
     if (!aligned_16(q_latent) || !aligned_16(q) || !aligned_16(out_packed) || !aligned_16(out_rows)) return TAH_E_ALIGN;
+    if (decode_on_tiles(L)) {
+        LatentDecode d{};
+        d.q_latent = static_cast<const __bf16*>(q_latent); d.q_latent_hs = q_latent_hs;
+        d.q_rot = static_cast<const __bf16*>(q) + L->dim_pad; d.q_rs = q_rs;
+        d.ring = static_cast<const __bf16*>(L->ring); d.slot = slot; d.pos = pos; d.part = static_cast<float*>(workspace);
+        d.heads = L->heads; d.dim_pad = L->dim_pad; d.rot_pad = L->rot_pad; d.rank_pad = L->rank_pad; d.capacity = L->capacity; d.nslots = L->nslots;
+        d.window = L->window; d.rows = rows; d.scale_log2 = L->scale * kLog2e;
+        decode_split(L->heads, rows, L->window, d.splits, d.tiles_per_split);
+        const int hp = (L->heads + 15) / 16 * 16;
+        if (!workspace || workspace_bytes < (size_t)rows * hp * d.splits * (L->rank_pad + 2) * sizeof(float)) return TAH_E_WORKSPACE;
+        hipStream_t st = static_cast<hipStream_t>(stream);
+        const int lp = L->rank_pad + L->rot_pad;
+        int rc;
+        if (lp <= 128) rc = launch_latent_decode<2, 4>(d, st);
+        else if (lp <= 320) rc = launch_latent_decode<5, 10>(d, st);
+        else if (lp <= 576) rc = launch_latent_decode<9, 18>(d, st);
+        else rc = launch_latent_decode<16, 32>(d, st);
+        if (rc != TAH_OK) return rc;
+        hipLaunchKernelGGL(latent_merge_kernel, dim3(L->heads, rows), dim3(kLatThreads), 0, st, static_cast<const float*>(workspace), hp, (int)d.splits,
+                           (int)L->rank_pad, (int)rows, static_cast<__bf16*>(out_packed), static_cast<__bf16*>(out_rows));
+        return launch_status();
+    }
     AttendRows a{};
     a.q1 = q_latent; a.q1_rs = L->rank_pad; a.q1_hs = q_latent_hs; a.n1 = L->rank_pad;
     a.q2 = static_cast<const char*>(q) + (size_t)L->dim_pad * elem_bytes(L->dtype); a.q2_rs = q_rs; a.q2_hs = L->dim_pad + L->rot_pad; a.n2 = L->rot_pad;

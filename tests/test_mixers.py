@@ -1,0 +1,115 @@
+"""Layer mechanisms (tah_amd.mixers, include/tah_mixers.h), each alone, against the plain oracle: on the CPU execution build
+at small sizes, on the GPU at those and at larger ones."""
+import pytest
+
+from tests import emu_util
+from tests import zozosun_cases as Z
+
+needs_clang = pytest.mark.skipif(not emu_util.have_host_clang(), reason="host clang++ not available")
+BOTH = pytest.mark.parametrize("dtype", ["f32", "bf16"])
+
+
+def delta(heads, kv, dim, vdim, conv, eps=1e-4):
+    return {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv, "eps": eps}
+
+
+def latent(heads, dim, rot, vdim, rank, window, base=50.0, scale=0.4):
+    return Z.latent_of(heads, dim, rot, vdim, rank, window, base, scale)["mixer"]
+
+
+# (sizes, lengths, portions per sequence)
+DELTA_SMALL = [(delta(2, 1, 6, 5, 3), (5, 3), ((2, 3), (3,))), (delta(2, 2, 12, 8, 4), (7, 2), ((7,), (2,)))]
+DELTA_GPU = DELTA_SMALL + [
+    (delta(6, 3, 40, 24, 4), (70, 33), ((37, 2, 31), (2, 31))), (delta(4, 4, 64, 64, 2), (130, 5), ((128, 2), (3, 2))),
+    (delta(8, 2, 128, 128, 4), (200, 65), ((64, 17, 119), (65,))), (delta(2, 1, 256, 96, 4), (40, 40), ((40,), (17, 23))),
+    (delta(3, 1, 17, 130, 1), (30, 9), ((16, 14), (9,))), (delta(2, 2, 100, 256, 5), (21, 2), ((5, 16), (2,))),
+    (delta(5, 5, 32, 512, 3), (19, 18), ((19,), (2, 16))),
+]
+# (sizes, prompt, portions, decoded tokens, ring capacity)
+LATENT_SMALL = [(latent(2, 8, 4, 6, 10, 4), 9, (2, 5, 2), 3, None), (latent(1, 32, 6, 16, 40, 3), 6, (6,), 2, 5)]
+LATENT_GPU = LATENT_SMALL + [
+    (latent(3, 24, 8, 20, 48, 40), 150, (64, 2, 84), 45, None), (latent(16, 128, 64, 128, 512, 100), 300, (300,), 70, 130),
+    (latent(20, 64, 32, 64, 96, 65), 129, (1 + 63, 65), 66, 65), (latent(5, 64, 16, 200, 64, 7), 40, (7, 2, 31), 9, None),
+    (latent(2, 96, 32, 96, 288, 128), 260, (128, 132), 4, 200), (latent(33, 32, 32, 32, 32, 2), 20, (20,), 3, None),
+    (latent(4, 200, 40, 48, 700, 33), 70, (3, 67), 5, None), (latent(2, 400, 6, 300, 64, 9), 21, (21,), 3, None),
+    (latent(2, 32, 2, 16, 960, 5), 12, (12,), 2, None),
+]
+MOE_SMALL = [(5, 40, 12, 4, 2, 9), (3, 32, 32, 3, 1, 0)]
+MOE_GPU = MOE_SMALL + [(32, 96, 48, 16, 4, 64), (200, 160, 96, 8, 8, 32), (700, 256, 192, 64, 6, 128), (31, 512, 100, 7, 3, 0), (300, 72, 40, 5, 5, 17)]
+
+
+# ── CPU execution build ──────────────────────────────────────────────────────────────────────────────────────────────
+@needs_clang
+@BOTH
+def test_rows_on_cpu_shim(dtype):
+    with emu_util.emulated():
+        Z.rows_case("cpu", Z.DTYPES[dtype])
+
+
+@needs_clang
+def test_linear_batches_on_cpu_shim():
+    with emu_util.emulated():
+        Z.linear_batch_case("cpu", 3, 16, 32, 3)
+
+
+@needs_clang
+@BOTH
+@pytest.mark.parametrize("case", range(len(DELTA_SMALL)))
+def test_delta_rule_on_cpu_shim(dtype, case):
+    m, lens, cuts = DELTA_SMALL[case]
+    with emu_util.emulated():
+        Z.delta_case("cpu", Z.DTYPES[dtype], m, lens, cuts, steps=2)
+
+
+@needs_clang
+@BOTH
+@pytest.mark.parametrize("case", range(len(LATENT_SMALL)))
+def test_latent_attention_on_cpu_shim(dtype, case):
+    m, total, cuts, steps, cap = LATENT_SMALL[case]
+    with emu_util.emulated():
+        Z.latent_case("cpu", Z.DTYPES[dtype], m, total, cuts, steps, cap)
+
+
+@needs_clang
+@BOTH
+@pytest.mark.parametrize("case", range(len(MOE_SMALL)))
+def test_mixture_of_experts_on_cpu_shim(dtype, case):
+    with emu_util.emulated():
+        Z.moe_case("cpu", Z.DTYPES[dtype], *MOE_SMALL[case])
+
+
+# ── GPU ──────────────────────────────────────────────────────────────────────────────────────────────────────────────
+@pytest.mark.gpu
+@BOTH
+@pytest.mark.parametrize("rows,width,cols", [(5, 72, 96), (32, 2048, 2048), (40, 100, 104), (3, 5000, 5024), (2, 16384, 16384)])
+def test_rows_gpu(dtype, rows, width, cols):
+    Z.rows_case("cuda", Z.DTYPES[dtype], rows, width, cols)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("rows,n,k,batch", [(3, 16, 32, 3), (32, 512, 128, 16), (20, 128, 512, 16), (7, 48, 96, 1), (32, 96, 256, 5)])
+def test_linear_batches_gpu(rows, n, k, batch):
+    Z.linear_batch_case("cuda", rows, n, k, batch)
+
+
+@pytest.mark.gpu
+@BOTH
+@pytest.mark.parametrize("case", range(len(DELTA_GPU)))
+def test_delta_rule_gpu(dtype, case):
+    m, lens, cuts = DELTA_GPU[case]
+    Z.delta_case("cuda", Z.DTYPES[dtype], m, lens, cuts, steps=4)
+
+
+@pytest.mark.gpu
+@BOTH
+@pytest.mark.parametrize("case", range(len(LATENT_GPU)))
+def test_latent_attention_gpu(dtype, case):
+    m, total, cuts, steps, cap = LATENT_GPU[case]
+    Z.latent_case("cuda", Z.DTYPES[dtype], m, total, cuts, steps, cap)
+
+
+@pytest.mark.gpu
+@BOTH
+@pytest.mark.parametrize("case", range(len(MOE_GPU)))
+def test_mixture_of_experts_gpu(dtype, case):
+    Z.moe_case("cuda", Z.DTYPES[dtype], *MOE_GPU[case])
