@@ -728,6 +728,87 @@ def bench_e2e_decode(new_tokens: int, B: int = 32, prompt_len: int = 512, temper
             "prefill_s": prefill_s, "weight_bytes": params * 2, "mean_context_at_end": ctx}
 
 
+STACK_SIZES = {  # prompts (sequences x tokens), and decode batches at a context
+    "prefill": [(1, 8192), (4, 2048), (1, 1024)],
+    "decode": [(32, 1536), (8, 1536), (1, 1536)],
+}
+
+
+def stack_config(layers: int = 12, width: int = 2048, vocab: int = 151936):
+    """A Zozosun model with the layer sizes of a few-billion-parameter model: three delta-rule layers to each latent-attention
+    layer, every second feed-forward a mixture of 64 experts."""
+    delta = {"heads": 32, "kv_heads": 16, "dim": 128, "vdim": 128, "conv": 4}
+    latent = {"heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "rot": {"base": 1e6, "dims": 64},
+              "mask": {"size": 1024}}
+    dense = {"kind": "dense", "ff": 6144}
+    moe = {"kind": "moe", "router": {"experts": 64, "top": 8}, "expert": {"ff": 768}, "shared": {"ff": 768}}
+    out = []
+    for i in range(layers):
+        is_latent = i % 4 == 3
+        out.append({"type": "latent_attention" if is_latent else "delta", "mixer": dict(latent if is_latent else delta),
+                    "mlp": moe if i % 2 else dense})
+    return {"architecture": "Zozosun", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out}
+
+
+def bench_stack(steps: int, warmup: int, layers: int = 12):
+    """Prefill and decode throughput of a Zozosun model at the layer sizes of a real one (random weights), beside the Qwen3
+    engine with as many layers of the same width and vocabulary (no token takes a second iteration there)."""
+    import torch
+
+    from tah_amd import zozosun
+    from tah_amd.engine import EngineConfig, TaHDecodeEngine, Weights
+
+    cfg = stack_config(layers)
+    model = zozosun.load(cfg, zozosun.random_tensors(cfg, "cuda", seed=1), "cuda")
+    w = Weights.random_init(EngineConfig(layers=layers), "cuda", seed=1239)
+    w.threshold = 2.0  # above every probability: one iteration per token
+    g = torch.Generator().manual_seed(5)
+    yield
+
+    def build(kind, B, length):
+        if kind == "zozosun":
+            return zozosun.engine(model, B, length)
+        return TaHDecodeEngine(w, B, length, max_hard=512)
+
+    def timed(f, n):
+        for _ in range(max(1, min(warmup, 3))):
+            f()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            f()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / n
+
+    out = {"workload": f"{layers} layers, width 2048, vocab 151936, bf16, random weights; zozosun: gated delta rule (32 heads of 128 x 128, "
+                       "convolutions of 4) in three of four layers, latent attention (16 heads, 128 + 64, rank 512, window 1024) in the fourth, "
+                       "feed-forward 6144 or 64 experts of 768 (8 per token) and a shared one; qwen3: 16 / 8 heads of 128, feed-forward 6144"}
+    for kind in ("zozosun", "qwen3"):
+        res = out[kind] = {}
+        for B, T in STACK_SIZES["prefill"]:
+            eng = build(kind, B, T)
+            ids = torch.randint(0, cfg["vocab"], (B * T,), generator=g).cuda()
+            cu = torch.arange(0, B * T + 1, T, dtype=torch.int32, device="cuda")
+            s = timed(lambda: eng.prefill(ids, cu), max(2, steps // 10))
+            res[f"prefill_{B}x{T}"] = {"ms": s * 1e3, "tokens_per_s": B * T / s}
+            del eng
+        for B, ctx in STACK_SIZES["decode"]:
+            new = 64
+            eng = build(kind, B, ctx + 4 * new + 8)
+            ids = torch.randint(0, cfg["vocab"], (B * ctx,), generator=g).cuda()
+            cu = torch.arange(0, B * ctx + 1, ctx, dtype=torch.int32, device="cuda")
+            first, _ = eng.prefill(ids, cu)
+            eng.generate(first, 8)           # captures the step
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            eng.generate(first, new)
+            torch.cuda.synchronize()
+            s = (time.perf_counter() - t0) / (new - 1)
+            res[f"decode_{B}x{ctx}"] = {"ms_per_token": s * 1e3, "tokens_per_s": B / s}
+            del eng
+    return out
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -741,8 +822,9 @@ def main() -> int:
     ap.add_argument("--spinup", type=int, default=200,
                     help="untimed launches of the headline kernel before its warm-up steps (the GPU's clock needs tens of "
                          "milliseconds of work to leave its idle state)")
-    ap.add_argument("--only", choices=["all", "fwd", "decode", "fwd_bwd", "host_layer", "context", "qk_prep", "topk_mix", "sample_rows", "e2e"], default="all",
-                    help="profiling aid: run only one leg (the JSON line then lacks the other legs)")
+    ap.add_argument("--only", choices=["all", "fwd", "decode", "fwd_bwd", "host_layer", "context", "qk_prep", "topk_mix", "sample_rows", "e2e", "stack"], default="all",
+                    help="run only one leg (the JSON line then lacks the other legs); stack: prefill and decode of a Zozosun model "
+                         "beside the Qwen3 engine, not part of all")
     ap.add_argument("--calib-copy", action="store_true",
                     help="profiling aid: also run one plain 256 MiB device copy (known traffic for counter scaling)")
     args = ap.parse_args()
@@ -798,6 +880,8 @@ def main() -> int:
         legs.append(("sample_rows", bench_sample_rows(args.steps, args.warmup)))
     if args.only in ("all", "e2e"):
         legs.append(("e2e_decode", bench_e2e_decode(args.e2e_tokens, temperature=args.e2e_temperature, top_k=args.e2e_top_k)))
+    if args.only == "stack":
+        legs.append(("stack", bench_stack(args.steps, args.warmup)))
     for _, leg in legs:
         next(leg)  # runs the leg up to its `yield`: inputs built and resident
     sched = launch_order(ops, dev)

@@ -170,14 +170,15 @@ int tah_latent_decode(const tah_latent_layer* layer, const int32_t* slot, const 
 int tah_moe_route(const float* x, const void* router, const void* gate_w, int32_t rows, int32_t cols, int32_t experts,
                   int32_t top, int32_t* index, float* weight, float* shared_gate, int32_t dtype, tah_stream_t stream);
 /* Rows sorted by expert, every expert's rows padded to whole tiles of TAH_MOE_TILE: source row of every place (-1:
- * padding), the expert of every tile (-1 past the last), and the place of every (row, choice).
- * places, tiles: capacities; tah_moe_places(rows, top, experts) places are enough. */
+ * padding), the expert of every tile (-1 past the last) and behind them the number of tiles used, and the place of
+ * every (row, choice).  source holds tah_moe_places(rows, top, experts) places, tile_expert a tile for each TAH_MOE_TILE
+ * of them and one entry more. */
 enum { TAH_MOE_TILE = 128 };
 int32_t tah_moe_places(int32_t rows, int32_t top, int32_t experts);
 int tah_moe_plan(const int32_t* index, int32_t rows, int32_t top, int32_t experts, int32_t* source, int32_t* tile_expert,
                  int32_t* place, tah_stream_t stream);
 /* Product of the sorted rows with their experts' weights.  TAH_LINEAR_GATE_UP: w [experts, 2 n, k] (gate rows, then up
- * rows), x row source[place], out = silu(gate) * up [places, n]; TAH_LINEAR_PLAIN: w [experts, n, k], x row `place`. */
+ * rows), x row source[place] (`tiles` without the entry behind them), out = silu(gate) * up [places, n]; TAH_LINEAR_PLAIN: w [experts, n, k], x row `place`. */
 int tah_moe_linear(const void* x, int64_t x_row_stride, const void* w, const int32_t* source, const int32_t* tile_expert,
                    int32_t tiles, int32_t n, int32_t k, int32_t kind, void* out, int64_t out_row_stride, int32_t dtype,
                    tah_stream_t stream);

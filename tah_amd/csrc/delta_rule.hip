@@ -268,6 +268,90 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_prepare_kernel(const tah_
     }
 }
 
+__device__ __forceinline__ float silu_act(float x, __bf16*) { return x * fast_rcp(1.0f + fast_exp2(-x * kLog2e)); }  // an activation of a bf16 model
+__device__ __forceinline__ float silu_act(float x, float*) { return silu_exact(x); }
+
+// The same for heads of whole eight-channel units, a power of two of them: a thread owns eight channels and keeps the
+// last inputs of its convolutions in registers; the lanes of a q or k head add up their squares.  grid.y: 256 units
+// each, then one for the gates.
+template <class E, int TAPS>
+__global__ __launch_bounds__(kDeltaThreads) void delta_prepare_units_kernel(const tah_delta_layer L, const tah_portions P, float* q, float* k, float* v,
+                                                                            float* lg, float* beta) {
+    const int tid = threadIdx.x, t0 = blockIdx.x * kPrepTokens, tn = t0 + kPrepTokens < P.rows ? t0 + kPrepTokens : P.rows;
+    const E* const proj = static_cast<const E*>(L.proj);
+    if (blockIdx.y == gridDim.y - 1) {
+        for (int i = tid; i < (tn - t0) * L.heads; i += kDeltaThreads) {
+            const int t = t0 + i / L.heads, h = i % L.heads;
+            const E* pr = proj + (int64_t)t * L.proj_row_stride;
+            lg[(int64_t)t * L.heads + h] = decay_log(L, (float)pr[L.a_col + h], h);
+            beta[(int64_t)t * L.heads + h] = sigmoid_exact((float)pr[L.b_col + h]);
+        }
+        return;
+    }
+    const int qk = L.kv_heads * L.dim, nch = 2 * qk + L.heads * L.vdim;
+    int ch = 8 * (blockIdx.y * kDeltaThreads + tid);
+    const bool on = ch < nch;
+    ch = on ? ch : 0;  // (lanes past the end take part in the sums of nobody)
+    const bool is_q = ch < qk, is_v = ch >= 2 * qk;
+    const E* const src = proj + proj_col(L, ch);
+    float* const dst = is_q ? q + ch : (is_v ? v + ch - 2 * qk : k + ch - qk);
+    const int64_t dst_rs = is_v ? (int64_t)L.heads * L.vdim : qk;
+    const int lanes = L.dim / 8;  // of a q or k head
+    const float scale = is_q ? 1.0f / sqrtf((float)L.dim) : 1.0f;
+    float w[TAPS][8], hist[TAPS > 1 ? TAPS - 1 : 1][8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[j][i] = L.conv[(int64_t)(ch + i) * TAPS + j];
+    constexpr int kAhead = 4;
+    for (int tb = t0; tb < tn; tb += kAhead) {
+        float x[kAhead][8];
+#pragma unroll
+        for (int a = 0; a < kAhead; ++a) load8(src + (int64_t)(tb + a < tn ? tb + a : tn - 1) * L.proj_row_stride, x[a]);
+#pragma unroll
+        for (int a = 0; a < kAhead; ++a) {
+            const int t = tb + a;
+            if (t >= tn) break;
+            const int b = P.row_seq[t], first = P.cu[b];
+            if (t == t0 || t == first) {  // what came before: earlier rows of the portion, the state, or nothing
+                const int pos = P.pos0[b] + t - first, slot = P.slot[b];
+                const E* cs = static_cast<const E*>(L.conv_state) + (int64_t)(slot < 0 ? 0 : slot) * TAPS * nch + ch;
+#pragma unroll
+                for (int j = 1; j < TAPS; ++j) {
+                    if (t - j >= first) load8(src + (int64_t)(t - j) * L.proj_row_stride, hist[j - 1]);
+                    else if (pos - j >= 0 && slot >= 0) load8(cs + (int64_t)((pos - j) % TAPS) * nch, hist[j - 1]);
+                    else {
+#pragma unroll
+                        for (int i = 0; i < 8; ++i) hist[j - 1][i] = 0.f;
+                    }
+                }
+            }
+            float y[8], ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                float s = w[TAPS - 1][i] * x[a][i];
+#pragma unroll
+                for (int j = 1; j < TAPS; ++j) s += w[TAPS - 1 - j][i] * hist[j - 1][i];
+                y[i] = silu_act(s, static_cast<E*>(nullptr));
+                ss += y[i] * y[i];
+            }
+            for (int m = 1; m < lanes; m <<= 1) ss += __shfl_xor(ss, m);
+            const float r = is_v ? 1.0f : scale / sqrtf(ss + kUnitEps);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[i] *= r;
+            if (on) store8(dst + (int64_t)t * dst_rs, y);
+#pragma unroll
+            for (int j = TAPS - 1; j > 1; --j)
+#pragma unroll
+                for (int i = 0; i < 8; ++i) hist[j - 1][i] = hist[j - 2][i];
+            if constexpr (TAPS > 1) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) hist[0][i] = x[a][i];
+            }
+        }
+    }
+}
+
 // The convolution's inputs of a portion's last tokens, into the ring.  (After delta_prepare_kernel has read the old ones.)
 template <class E>
 __global__ __launch_bounds__(kDeltaThreads) void conv_tail_kernel(const tah_delta_layer L, const tah_portions P) {
@@ -427,6 +511,40 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_finish_kernel(const tah_d
         for (int c = L.heads * L.vdim + lane; c < out_cols; c += kWave) y[c] = (E)0.f;
 }
 
+// the same for values of whole eight-column units, a power of two of them per head: one thread per unit
+template <class E>
+__global__ __launch_bounds__(kDeltaThreads) void delta_finish_units_kernel(const tah_delta_layer L, const float* o, int64_t units, E* out, int64_t out_rs,
+                                                                           int out_cols) {
+    int64_t u = (int64_t)blockIdx.x * kDeltaThreads + threadIdx.x;
+    const bool on = u < units;
+    u = on ? u : units - 1;
+    const int per_row = L.heads * L.vdim / 8, lanes = L.vdim / 8;
+    const int64_t row = u / per_row;
+    const int c = 8 * (int)(u % per_row);
+    float x[8], gate[8], nw[8], ss = 0.f;
+    load8(o + row * L.heads * L.vdim + c, x);
+    load8(static_cast<const E*>(L.proj) + row * L.proj_row_stride + L.gate_col + c, gate);
+    load8(L.norm + c % L.vdim, nw);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+    for (int m = 1; m < lanes; m <<= 1) ss += __shfl_xor(ss, m);
+    const float r = 1.0f / sqrtf(ss / (float)L.vdim + L.eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = x[i] * r * nw[i] * silu_act(gate[i], static_cast<E*>(nullptr));
+    if (!on) return;
+    store8(out + row * out_rs + c, x);
+    if (c + 8 == L.heads * L.vdim)
+        for (int i = c + 8; i < out_cols; ++i) out[row * out_rs + i] = (E)0.f;
+}
+
+// a head of d channels is whole eight-channel units, a power of two of them, at most a wave's lanes
+bool in_units(int d) { return d % 8 == 0 && d <= 512 && (d & (d - 1)) == 0; }
+// projection rows that eight-element loads can address
+bool unit_rows(const tah_delta_layer& L) {
+    return aligned_16(L.proj) && L.proj_row_stride % 8 == 0 && aligned_16(L.conv_state) && aligned_16(L.norm) && L.q_col % 8 == 0 && L.k_col % 8 == 0 &&
+           L.v_col % 8 == 0 && L.gate_col % 8 == 0;
+}
+
 int check_layer(const tah_delta_layer* L) {
     if (!L) return TAH_E_NULL;
     if (L->heads <= 0 || L->kv_heads <= 0 || L->heads % L->kv_heads != 0 || L->dim <= 0 || L->vdim <= 0 || L->taps <= 0 || L->nslots <= 0 ||
@@ -465,6 +583,17 @@ void dispatch_step(const tah_delta_layer& L, const int32_t* slot, const int32_t*
 }
 template <class E>
 void launch_prepare(const tah_delta_layer& L, const tah_portions& P, float* q, float* k, float* v, float* lg, float* beta, hipStream_t st) {
+    const int nch = 2 * L.kv_heads * L.dim + L.heads * L.vdim;
+    const dim3 tail((nch + kDeltaThreads - 1) / kDeltaThreads, P.nseq);
+    if (L.taps >= 1 && L.taps <= 4 && in_units(L.dim) && L.vdim % 8 == 0 && unit_rows(L) && aligned_16(q) && aligned_16(k) && aligned_16(v)) {
+        const dim3 grid((P.rows + kPrepTokens - 1) / kPrepTokens, (nch / 8 + kDeltaThreads - 1) / kDeltaThreads + 1);
+        if (L.taps == 1) hipLaunchKernelGGL((delta_prepare_units_kernel<E, 1>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+        else if (L.taps == 2) hipLaunchKernelGGL((delta_prepare_units_kernel<E, 2>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+        else if (L.taps == 3) hipLaunchKernelGGL((delta_prepare_units_kernel<E, 3>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+        else hipLaunchKernelGGL((delta_prepare_units_kernel<E, 4>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
+        hipLaunchKernelGGL((conv_tail_kernel<E>), tail, dim3(kDeltaThreads), 0, st, L, P);
+        return;
+    }
     constexpr int per_block = kPrepTokens * (kDeltaThreads / kWave);
     const dim3 grid((P.rows + per_block - 1) / per_block, 2 * L.kv_heads + L.heads + 1);
     const int d = L.dim > L.vdim ? L.dim : L.vdim;
@@ -472,8 +601,20 @@ void launch_prepare(const tah_delta_layer& L, const tah_portions& P, float* q, f
     else if (d <= 128) hipLaunchKernelGGL((delta_prepare_kernel<E, 2>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
     else if (d <= 256) hipLaunchKernelGGL((delta_prepare_kernel<E, 4>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
     else hipLaunchKernelGGL((delta_prepare_kernel<E, 8>), grid, dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg, beta);
-    const int nch = 2 * L.kv_heads * L.dim + L.heads * L.vdim;
-    hipLaunchKernelGGL((conv_tail_kernel<E>), dim3((nch + kDeltaThreads - 1) / kDeltaThreads, P.nseq), dim3(kDeltaThreads), 0, st, L, P);
+    hipLaunchKernelGGL((conv_tail_kernel<E>), tail, dim3(kDeltaThreads), 0, st, L, P);
+}
+
+template <class E>
+void launch_finish(const tah_delta_layer& L, const float* o, int rows, void* out, int64_t out_rs, int out_cols, hipStream_t st) {
+    const int64_t items = (int64_t)rows * L.heads;
+    if (in_units(L.vdim) && unit_rows(L) && aligned_16(o) && aligned_16(out) && out_rs % 8 == 0) {
+        const int64_t units = items * L.vdim / 8;
+        hipLaunchKernelGGL((delta_finish_units_kernel<E>), dim3((unsigned)((units + kDeltaThreads - 1) / kDeltaThreads)), dim3(kDeltaThreads), 0, st, L, o,
+                           units, static_cast<E*>(out), out_rs, out_cols);
+    } else {
+        hipLaunchKernelGGL((delta_finish_kernel<E>), dim3((unsigned)((items + kDeltaThreads / kWave - 1) / (kDeltaThreads / kWave))), dim3(kDeltaThreads), 0,
+                           st, L, o, items, static_cast<E*>(out), out_rs, out_cols);
+    }
 }
 
 }  // namespace
@@ -531,12 +672,8 @@ extern "C" int tah_delta_finish(const tah_delta_layer* L, const float* o, int32_
     if (rows < 0 || out_cols < L->heads * L->vdim || (rows > 1 && out_rs < out_cols)) return TAH_E_SHAPE;
     if (rows == 0) return TAH_OK;
     if (!o || !out) return TAH_E_NULL;
-    const int64_t items = (int64_t)rows * L->heads;
-    const dim3 grid((unsigned)((items + kDeltaThreads / kWave - 1) / (kDeltaThreads / kWave)));
     hipStream_t st = static_cast<hipStream_t>(stream);
-    if (L->dtype == TAH_DT_BF16)
-        hipLaunchKernelGGL((delta_finish_kernel<__bf16>), grid, dim3(kDeltaThreads), 0, st, *L, o, items, static_cast<__bf16*>(out), out_rs, out_cols);
-    else
-        hipLaunchKernelGGL((delta_finish_kernel<float>), grid, dim3(kDeltaThreads), 0, st, *L, o, items, static_cast<float*>(out), out_rs, out_cols);
+    if (L->dtype == TAH_DT_BF16) launch_finish<__bf16>(*L, o, rows, out, out_rs, out_cols, st);
+    else launch_finish<float>(*L, o, rows, out, out_rs, out_cols, st);
     return launch_status();
 }

@@ -7,7 +7,7 @@
 //    the per-head products.
 //  * latent_context_kernel / latent_append_kernel: the rows a batch of portions can see, packed (old ones from the
 //    ring, new ones from the portion), then the new rows into the ring.
-//  * attend_tile_kernel (bf16): portions.  128 query rows of one head per workgroup against 64 keys at a time, on the
+//  * attend_tile_kernel (bf16): portions.  256 query rows of one head per workgroup (32 per wave) against 64 keys at a time, on the
 //    matrix cores: S^T = K Q^T, so that a query's scores sit in one lane column and the softmax needs two shuffles, and
 //    O^T = V^T P^T with V^T read from the row-major tile by transpose reads.  Keys outside the window are not visited.
 //  * latent_decode_kernel / latent_merge_kernel (bf16): single tokens.  All heads (sixteen at a time) of one row share a
@@ -207,7 +207,7 @@ __global__ __launch_bounds__(kLatThreads) void attend_rows_kernel(const AttendRo
 }
 
 // ---- bf16 on the matrix cores ------------------------------------------------------------------------------------
-constexpr int kTileKeys = 64, kTileRows = 128;
+constexpr int kTileKeys = 64;
 constexpr float kNoScore = -1e30f;  // below every score, and finite: differences of it are numbers
 
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
@@ -234,9 +234,10 @@ struct AttendTile {
     float scale_log2;
 };
 
-// NQ: 32-wide steps of a query row (at most), NV: 16-wide tiles of a value row (at most).
-template <int NQ, int NV>
-__global__ __launch_bounds__(kLatThreads) void attend_tile_kernel(const AttendTile p) {
+// NQ: 32-wide steps of a query row (at most), NV: 16-wide tiles of a value row (at most), W: waves, 32 query rows each.
+template <int NQ, int NV, int W>
+__global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile p) {
+    constexpr int kTileRows = 32 * W, kTileThreads = W * kWave;
     HIP_DYNAMIC_SHARED(unsigned char, tile_lds)
     int tile = blockIdx.x, b = 0, row0 = 0, row_end = 0;
     if (!find_tile(p.cu, p.nseq, kTileRows, tile, b, row0, row_end)) return;
@@ -271,44 +272,48 @@ __global__ __launch_bounds__(kLatThreads) void attend_tile_kernel(const AttendTi
     for (int i = 0; i < NV; ++i)
 #pragma unroll
         for (int t = 0; t < 2; ++t) acc[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    // a thread's sixteen-byte units of a tile: NQ of the keys, NV / 2 of the values
-    constexpr int UV = (NV + 1) / 2;
+    // a thread's sixteen-byte units of a tile, of the keys and of the values: where they come from and go to
+    constexpr int UK = (kTileKeys * NQ * 4 + kTileThreads - 1) / kTileThreads, UV = (kTileKeys * NV * 2 + kTileThreads - 1) / kTileThreads;
     const int uk = dq / 8, ukn = p.dim_pad / 8, uv = p.vdim_pad / 8;
-    bf16x8 fk[NQ], fv[UV];
+    const __bf16 *gk[UK], *gv[UV];
+    int kkey[UK], vkey[UV], kdst[UK], vdst[UV];
+    int64_t krs[UK];
+    bf16x8 fk[UK], fv[UV];
+#pragma unroll
+    for (int i = 0; i < UK; ++i) {
+        const int u = tid + kTileThreads * i, key = u / uk, x = u % uk;
+        kkey[i] = u < kTileKeys * uk ? key : -1;
+        kdst[i] = key * ks + 8 * x;
+        gk[i] = x < ukn ? p.k + (int64_t)k0 * p.k_rs + (int64_t)h * p.dim_pad + 8 * x : p.ctx + (int64_t)k0 * p.ctx_rs + 8 * (x - ukn);
+        krs[i] = x < ukn ? p.k_rs : p.ctx_rs;
+    }
+#pragma unroll
+    for (int i = 0; i < UV; ++i) {
+        const int u = tid + kTileThreads * i, key = u / uv, x = u % uv;
+        vkey[i] = u < kTileKeys * uv ? key : -1;
+        vdst[i] = key * vs + 8 * x;
+        gv[i] = p.v + (int64_t)k0 * p.v_rs + (int64_t)h * p.vdim_pad + 8 * x;
+    }
     auto fetch = [&](int j0) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < NQ; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (i < nq) {
-                const int key = u / uk, x = u % uk;
-                int j = j0 + key;
-                j = (j < lk ? j : lk - 1) + k0;
-                fk[i] = *reinterpret_cast<const bf16x8*>(x < ukn ? p.k + j * p.k_rs + (int64_t)h * p.dim_pad + 8 * x : p.ctx + j * p.ctx_rs + 8 * (x - ukn));
-            }
+        for (int i = 0; i < UK; ++i) {
+            const int j = j0 + kkey[i];
+            if (kkey[i] >= 0) fk[i] = *reinterpret_cast<const bf16x8*>(gk[i] + (j < lk ? j : lk - 1) * krs[i]);
         }
 #pragma unroll
         for (int i = 0; i < UV; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (u < kTileKeys * uv) {
-                const int key = u / uv, x = u % uv;
-                int j = j0 + key;
-                j = (j < lk ? j : lk - 1) + k0;
-                fv[i] = *reinterpret_cast<const bf16x8*>(p.v + j * p.v_rs + (int64_t)h * p.vdim_pad + 8 * x);
-            }
+            const int j = j0 + vkey[i];
+            if (vkey[i] >= 0) fv[i] = *reinterpret_cast<const bf16x8*>(gv[i] + (j < lk ? j : lk - 1) * p.v_rs);
         }
     };
     fetch(j_lo);
     for (int j0 = j_lo; j0 <= j_hi; j0 += kTileKeys) {
 #pragma unroll
-        for (int i = 0; i < NQ; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (i < nq) *reinterpret_cast<bf16x8*>(kt + (u / uk) * ks + 8 * (u % uk)) = fk[i];
-        }
+        for (int i = 0; i < UK; ++i)
+            if (kkey[i] >= 0) *reinterpret_cast<bf16x8*>(kt + kdst[i]) = fk[i];
 #pragma unroll
-        for (int i = 0; i < UV; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (u < kTileKeys * uv) *reinterpret_cast<bf16x8*>(vt + (u / uv) * vs + 8 * (u % uv)) = fv[i];
-        }
+        for (int i = 0; i < UV; ++i)
+            if (vkey[i] >= 0) *reinterpret_cast<bf16x8*>(vt + vdst[i]) = fv[i];
         __syncthreads();
         if (j0 + kTileKeys <= j_hi) fetch(j0 + kTileKeys);
         // (uniform per wave) does this wave see anything of the tile, and does it see all of it?
@@ -403,7 +408,7 @@ struct LatentDecode {
     const __bf16 *q_latent, *q_rot, *ring;
     int64_t q_latent_hs, q_rs;
     const int32_t *slot, *pos;
-    float* part;  // [rows][heads padded to 16][splits]: rank_pad sums, the maximum, the sum of weights
+    float* part;  // [rows][heads padded to 16][splits][rank_pad + 4]: sums, the maximum, the sum of weights
     int32_t heads, dim_pad, rot_pad, rank_pad, capacity, nslots, window, rows, splits, tiles_per_split;
     float scale_log2;
 };
@@ -432,14 +437,23 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
     end = end < pos ? end : pos;
     if (!live) end = begin - 1;
     bf16x8 fk[NU];
+    int key[NU], dst[NU];
+#pragma unroll
+    for (int i = 0; i < NU; ++i) {
+        const int u = tid + kLatThreads * i;
+        key[i] = u < units ? u / upk : -1;
+        dst[i] = (u / upk) * ks + 8 * (u % upk);
+    }
+    // a key's row of the ring: the first one's, advanced, wrapped at most once per tile (a tile is not longer than the ring,
+    // or the positions past `end` repeat the last)
     auto fetch = [&](int j0) __attribute__((always_inline)) {
+        const int r0 = j0 % p.capacity;
 #pragma unroll
         for (int i = 0; i < NU; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (u < units) {
-                int j = j0 + u / upk;
-                j = j < end ? j : end;
-                fk[i] = *reinterpret_cast<const bf16x8*>(ring + (int64_t)(j % p.capacity) * lp + 8 * (u % upk));
+            if (key[i] >= 0) {
+                int r = r0 + (j0 + key[i] < end ? key[i] : end - j0);
+                r = r >= p.capacity ? r - p.capacity : r;
+                fk[i] = *reinterpret_cast<const bf16x8*>(ring + (int64_t)r * lp + dst[i] - key[i] * ks);
             }
         }
     };
@@ -458,10 +472,8 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
     float m = kNoScore, l = 0.f;
     for (int j0 = begin; j0 <= end; j0 += kTileKeys) {
 #pragma unroll
-        for (int i = 0; i < NU; ++i) {
-            const int u = tid + kLatThreads * i;
-            if (u < units) *reinterpret_cast<bf16x8*>(kt + (u / upk) * ks + 8 * (u % upk)) = fk[i];
-        }
+        for (int i = 0; i < NU; ++i)
+            if (key[i] >= 0) *reinterpret_cast<bf16x8*>(kt + dst[i]) = fk[i];
         __syncthreads();
         if (j0 + kTileKeys <= end) fetch(j0 + kTileKeys);
         // scores of this wave's sixteen keys: register r of lane (c, g) is key 16 wave + 4 g + r, head c
@@ -520,15 +532,12 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
     if (g == 0) sum_[wave][c] = l;
     __syncthreads();
     const int hp = gridDim.y * 16;
-    float* const out = p.part + (((int64_t)row * hp + blockIdx.y * 16 + c) * p.splits + blockIdx.x) * (p.rank_pad + 2);
+    float* const out = p.part + (((int64_t)row * hp + blockIdx.y * 16 + c) * p.splits + blockIdx.x) * (p.rank_pad + 4);
     if (begin <= end) {
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
             const int t = wave + kLatWaves * i;
-            if (t < nt) {
-#pragma unroll
-                for (int r = 0; r < 4; ++r) out[16 * t + 4 * g + r] = acc[i][r];
-            }
+            if (t < nt) *reinterpret_cast<f32x4*>(out + 16 * t + 4 * g) = acc[i];
         }
     }
     if (tid < 16) {
@@ -537,28 +546,40 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
     }
 }
 
-// grid (heads, rows)
+// grid (heads, rows); four latent columns per thread
 __global__ __launch_bounds__(kLatThreads) void latent_merge_kernel(const float* part, int hp, int splits, int rank_pad, int rows, __bf16* out_packed,
                                                                    __bf16* out_rows) {
-    const int h = blockIdx.x, row = blockIdx.y;
-    const float* const base = part + ((int64_t)row * hp + h) * splits * (rank_pad + 2);
+    const int h = blockIdx.x, row = blockIdx.y, i = 4 * threadIdx.x, ps = rank_pad + 4;
+    const float* const base = part + ((int64_t)row * hp + h) * splits * ps;
+    if (i >= rank_pad) return;
     float m = kNoScore, l = 0.f;
-    for (int s = 0; s < splits; ++s)
-        if (base[(int64_t)s * (rank_pad + 2) + rank_pad + 1] > 0.f) m = fmaxf(m, base[(int64_t)s * (rank_pad + 2) + rank_pad]);
-    for (int s = 0; s < splits; ++s) {
-        const float* x = base + (int64_t)s * (rank_pad + 2) + rank_pad;
-        if (x[1] > 0.f) l += x[1] * fast_exp2(x[0] - m);
-    }
-    for (int i = threadIdx.x; i < rank_pad; i += kLatThreads) {
-        float y = 0.f;
-        for (int s = 0; s < splits; ++s) {
-            const float* x = base + (int64_t)s * (rank_pad + 2);
-            if (x[rank_pad + 1] > 0.f) y += x[i] * fast_exp2(x[rank_pad] - m);
+    f32x4 y = {0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < splits; s0 += 4) {
+        f32x4 v[4];
+        float vm[4], vl[4];
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+            const float* p = base + (int64_t)(s0 + x < splits ? s0 + x : splits - 1) * ps;
+            v[x] = *reinterpret_cast<const f32x4*>(p + i);
+            vm[x] = p[rank_pad];
+            vl[x] = s0 + x < splits ? p[rank_pad + 1] : 0.f;
         }
-        y = l > 0.f ? y / l : 0.f;
-        if (out_packed) out_packed[(int64_t)h * 32 * rank_pad + rows_form_elem(row, i)] = (__bf16)y;
-        if (out_rows) out_rows[((int64_t)h * rows + row) * rank_pad + i] = (__bf16)y;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+            if (!(vl[x] > 0.f)) continue;  // saw nothing: its sums were not written
+            const float mn = fmaxf(m, vm[x]), a = fast_exp2(m - mn), b = fast_exp2(vm[x] - mn);
+            m = mn;
+            l = l * a + vl[x] * b;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) y[e] = y[e] * a + v[x][e] * b;
+        }
     }
+    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    bf16x4 o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (__bf16)(y[e] * inv);
+    if (out_packed) *reinterpret_cast<bf16x4*>(out_packed + (int64_t)h * 32 * rank_pad + rows_form_elem(row, i)) = o;
+    if (out_rows) *reinterpret_cast<bf16x4*>(out_rows + ((int64_t)h * rows + row) * rank_pad + i) = o;
 }
 
 int check_layer(const tah_latent_layer* L) {
@@ -585,18 +606,18 @@ void launch_attend_rows(const AttendRows& p, int heads, int dtype, hipStream_t s
 }
 size_t elem_bytes(int dtype) { return dtype == TAH_DT_BF16 ? 2 : 4; }
 
-template <int NQ, int NV>
-int launch_attend_tile(const AttendTile& p, int slots, int heads, hipStream_t st) {
+template <int NQ, int NV, int W>
+int launch_attend_tile(const AttendTile& p, int rows, int heads, hipStream_t st) {
     const size_t lds = (size_t)kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 8) * 2;
-    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV>), hipFuncAttributeMaxDynamicSharedMemorySize,
+    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV, W>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                            (int)lds) != hipSuccess)
         return TAH_E_LAUNCH;
-    hipLaunchKernelGGL((attend_tile_kernel<NQ, NV>), dim3(slots, heads), dim3(kLatThreads), lds, st, p);
+    hipLaunchKernelGGL((attend_tile_kernel<NQ, NV, W>), dim3(rows / (32 * W) + p.nseq, heads), dim3(W * kWave), lds, st, p);
     return launch_status();
 }
 
 // how a decode call splits its window: enough workgroups for the chip, whole tiles of 64 keys each
-constexpr int kDecodeGroups = 512;
+constexpr int kDecodeGroups = 256;
 void decode_split(int heads, int rows, int window, int& splits, int& tiles_per_split) {
     const int tiles = (window + kTileKeys - 1) / kTileKeys, groups = rows * ((heads + 15) / 16);
     int want = groups > 0 ? kDecodeGroups / groups : 1;
@@ -682,10 +703,9 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
         t.dim_pad = L->dim_pad; t.rot_pad = L->rot_pad; t.vdim_pad = L->vdim_pad; t.window = L->window;
         t.scale_log2 = L->scale * kLog2e;
         hipStream_t st = static_cast<hipStream_t>(stream);
-        const int slots = p->rows / kTileRows + p->nseq;
-        if (nq <= 4 && nv <= 4) return launch_attend_tile<4, 4>(t, slots, L->heads, st);
-        if (nq <= 6 && nv <= 8) return launch_attend_tile<6, 8>(t, slots, L->heads, st);
-        return launch_attend_tile<10, 16>(t, slots, L->heads, st);
+        if (nq <= 4 && nv <= 4) return launch_attend_tile<4, 4, 8>(t, p->rows, L->heads, st);
+        if (nq <= 6 && nv <= 8) return launch_attend_tile<6, 8, 8>(t, p->rows, L->heads, st);
+        return launch_attend_tile<10, 16, 4>(t, p->rows, L->heads, st);
     }
     AttendRows a{};
     a.q1 = q; a.q1_rs = q_rs; a.q1_hs = L->dim_pad + L->rot_pad; a.n1 = L->dim_pad;
@@ -702,8 +722,8 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
 
 extern "C" size_t tah_latent_decode_workspace(const tah_latent_layer* L, int32_t rows) {
     if (tah::check_layer(L) != TAH_OK || rows <= 0 || !tah::decode_on_tiles(L)) return 0;
-    const size_t groups = (size_t)rows * ((L->heads + 15) / 16);
-    return (groups > tah::kDecodeGroups ? groups : (size_t)tah::kDecodeGroups) * 16 * (L->rank_pad + 2) * sizeof(float);  // enough for fewer rows too
+    const size_t groups = (size_t)rows * ((L->heads + 15) / 16);  // (rank_pad <= 4 * kLatThreads: one pass of the merge)
+    return (groups > tah::kDecodeGroups ? groups : (size_t)tah::kDecodeGroups) * 16 * (L->rank_pad + 4) * sizeof(float);  // enough for fewer rows too
 }
 
 extern "C" int tah_latent_decode(const tah_latent_layer* L, const int32_t* slot, const int32_t* pos, int32_t rows, const void* q_latent,
@@ -724,7 +744,7 @@ extern "C" int tah_latent_decode(const tah_latent_layer* L, const int32_t* slot,
         d.window = L->window; d.rows = rows; d.scale_log2 = L->scale * kLog2e;
         decode_split(L->heads, rows, L->window, d.splits, d.tiles_per_split);
         const int hp = (L->heads + 15) / 16 * 16;
-        if (!workspace || workspace_bytes < (size_t)rows * hp * d.splits * (L->rank_pad + 2) * sizeof(float)) return TAH_E_WORKSPACE;
+        if (!workspace || workspace_bytes < (size_t)rows * hp * d.splits * (L->rank_pad + 4) * sizeof(float)) return TAH_E_WORKSPACE;
         hipStream_t st = static_cast<hipStream_t>(stream);
         const int lp = L->rank_pad + L->rot_pad;
         int rc;

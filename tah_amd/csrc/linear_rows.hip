@@ -403,7 +403,7 @@ void launch(LinParams& p, int groups, int batch, hipStream_t st) {
     p.groups = groups;
     if (p.rows <= 16)
         hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(groups, batch), dim3(kLinThreads), 0, st, p);
-    else if (groups < kSplitRowsBelowGroups)
+    else if (groups * batch < kSplitRowsBelowGroups)
         hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 1>), dim3(2 * groups, batch), dim3(kLinThreads), 0, st, p);
     else
         hipLaunchKernelGGL((linear_rows_kernel<NC, CH, EPI, PW, 2>), dim3(groups, batch), dim3(kLinThreads), 0, st, p);
@@ -504,12 +504,21 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
         }
     } else if (!gate_up && a->input_norm == TAH_NORM_LAYER) {
         launch<1, 4, kPlainLayerNorm, 0>(p, a->n / kTileCols, batch, st);
+    } else if (!gate_up && batch > 1 && a->n % (2 * kTileCols) == 0 && a->n / (2 * kTileCols) * batch >= kSplitRowsBelowGroups) {
+        // many products of one size: two tiles per workgroup halve the workgroups and the reads of the rows' operand
+        const int groups = a->n / (2 * kTileCols);
+        if (pw == 2) launch<2, 2, kPlain, 2>(p, groups, batch, st);
+        else if (pw == 3) launch<2, 3, kPlain, 3>(p, groups, batch, st);
+        else if (pw == 4) launch<2, 4, kPlain, 4>(p, groups, batch, st);
+        else if (pw == 8) launch<2, 4, kPlain, 8>(p, groups, batch, st);
+        else launch<2, 2, kPlain, 0>(p, groups, batch, st);
     } else if (!gate_up) {
         const int groups = a->n / kTileCols;
         if (p.norm) {
             if (pw == 8) launch<1, 8, kPlainNorm, 8>(p, groups, batch, st);
             else launch<1, 4, kPlainNorm, 0>(p, groups, batch, st);
         } else if (pw == 8) launch<1, 8, kPlain, 8>(p, groups, batch, st);
+        else if (pw == 16) launch<1, 8, kPlain, 16>(p, groups, batch, st);
         else if (pw == 24) launch<1, 8, kPlain, 24>(p, groups, batch, st);
         else launch<1, 4, kPlain, 0>(p, groups, batch, st);
     } else if (g24) {

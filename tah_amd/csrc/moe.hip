@@ -3,7 +3,7 @@
 // expert that some row chose over all rows.)
 //
 //  * moe_route_kernel: router logits in float32 from the float32 rows, the largest ones and their softmax; RB rows per
-//    workgroup share the router's weights.
+//    workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
 //  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
 //  * moe_tile_kernel: bf16 tiles of 128 places x 128 weight rows on the matrix cores, both operands staged through LDS
 //    by asynchronous copies, two stages; gate and up rows of the same columns share a wave, which applies the gate.
@@ -16,7 +16,6 @@ namespace tah {
 namespace {
 
 constexpr int kMoeThreads = 256;
-constexpr int kMoeWaves = kMoeThreads / kWave;
 constexpr int kMaxExperts = 1024;
 constexpr int kMaxTop = 64;
 constexpr int kTile = TAH_MOE_TILE;
@@ -24,43 +23,54 @@ constexpr int kTile = TAH_MOE_TILE;
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
 // LDS: rows [RB][cols] float32, logits [RB][experts + 1]
-template <class E, int RB>
-__global__ __launch_bounds__(kMoeThreads) void moe_route_kernel(const float* x, const E* router, const E* gate_w, int rows, int cols, int experts,
+template <class E, int RB, int EB, int kThreads>
+__global__ __launch_bounds__(kThreads) void moe_route_kernel(const float* x, const E* router, const E* gate_w, int rows, int cols, int experts,
                                                                 int top, int32_t* index, float* weight, float* shared_gate) {
     HIP_DYNAMIC_SHARED(float, sm)
     float* const xs = sm;
     float* const z = sm + RB * cols;
+    constexpr int kWaves = kThreads / kWave;
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, row0 = blockIdx.x * RB;
-    const int zs = experts + 1;
-    for (int i = 4 * tid; i < RB * cols; i += 4 * kMoeThreads) {
+    const int zs = experts + 1, total = experts + (gate_w ? 1 : 0);
+    for (int i = 4 * tid; i < RB * cols; i += 4 * kThreads) {
         const int r = row0 + i / cols;
         *reinterpret_cast<f32x4*>(xs + i) = r < rows ? *reinterpret_cast<const f32x4*>(x + (int64_t)r * cols + i % cols) : f32x4{0.f, 0.f, 0.f, 0.f};
     }
     __syncthreads();
-    for (int e = wave; e < experts + (gate_w ? 1 : 0); e += kMoeWaves) {
-        const E* w = e < experts ? router + (int64_t)e * cols : gate_w;
-        float s[RB];
+    for (int e0 = EB * wave; e0 < total; e0 += EB * kWaves) {
+        const E* w[EB];
+        float s[EB][RB];
 #pragma unroll
-        for (int r = 0; r < RB; ++r) s[r] = 0.f;
+        for (int x = 0; x < EB; ++x) {
+            const int e = e0 + x;
+            w[x] = e < experts ? router + (int64_t)e * cols : (e < total ? gate_w : router);  // (past the end: computed, not stored)
+#pragma unroll
+            for (int r = 0; r < RB; ++r) s[x][r] = 0.f;
+        }
         for (int c = 8 * lane; c < cols; c += 8 * kWave) {
-            float v[8];
-            load8(w + c, v);
+            float v[EB][8];
+#pragma unroll
+            for (int x = 0; x < EB; ++x) load8(w[x] + c, v[x]);
 #pragma unroll
             for (int r = 0; r < RB; ++r) {
                 float y[8];
                 load8(xs + r * cols + c, y);
 #pragma unroll
-                for (int i = 0; i < 8; ++i) s[r] += v[i] * y[i];
+                for (int x = 0; x < EB; ++x)
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) s[x][r] += v[x][i] * y[i];
             }
         }
 #pragma unroll
-        for (int r = 0; r < RB; ++r) {
-            const float t = wave_sum(s[r]);
-            if (lane == 0) z[r * zs + e] = t;
-        }
+        for (int x = 0; x < EB; ++x)
+#pragma unroll
+            for (int r = 0; r < RB; ++r) {
+                const float t = wave_sum(s[x][r]);
+                if (lane == 0 && e0 + x < total) z[r * zs + e0 + x] = t;
+            }
     }
     __syncthreads();
-    for (int r = wave; r < RB; r += kMoeWaves) {
+    for (int r = wave; r < RB; r += kWaves) {
         const int row = row0 + r;
         if (row >= rows) break;
         float* const zr = z + r * zs;
@@ -120,6 +130,7 @@ __global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(const int32_t* i
     for (int t = 0; t < mine; ++t) tile_expert[t0 + t] = tid;
     for (int i = n; i < mine * kTile; ++i) source[t0 * kTile + i] = -1;
     for (int t = used + tid; t < tiles; t += kPlanThreads) tile_expert[t] = -1;
+    if (tid == 0) tile_expert[tiles] = used;
     __syncthreads();
     for (int i = tid; i < pairs; i += kPlanThreads) {
         const int at = atomicAdd(&cursor[index[i]], 1);
@@ -134,8 +145,19 @@ struct MoeGemm {
     const int32_t *source, *tile_expert;
     void* out;
     int64_t x_rs, out_rs;
-    int32_t n, k;
+    int32_t n, k, tiles, col_tiles;
 };
+
+// Which tile of places and which tile of columns a workgroup takes.  Workgroups go to the XCDs round robin; an XCD gets a
+// run of consecutive place tiles with all their columns, so that an expert's weights and a place's row are read into
+// one L2 only.  False: nothing to do.
+__device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int& tile, int& col_tile) {
+    const int used = p.tile_expert[p.tiles], per = (used + 7) / 8;
+    const int xcd = blockIdx.x % 8, i = blockIdx.x / 8;
+    tile = xcd * per + i / p.col_tiles;
+    col_tile = i % p.col_tiles;
+    return i / p.col_tiles < per && tile < used;
+}
 
 // ---- bf16 tiles ------------------------------------------------------------------------------------------------
 constexpr int kStageK = 64;
@@ -145,13 +167,14 @@ constexpr int kStageBytes = 2 * kTile * kStageK * 2;  // both operands of one st
 template <bool GATE>
 __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) {
     HIP_DYNAMIC_SHARED(unsigned char, lds)
-    const int expert = p.tile_expert[blockIdx.y];
-    if (expert < 0) return;
+    int tile, col_tile;
+    if (!moe_tile_of(p, tile, col_tile)) return;
+    const int expert = p.tile_expert[tile];
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 2, wn = wave % 2;
     const __bf16* const x = static_cast<const __bf16*>(p.x);
     const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
     constexpr int kCols = GATE ? kTile / 2 : kTile;  // output columns of a tile
-    const int n0 = blockIdx.x * kCols;
+    const int n0 = col_tile * kCols;
     // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
     // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
     const __bf16 *ga[4], *gb[4];
@@ -160,7 +183,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
     for (int i = 0; i < 4; ++i) {
         const int r = 8 * (4 * wave + i) + lane / 8;
         chunk[i] = (lane % 8) ^ ((r >> 1) & 7);
-        int src = GATE ? p.source[blockIdx.y * kTile + r] : blockIdx.y * kTile + r;
+        int src = GATE ? p.source[tile * kTile + r] : tile * kTile + r;
         src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
         ga[i] = x + (int64_t)src * p.x_rs;
         int wr;
@@ -221,7 +244,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
     __bf16* const out = static_cast<__bf16*>(p.out);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        __bf16* const row = out + ((int64_t)blockIdx.y * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
+        __bf16* const row = out + ((int64_t)tile * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
         if constexpr (GATE) {
 #pragma unroll
             for (int i = 0; i < 2; ++i) {
@@ -251,9 +274,10 @@ constexpr int kPlainK = 16, kPlainCols = 32;
 template <bool GATE>
 __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p) {
     __shared__ float a[kPlainK][kTile + 1], g[kPlainK][kPlainCols + 1], u[GATE ? kPlainK : 1][kPlainCols + 1];
-    const int expert = p.tile_expert[blockIdx.y];
-    if (expert < 0) return;
-    const int tid = threadIdx.x, tc = tid % kPlainCols, tr = tid / kPlainCols, n0 = blockIdx.x * kPlainCols;
+    int tile, col_tile;
+    if (!moe_tile_of(p, tile, col_tile)) return;
+    const int expert = p.tile_expert[tile];
+    const int tid = threadIdx.x, tc = tid % kPlainCols, tr = tid / kPlainCols, n0 = col_tile * kPlainCols;
     const float* const x = static_cast<const float*>(p.x);
     const float* const w = static_cast<const float*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
     float sg[16], su[16];
@@ -262,7 +286,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p)
     for (int k0 = 0; k0 < p.k; k0 += kPlainK) {
         for (int i = tid; i < kTile * kPlainK; i += kMoeThreads) {
             const int r = i / kPlainK, c = i % kPlainK;
-            const int src = GATE ? p.source[blockIdx.y * kTile + r] : blockIdx.y * kTile + r;
+            const int src = GATE ? p.source[tile * kTile + r] : tile * kTile + r;
             a[c][r] = src >= 0 ? x[(int64_t)src * p.x_rs + k0 + c] : 0.f;
         }
         for (int i = tid; i < kPlainCols * kPlainK; i += kMoeThreads) {
@@ -286,7 +310,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p)
     if (n0 + tc >= p.n) return;
 #pragma unroll
     for (int i = 0; i < 16; ++i)
-        static_cast<float*>(p.out)[((int64_t)blockIdx.y * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = GATE ? silu_exact(sg[i]) * su[i] : sg[i];
+        static_cast<float*>(p.out)[((int64_t)tile * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = GATE ? silu_exact(sg[i]) * su[i] : sg[i];
 }
 
 template <class E>
@@ -296,10 +320,10 @@ void launch_route(const float* x, const void* router, const void* gate_w, int ro
     const E* const gw = static_cast<const E*>(gate_w);
     const auto lds = [&](int rb) { return (size_t)rb * (cols + experts + 1) * sizeof(float); };
     if (rows > 256 && lds(8) <= 65536)  // many rows: eight share a pass over the router's weights
-        hipLaunchKernelGGL((moe_route_kernel<E, 8>), dim3((rows + 7) / 8), dim3(kMoeThreads), lds(8), st, x, rt, gw, rows, cols, experts, top, index,
+        hipLaunchKernelGGL((moe_route_kernel<E, 8, 4, 256>), dim3((rows + 7) / 8), dim3(256), lds(8), st, x, rt, gw, rows, cols, experts, top, index,
                            weight, shared_gate);
-    else
-        hipLaunchKernelGGL((moe_route_kernel<E, 1>), dim3(rows), dim3(kMoeThreads), lds(1), st, x, rt, gw, rows, cols, experts, top, index, weight,
+    else  // few rows: what counts is how much of the router's weights one row has in flight
+        hipLaunchKernelGGL((moe_route_kernel<E, 1, 2, 1024>), dim3(rows), dim3(1024), lds(1), st, x, rt, gw, rows, cols, experts, top, index, weight,
                            shared_gate);
 }
 
@@ -348,16 +372,17 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
     if (tiles == 0) return TAH_OK;
     if (!x || !w || !tile_expert || !out || (kind == TAH_LINEAR_GATE_UP && !source)) return TAH_E_NULL;
     if (!aligned_16(x) || !aligned_16(w) || !aligned_16(out)) return TAH_E_ALIGN;
-    const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k};
     const bool gate = kind == TAH_LINEAR_GATE_UP;
+    const int cols = dtype == TAH_DT_F32 ? kPlainCols : (gate ? kTile / 2 : kTile);
+    const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k, tiles, (n + cols - 1) / cols};
+    const int64_t groups = (int64_t)((tiles + 7) / 8) * 8 * p.col_tiles;  // whole rounds over the XCDs
+    if (groups > 0x7fffffff) return TAH_E_SHAPE;
+    const dim3 grid((unsigned)groups);
     hipStream_t st = static_cast<hipStream_t>(stream);
     if (dtype == TAH_DT_BF16) {
-        const int cols = gate ? kTile / 2 : kTile;
-        const dim3 grid((n + cols - 1) / cols, tiles);
         if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
         else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
     } else {
-        const dim3 grid((n + kPlainCols - 1) / kPlainCols, tiles);
         if (gate) hipLaunchKernelGGL((moe_plain_kernel<true>), grid, dim3(kMoeThreads), 0, st, p);
         else hipLaunchKernelGGL((moe_plain_kernel<false>), grid, dim3(kMoeThreads), 0, st, p);
     }

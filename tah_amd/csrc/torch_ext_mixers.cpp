@@ -285,7 +285,7 @@ void moe_route(const Tensor& x, const Tensor& router, const optional<Tensor>& ga
              "tah_moe_route");
 }
 
-// -> source [places], tile_expert [tiles], place [rows, top]
+// -> source [places], tile_expert [tiles and their number], place [rows, top]
 std::vector<Tensor> moe_plan(const Tensor& index, int64_t experts) {
     need_lib();
     Dev d; d.see(index);
@@ -293,7 +293,7 @@ std::vector<Tensor> moe_plan(const Tensor& index, int64_t experts) {
     flat(index, at::kInt, -1, "moe_plan: index");
     const int64_t rows = index.size(0), top = index.size(1);
     const int64_t places = g.moe_places((int32_t)rows, (int32_t)top, (int32_t)experts);
-    Tensor source = at::empty({places}, index.options()), tile = at::empty({places / TAH_MOE_TILE}, index.options()), place = at::empty_like(index);
+    Tensor source = at::empty({places}, index.options()), tile = at::empty({places / TAH_MOE_TILE + 1}, index.options()), place = at::empty_like(index);
     check_rc(g.moe_plan(at_<int32_t>(index), (int32_t)rows, (int32_t)top, (int32_t)experts, at_<int32_t>(source), at_<int32_t>(tile), at_<int32_t>(place),
                         d.stream()),
              "tah_moe_plan");
@@ -304,7 +304,7 @@ Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& source, const 
     need_lib();
     Dev d; d.see(x); d.see(w); d.see(source); d.see(tile_expert);
     TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && (!gate_up || w.size(1) % 2 == 0), "moe_linear: w must be a contiguous [experts, n, k] tensor");
-    const int64_t n = gate_up ? w.size(1) / 2 : w.size(1), k = w.size(2), tiles = tile_expert.numel();
+    const int64_t n = gate_up ? w.size(1) / 2 : w.size(1), k = w.size(2), tiles = tile_expert.numel() - 1;
     flat(tile_expert, at::kInt, -1, "moe_linear: tile_expert"); flat(source, at::kInt, tiles * TAH_MOE_TILE, "moe_linear: source");
     const int64_t rs = matrix(x, w.scalar_type(), gate_up ? 1 : tiles * TAH_MOE_TILE, k, "moe_linear: x");
     Tensor out = at::empty({tiles * TAH_MOE_TILE, n}, x.options());

@@ -18,7 +18,8 @@ def latent(heads, dim, rot, vdim, rank, window, base=50.0, scale=0.4):
 
 
 # (sizes, lengths, portions per sequence)
-DELTA_SMALL = [(delta(2, 1, 6, 5, 3), (5, 3), ((2, 3), (3,))), (delta(2, 2, 12, 8, 4), (7, 2), ((7,), (2,)))]
+DELTA_SMALL = [(delta(2, 1, 6, 5, 3), (5, 3), ((2, 3), (3,))), (delta(2, 2, 12, 8, 4), (7, 2), ((7,), (2,))),
+               (delta(2, 1, 16, 32, 3), (5, 4), ((3, 2), (4,)))]
 DELTA_GPU = DELTA_SMALL + [
     (delta(6, 3, 40, 24, 4), (70, 33), ((37, 2, 31), (2, 31))), (delta(4, 4, 64, 64, 2), (130, 5), ((128, 2), (3, 2))),
     (delta(8, 2, 128, 128, 4), (200, 65), ((64, 17, 119), (65,))), (delta(2, 1, 256, 96, 4), (40, 40), ((40,), (17, 23))),

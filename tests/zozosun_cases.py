@@ -132,13 +132,14 @@ def delta_layer(dev, dtype, m, nslots, g, slow=True):
     H, KH, D, V, taps = m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"]
     nch = 2 * KH * D + H * V
     w = {"conv": rnd(g, nch, taps) * taps ** -0.5, "A_log": rnd(g, H) * 0.3 + (-5.0 if slow else 0.5), "dt_bias": rnd(g, H), "norm": 1 + 0.2 * rnd(g, V)}
-    at, cols = 3, []
+    at, cols = (8 if D % 8 == 0 else 3), []   # (both the vector form and the element form of the kernels)
     for n in (KH * D, KH * D, H * V, H * V, H, H):  # q k v gate b a
         cols.append(at)
         at += n
     f = lambda t: t.float().to(dev)
     cs = torch.full((nslots, taps, nch), 7.0, dtype=dtype, device=dev)
     S = torch.full((nslots, H, D, V), -3.0, device=dev)
+    at = (at + 7) // 8 * 8
     return ops.lib().DeltaLayer(f(w["conv"]), f(w["A_log"]), f(w["dt_bias"]), f(w["norm"]), cs, S, H, KH, D, V, cols, m["eps"]), w, cols, at, S
 
 
