@@ -97,7 +97,8 @@ int tah_delta_step(const tah_delta_layer* layer, const int32_t* slot, const int3
 
 /* Portions of sequences.  tah_delta_prepare: q, k [T, kv_heads, dim], v [T, heads, vdim], the decay's logarithm and
  * beta [T, heads], all float32, and the convolution's state; row_seq int32 [T]: a row's sequence.
- * tah_delta_scan: the recurrence, o float32 [T, heads, vdim], and the new states.
+ * tah_delta_scan: the recurrence, o float32 [T, heads, vdim], and the new states; workspace as large as
+ * tah_delta_scan_workspace says (0: none), which depends on the sizes and counts alone.
  * tah_delta_finish: norm and gate, out element type [T, out_row_stride]. */
 typedef struct tah_portions {
     const int32_t *cu, *slot, *pos0; /* [nseq + 1], [nseq], [nseq] */
@@ -107,7 +108,8 @@ typedef struct tah_portions {
 int tah_delta_prepare(const tah_delta_layer* layer, const tah_portions* p, float* q, float* k, float* v, float* log_decay,
                       float* beta, tah_stream_t stream);
 int tah_delta_scan(const tah_delta_layer* layer, const tah_portions* p, const float* q, const float* k, const float* v,
-                   const float* log_decay, const float* beta, float* o, tah_stream_t stream);
+                   const float* log_decay, const float* beta, float* o, void* workspace, size_t workspace_bytes, tah_stream_t stream);
+size_t tah_delta_scan_workspace(const tah_delta_layer* layer, int32_t nseq, int32_t rows);
 int tah_delta_finish(const tah_delta_layer* layer, const float* o, int32_t rows, void* out, int64_t out_row_stride,
                      int32_t out_cols, tah_stream_t stream);
 

@@ -349,7 +349,8 @@ PROTOTYPES = {
     "tah_activate_rows": (C.c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int32, c_int32, c_int32, c_int32, c_void_p]),
     "tah_delta_step": (C.c_int, [C.POINTER(DeltaLayer), c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int32, c_void_p]),
     "tah_delta_prepare": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 6),
-    "tah_delta_scan": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 7),
+    "tah_delta_scan": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 7 + [C.c_size_t, c_void_p]),
+    "tah_delta_scan_workspace": (C.c_size_t, [C.POINTER(DeltaLayer), c_int32, c_int32]),
     "tah_delta_finish": (C.c_int, [C.POINTER(DeltaLayer), c_void_p, c_int32, c_void_p, c_int64, c_int32, c_void_p]),
     "tah_latent_prep": (C.c_int, [C.POINTER(LatentLayer), C.POINTER(LatentPrepArgs), c_void_p]),
     "tah_latent_context": (C.c_int, [C.POINTER(LatentLayer), C.POINTER(Portions), c_void_p, c_int32, c_void_p, c_void_p, c_void_p]),

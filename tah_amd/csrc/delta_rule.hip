@@ -10,7 +10,16 @@
 //  * delta_prepare_kernel / delta_scan_kernel / delta_finish_kernel: portions of many tokens.  Columns of the state do
 //    not interact, so a head is split over workgroups of 16 columns: a wave owns 4 columns, 16 lanes share a column's
 //    rows and reduce over them with DPP row rotations; k and q of the next 16 tokens are fetched while the current 16
-//    run.  State and inputs are float32 throughout (no reduced-precision matrix instruction touches the recurrence).
+//    run.
+//  * delta_chunk_kernel / delta_chunk_scan_kernel: the same for long portions, 32 tokens at a time, on the float32
+//    matrix instruction.  With G_t the running sum of the decays' logarithms since the chunk's start and S the state
+//    there, the chunk's writes u satisfy
+//        u_t + beta_t sum_{s<t} exp(G_t - G_s) (k_t . k_s) u_s = beta_t (v_t - exp(G_t) S^T k_t),
+//    a unit lower triangular system.  The first kernel solves it for all chunks at once, for the two parts of the right
+//    hand side: U0 (from v) and W (from k), so that u = U0 - W S; and forms P[t][s] = exp(G_t - G_s) (q_t . k_s), s <= t.
+//    The second walks the chunks of a sequence: u = U0 - W S, o_t = exp(G_t) S^T q_t + (P u)_t,
+//    S <- exp(G_last) S + sum_s exp(G_last - G_s) k_s u_s^T, a workgroup holding sixteen columns of a head's state.
+//  State and inputs are float32 throughout: no reduced-precision matrix instruction touches the recurrence.
 //
 // The convolution's inputs of the last `taps` tokens are kept as a ring (token p at p % taps): a step writes the entry
 // that no row of the step reads, so workgroups that share channels need no order among themselves.
@@ -491,6 +500,258 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_scan_kernel(const tah_del
         }
 }
 
+// ---- long portions, 32 tokens at a time -------------------------------------------------------------------------
+constexpr int kChunk = 32;
+
+__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// running sums of a chunk's decay logarithms: lane t < 32 ends with G_t (lanes of 32 and more repeat lane 31)
+__device__ __forceinline__ float chunk_decay(const float* lg, int heads, int h, int row0, int n, int lane) {
+    float x = lane < n ? lg[(int64_t)(row0 + lane) * heads + h] : 0.f;
+#pragma unroll
+    for (int o = 1; o < kChunk; o <<= 1) {
+        const float y = __shfl_up(x, o);
+        if (lane >= o && lane < kChunk) x += y;
+    }
+    return __shfl(x, lane < kChunk ? lane : kChunk - 1);
+}
+
+// what the first kernel leaves per (chunk, head), in floats: W [32][dim], U0 [32][vdim], P [32][32]
+__device__ __host__ __forceinline__ int64_t chunk_floats(int dim, int vdim) { return kChunk * (int64_t)(dim + vdim + kChunk); }
+
+// grid (chunk slots, heads).  NT: 16-wide tiles of dim.
+template <int NT>
+__global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
+                                                                    const float* v, const float* lg, const float* beta, float* work) {
+    constexpr int D = 16 * NT, kStride = D + 4;
+    __shared__ __align__(16) float kl[kChunk][kStride], ql[kChunk][kStride];
+    __shared__ __align__(16) float al[kChunk][kChunk + 4];
+    __shared__ float gl[kChunk], bl[kChunk];
+    int slot = blockIdx.x, b = 0, row0 = 0, row_end = 0;
+    if (!find_tile(P.cu, P.nseq, kChunk, slot, b, row0, row_end)) return;
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int h = blockIdx.y, kh = h / (L.heads / L.kv_heads), n = row_end - row0;
+    float* const out = work + ((int64_t)blockIdx.x * L.heads + h) * chunk_floats(D, L.vdim);
+    float* const out_u = out + kChunk * D;
+    float* const out_p = out_u + kChunk * L.vdim;
+    for (int u = tid; u < kChunk * D / 4; u += kDeltaThreads) {
+        const int t = u / (D / 4), i = 4 * (u % (D / 4));
+        f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
+        if (t < n) {
+            const int64_t at = ((int64_t)(row0 + t) * L.kv_heads + kh) * D + i;
+            x = *reinterpret_cast<const f32x4*>(k + at);
+            y = *reinterpret_cast<const f32x4*>(q + at);
+        }
+        *reinterpret_cast<f32x4*>(&kl[t][i]) = x;
+        *reinterpret_cast<f32x4*>(&ql[t][i]) = y;
+    }
+    if (wave == 0) {
+        const float x = chunk_decay(lg, L.heads, h, row0, n, lane);
+        if (lane < kChunk) {
+            gl[lane] = x;
+            bl[lane] = lane < n ? beta[(int64_t)(row0 + lane) * L.heads + h] : 0.f;
+        }
+    }
+    __syncthreads();
+    // six tiles of 16 x 16: the lower ones of K K^T and of Q K^T
+    for (int id = wave; id < 6; id += kDeltaThreads / kWave) {
+        const bool is_p = id >= 3;
+        const int i = id % 3 == 0 ? 0 : 1, j = id % 3 == 2 ? 1 : 0;
+        const float* const a = is_p ? &ql[16 * i + c][4 * g] : &kl[16 * i + c][4 * g];
+        const float* const bb = &kl[16 * j + c][4 * g];
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = acc;
+#pragma unroll
+        for (int s = 0; s < NT; ++s) {
+            const f32x4 x = *reinterpret_cast<const f32x4*>(a + 16 * s), y = *reinterpret_cast<const f32x4*>(bb + 16 * s);
+#pragma unroll
+            for (int e = 0; e < 4; e += 2) {
+                acc = mfma_f32(x[e], y[e], acc);
+                acc2 = mfma_f32(x[e + 1], y[e + 1], acc2);
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = 16 * i + 4 * g + r, s = 16 * j + c;
+            const float w = t >= s ? (acc[r] + acc2[r]) * expf(gl[t] - gl[s]) : 0.f;
+            if (is_p) out_p[t * kChunk + s] = w;
+            else al[t][s] = bl[t] * w;
+        }
+    }
+    if (wave == 3) {  // the tile above the diagonal
+#pragma unroll
+        for (int r = 0; r < 4; ++r) out_p[(4 * g + r) * kChunk + 16 + c] = 0.f;
+    }
+    __syncthreads();
+    // the triangular system, one column of a right hand side per thread: columns of v, then of k
+    for (int col = tid; col < L.vdim + D; col += kDeltaThreads) {
+        const bool is_k = col >= L.vdim;
+        const int i = is_k ? col - L.vdim : col;
+        float x[kChunk];
+#pragma unroll
+        for (int t = 0; t < kChunk; ++t) {
+            if (is_k) x[t] = bl[t] * expf(gl[t]) * kl[t][i];
+            else x[t] = t < n ? bl[t] * v[((int64_t)(row0 + t) * L.heads + h) * L.vdim + i] : 0.f;
+        }
+#pragma unroll
+        for (int t = 1; t < kChunk; ++t) {
+#pragma unroll
+            for (int s4 = 0; s4 < (t + 3) / 4; ++s4) {
+                const f32x4 a = *reinterpret_cast<const f32x4*>(&al[t][4 * s4]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (4 * s4 + e < t) x[t] -= a[e] * x[4 * s4 + e];
+            }
+        }
+        float* const dst = is_k ? out + i : out_u + i;
+        const int ds = is_k ? D : L.vdim;
+#pragma unroll
+        for (int t = 0; t < kChunk; ++t) dst[t * ds] = x[t];
+    }
+}
+
+// grid (16-column slices, heads, sequences).  Waves 0 and 1 form u, waves 2 and 3 the results; each holds every fourth
+// 16-row tile of the state's slice, register r of lane (c, g) of tile i being S[16 i + c][4 g + r].
+template <int NT>
+__global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
+                                                                         const float* lg, const float* work, float* o) {
+    constexpr int D = 16 * NT, kOwn = (NT + 3) / 4;
+    __shared__ __align__(16) float st[16][D + 4];           // S^T
+    __shared__ __align__(16) float ut[16][kChunk + 4], us[16][kChunk + 4];  // u^T, and times exp(G_last - G_s)
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int h = blockIdx.y, b = blockIdx.z, kh = h / (L.heads / L.kv_heads), v0 = 16 * blockIdx.x;
+    const int first = P.cu[b], n = P.cu[b + 1] - first, slot = P.slot[b];
+    if (n <= 0 || slot < 0 || slot >= L.nslots) return;
+    int64_t chunk0 = 0;  // chunks of the sequences before
+    for (int x = 0; x < b; ++x) chunk0 += (P.cu[x + 1] - P.cu[x] + kChunk - 1) / kChunk;
+    const int64_t wf = chunk_floats(D, L.vdim);
+    float* const S = L.state + ((int64_t)slot * L.heads + h) * D * L.vdim + v0 + 4 * g;
+    const bool fresh = P.pos0[b] == 0;
+    f32x4 s[kOwn];
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+        const int d = wave + 4 * i;
+        s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (d < NT) {
+            if (!fresh) s[i] = *reinterpret_cast<const f32x4*>(S + (int64_t)(16 * d + c) * L.vdim);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) st[4 * g + r][16 * d + c] = s[i][r];
+        }
+    }
+    const bool former = wave < 2;
+    const int tr = 16 * (wave % 2);  // the wave's rows of a chunk
+    struct Loads {
+        f32x4 a[NT], p[2];
+        float u0[4], kk[kOwn][8], decay;
+    } cur, nxt;
+    auto fetch = [&](int ch, Loads& x) __attribute__((always_inline)) {
+        const int row0 = first + ch * kChunk, m = n - ch * kChunk < kChunk ? n - ch * kChunk : kChunk;
+        const float* const w = work + ((chunk0 + ch) * L.heads + h) * wf;
+        const float* const wu = w + kChunk * D;
+        const float* const wp = wu + kChunk * L.vdim;
+        const int t = tr + c < m ? tr + c : m - 1;
+        const float* const a = former ? w + (tr + c) * D : q + ((int64_t)(row0 + t) * L.kv_heads + kh) * D;
+#pragma unroll
+        for (int i = 0; i < NT; ++i) x.a[i] = *reinterpret_cast<const f32x4*>(a + 16 * i + 4 * g);
+        if (former) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) x.u0[r] = wu[(tr + 4 * g + r) * L.vdim + v0 + c];
+        } else {
+#pragma unroll
+            for (int i = 0; i < 2; ++i) x.p[i] = *reinterpret_cast<const f32x4*>(wp + (tr + c) * kChunk + 16 * i + 4 * g);
+        }
+#pragma unroll
+        for (int i = 0; i < kOwn; ++i) {
+            const int d = wave + 4 * i < NT ? wave + 4 * i : 0;
+#pragma unroll
+            for (int y = 0; y < 8; ++y) {
+                const int tk = 16 * (y / 4) + 4 * g + y % 4;
+                x.kk[i][y] = k[((int64_t)(row0 + (tk < m ? tk : m - 1)) * L.kv_heads + kh) * D + 16 * d + c];
+            }
+        }
+        x.decay = lane < m ? lg[(int64_t)(row0 + lane) * L.heads + h] : 0.f;
+    };
+    const int chunks = (n + kChunk - 1) / kChunk;
+    fetch(0, cur);
+    __syncthreads();
+    for (int ch = 0; ch < chunks; ++ch) {
+        if (ch + 1 < chunks) fetch(ch + 1, nxt);
+        float G = cur.decay;
+#pragma unroll
+        for (int x = 1; x < kChunk; x <<= 1) {
+            const float y = __shfl_up(G, x);
+            if (lane >= x && lane < kChunk) G += y;
+        }
+        const float last = __shfl(G, kChunk - 1);
+        float gr[4];  // G of the wave's rows 4 g + r
+#pragma unroll
+        for (int r = 0; r < 4; ++r) gr[r] = __shfl(G, tr + 4 * g + r);
+        // W S or Q S
+        f32x4 x0 = {0.f, 0.f, 0.f, 0.f}, x1 = x0;
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            const f32x4 y = *reinterpret_cast<const f32x4*>(&st[c][16 * i + 4 * g]);
+            x0 = mfma_f32(cur.a[i][0], y[0], x0);
+            x1 = mfma_f32(cur.a[i][1], y[1], x1);
+            x0 = mfma_f32(cur.a[i][2], y[2], x0);
+            x1 = mfma_f32(cur.a[i][3], y[3], x1);
+        }
+        f32x4 res;
+        if (former) {
+            f32x4 u, w;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                u[r] = cur.u0[r] - (x0[r] + x1[r]);
+                w[r] = u[r] * expf(last - gr[r]);
+            }
+            *reinterpret_cast<f32x4*>(&ut[c][tr + 4 * g]) = u;
+            *reinterpret_cast<f32x4*>(&us[c][tr + 4 * g]) = w;
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) res[r] = (x0[r] + x1[r]) * expf(gr[r]);
+        }
+        __syncthreads();
+        const float gc = expf(last);
+        f32x4 uw[2];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) uw[i] = *reinterpret_cast<const f32x4*>(&us[c][16 * i + 4 * g]);
+#pragma unroll
+        for (int i = 0; i < kOwn; ++i) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s[i][r] *= gc;
+#pragma unroll
+            for (int y = 0; y < 8; ++y) s[i] = mfma_f32(uw[y / 4][y % 4], cur.kk[i][y], s[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < kOwn; ++i) {
+            const int d = wave + 4 * i;
+            if (d < NT) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) st[4 * g + r][16 * d + c] = s[i][r];
+            }
+        }
+        if (!former) {
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const f32x4 u = *reinterpret_cast<const f32x4*>(&ut[c][16 * i + 4 * g]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) res = mfma_f32(cur.p[i][e], u[e], res);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int t = ch * kChunk + tr + 4 * g + r;
+                if (t < n) o[((int64_t)(first + t) * L.heads + h) * L.vdim + v0 + c] = res[r];
+            }
+        }
+        __syncthreads();
+        cur = nxt;
+    }
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i) {
+        const int d = wave + 4 * i;
+        if (d < NT) *reinterpret_cast<f32x4*>(S + (int64_t)(16 * d + c) * L.vdim) = s[i];
+    }
+}
+
 // one wave per (row, head)
 template <class E>
 __global__ __launch_bounds__(kDeltaThreads) void delta_finish_kernel(const tah_delta_layer L, const float* o, int64_t items, E* out, int64_t out_rs,
@@ -604,6 +865,22 @@ void launch_prepare(const tah_delta_layer& L, const tah_portions& P, float* q, f
     hipLaunchKernelGGL((conv_tail_kernel<E>), tail, dim3(kDeltaThreads), 0, st, L, P);
 }
 
+// Portions long enough, and sizes in whole tiles, for the chunked form.
+constexpr int kChunkedFromRows = 48;  // rows per sequence, on average
+bool chunked(const tah_delta_layer& L, int rows, int nseq) {
+    const bool tiles = L.dim == 16 || L.dim == 32 || L.dim == 64 || L.dim == 128 || L.dim == 256;
+    return tiles && L.vdim % 16 == 0 && nseq > 0 && rows / nseq >= kChunkedFromRows;
+}
+int64_t chunk_slots(int rows, int nseq) { return (int64_t)rows / kChunk + nseq; }
+
+template <int NT>
+void launch_chunked(const tah_delta_layer& L, const tah_portions& P, const float* q, const float* k, const float* v, const float* lg, const float* beta,
+                    float* o, float* work, hipStream_t st) {
+    hipLaunchKernelGGL((delta_chunk_kernel<NT>), dim3((unsigned)chunk_slots(P.rows, P.nseq), L.heads), dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg,
+                       beta, work);
+    hipLaunchKernelGGL((delta_chunk_scan_kernel<NT>), dim3(L.vdim / 16, L.heads, P.nseq), dim3(kDeltaThreads), 0, st, L, P, q, k, lg, work, o);
+}
+
 template <class E>
 void launch_finish(const tah_delta_layer& L, const float* o, int rows, void* out, int64_t out_rs, int out_cols, hipStream_t st) {
     const int64_t items = (int64_t)rows * L.heads;
@@ -649,8 +926,14 @@ extern "C" int tah_delta_prepare(const tah_delta_layer* L, const tah_portions* p
     return launch_status();
 }
 
+extern "C" size_t tah_delta_scan_workspace(const tah_delta_layer* L, int32_t nseq, int32_t rows) {
+    using namespace tah;
+    if (check_layer(L) != TAH_OK || nseq <= 0 || rows <= 0 || !chunked(*L, rows, nseq)) return 0;
+    return (size_t)(chunk_slots(rows, nseq) * L->heads * chunk_floats(L->dim, L->vdim)) * sizeof(float);
+}
+
 extern "C" int tah_delta_scan(const tah_delta_layer* L, const tah_portions* p, const float* q, const float* k, const float* v, const float* lg,
-                              const float* beta, float* o, tah_stream_t stream) {
+                              const float* beta, float* o, void* workspace, size_t workspace_bytes, tah_stream_t stream) {
     using namespace tah;
     if (const int rc = check_layer(L)) return rc;
     if (const int rc = check_portions(p)) return rc;
@@ -659,6 +942,17 @@ extern "C" int tah_delta_scan(const tah_delta_layer* L, const tah_portions* p, c
     if (!aligned_16(q) || !aligned_16(k)) return TAH_E_ALIGN;
     const dim3 grid((L->vdim + kScanCols - 1) / kScanCols, L->heads, p->nseq);
     hipStream_t st = static_cast<hipStream_t>(stream);
+    if (const size_t need = tah_delta_scan_workspace(L, p->nseq, p->rows)) {
+        if (!workspace || workspace_bytes < need) return TAH_E_WORKSPACE;
+        if (!aligned_16(workspace)) return TAH_E_ALIGN;
+        float* const w = static_cast<float*>(workspace);
+        if (L->dim == 16) launch_chunked<1>(*L, *p, q, k, v, lg, beta, o, w, st);
+        else if (L->dim == 32) launch_chunked<2>(*L, *p, q, k, v, lg, beta, o, w, st);
+        else if (L->dim == 64) launch_chunked<4>(*L, *p, q, k, v, lg, beta, o, w, st);
+        else if (L->dim == 128) launch_chunked<8>(*L, *p, q, k, v, lg, beta, o, w, st);
+        else launch_chunked<16>(*L, *p, q, k, v, lg, beta, o, w, st);
+        return launch_status();
+    }
     if (L->dim <= 64) hipLaunchKernelGGL((delta_scan_kernel<1>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);
     else if (L->dim <= 128) hipLaunchKernelGGL((delta_scan_kernel<2>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);
     else hipLaunchKernelGGL((delta_scan_kernel<4>), grid, dim3(kDeltaThreads), 0, st, *L, *p, q, k, v, lg, beta, o);

@@ -246,6 +246,26 @@ inline emu_f32x4 emu_mfma_16x16x32_bf16(emu_bf16x8 a, emu_bf16x8 b, emu_f32x4 c,
     emu::wave_sync();
     return d;
 }
+// 16x16x4 f32: A[i=l%16][k=l/16], B[k=l/16][j=l%16], C/D as above
+inline emu_f32x4 emu_mfma_16x16x4_f32(float a, float b, emu_f32x4 c, int, int, int) {
+    float s[2] = {a, b};
+    memcpy(emu::t_wave->box[emu::t_lane], s, sizeof(s));
+    emu::wave_sync();
+    const int l = emu::t_lane, j = l % 16;
+    emu_f32x4 d = c;
+    for (int r = 0; r < 4; ++r) {
+        const int i = 4 * (l / 16) + r;
+        for (int k = 0; k < 4; ++k) {
+            float sa[2], sb[2];
+            memcpy(sa, emu::t_wave->box[i + 16 * k], sizeof(sa));
+            memcpy(sb, emu::t_wave->box[j + 16 * k], sizeof(sb));
+            d[r] += sa[0] * sb[1];
+        }
+    }
+    emu::wave_sync();
+    return d;
+}
+#define __builtin_amdgcn_mfma_f32_16x16x4f32 emu_mfma_16x16x4_f32
 #define __builtin_amdgcn_mfma_f32_32x32x16_bf16 emu_mfma_32x32x16_bf16
 #define __builtin_amdgcn_mfma_f32_16x16x32_bf16 emu_mfma_16x16x32_bf16
 

@@ -214,6 +214,8 @@ __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __
 
 __device__ __forceinline__ bf16x8 join8(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
 
+__device__ __forceinline__ bf16x4 to_bf16x4(const float (&w)[4]) { return __builtin_convertvector((f32x4{w[0], w[1], w[2], w[3]}), bf16x4); }
+
 // x over the four lane groups that share l % 16
 __device__ __forceinline__ float groups_max(float x) {
     x = fmaxf(x, __shfl_xor(x, 16));
@@ -336,31 +338,41 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
             bf16x8 ph[2][2], pl[2][2];  // [pair of key tiles][query tile]
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
-                float mx = kNoScore;
+                if (!all) {
 #pragma unroll
-                for (int x = 0; x < 4; ++x)
+                    for (int x = 0; x < 4; ++x)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        float y = sc[x][t][r] * p.scale_log2;
-                        const int j = j0 + 16 * x + 4 * g + r;
-                        if (!all && (j > own[t] || j <= own[t] - p.window)) y = kNegInf;
-                        sc[x][t][r] = y;
-                        mx = fmaxf(mx, y);
-                    }
-                mx = fmaxf(m[t], groups_max(mx));
+                        for (int r = 0; r < 4; ++r) {
+                            const int j = j0 + 16 * x + 4 * g + r;
+                            if (j > own[t] || j <= own[t] - p.window) sc[x][t][r] = kNegInf;
+                        }
+                }
+                // (maximum before the scale, which is positive; scale and difference are one multiply-add)
+                float mx = fmaxf(fmaxf(sc[0][t][0], sc[0][t][1]), fmaxf(sc[0][t][2], sc[0][t][3]));
+#pragma unroll
+                for (int x = 1; x < 4; ++x) mx = fmaxf(mx, fmaxf(fmaxf(sc[x][t][0], sc[x][t][1]), fmaxf(sc[x][t][2], sc[x][t][3])));
+                mx = fmaxf(m[t], groups_max(mx) * p.scale_log2);
                 const float a = fast_exp2(m[t] - mx);
                 m[t] = mx;
                 float sum = 0.f;
 #pragma unroll
-                for (int x = 0; x < 4; ++x)
+                for (int x = 0; x < 4; ++x) {
+                    float w[4];
 #pragma unroll
                     for (int r = 0; r < 4; ++r) {
-                        const float w = fast_exp2(sc[x][t][r] - mx);
-                        sum += w;
-                        const __bf16 hi = (__bf16)w;
-                        ph[x / 2][t][4 * (x % 2) + r] = hi;
-                        pl[x / 2][t][4 * (x % 2) + r] = (__bf16)(w - (float)hi);
+                        w[r] = fast_exp2(__builtin_fmaf(sc[x][t][r], p.scale_log2, -mx));
+                        sum += w[r];
                     }
+                    const bf16x4 hi = to_bf16x4(w);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) w[r] -= (float)hi[r];
+                    const bf16x4 lo = to_bf16x4(w);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        ph[x / 2][t][4 * (x % 2) + r] = hi[r];
+                        pl[x / 2][t][4 * (x % 2) + r] = lo[r];
+                    }
+                }
                 l[t] = l[t] * a + sum;
                 if (__ballot(a != 1.0f) != 0) {
 #pragma unroll
@@ -477,10 +489,17 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
         __syncthreads();
         if (j0 + kTileKeys <= end) fetch(j0 + kTileKeys);
         // scores of this wave's sixteen keys: register r of lane (c, g) is key 16 wave + 4 g + r, head c
-        f32x4 sc = f32x4{0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < steps; ++s)
-            sc = mfma16(*reinterpret_cast<const bf16x8*>(kt + (16 * wave + c) * ks + 32 * s + 8 * g),
-                        *reinterpret_cast<const bf16x8*>(qt + c * ks + 32 * s + 8 * g), sc);
+        f32x4 sc = f32x4{0.f, 0.f, 0.f, 0.f}, sc2 = sc;
+#pragma unroll
+        for (int s = 0; s < NU; ++s)  // (a row has as many steps of 32 as a thread has units of a tile)
+            if (s < steps) {
+                const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + (16 * wave + c) * ks + 32 * s + 8 * g);
+                const bf16x8 b = *reinterpret_cast<const bf16x8*>(qt + c * ks + 32 * s + 8 * g);
+                if (s % 2) sc2 = mfma16(a, b, sc2);
+                else sc = mfma16(a, b, sc);
+            }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[r] += sc2[r];
         float mw = kNoScore;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
@@ -693,7 +712,7 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
     if (!cu_k || !q || !k || !v || !ctx || !out) return TAH_E_NULL;
     if (!aligned_16(q) || !aligned_16(k) || !aligned_16(v) || !aligned_16(ctx) || !aligned_16(out)) return TAH_E_ALIGN;
     const int nq = (L->dim_pad + L->rot_pad) / 32, nv = (L->vdim_pad + 15) / 16;
-    if (L->dtype == TAH_DT_BF16 && nq <= 10 && nv <= 16) {
+    if (L->dtype == TAH_DT_BF16 && nq <= 10 && nv <= 16 && L->scale > 0.f) {
         AttendTile t{};
         t.q = static_cast<const __bf16*>(q); t.k = static_cast<const __bf16*>(k); t.v = static_cast<const __bf16*>(v);
         t.ctx = static_cast<const __bf16*>(ctx) + L->rank_pad;

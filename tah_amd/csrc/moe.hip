@@ -6,7 +6,7 @@
 //    workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
 //  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
 //  * moe_tile_kernel: bf16 tiles of 128 places x 128 weight rows on the matrix cores, both operands staged through LDS
-//    by asynchronous copies, two stages; gate and up rows of the same columns share a wave, which applies the gate.
+//    by asynchronous copies, three stages ahead; gate and up rows of the same columns share a wave, which applies the gate.
 //  * moe_plain_kernel: the same product in float32 arithmetic (the float32 form of a model).
 #include <hip/hip_runtime.h>
 
@@ -160,8 +160,12 @@ __device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int& tile, int& co
 }
 
 // ---- bf16 tiles ------------------------------------------------------------------------------------------------
-constexpr int kStageK = 64;
-constexpr int kStageBytes = 2 * kTile * kStageK * 2;  // both operands of one stage: 128 x 64 bf16 each
+constexpr int kStageK = 32;
+constexpr int kStages = 4;
+constexpr int kStageBytes = 2 * kTile * kStageK * 2;  // both operands of one stage: 128 x 32 bf16 each
+// LDS tile of rows x 32 bf16 (64 B per row, 4 chunks of 16 B): chunks permuted so that sixteen rows' reads of one logical
+// chunk touch sixteen different places of 256 bytes
+__device__ __forceinline__ int rowmajor32_off(int row, int chunk) { return row * 64 + ((chunk ^ ((row >> 2) & 3)) << 4); }
 
 // Four waves, 2 x 2: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
 template <bool GATE>
@@ -175,17 +179,16 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
     const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
     constexpr int kCols = GATE ? kTile / 2 : kTile;  // output columns of a tile
     const int n0 = col_tile * kCols;
-    // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
-    // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
-    const __bf16 *ga[4], *gb[4];
-    int chunk[4];
+    // This lane's part of the copies: of every sixteen rows a wave copies, row lane / 4, sixteen bytes at the logical chunk
+    // that lies at place lane % 4 of the row in LDS.
+    const __bf16 *ga[2], *gb[2];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int r = 8 * (4 * wave + i) + lane / 8;
-        chunk[i] = (lane % 8) ^ ((r >> 1) & 7);
+    for (int i = 0; i < 2; ++i) {
+        const int r = 16 * (2 * wave + i) + lane / 4;
+        const int chunk = (lane % 4) ^ ((r >> 2) & 3);
         int src = GATE ? p.source[tile * kTile + r] : tile * kTile + r;
         src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
-        ga[i] = x + (int64_t)src * p.x_rs;
+        ga[i] = x + (int64_t)src * p.x_rs + 8 * chunk;
         int wr;
         if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
             int c = n0 + 32 * (r / 64) + r % 32;
@@ -194,51 +197,43 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
         } else {
             wr = n0 + r < p.n ? n0 + r : p.n - 1;
         }
-        gb[i] = w + (int64_t)wr * p.k;
+        gb[i] = w + (int64_t)wr * p.k + 8 * chunk;
     }
-    auto stage = [&](int s, int k0) __attribute__((always_inline)) {
-        unsigned char* const base = lds + s * kStageBytes;
-        const int valid = (p.k - k0) / 8;  // chunks of this stage inside the rows
+    auto stage = [&](int s) __attribute__((always_inline)) {
+        unsigned char* const base = lds + (s % kStages) * kStageBytes;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int c = chunk[i] < valid ? chunk[i] : 0;
-            async_copy_16B(ga[i] + k0 + 8 * c, base + (4 * wave + i) * 1024);
-        }
+        for (int i = 0; i < 2; ++i) async_copy_16B(ga[i] + s * kStageK, base + (2 * wave + i) * 1024);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int c = chunk[i] < valid ? chunk[i] : 0;
-            async_copy_16B(gb[i] + k0 + 8 * c, base + kTile * kStageK * 2 + (4 * wave + i) * 1024);
-        }
+        for (int i = 0; i < 2; ++i) async_copy_16B(gb[i] + s * kStageK, base + kTile * kStageK * 2 + (2 * wave + i) * 1024);
     };
     f32x4 acc[4][4];  // [weight tile][place tile]
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int stages = (p.k + kStageK - 1) / kStageK;
-    stage(0, 0);
-    TAH_WAIT_VMEM();
-    __syncthreads();
+    const int stages = p.k / kStageK;
+    TAH_WAIT_VMEM();  // (the places' sources: from here on only copies are on their way)
+    for (int s = 0; s < kStages - 1 && s < stages; ++s) stage(s);
     for (int s = 0; s < stages; ++s) {
-        if (s + 1 < stages) stage((s + 1) & 1, (s + 1) * kStageK);
-        const unsigned char* const a = lds + (s & 1) * kStageBytes;
+        // four copies per stage: all but those of the (at most two) stages behind this one have landed
+        const int behind = stages - 1 - s;
+        if (behind >= 2) TAH_WAIT_VMEM_N(8);
+        else if (behind == 1) TAH_WAIT_VMEM_N(4);
+        else TAH_WAIT_VMEM();
+        __syncthreads();  // every wave's copies of stage s are in, and nobody reads stage s - 1 any more
+        if (s + kStages - 1 < stages) stage(s + kStages - 1);
+        const unsigned char* const a = lds + (s % kStages) * kStageBytes;
         const unsigned char* const b = a + kTile * kStageK * 2;
+        bf16x8 fx[4], fw[4];
 #pragma unroll
-        for (int h = 0; h < 2; ++h) {
-            if (s * kStageK + 32 * h >= p.k) break;  // (uniform)
-            bf16x8 fx[4], fw[4];
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor64_off(64 * wm + 16 * j + lane % 16, 4 * h + lane / 16));
-                fw[j] = *reinterpret_cast<const bf16x8*>(b + rowmajor64_off(64 * wn + 16 * j + lane % 16, 4 * h + lane / 16));
-            }
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-#pragma unroll
-                for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
+        for (int j = 0; j < 4; ++j) {
+            fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor32_off(64 * wm + 16 * j + lane % 16, lane / 16));
+            fw[j] = *reinterpret_cast<const bf16x8*>(b + rowmajor32_off(64 * wn + 16 * j + lane % 16, lane / 16));
         }
-        TAH_WAIT_VMEM();
-        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
     }
     // accumulator (i, j) register r of lane l: weight row 16 i + 4 (l / 16) + r, place 16 j + l % 16
     __bf16* const out = static_cast<__bf16*>(p.out);
@@ -319,8 +314,8 @@ void launch_route(const float* x, const void* router, const void* gate_w, int ro
     const E* const rt = static_cast<const E*>(router);
     const E* const gw = static_cast<const E*>(gate_w);
     const auto lds = [&](int rb) { return (size_t)rb * (cols + experts + 1) * sizeof(float); };
-    if (rows > 256 && lds(8) <= 65536)  // many rows: eight share a pass over the router's weights
-        hipLaunchKernelGGL((moe_route_kernel<E, 8, 4, 256>), dim3((rows + 7) / 8), dim3(256), lds(8), st, x, rt, gw, rows, cols, experts, top, index,
+    if (rows > 256 && lds(4) <= 65536)  // many rows: four share a pass over the router's weights
+        hipLaunchKernelGGL((moe_route_kernel<E, 4, 4, 256>), dim3((rows + 3) / 4), dim3(256), lds(4), st, x, rt, gw, rows, cols, experts, top, index,
                            weight, shared_gate);
     else  // few rows: what counts is how much of the router's weights one row has in flight
         hipLaunchKernelGGL((moe_route_kernel<E, 1, 2, 1024>), dim3(rows), dim3(1024), lds(1), st, x, rt, gw, rows, cols, experts, top, index, weight,
@@ -380,8 +375,8 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
     const dim3 grid((unsigned)groups);
     hipStream_t st = static_cast<hipStream_t>(stream);
     if (dtype == TAH_DT_BF16) {
-        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
-        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), 2 * kStageBytes, st, p);
+        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
+        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
     } else {
         if (gate) hipLaunchKernelGGL((moe_plain_kernel<true>), grid, dim3(kMoeThreads), 0, st, p);
         else hipLaunchKernelGGL((moe_plain_kernel<false>), grid, dim3(kMoeThreads), 0, st, p);

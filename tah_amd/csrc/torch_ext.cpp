@@ -69,6 +69,7 @@ void load_library(const std::string& path, bool allow_host) {
     bind(g.delta_step, "tah_delta_step");
     bind(g.delta_prepare, "tah_delta_prepare");
     bind(g.delta_scan, "tah_delta_scan");
+    bind(g.delta_scan_workspace, "tah_delta_scan_workspace");
     bind(g.delta_finish, "tah_delta_finish");
     bind(g.latent_prep, "tah_latent_prep");
     bind(g.latent_context, "tah_latent_context");

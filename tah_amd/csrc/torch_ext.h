@@ -67,6 +67,7 @@ struct Api {
     Entry<decltype(&tah_delta_step)> delta_step;
     Entry<decltype(&tah_delta_prepare)> delta_prepare;
     Entry<decltype(&tah_delta_scan)> delta_scan;
+    Entry<decltype(&tah_delta_scan_workspace)> delta_scan_workspace;
     Entry<decltype(&tah_delta_finish)> delta_finish;
     Entry<decltype(&tah_latent_prep)> latent_prep;
     Entry<decltype(&tah_latent_context)> latent_context;

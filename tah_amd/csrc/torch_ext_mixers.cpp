@@ -174,7 +174,10 @@ struct DeltaLayer {
         Tensor q = at::empty({P.rows, L.kv_heads, L.dim}, f32), k = at::empty_like(q), v = at::empty({P.rows, L.heads, L.vdim}, f32);
         Tensor lg = at::empty({P.rows, L.heads}, f32), beta = at::empty_like(lg), o = at::empty_like(v);
         check_rc(g.delta_prepare(&l, &P, at_<float>(q), at_<float>(k), at_<float>(v), at_<float>(lg), at_<float>(beta), d.stream()), "tah_delta_prepare");
-        check_rc(g.delta_scan(&l, &P, at_<float>(q), at_<float>(k), at_<float>(v), at_<float>(lg), at_<float>(beta), at_<float>(o), d.stream()),
+        const size_t bytes = g.delta_scan_workspace(&l, P.nseq, P.rows);
+        Tensor work = at::empty({(int64_t)bytes}, proj.options().dtype(at::kByte));
+        check_rc(g.delta_scan(&l, &P, at_<float>(q), at_<float>(k), at_<float>(v), at_<float>(lg), at_<float>(beta), at_<float>(o), mptr(work), bytes,
+                              d.stream()),
                  "tah_delta_scan");
         check_rc(g.delta_finish(&l, at_<float>(o), P.rows, mptr(out), rs, (int32_t)out.size(1), d.stream()), "tah_delta_finish");
     }

@@ -19,12 +19,14 @@ def latent(heads, dim, rot, vdim, rank, window, base=50.0, scale=0.4):
 
 # (sizes, lengths, portions per sequence)
 DELTA_SMALL = [(delta(2, 1, 6, 5, 3), (5, 3), ((2, 3), (3,))), (delta(2, 2, 12, 8, 4), (7, 2), ((7,), (2,))),
-               (delta(2, 1, 16, 32, 3), (5, 4), ((3, 2), (4,)))]
+               (delta(2, 1, 16, 32, 3), (5, 4), ((3, 2), (4,))),
+               (delta(2, 1, 16, 16, 4), (100, 49), ((50, 50), (49,)))]   # long enough for the chunked form
 DELTA_GPU = DELTA_SMALL + [
     (delta(6, 3, 40, 24, 4), (70, 33), ((37, 2, 31), (2, 31))), (delta(4, 4, 64, 64, 2), (130, 5), ((128, 2), (3, 2))),
     (delta(8, 2, 128, 128, 4), (200, 65), ((64, 17, 119), (65,))), (delta(2, 1, 256, 96, 4), (40, 40), ((40,), (17, 23))),
     (delta(3, 1, 17, 130, 1), (30, 9), ((16, 14), (9,))), (delta(2, 2, 100, 256, 5), (21, 2), ((5, 16), (2,))),
-    (delta(5, 5, 32, 512, 3), (19, 18), ((19,), (2, 16))),
+    (delta(5, 5, 32, 512, 3), (19, 18), ((19,), (2, 16))), (delta(4, 2, 128, 64, 4), (333, 97), ((96, 64, 173), (97,))),
+    (delta(2, 1, 256, 32, 2), (161, 70), ((100, 61), (70,))), (delta(6, 3, 32, 48, 4), (520, 520), ((255, 265), (256, 264))),
 ]
 # (sizes, prompt, portions, decoded tokens, ring capacity)
 LATENT_SMALL = [(latent(2, 8, 4, 6, 10, 4), 9, (2, 5, 2), 3, None), (latent(1, 32, 6, 16, 40, 3), 6, (6,), 2, 5)]
