@@ -526,7 +526,7 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
     constexpr int D = 16 * NT, kStride = D + 4;
     __shared__ __align__(16) float kl[kChunk][kStride], ql[kChunk][kStride];
     __shared__ __align__(16) float al[kChunk][kChunk + 4];
-    __shared__ float gl[kChunk], bl[kChunk];
+    __shared__ float gl[kChunk], bl[kChunk], be[kChunk];  // G, beta, beta exp(G)
     int slot = blockIdx.x, b = 0, row0 = 0, row_end = 0;
     if (!find_tile(P.cu, P.nseq, kChunk, slot, b, row0, row_end)) return;
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
@@ -550,6 +550,7 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
         if (lane < kChunk) {
             gl[lane] = x;
             bl[lane] = lane < n ? beta[(int64_t)(row0 + lane) * L.heads + h] : 0.f;
+            be[lane] = bl[lane] * expf(x);
         }
     }
     __syncthreads();
@@ -589,11 +590,12 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
         float x[kChunk];
 #pragma unroll
         for (int t = 0; t < kChunk; ++t) {
-            if (is_k) x[t] = bl[t] * expf(gl[t]) * kl[t][i];
+            if (is_k) x[t] = be[t] * kl[t][i];
             else x[t] = t < n ? bl[t] * v[((int64_t)(row0 + t) * L.heads + h) * L.vdim + i] : 0.f;
         }
 #pragma unroll
         for (int t = 1; t < kChunk; ++t) {
+            if (t % 2) asm volatile("" ::: "memory");  // (the matrix is read row by row, not all of it into registers)
 #pragma unroll
             for (int s4 = 0; s4 < (t + 3) / 4; ++s4) {
                 const f32x4 a = *reinterpret_cast<const f32x4*>(&al[t][4 * s4]);
@@ -609,7 +611,8 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
     }
 }
 
-// grid (16-column slices, heads, sequences).  Waves 0 and 1 form u, waves 2 and 3 the results; each holds every fourth
+// One workgroup per 16-column slice of a (sequence, head).  Workgroups go to the XCDs round robin: the slices of a head are
+// placed on one XCD, whose L2 then fetches what they share once.  Waves 0 and 1 form u, waves 2 and 3 the results; each holds every fourth
 // 16-row tile of the state's slice, register r of lane (c, g) of tile i being S[16 i + c][4 g + r].
 template <int NT>
 __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
@@ -618,7 +621,9 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const t
     __shared__ __align__(16) float st[16][D + 4];           // S^T
     __shared__ __align__(16) float ut[16][kChunk + 4], us[16][kChunk + 4];  // u^T, and times exp(G_last - G_s)
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
-    const int h = blockIdx.y, b = blockIdx.z, kh = h / (L.heads / L.kv_heads), v0 = 16 * blockIdx.x;
+    const int slices = L.vdim / 16, item = blockIdx.x / 8 / slices * 8 + blockIdx.x % 8;
+    if (item >= L.heads * P.nseq) return;
+    const int h = item % L.heads, b = item / L.heads, kh = h / (L.heads / L.kv_heads), v0 = 16 * (blockIdx.x / 8 % slices);
     const int first = P.cu[b], n = P.cu[b + 1] - first, slot = P.slot[b];
     if (n <= 0 || slot < 0 || slot >= L.nslots) return;
     int64_t chunk0 = 0;  // chunks of the sequences before
@@ -878,7 +883,7 @@ void launch_chunked(const tah_delta_layer& L, const tah_portions& P, const float
                     float* o, float* work, hipStream_t st) {
     hipLaunchKernelGGL((delta_chunk_kernel<NT>), dim3((unsigned)chunk_slots(P.rows, P.nseq), L.heads), dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg,
                        beta, work);
-    hipLaunchKernelGGL((delta_chunk_scan_kernel<NT>), dim3(L.vdim / 16, L.heads, P.nseq), dim3(kDeltaThreads), 0, st, L, P, q, k, lg, work, o);
+    hipLaunchKernelGGL((delta_chunk_scan_kernel<NT>), dim3((unsigned)((L.heads * P.nseq + 7) / 8 * 8 * (L.vdim / 16))), dim3(kDeltaThreads), 0, st, L, P, q, k, lg, work, o);
 }
 
 template <class E>

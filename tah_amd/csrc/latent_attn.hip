@@ -232,22 +232,32 @@ struct AttendTile {
     __bf16* out;
     int64_t out_rs;
     const int32_t *cu, *cu_k;
-    int32_t nseq, dim_pad, rot_pad, vdim_pad, window;
+    int32_t nseq, dim_pad, rot_pad, vdim_pad, window, heads, slots;
     float scale_log2;
 };
 
-// NQ: 32-wide steps of a query row (at most), NV: 16-wide tiles of a value row (at most), W: waves, 32 query rows each.
-template <int NQ, int NV, int W>
+// NQ: 32-wide steps of a query row (at most), NV: 16-wide tiles of a value row (at most; kExact: just so many, and no
+// branch stands between a tile's products), W: waves, 32 query rows each.
+template <int NQ, int NV, int W, bool kExact>
 __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile p) {
     constexpr int kTileRows = 32 * W, kTileThreads = W * kWave;
     HIP_DYNAMIC_SHARED(unsigned char, tile_lds)
-    int tile = blockIdx.x, b = 0, row0 = 0, row_end = 0;
+    // (workgroups go to the XCDs round robin: where the heads divide among them, a head's tiles share an XCD and its L2)
+    int tile, b = 0, row0 = 0, row_end = 0, h;
+    if (p.heads % 8 == 0) {
+        tile = blockIdx.x / 8 % p.slots;
+        h = blockIdx.x / 8 / p.slots * 8 + blockIdx.x % 8;
+    } else {
+        tile = blockIdx.x % p.slots;
+        h = blockIdx.x / p.slots;
+    }
     if (!find_tile(p.cu, p.nseq, kTileRows, tile, b, row0, row_end)) return;
-    const int h = blockIdx.y, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
-    const int dq = p.dim_pad + p.rot_pad, nq = dq / 32, nv = p.vdim_pad / 16;
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int dq = p.dim_pad + p.rot_pad, nq = kExact ? NQ : dq / 32, nv = kExact ? NV : p.vdim_pad / 16;
     const int ks = dq + 8, vs = p.vdim_pad + 8;  // row strides in LDS: rows start in different banks
     __bf16* const kt = reinterpret_cast<__bf16*>(tile_lds);
     __bf16* const vt = kt + kTileKeys * ks;
+    const int buffer = kTileKeys * (ks + vs);  // two of them: the next tile is written while this one is read
     const int first = p.cu[b], n = p.cu[b + 1] - first, k0 = p.cu_k[b], lk = p.cu_k[b + 1] - k0;
     // a query row's own key, as a context row of its sequence: row - first + lk - n
     const int shift = lk - n - first;
@@ -261,7 +271,7 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
         own[t] = r + shift;
 #pragma unroll
         for (int s = 0; s < NQ; ++s)
-            if (s < nq) q[t][s] = *reinterpret_cast<const bf16x8*>(p.q + (int64_t)r * p.q_rs + (int64_t)h * dq + 32 * s + 8 * g);
+            if (kExact || s < nq) q[t][s] = *reinterpret_cast<const bf16x8*>(p.q + (int64_t)r * p.q_rs + (int64_t)h * dq + 32 * s + 8 * g);
     }
     const int own_lo = (wrow < row_end ? wrow : row_end - 1) + shift;
     const int own_hi = (wrow + 31 < row_end ? wrow + 31 : row_end - 1) + shift;
@@ -308,16 +318,21 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
             if (vkey[i] >= 0) fv[i] = *reinterpret_cast<const bf16x8*>(gv[i] + (j < lk ? j : lk - 1) * p.v_rs);
         }
     };
-    fetch(j_lo);
-    for (int j0 = j_lo; j0 <= j_hi; j0 += kTileKeys) {
+    auto store = [&](int at) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < UK; ++i)
-            if (kkey[i] >= 0) *reinterpret_cast<bf16x8*>(kt + kdst[i]) = fk[i];
+            if (kkey[i] >= 0) *reinterpret_cast<bf16x8*>(kt + at + kdst[i]) = fk[i];
 #pragma unroll
         for (int i = 0; i < UV; ++i)
-            if (vkey[i] >= 0) *reinterpret_cast<bf16x8*>(vt + vdst[i]) = fv[i];
-        __syncthreads();
-        if (j0 + kTileKeys <= j_hi) fetch(j0 + kTileKeys);
+            if (vkey[i] >= 0) *reinterpret_cast<bf16x8*>(vt + at + vdst[i]) = fv[i];
+    };
+    fetch(j_lo);
+    store(0);
+    int now = 0;
+    for (int j0 = j_lo; j0 <= j_hi; j0 += kTileKeys, now = buffer - now) {
+        const bool more = j0 + kTileKeys <= j_hi;
+        if (more) fetch(j0 + kTileKeys);
+        __syncthreads();  // this tile is written, and nobody reads the other buffer any more
         // (uniform per wave) does this wave see anything of the tile, and does it see all of it?
         const bool any = j0 <= own_hi && j0 + kTileKeys - 1 > own_lo - p.window;
         const bool all = j0 + kTileKeys - 1 <= own_lo && j0 > own_hi - p.window;
@@ -329,8 +344,8 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
                 for (int t = 0; t < 2; ++t) sc[x][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int s = 0; s < NQ; ++s)
-                    if (s < nq) {
-                        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + (16 * x + c) * ks + 32 * s + 8 * g);
+                    if (kExact || s < nq) {
+                        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + now + (16 * x + c) * ks + 32 * s + 8 * g);
 #pragma unroll
                         for (int t = 0; t < 2; ++t) sc[x][t] = mfma16(a, q[t][s], sc[x][t]);
                     }
@@ -383,10 +398,10 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
             }
 #pragma unroll
             for (int i = 0; i < NV; ++i)
-                if (i < nv) {
+                if (kExact || i < nv) {
 #pragma unroll
                     for (int x = 0; x < 2; ++x) {
-                        const __bf16* at = vt + (32 * x + 4 * g + c / 4) * vs + 16 * i + 4 * (c % 4);
+                        const __bf16* at = vt + now + (32 * x + 4 * g + c / 4) * vs + 16 * i + 4 * (c % 4);
                         const bf16x8 a = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
                                                lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * vs)));
 #pragma unroll
@@ -397,7 +412,7 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
                     }
                 }
         }
-        __syncthreads();
+        if (more) store(buffer - now);
     }
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
@@ -406,7 +421,7 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
         if (r < row_end) {
 #pragma unroll
             for (int i = 0; i < NV; ++i)
-                if (i < nv) {
+                if (kExact || i < nv) {
                     bf16x4 y;
 #pragma unroll
                     for (int e = 0; e < 4; ++e) y[e] = (__bf16)(acc[i][t][e] * inv);
@@ -426,13 +441,13 @@ struct LatentDecode {
 };
 
 // grid (splits, groups of 16 heads, rows).  NT: 16-wide tiles of the latent per wave (at most); NU: 16-byte units of a key
-// tile per thread (at most).
-template <int NT, int NU>
+// tile per thread, and of steps of 32 of a row (at most; kExact: just so many).
+template <int NT, int NU, bool kExact>
 __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const LatentDecode p) {
     HIP_DYNAMIC_SHARED(unsigned char, dec_lds)
     __shared__ float mx_[kLatWaves][16], sum_[kLatWaves][16];
     const int row = blockIdx.z, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
-    const int lp = p.rank_pad + p.rot_pad, steps = lp / 32, nt = p.rank_pad / 16, ks = lp + 8, ps = kTileKeys + 8;
+    const int lp = kExact ? 32 * NU : p.rank_pad + p.rot_pad, steps = lp / 32, nt = kExact ? kLatWaves * NT : p.rank_pad / 16, ks = lp + 8, ps = kTileKeys + 8;
     __bf16* const kt = reinterpret_cast<__bf16*>(dec_lds);  // [64 keys][ks]
     __bf16* const qt = kt + kTileKeys * ks;                 // [16 heads][ks]
     __bf16* const pt = qt + 16 * ks;                        // [2 terms][16 heads][ps]
@@ -453,7 +468,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
 #pragma unroll
     for (int i = 0; i < NU; ++i) {
         const int u = tid + kLatThreads * i;
-        key[i] = u < units ? u / upk : -1;
+        key[i] = kExact || u < units ? u / upk : -1;
         dst[i] = (u / upk) * ks + 8 * (u % upk);
     }
     // a key's row of the ring: the first one's, advanced, wrapped at most once per tile (a tile is not longer than the ring,
@@ -492,7 +507,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
         f32x4 sc = f32x4{0.f, 0.f, 0.f, 0.f}, sc2 = sc;
 #pragma unroll
         for (int s = 0; s < NU; ++s)  // (a row has as many steps of 32 as a thread has units of a tile)
-            if (s < steps) {
+            if (kExact || s < steps) {
                 const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + (16 * wave + c) * ks + 32 * s + 8 * g);
                 const bf16x8 b = *reinterpret_cast<const bf16x8*>(qt + c * ks + 32 * s + 8 * g);
                 if (s % 2) sc2 = mfma16(a, b, sc2);
@@ -536,7 +551,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_decode_kernel(const Latent
 #pragma unroll
             for (int i = 0; i < NT; ++i) {
                 const int t = wave + kLatWaves * i;
-                if (t < nt) {
+                if (kExact || t < nt) {
                     const __bf16* at = kt + (32 * x + 4 * g + c / 4) * ks + 16 * t + 4 * (c % 4);
                     const bf16x8 v = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
                                            lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * ks)));
@@ -625,13 +640,14 @@ void launch_attend_rows(const AttendRows& p, int heads, int dtype, hipStream_t s
 }
 size_t elem_bytes(int dtype) { return dtype == TAH_DT_BF16 ? 2 : 4; }
 
-template <int NQ, int NV, int W>
-int launch_attend_tile(const AttendTile& p, int rows, int heads, hipStream_t st) {
-    const size_t lds = (size_t)kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 8) * 2;
-    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV, W>), hipFuncAttributeMaxDynamicSharedMemorySize,
-                                           (int)lds) != hipSuccess)
+template <int NQ, int NV, int W, bool kExact>
+int launch_attend_tile(AttendTile p, int rows, hipStream_t st) {
+    const size_t lds = (size_t)2 * kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 8) * 2;
+    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV, W, kExact>),
+                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
         return TAH_E_LAUNCH;
-    hipLaunchKernelGGL((attend_tile_kernel<NQ, NV, W>), dim3(rows / (32 * W) + p.nseq, heads), dim3(W * kWave), lds, st, p);
+    p.slots = rows / (32 * W) + p.nseq;
+    hipLaunchKernelGGL((attend_tile_kernel<NQ, NV, W, kExact>), dim3((unsigned)(p.slots * p.heads)), dim3(W * kWave), lds, st, p);
     return launch_status();
 }
 
@@ -648,13 +664,13 @@ size_t decode_lds(int lp) { return ((size_t)(kTileKeys + 16) * (lp + 8) + 2 * 16
 constexpr size_t kLdsBytes = 160 * 1024 - 1024;  // a compute unit's LDS, less the kernel's static part
 bool decode_on_tiles(const tah_latent_layer* L) { return L->dtype == TAH_DT_BF16 && decode_lds(L->rank_pad + L->rot_pad) <= kLdsBytes; }
 
-template <int NT, int NU>
+template <int NT, int NU, bool kExact>
 int launch_latent_decode(const LatentDecode& p, hipStream_t st) {
     const size_t lds = decode_lds(p.rank_pad + p.rot_pad);
-    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NT, NU>), hipFuncAttributeMaxDynamicSharedMemorySize,
+    if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NT, NU, kExact>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                            (int)lds) != hipSuccess)
         return TAH_E_LAUNCH;
-    hipLaunchKernelGGL((latent_decode_kernel<NT, NU>), dim3(p.splits, (p.heads + 15) / 16, p.rows), dim3(kLatThreads), lds, st, p);
+    hipLaunchKernelGGL((latent_decode_kernel<NT, NU, kExact>), dim3(p.splits, (p.heads + 15) / 16, p.rows), dim3(kLatThreads), lds, st, p);
     return launch_status();
 }
 
@@ -722,9 +738,11 @@ extern "C" int tah_latent_attend(const tah_latent_layer* L, const tah_portions* 
         t.dim_pad = L->dim_pad; t.rot_pad = L->rot_pad; t.vdim_pad = L->vdim_pad; t.window = L->window;
         t.scale_log2 = L->scale * kLog2e;
         hipStream_t st = static_cast<hipStream_t>(stream);
-        if (nq <= 4 && nv <= 4) return launch_attend_tile<4, 4, 8>(t, p->rows, L->heads, st);
-        if (nq <= 6 && nv <= 8) return launch_attend_tile<6, 8, 8>(t, p->rows, L->heads, st);
-        return launch_attend_tile<10, 16, 4>(t, p->rows, L->heads, st);
+        t.heads = L->heads;
+        if (nq == 6 && nv == 8) return launch_attend_tile<6, 8, 8, true>(t, p->rows, st);
+        if (nq <= 4 && nv <= 4) return launch_attend_tile<4, 4, 8, false>(t, p->rows, st);
+        if (nq <= 6 && nv <= 8) return launch_attend_tile<6, 8, 8, false>(t, p->rows, st);
+        return launch_attend_tile<10, 16, 4, false>(t, p->rows, st);
     }
     AttendRows a{};
     a.q1 = q; a.q1_rs = q_rs; a.q1_hs = L->dim_pad + L->rot_pad; a.n1 = L->dim_pad;
@@ -767,10 +785,11 @@ extern "C" int tah_latent_decode(const tah_latent_layer* L, const int32_t* slot,
         hipStream_t st = static_cast<hipStream_t>(stream);
         const int lp = L->rank_pad + L->rot_pad;
         int rc;
-        if (lp <= 128) rc = launch_latent_decode<2, 4>(d, st);
-        else if (lp <= 320) rc = launch_latent_decode<5, 10>(d, st);
-        else if (lp <= 576) rc = launch_latent_decode<9, 18>(d, st);
-        else rc = launch_latent_decode<16, 32>(d, st);
+        if (lp == 576 && L->rank_pad == 512) rc = launch_latent_decode<8, 18, true>(d, st);
+        else if (lp <= 128) rc = launch_latent_decode<2, 4, false>(d, st);
+        else if (lp <= 320) rc = launch_latent_decode<5, 10, false>(d, st);
+        else if (lp <= 576) rc = launch_latent_decode<9, 18, false>(d, st);
+        else rc = launch_latent_decode<16, 32, false>(d, st);
         if (rc != TAH_OK) return rc;
         hipLaunchKernelGGL(latent_merge_kernel, dim3(L->heads, rows), dim3(kLatThreads), 0, st, static_cast<const float*>(workspace), hp, (int)d.splits,
                            (int)L->rank_pad, (int)rows, static_cast<__bf16*>(out_packed), static_cast<__bf16*>(out_rows));

@@ -5,8 +5,8 @@
 //  * moe_route_kernel: router logits in float32 from the float32 rows, the largest ones and their softmax; RB rows per
 //    workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
 //  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
-//  * moe_tile_kernel: bf16 tiles of 128 places x 128 weight rows on the matrix cores, both operands staged through LDS
-//    by asynchronous copies, three stages ahead; gate and up rows of the same columns share a wave, which applies the gate.
+//  * moe_tile_kernel: bf16 tiles of 128 places x 256 weight rows on the matrix cores, both operands staged through LDS
+//    by asynchronous copies, two stages ahead; gate and up rows of the same columns share a wave, which applies the gate.
 //  * moe_plain_kernel: the same product in float32 arithmetic (the float32 form of a model).
 #include <hip/hip_runtime.h>
 
@@ -160,14 +160,12 @@ __device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int& tile, int& co
 }
 
 // ---- bf16 tiles ------------------------------------------------------------------------------------------------
-constexpr int kStageK = 32;
-constexpr int kStages = 4;
-constexpr int kStageBytes = 2 * kTile * kStageK * 2;  // both operands of one stage: 128 x 32 bf16 each
-// LDS tile of rows x 32 bf16 (64 B per row, 4 chunks of 16 B): chunks permuted so that sixteen rows' reads of one logical
-// chunk touch sixteen different places of 256 bytes
-__device__ __forceinline__ int rowmajor32_off(int row, int chunk) { return row * 64 + ((chunk ^ ((row >> 2) & 3)) << 4); }
+constexpr int kStageK = 64;     // a whole 128-byte line of every row per stage
+constexpr int kStages = 3;
+constexpr int kTileW = 256;     // weight rows of a tile
+constexpr int kStageBytes = (kTile + kTileW) * kStageK * 2;
 
-// Four waves, 2 x 2: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
+// Four waves, 2 x 2: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 128 wn ... + 127 of the tile.
 template <bool GATE>
 __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) {
     HIP_DYNAMIC_SHARED(unsigned char, lds)
@@ -177,63 +175,75 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 2, wn = wave % 2;
     const __bf16* const x = static_cast<const __bf16*>(p.x);
     const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
-    constexpr int kCols = GATE ? kTile / 2 : kTile;  // output columns of a tile
+    constexpr int kCols = GATE ? kTileW / 2 : kTileW;  // output columns of a tile
     const int n0 = col_tile * kCols;
-    // This lane's part of the copies: of every sixteen rows a wave copies, row lane / 4, sixteen bytes at the logical chunk
-    // that lies at place lane % 4 of the row in LDS.
-    const __bf16 *ga[2], *gb[2];
+    // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
+    // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
+    constexpr int kA = kTile / 8 / 4, kB = kTileW / 8 / 4;  // copies per wave and stage: 4 and 8
+    const __bf16 *ga[kA], *gb[kB];
+    const int chunk = (lane % 8) ^ ((lane / 16) & 7);  // ((row >> 1) & 7 with row = 8 i + lane / 8: i's part is even)
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-        const int r = 16 * (2 * wave + i) + lane / 4;
-        const int chunk = (lane % 4) ^ ((r >> 2) & 3);
+    for (int i = 0; i < kA; ++i) {
+        const int r = 8 * (kA * wave + i) + lane / 8;
         int src = GATE ? p.source[tile * kTile + r] : tile * kTile + r;
         src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
-        ga[i] = x + (int64_t)src * p.x_rs + 8 * chunk;
+        ga[i] = x + (int64_t)src * p.x_rs;
+    }
+#pragma unroll
+    for (int i = 0; i < kB; ++i) {
+        const int r = 8 * (kB * wave + i) + lane / 8;
         int wr;
-        if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
-            int c = n0 + 32 * (r / 64) + r % 32;
+        if constexpr (GATE) {  // rows of the tile: 64 gate, 64 up of the first 64 columns, then of the next
+            int c = n0 + 64 * (r / 128) + r % 64;
             c = c < p.n ? c : p.n - 1;
-            wr = (r / 32) % 2 ? p.n + c : c;
+            wr = (r / 64) % 2 ? p.n + c : c;
         } else {
             wr = n0 + r < p.n ? n0 + r : p.n - 1;
         }
-        gb[i] = w + (int64_t)wr * p.k + 8 * chunk;
+        gb[i] = w + (int64_t)wr * p.k;
     }
     auto stage = [&](int s) __attribute__((always_inline)) {
         unsigned char* const base = lds + (s % kStages) * kStageBytes;
+        const int k0 = s * kStageK, valid = (p.k - k0) / 8;  // chunks of this stage inside the rows
 #pragma unroll
-        for (int i = 0; i < 2; ++i) async_copy_16B(ga[i] + s * kStageK, base + (2 * wave + i) * 1024);
+        for (int i = 0; i < kA; ++i) {
+            const int c = chunk ^ ((4 * (kA * wave + i)) & 7);
+            async_copy_16B(ga[i] + k0 + 8 * (c < valid ? c : 0), base + (kA * wave + i) * 1024);
+        }
 #pragma unroll
-        for (int i = 0; i < 2; ++i) async_copy_16B(gb[i] + s * kStageK, base + kTile * kStageK * 2 + (2 * wave + i) * 1024);
+        for (int i = 0; i < kB; ++i) {
+            const int c = chunk ^ ((4 * (kB * wave + i)) & 7);
+            async_copy_16B(gb[i] + k0 + 8 * (c < valid ? c : 0), base + kTile * kStageK * 2 + (kB * wave + i) * 1024);
+        }
     };
-    f32x4 acc[4][4];  // [weight tile][place tile]
+    f32x4 acc[8][4];  // [weight tile][place tile]
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < 8; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int stages = p.k / kStageK;
+    const int stages = (p.k + kStageK - 1) / kStageK;
     TAH_WAIT_VMEM();  // (the places' sources: from here on only copies are on their way)
     for (int s = 0; s < kStages - 1 && s < stages; ++s) stage(s);
     for (int s = 0; s < stages; ++s) {
-        // four copies per stage: all but those of the (at most two) stages behind this one have landed
-        const int behind = stages - 1 - s;
-        if (behind >= 2) TAH_WAIT_VMEM_N(8);
-        else if (behind == 1) TAH_WAIT_VMEM_N(4);
+        if (s + 1 < stages) TAH_WAIT_VMEM_N(kA + kB);  // all but the next stage's copies have landed
         else TAH_WAIT_VMEM();
         __syncthreads();  // every wave's copies of stage s are in, and nobody reads stage s - 1 any more
         if (s + kStages - 1 < stages) stage(s + kStages - 1);
         const unsigned char* const a = lds + (s % kStages) * kStageBytes;
         const unsigned char* const b = a + kTile * kStageK * 2;
-        bf16x8 fx[4], fw[4];
+        auto multiply = [&](int h) __attribute__((always_inline)) {
+            bf16x8 fx[4], fw[8];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor32_off(64 * wm + 16 * j + lane % 16, lane / 16));
-            fw[j] = *reinterpret_cast<const bf16x8*>(b + rowmajor32_off(64 * wn + 16 * j + lane % 16, lane / 16));
-        }
+            for (int j = 0; j < 4; ++j) fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor64_off(64 * wm + 16 * j + lane % 16, 4 * h + lane / 16));
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
+            for (int i = 0; i < 8; ++i) fw[i] = *reinterpret_cast<const bf16x8*>(b + rowmajor64_off(128 * wn + 16 * i + lane % 16, 4 * h + lane / 16));
 #pragma unroll
-            for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
+            for (int i = 0; i < 8; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
+        };
+        multiply(0);
+        if (s * kStageK + 32 < p.k) multiply(1);  // (uniform)
     }
     // accumulator (i, j) register r of lane l: weight row 16 i + 4 (l / 16) + r, place 16 j + l % 16
     __bf16* const out = static_cast<__bf16*>(p.out);
@@ -242,17 +252,17 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
         __bf16* const row = out + ((int64_t)tile * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
         if constexpr (GATE) {
 #pragma unroll
-            for (int i = 0; i < 2; ++i) {
-                const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
+            for (int i = 0; i < 4; ++i) {
+                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
                 bf16x4 y;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
+                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[4 + i][j][r]);
                 if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
             }
         } else {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
+            for (int i = 0; i < 8; ++i) {
+                const int c = n0 + 128 * wn + 16 * i + 4 * (lane / 16);
                 bf16x4 y;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) y[r] = (__bf16)acc[i][j][r];
@@ -368,13 +378,15 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
     if (!x || !w || !tile_expert || !out || (kind == TAH_LINEAR_GATE_UP && !source)) return TAH_E_NULL;
     if (!aligned_16(x) || !aligned_16(w) || !aligned_16(out)) return TAH_E_ALIGN;
     const bool gate = kind == TAH_LINEAR_GATE_UP;
-    const int cols = dtype == TAH_DT_F32 ? kPlainCols : (gate ? kTile / 2 : kTile);
+    const int cols = dtype == TAH_DT_F32 ? kPlainCols : (gate ? kTileW / 2 : kTileW);
     const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k, tiles, (n + cols - 1) / cols};
     const int64_t groups = (int64_t)((tiles + 7) / 8) * 8 * p.col_tiles;  // whole rounds over the XCDs
     if (groups > 0x7fffffff) return TAH_E_SHAPE;
     const dim3 grid((unsigned)groups);
     hipStream_t st = static_cast<hipStream_t>(stream);
     if (dtype == TAH_DT_BF16) {
+        const void* f = gate ? reinterpret_cast<const void*>(&moe_tile_kernel<true>) : reinterpret_cast<const void*>(&moe_tile_kernel<false>);
+        if (hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, kStages * kStageBytes) != hipSuccess) return TAH_E_LAUNCH;
         if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
         else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
     } else {
