@@ -502,10 +502,12 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_scan_kernel(const tah_del
 
 // ---- long portions, 32 tokens at a time -------------------------------------------------------------------------
 constexpr int kChunk = 32;
+constexpr int kChunkThreads = 128;
 
 __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-// running sums of a chunk's decay logarithms: lane t < 32 ends with G_t (lanes of 32 and more repeat lane 31)
+// running sums of a chunk's decay logarithms: lane t < 32 ends with G_t (lanes of 32 and more repeat lane 31; rows past the
+// end do not decay)
 __device__ __forceinline__ float chunk_decay(const float* lg, int heads, int h, int row0, int n, int lane) {
     float x = lane < n ? lg[(int64_t)(row0 + lane) * heads + h] : 0.f;
 #pragma unroll
@@ -516,12 +518,13 @@ __device__ __forceinline__ float chunk_decay(const float* lg, int heads, int h, 
     return __shfl(x, lane < kChunk ? lane : kChunk - 1);
 }
 
-// what the first kernel leaves per (chunk, head), in floats: W [32][dim], U0 [32][vdim], P [32][32]
-__device__ __host__ __forceinline__ int64_t chunk_floats(int dim, int vdim) { return kChunk * (int64_t)(dim + vdim + kChunk); }
+// what the first kernel leaves per (chunk, head), in floats: W [32][dim], U0 [32][vdim], P [32][32], and
+// exp(G_t), exp(G_last - G_t) [32] each
+__device__ __host__ __forceinline__ int chunk_floats(int dim, int vdim) { return kChunk * (dim + vdim + kChunk + 2); }
 
 // grid (chunk slots, heads).  NT: 16-wide tiles of dim.
 template <int NT>
-__global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
+__global__ __launch_bounds__(kChunkThreads) void delta_chunk_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
                                                                     const float* v, const float* lg, const float* beta, float* work) {
     constexpr int D = 16 * NT, kStride = D + 4;
     __shared__ __align__(16) float kl[kChunk][kStride], ql[kChunk][kStride];
@@ -534,7 +537,7 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
     float* const out = work + ((int64_t)blockIdx.x * L.heads + h) * chunk_floats(D, L.vdim);
     float* const out_u = out + kChunk * D;
     float* const out_p = out_u + kChunk * L.vdim;
-    for (int u = tid; u < kChunk * D / 4; u += kDeltaThreads) {
+    for (int u = tid; u < kChunk * D / 4; u += kChunkThreads) {
         const int t = u / (D / 4), i = 4 * (u % (D / 4));
         f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
         if (t < n) {
@@ -547,15 +550,18 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
     }
     if (wave == 0) {
         const float x = chunk_decay(lg, L.heads, h, row0, n, lane);
+        const float last = __shfl(x, kChunk - 1);
         if (lane < kChunk) {
             gl[lane] = x;
             bl[lane] = lane < n ? beta[(int64_t)(row0 + lane) * L.heads + h] : 0.f;
             be[lane] = bl[lane] * expf(x);
+            out_p[kChunk * kChunk + lane] = expf(x);
+            out_p[kChunk * kChunk + kChunk + lane] = expf(last - x);
         }
     }
     __syncthreads();
     // six tiles of 16 x 16: the lower ones of K K^T and of Q K^T
-    for (int id = wave; id < 6; id += kDeltaThreads / kWave) {
+    for (int id = wave; id < 6; id += kChunkThreads / kWave) {
         const bool is_p = id >= 3;
         const int i = id % 3 == 0 ? 0 : 1, j = id % 3 == 2 ? 1 : 0;
         const float* const a = is_p ? &ql[16 * i + c][4 * g] : &kl[16 * i + c][4 * g];
@@ -578,20 +584,26 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
             else al[t][s] = bl[t] * w;
         }
     }
-    if (wave == 3) {  // the tile above the diagonal
+    if (wave == kChunkThreads / kWave - 1) {  // the tile above the diagonal
 #pragma unroll
         for (int r = 0; r < 4; ++r) out_p[(4 * g + r) * kChunk + 16 + c] = 0.f;
     }
     __syncthreads();
-    // the triangular system, one column of a right hand side per thread: columns of v, then of k
-    for (int col = tid; col < L.vdim + D; col += kDeltaThreads) {
-        const bool is_k = col >= L.vdim;
-        const int i = is_k ? col - L.vdim : col;
-        float x[kChunk];
+    // the triangular system, two columns of the right hand sides per thread (a matrix entry, read from LDS by all lanes at
+    // once, then serves two): columns of v, then of k
+    const int cols = L.vdim + D;  // (even)
+    for (int col = tid; col < cols / 2; col += kChunkThreads) {
+        float x[2][kChunk];
 #pragma unroll
-        for (int t = 0; t < kChunk; ++t) {
-            if (is_k) x[t] = be[t] * kl[t][i];
-            else x[t] = t < n ? bl[t] * v[((int64_t)(row0 + t) * L.heads + h) * L.vdim + i] : 0.f;
+        for (int y = 0; y < 2; ++y) {
+            const int i = col + y * (cols / 2);
+            if (i >= L.vdim) {
+#pragma unroll
+                for (int t = 0; t < kChunk; ++t) x[y][t] = be[t] * kl[t][i - L.vdim];
+            } else {
+#pragma unroll
+                for (int t = 0; t < kChunk; ++t) x[y][t] = bl[t] * v[((int64_t)(row0 + (t < n ? t : n - 1)) * L.heads + h) * L.vdim + i];  // (beta is 0 past the end)
+            }
         }
 #pragma unroll
         for (int t = 1; t < kChunk; ++t) {
@@ -601,26 +613,37 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_kernel(const tah_de
                 const f32x4 a = *reinterpret_cast<const f32x4*>(&al[t][4 * s4]);
 #pragma unroll
                 for (int e = 0; e < 4; ++e)
-                    if (4 * s4 + e < t) x[t] -= a[e] * x[4 * s4 + e];
+                    if (4 * s4 + e < t) {
+                        x[0][t] -= a[e] * x[0][4 * s4 + e];
+                        x[1][t] -= a[e] * x[1][4 * s4 + e];
+                    }
             }
         }
-        float* const dst = is_k ? out + i : out_u + i;
-        const int ds = is_k ? D : L.vdim;
 #pragma unroll
-        for (int t = 0; t < kChunk; ++t) dst[t * ds] = x[t];
+        for (int y = 0; y < 2; ++y) {
+            const int i = col + y * (cols / 2);
+            if (i >= L.vdim) {
+#pragma unroll
+                for (int t = 0; t < kChunk; ++t) out[t * D + i - L.vdim] = x[y][t];
+            } else {
+#pragma unroll
+                for (int t = 0; t < kChunk; ++t) out_u[t * L.vdim + i] = x[y][t];
+            }
+        }
     }
 }
 
 // One workgroup per 16-column slice of a (sequence, head).  Workgroups go to the XCDs round robin: the slices of a head are
-// placed on one XCD, whose L2 then fetches what they share once.  Waves 0 and 1 form u, waves 2 and 3 the results; each holds every fourth
-// 16-row tile of the state's slice, register r of lane (c, g) of tile i being S[16 i + c][4 g + r].
+// placed on one XCD, whose L2 then fetches what they share once.  Waves 0 and 1 form u, waves 2 and 3 the results; a
+// wave holds 16 kOwn rows of the state's slice: register r of lane (c, g) of its tile i is S[kOwn (16 wave + c) + i][4 g + r].
 template <int NT>
 __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const tah_delta_layer L, const tah_portions P, const float* q, const float* k,
-                                                                         const float* lg, const float* work, float* o) {
+                                                                         const float* work, float* o) {
     constexpr int D = 16 * NT, kOwn = (NT + 3) / 4;
+    typedef __attribute__((__vector_size__(kOwn * sizeof(float)))) float own_t;
     __shared__ __align__(16) float st[16][D + 4];           // S^T
     __shared__ __align__(16) float ut[16][kChunk + 4], us[16][kChunk + 4];  // u^T, and times exp(G_last - G_s)
-    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
+    const int lane = threadIdx.x % kWave, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), c = lane % 16, g = lane / 16;
     const int slices = L.vdim / 16, item = blockIdx.x / 8 / slices * 8 + blockIdx.x % 8;
     if (item >= L.heads * P.nseq) return;
     const int h = item % L.heads, b = item / L.heads, kh = h / (L.heads / L.kv_heads), v0 = 16 * (blockIdx.x / 8 % slices);
@@ -628,68 +651,72 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const t
     if (n <= 0 || slot < 0 || slot >= L.nslots) return;
     int64_t chunk0 = 0;  // chunks of the sequences before
     for (int x = 0; x < b; ++x) chunk0 += (P.cu[x + 1] - P.cu[x] + kChunk - 1) / kChunk;
-    const int64_t wf = chunk_floats(D, L.vdim);
-    float* const S = L.state + ((int64_t)slot * L.heads + h) * D * L.vdim + v0 + 4 * g;
-    const bool fresh = P.pos0[b] == 0;
+    const int wf = chunk_floats(D, L.vdim), rs = L.kv_heads * D;
+    const bool holds = wave * kOwn < NT, fresh = P.pos0[b] == 0;
+    const int own = holds ? kOwn * (16 * wave + c) : 0;  // its first row of the state
+    float* const S = L.state + ((int64_t)slot * L.heads + h) * D * L.vdim + (int64_t)own * L.vdim + v0 + 4 * g;
     f32x4 s[kOwn];
+    auto publish = [&]() __attribute__((always_inline)) {
+        if (!holds) return;
 #pragma unroll
-    for (int i = 0; i < kOwn; ++i) {
-        const int d = wave + 4 * i;
-        s[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (d < NT) {
-            if (!fresh) s[i] = *reinterpret_cast<const f32x4*>(S + (int64_t)(16 * d + c) * L.vdim);
+        for (int r = 0; r < 4; ++r) {
+            own_t y;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) st[4 * g + r][16 * d + c] = s[i][r];
+            for (int i = 0; i < kOwn; ++i) y[i] = s[i][r];
+            *reinterpret_cast<own_t*>(&st[4 * g + r][own]) = y;
         }
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < kOwn; ++i)
+        s[i] = holds && !fresh ? *reinterpret_cast<const f32x4*>(S + (int64_t)i * L.vdim) : f32x4{0.f, 0.f, 0.f, 0.f};
+    publish();
     const bool former = wave < 2;
     const int tr = 16 * (wave % 2);  // the wave's rows of a chunk
     struct Loads {
-        f32x4 a[NT], p[2];
-        float u0[4], kk[kOwn][8], decay;
-    } cur, nxt;
+        f32x4 a[NT], p[2], u0, gam;
+        own_t kk[8];
+        float all;
+    } buf0, buf1;
+    const int chunks = (n + kChunk - 1) / kChunk;
+    // (uniform bases and 32-bit offsets; no branch around or between the loads of a chunk: the compiler then knows which are
+    // still on their way)
     auto fetch = [&](int ch, Loads& x) __attribute__((always_inline)) {
         const int row0 = first + ch * kChunk, m = n - ch * kChunk < kChunk ? n - ch * kChunk : kChunk;
         const float* const w = work + ((chunk0 + ch) * L.heads + h) * wf;
-        const float* const wu = w + kChunk * D;
-        const float* const wp = wu + kChunk * L.vdim;
-        const int t = tr + c < m ? tr + c : m - 1;
-        const float* const a = former ? w + (tr + c) * D : q + ((int64_t)(row0 + t) * L.kv_heads + kh) * D;
+        const float* const wu = w + kChunk * D + v0;
+        const float* const wp = w + kChunk * (D + L.vdim);
+        const float* const wg = wp + kChunk * kChunk;
+        const float* const kb = k + ((int64_t)row0 * L.kv_heads + kh) * D;
+        const float* const ab = former ? w : q + ((int64_t)row0 * L.kv_heads + kh) * D;
+        const unsigned ao = former ? (tr + c) * D : (tr + c < m ? tr + c : m - 1) * rs;
 #pragma unroll
-        for (int i = 0; i < NT; ++i) x.a[i] = *reinterpret_cast<const f32x4*>(a + 16 * i + 4 * g);
-        if (former) {
+        for (int i = 0; i < NT; ++i) x.a[i] = *reinterpret_cast<const f32x4*>(ab + (ao + 16 * i + 4 * g));
 #pragma unroll
-            for (int r = 0; r < 4; ++r) x.u0[r] = wu[(tr + 4 * g + r) * L.vdim + v0 + c];
-        } else {
+        for (int r = 0; r < 4; ++r) x.u0[r] = wu[(unsigned)((tr + 4 * g + r) * L.vdim + c)];
 #pragma unroll
-            for (int i = 0; i < 2; ++i) x.p[i] = *reinterpret_cast<const f32x4*>(wp + (tr + c) * kChunk + 16 * i + 4 * g);
+        for (int i = 0; i < 2; ++i) x.p[i] = *reinterpret_cast<const f32x4*>(wp + (unsigned)((tr + c) * kChunk + 16 * i + 4 * g));
+        x.gam = *reinterpret_cast<const f32x4*>(wg + (unsigned)((former ? kChunk : 0) + tr + 4 * g));
+        x.all = wg[kChunk - 1];  // exp(G_last)
+#pragma unroll
+        for (int y = 0; y < 8; ++y) {
+            const int tk = 16 * (y / 4) + 4 * g + y % 4;
+            x.kk[y] = *reinterpret_cast<const own_t*>(kb + (unsigned)((tk < m ? tk : m - 1) * rs + own));
         }
-#pragma unroll
-        for (int i = 0; i < kOwn; ++i) {
-            const int d = wave + 4 * i < NT ? wave + 4 * i : 0;
-#pragma unroll
-            for (int y = 0; y < 8; ++y) {
-                const int tk = 16 * (y / 4) + 4 * g + y % 4;
-                x.kk[i][y] = k[((int64_t)(row0 + (tk < m ? tk : m - 1)) * L.kv_heads + kh) * D + 16 * d + c];
-            }
-        }
-        x.decay = lane < m ? lg[(int64_t)(row0 + lane) * L.heads + h] : 0.f;
     };
-    const int chunks = (n + kChunk - 1) / kChunk;
-    fetch(0, cur);
-    __syncthreads();
-    for (int ch = 0; ch < chunks; ++ch) {
-        if (ch + 1 < chunks) fetch(ch + 1, nxt);
-        float G = cur.decay;
+    // the results of a chunk are written during the next one, so that no load waits behind a store just issued
+    f32x4 done = {0.f, 0.f, 0.f, 0.f};
+    auto flush = [&](int ch) __attribute__((always_inline)) {
+        if (former || ch < 0) return;
+        float* const ob = o + ((int64_t)(first + ch * kChunk) * L.heads + h) * L.vdim + v0;
 #pragma unroll
-        for (int x = 1; x < kChunk; x <<= 1) {
-            const float y = __shfl_up(G, x);
-            if (lane >= x && lane < kChunk) G += y;
+        for (int r = 0; r < 4; ++r) {
+            const int t = tr + 4 * g + r;
+            if (ch * kChunk + t < n) ob[(unsigned)(t * L.heads * L.vdim + c)] = done[r];
         }
-        const float last = __shfl(G, kChunk - 1);
-        float gr[4];  // G of the wave's rows 4 g + r
-#pragma unroll
-        for (int r = 0; r < 4; ++r) gr[r] = __shfl(G, tr + 4 * g + r);
+    };
+    auto step = [&](int ch, const Loads& cur, Loads& nxt) __attribute__((always_inline)) {
+        fetch(ch + 1 < chunks ? ch + 1 : ch, nxt);
+        __builtin_amdgcn_sched_barrier(0);
         // W S or Q S
         f32x4 x0 = {0.f, 0.f, 0.f, 0.f}, x1 = x0;
 #pragma unroll
@@ -700,40 +727,34 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const t
             x0 = mfma_f32(cur.a[i][2], y[2], x0);
             x1 = mfma_f32(cur.a[i][3], y[3], x1);
         }
+        flush(ch - 1);
         f32x4 res;
         if (former) {
             f32x4 u, w;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 u[r] = cur.u0[r] - (x0[r] + x1[r]);
-                w[r] = u[r] * expf(last - gr[r]);
+                w[r] = u[r] * cur.gam[r];
             }
             *reinterpret_cast<f32x4*>(&ut[c][tr + 4 * g]) = u;
             *reinterpret_cast<f32x4*>(&us[c][tr + 4 * g]) = w;
         } else {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) res[r] = (x0[r] + x1[r]) * expf(gr[r]);
+            for (int r = 0; r < 4; ++r) res[r] = (x0[r] + x1[r]) * cur.gam[r];
         }
         __syncthreads();
-        const float gc = expf(last);
         f32x4 uw[2];
 #pragma unroll
         for (int i = 0; i < 2; ++i) uw[i] = *reinterpret_cast<const f32x4*>(&us[c][16 * i + 4 * g]);
 #pragma unroll
-        for (int i = 0; i < kOwn; ++i) {
+        for (int i = 0; i < kOwn; ++i)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) s[i][r] *= gc;
+            for (int r = 0; r < 4; ++r) s[i][r] *= cur.all;
 #pragma unroll
-            for (int y = 0; y < 8; ++y) s[i] = mfma_f32(uw[y / 4][y % 4], cur.kk[i][y], s[i]);
-        }
+        for (int y = 0; y < 8; ++y)
 #pragma unroll
-        for (int i = 0; i < kOwn; ++i) {
-            const int d = wave + 4 * i;
-            if (d < NT) {
-#pragma unroll
-                for (int r = 0; r < 4; ++r) st[4 * g + r][16 * d + c] = s[i][r];
-            }
-        }
+            for (int i = 0; i < kOwn; ++i) s[i] = mfma_f32(uw[y / 4][y % 4], cur.kk[y][i], s[i]);
+        publish();
         if (!former) {
 #pragma unroll
             for (int i = 0; i < 2; ++i) {
@@ -741,20 +762,22 @@ __global__ __launch_bounds__(kDeltaThreads) void delta_chunk_scan_kernel(const t
 #pragma unroll
                 for (int e = 0; e < 4; ++e) res = mfma_f32(cur.p[i][e], u[e], res);
             }
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = ch * kChunk + tr + 4 * g + r;
-                if (t < n) o[((int64_t)(first + t) * L.heads + h) * L.vdim + v0 + c] = res[r];
-            }
+            done = res;
         }
         __syncthreads();
-        cur = nxt;
+    };
+    fetch(0, buf0);
+    __syncthreads();
+    for (int ch = 0;;) {
+        step(ch, buf0, buf1);
+        if (++ch == chunks) break;
+        step(ch, buf1, buf0);
+        if (++ch == chunks) break;
     }
+    flush(chunks - 1);
 #pragma unroll
-    for (int i = 0; i < kOwn; ++i) {
-        const int d = wave + 4 * i;
-        if (d < NT) *reinterpret_cast<f32x4*>(S + (int64_t)(16 * d + c) * L.vdim) = s[i];
-    }
+    for (int i = 0; i < kOwn; ++i)
+        if (holds) *reinterpret_cast<f32x4*>(S + (int64_t)i * L.vdim) = s[i];
 }
 
 // one wave per (row, head)
@@ -881,9 +904,9 @@ int64_t chunk_slots(int rows, int nseq) { return (int64_t)rows / kChunk + nseq; 
 template <int NT>
 void launch_chunked(const tah_delta_layer& L, const tah_portions& P, const float* q, const float* k, const float* v, const float* lg, const float* beta,
                     float* o, float* work, hipStream_t st) {
-    hipLaunchKernelGGL((delta_chunk_kernel<NT>), dim3((unsigned)chunk_slots(P.rows, P.nseq), L.heads), dim3(kDeltaThreads), 0, st, L, P, q, k, v, lg,
+    hipLaunchKernelGGL((delta_chunk_kernel<NT>), dim3((unsigned)chunk_slots(P.rows, P.nseq), L.heads), dim3(kChunkThreads), 0, st, L, P, q, k, v, lg,
                        beta, work);
-    hipLaunchKernelGGL((delta_chunk_scan_kernel<NT>), dim3((unsigned)((L.heads * P.nseq + 7) / 8 * 8 * (L.vdim / 16))), dim3(kDeltaThreads), 0, st, L, P, q, k, lg, work, o);
+    hipLaunchKernelGGL((delta_chunk_scan_kernel<NT>), dim3((unsigned)((L.heads * P.nseq + 7) / 8 * 8 * (L.vdim / 16))), dim3(kDeltaThreads), 0, st, L, P, q, k, work, o);
 }
 
 template <class E>

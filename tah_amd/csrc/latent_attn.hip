@@ -254,7 +254,7 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
     if (!find_tile(p.cu, p.nseq, kTileRows, tile, b, row0, row_end)) return;
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, c = lane % 16, g = lane / 16;
     const int dq = p.dim_pad + p.rot_pad, nq = kExact ? NQ : dq / 32, nv = kExact ? NV : p.vdim_pad / 16;
-    const int ks = dq + 8, vs = p.vdim_pad + 8;  // row strides in LDS: rows start in different banks
+    const int ks = dq + 8, vs = p.vdim_pad + 16;  // row strides in LDS: what a read takes from several rows lies in different banks
     __bf16* const kt = reinterpret_cast<__bf16*>(tile_lds);
     __bf16* const vt = kt + kTileKeys * ks;
     const int buffer = kTileKeys * (ks + vs);  // two of them: the next tile is written while this one is read
@@ -326,12 +326,20 @@ __global__ __launch_bounds__(W * kWave) void attend_tile_kernel(const AttendTile
         for (int i = 0; i < UV; ++i)
             if (vkey[i] >= 0) *reinterpret_cast<bf16x8*>(vt + at + vdst[i]) = fv[i];
     };
-    fetch(j_lo);
+    // Key tiles start at multiples of 64, and a workgroup begins with one whose number is a multiple of `cycle`, as many as
+    // a query tile can see: workgroups that run side by side read the same tiles at about the same time.
+    const int t_lo = j_lo / kTileKeys, t_hi = j_hi / kTileKeys, tiles = t_hi - t_lo + 1;
+    const int cycle = (p.window + kTileRows - 2) / kTileKeys + 2;
+    int tk = (t_lo + cycle - 1) / cycle * cycle;
+    tk = tk > t_hi ? t_lo : tk;
+    fetch(tk * kTileKeys);
     store(0);
     int now = 0;
-    for (int j0 = j_lo; j0 <= j_hi; j0 += kTileKeys, now = buffer - now) {
-        const bool more = j0 + kTileKeys <= j_hi;
-        if (more) fetch(j0 + kTileKeys);
+    for (int it = 0; it < tiles; ++it, now = buffer - now) {
+        const bool more = it + 1 < tiles;
+        const int j0 = tk * kTileKeys;
+        tk = tk < t_hi ? tk + 1 : t_lo;
+        if (more) fetch(tk * kTileKeys);
         __syncthreads();  // this tile is written, and nobody reads the other buffer any more
         // (uniform per wave) does this wave see anything of the tile, and does it see all of it?
         const bool any = j0 <= own_hi && j0 + kTileKeys - 1 > own_lo - p.window;
@@ -642,7 +650,7 @@ size_t elem_bytes(int dtype) { return dtype == TAH_DT_BF16 ? 2 : 4; }
 
 template <int NQ, int NV, int W, bool kExact>
 int launch_attend_tile(AttendTile p, int rows, hipStream_t st) {
-    const size_t lds = (size_t)2 * kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 8) * 2;
+    const size_t lds = (size_t)2 * kTileKeys * (p.dim_pad + p.rot_pad + 8 + p.vdim_pad + 16) * 2;
     if (lds > 65536 && hipFuncSetAttribute(reinterpret_cast<const void*>(&attend_tile_kernel<NQ, NV, W, kExact>),
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
         return TAH_E_LAUNCH;

@@ -163,23 +163,24 @@ __device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int& tile, int& co
 constexpr int kStageK = 64;     // a whole 128-byte line of every row per stage
 constexpr int kStages = 3;
 constexpr int kTileW = 256;     // weight rows of a tile
+constexpr int kTileWaves = 8;
 constexpr int kStageBytes = (kTile + kTileW) * kStageK * 2;
 
-// Four waves, 2 x 2: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 128 wn ... + 127 of the tile.
+// Eight waves, 2 x 4: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
 template <bool GATE>
-__global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) {
+__global__ __launch_bounds__(kTileWaves * kWave) void moe_tile_kernel(const MoeGemm p) {
     HIP_DYNAMIC_SHARED(unsigned char, lds)
     int tile, col_tile;
     if (!moe_tile_of(p, tile, col_tile)) return;
     const int expert = p.tile_expert[tile];
-    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 2, wn = wave % 2;
+    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 4, wn = wave % 4;
     const __bf16* const x = static_cast<const __bf16*>(p.x);
     const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
     constexpr int kCols = GATE ? kTileW / 2 : kTileW;  // output columns of a tile
     const int n0 = col_tile * kCols;
     // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
     // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
-    constexpr int kA = kTile / 8 / 4, kB = kTileW / 8 / 4;  // copies per wave and stage: 4 and 8
+    constexpr int kA = kTile / 8 / kTileWaves, kB = kTileW / 8 / kTileWaves;  // copies per wave and stage: 2 and 4
     const __bf16 *ga[kA], *gb[kB];
     const int chunk = (lane % 8) ^ ((lane / 16) & 7);  // ((row >> 1) & 7 with row = 8 i + lane / 8: i's part is even)
 #pragma unroll
@@ -193,10 +194,10 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
     for (int i = 0; i < kB; ++i) {
         const int r = 8 * (kB * wave + i) + lane / 8;
         int wr;
-        if constexpr (GATE) {  // rows of the tile: 64 gate, 64 up of the first 64 columns, then of the next
-            int c = n0 + 64 * (r / 128) + r % 64;
+        if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
+            int c = n0 + 32 * (r / 64) + r % 32;
             c = c < p.n ? c : p.n - 1;
-            wr = (r / 64) % 2 ? p.n + c : c;
+            wr = (r / 32) % 2 ? p.n + c : c;
         } else {
             wr = n0 + r < p.n ? n0 + r : p.n - 1;
         }
@@ -216,9 +217,9 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
             async_copy_16B(gb[i] + k0 + 8 * (c < valid ? c : 0), base + kTile * kStageK * 2 + (kB * wave + i) * 1024);
         }
     };
-    f32x4 acc[8][4];  // [weight tile][place tile]
+    f32x4 acc[4][4];  // [weight tile][place tile]
 #pragma unroll
-    for (int i = 0; i < 8; ++i)
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int stages = (p.k + kStageK - 1) / kStageK;
@@ -232,13 +233,13 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
         const unsigned char* const a = lds + (s % kStages) * kStageBytes;
         const unsigned char* const b = a + kTile * kStageK * 2;
         auto multiply = [&](int h) __attribute__((always_inline)) {
-            bf16x8 fx[4], fw[8];
+            bf16x8 fx[4], fw[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) fx[j] = *reinterpret_cast<const bf16x8*>(a + rowmajor64_off(64 * wm + 16 * j + lane % 16, 4 * h + lane / 16));
 #pragma unroll
-            for (int i = 0; i < 8; ++i) fw[i] = *reinterpret_cast<const bf16x8*>(b + rowmajor64_off(128 * wn + 16 * i + lane % 16, 4 * h + lane / 16));
+            for (int i = 0; i < 4; ++i) fw[i] = *reinterpret_cast<const bf16x8*>(b + rowmajor64_off(64 * wn + 16 * i + lane % 16, 4 * h + lane / 16));
 #pragma unroll
-            for (int i = 0; i < 8; ++i)
+            for (int i = 0; i < 4; ++i)
 #pragma unroll
                 for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(fw[i], fx[j], acc[i][j]);
         };
@@ -252,17 +253,17 @@ __global__ __launch_bounds__(kMoeThreads) void moe_tile_kernel(const MoeGemm p) 
         __bf16* const row = out + ((int64_t)tile * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
         if constexpr (GATE) {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
+            for (int i = 0; i < 2; ++i) {
+                const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
                 bf16x4 y;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[4 + i][j][r]);
+                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
                 if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
             }
         } else {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) {
-                const int c = n0 + 128 * wn + 16 * i + 4 * (lane / 16);
+            for (int i = 0; i < 4; ++i) {
+                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
                 bf16x4 y;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) y[r] = (__bf16)acc[i][j][r];
@@ -387,8 +388,8 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
     if (dtype == TAH_DT_BF16) {
         const void* f = gate ? reinterpret_cast<const void*>(&moe_tile_kernel<true>) : reinterpret_cast<const void*>(&moe_tile_kernel<false>);
         if (hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, kStages * kStageBytes) != hipSuccess) return TAH_E_LAUNCH;
-        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
-        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kMoeThreads), kStages * kStageBytes, st, p);
+        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
+        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
     } else {
         if (gate) hipLaunchKernelGGL((moe_plain_kernel<true>), grid, dim3(kMoeThreads), 0, st, p);
         else hipLaunchKernelGGL((moe_plain_kernel<false>), grid, dim3(kMoeThreads), 0, st, p);
