@@ -622,13 +622,10 @@ __global__ __launch_bounds__(kChunkThreads) void delta_chunk_kernel(const tah_de
 #pragma unroll
         for (int y = 0; y < 2; ++y) {
             const int i = col + y * (cols / 2);
-            if (i >= L.vdim) {
+            float* const dst = i >= L.vdim ? out + i - L.vdim : out_u + i;
+            const int ds = i >= L.vdim ? D : L.vdim;
 #pragma unroll
-                for (int t = 0; t < kChunk; ++t) out[t * D + i - L.vdim] = x[y][t];
-            } else {
-#pragma unroll
-                for (int t = 0; t < kChunk; ++t) out_u[t * L.vdim + i] = x[y][t];
-            }
+            for (int t = 0; t < kChunk; ++t) dst[t * ds] = x[y][t];
         }
     }
 }
