@@ -151,9 +151,9 @@ struct MoeGemm {
 // Which tile of places and which tile of columns a workgroup takes.  Workgroups go to the XCDs round robin; an XCD gets a
 // run of consecutive place tiles with all their columns, so that an expert's weights and a place's row are read into
 // one L2 only.  False: nothing to do.
-__device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int& tile, int& col_tile) {
-    const int used = p.tile_expert[p.tiles], per = (used + 7) / 8;
-    const int xcd = blockIdx.x % 8, i = blockIdx.x / 8;
+__device__ __forceinline__ bool moe_tile_of(const MoeGemm& p, int item, int& tile, int& col_tile) {
+    const int used = const_i32(p.tile_expert, p.tiles), per = (used + 7) / 8;
+    const int xcd = item % 8, i = item / 8;
     tile = xcd * per + i / p.col_tiles;
     col_tile = i % p.col_tiles;
     return i / p.col_tiles < per && tile < used;
@@ -164,47 +164,70 @@ constexpr int kStageK = 64;     // a whole 128-byte line of every row per stage
 constexpr int kStages = 3;
 constexpr int kTileW = 256;     // weight rows of a tile
 constexpr int kTileWaves = 8;
+constexpr int kTileWalkers = 256;  // workgroups: one per compute unit
 constexpr int kStageBytes = (kTile + kTileW) * kStageK * 2;
 
-// Eight waves, 2 x 4: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
+// A workgroup walks tiles blockIdx.x, blockIdx.x + gridDim.x, ... (gridDim.x % 8 == 0: all of one XCD) as one run of stages:
+// the first stages of the next tile are on their way while the last ones of this tile are multiplied and its result is
+// written.  Eight waves, 2 x 4: wave (wm, wn) computes places 64 wm ... + 63 against weight rows 64 wn ... + 63 of the tile.
 template <bool GATE>
 __global__ __launch_bounds__(kTileWaves * kWave) void moe_tile_kernel(const MoeGemm p) {
     HIP_DYNAMIC_SHARED(unsigned char, lds)
-    int tile, col_tile;
-    if (!moe_tile_of(p, tile, col_tile)) return;
-    const int expert = p.tile_expert[tile];
-    const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, wm = wave / 4, wn = wave % 4;
+    const int lane = threadIdx.x % kWave, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), wm = wave / 4, wn = wave % 4;
     const __bf16* const x = static_cast<const __bf16*>(p.x);
-    const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)expert * (GATE ? 2 : 1) * p.n * p.k;
     constexpr int kCols = GATE ? kTileW / 2 : kTileW;  // output columns of a tile
-    const int n0 = col_tile * kCols;
+    int tile, col_tile;
+    if (!moe_tile_of(p, blockIdx.x, tile, col_tile)) return;  // (an XCD's tiles come without gaps: nothing here, nothing further on)
+    int item = blockIdx.x, next = blockIdx.x;  // the tile being multiplied, and the one the copies are at
+    __bf16* const out = static_cast<__bf16*>(p.out);
     // This lane's part of the copies: of every eight rows a wave copies, row lane / 8, sixteen bytes at logical chunk
     // (lane % 8) ^ swizzle(row) -- the chunks of a row lie permuted in LDS so that the operand reads do not collide.
     constexpr int kA = kTile / 8 / kTileWaves, kB = kTileW / 8 / kTileWaves;  // copies per wave and stage: 2 and 4
     const __bf16 *ga[kA], *gb[kB];
     const int chunk = (lane % 8) ^ ((lane / 16) & 7);  // ((row >> 1) & 7 with row = 8 i + lane / 8: i's part is even)
+    auto point_at = [&](int tl, int ct) __attribute__((always_inline)) {
+        const __bf16* const w = static_cast<const __bf16*>(p.w) + (int64_t)const_i32(p.tile_expert, tl) * (GATE ? 2 : 1) * p.n * p.k;
+        const int c0 = ct * kCols;
 #pragma unroll
-    for (int i = 0; i < kA; ++i) {
-        const int r = 8 * (kA * wave + i) + lane / 8;
-        int src = GATE ? p.source[tile * kTile + r] : tile * kTile + r;
-        src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
-        ga[i] = x + (int64_t)src * p.x_rs;
-    }
-#pragma unroll
-    for (int i = 0; i < kB; ++i) {
-        const int r = 8 * (kB * wave + i) + lane / 8;
-        int wr;
-        if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
-            int c = n0 + 32 * (r / 64) + r % 32;
-            c = c < p.n ? c : p.n - 1;
-            wr = (r / 32) % 2 ? p.n + c : c;
-        } else {
-            wr = n0 + r < p.n ? n0 + r : p.n - 1;
+        for (int i = 0; i < kA; ++i) {
+            const int r = 8 * (kA * wave + i) + lane / 8;
+            int src = GATE ? p.source[tl * kTile + r] : tl * kTile + r;
+            src = src < 0 ? 0 : src;  // a padding place computes row 0 again; nobody reads it
+            ga[i] = x + (int64_t)src * p.x_rs;
         }
-        gb[i] = w + (int64_t)wr * p.k;
-    }
-    auto stage = [&](int s) __attribute__((always_inline)) {
-        unsigned char* const base = lds + (s % kStages) * kStageBytes;
+#pragma unroll
+        for (int i = 0; i < kB; ++i) {
+            const int r = 8 * (kB * wave + i) + lane / 8;
+            int wr;
+            if constexpr (GATE) {  // rows of the tile: 32 gate, 32 up of the first 32 columns, then of the next
+                int c = c0 + 32 * (r / 64) + r % 32;
+                c = c < p.n ? c : p.n - 1;
+                wr = (r / 32) % 2 ? p.n + c : c;
+            } else {
+                wr = c0 + r < p.n ? c0 + r : p.n - 1;
+            }
+            gb[i] = w + (int64_t)wr * p.k;
+        }
+    };
+    point_at(tile, col_tile);
+    const int stages = (p.k + kStageK - 1) / kStageK;
+    int ahead = 0, slot = 0;  // the stage of that tile the next copies are for, and their place in LDS
+    bool open = true;         // there is one
+    int pending = 0;          // stages whose copies are under way or in, not yet multiplied
+    auto stage = [&]() __attribute__((always_inline)) {
+        if (!open) return;
+        if (ahead == stages) {
+            int tl, ct;
+            next += gridDim.x;
+            open = moe_tile_of(p, next, tl, ct);
+            if (!open) return;
+            point_at(tl, ct);
+            ahead = 0;
+        }
+        ++pending;
+        const int s = ahead++;
+        unsigned char* const base = lds + slot * kStageBytes;
+        slot = slot + 1 < kStages ? slot + 1 : 0;
         const int k0 = s * kStageK, valid = (p.k - k0) / 8;  // chunks of this stage inside the rows
 #pragma unroll
         for (int i = 0; i < kA; ++i) {
@@ -222,15 +245,18 @@ __global__ __launch_bounds__(kTileWaves * kWave) void moe_tile_kernel(const MoeG
     for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int stages = (p.k + kStageK - 1) / kStageK;
-    TAH_WAIT_VMEM();  // (the places' sources: from here on only copies are on their way)
-    for (int s = 0; s < kStages - 1 && s < stages; ++s) stage(s);
-    for (int s = 0; s < stages; ++s) {
-        if (s + 1 < stages) TAH_WAIT_VMEM_N(kA + kB);  // all but the next stage's copies have landed
+    for (int s = 0; s < kStages - 1; ++s) stage();
+    int done = 0, at = 0;  // stages of `tile` that are multiplied; where the next one lies in LDS
+    while (pending > 0) {
+        // all but the copies of the one stage behind this one have landed (and the stores of a finished tile)
+        if (pending >= 2) TAH_WAIT_VMEM_N(kA + kB);
         else TAH_WAIT_VMEM();
-        __syncthreads();  // every wave's copies of stage s are in, and nobody reads stage s - 1 any more
-        if (s + kStages - 1 < stages) stage(s + kStages - 1);
-        const unsigned char* const a = lds + (s % kStages) * kStageBytes;
+        __syncthreads();  // every wave's copies of this stage are in, and nobody reads the one before any more
+        --pending;
+        stage();
+        const int s = done++;
+        const unsigned char* const a = lds + at * kStageBytes;
+        at = at + 1 < kStages ? at + 1 : 0;
         const unsigned char* const b = a + kTile * kStageK * 2;
         auto multiply = [&](int h) __attribute__((always_inline)) {
             bf16x8 fx[4], fw[4];
@@ -245,31 +271,39 @@ __global__ __launch_bounds__(kTileWaves * kWave) void moe_tile_kernel(const MoeG
         };
         multiply(0);
         if (s * kStageK + 32 < p.k) multiply(1);  // (uniform)
-    }
-    // accumulator (i, j) register r of lane l: weight row 16 i + 4 (l / 16) + r, place 16 j + l % 16
-    __bf16* const out = static_cast<__bf16*>(p.out);
+        if (done < stages) continue;
+        // accumulator (i, j) register r of lane l: weight row 16 i + 4 (l / 16) + r, place 16 j + l % 16
+        const int n0 = col_tile * kCols;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        __bf16* const row = out + ((int64_t)tile * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
-        if constexpr (GATE) {
+        for (int j = 0; j < 4; ++j) {
+            __bf16* const row = out + ((int64_t)tile * kTile + 64 * wm + 16 * j + lane % 16) * p.out_rs;
+            if constexpr (GATE) {
 #pragma unroll
-            for (int i = 0; i < 2; ++i) {
-                const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
-                bf16x4 y;
+                for (int i = 0; i < 2; ++i) {
+                    const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
+                    bf16x4 y;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
-                if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
-            }
-        } else {
+                    for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
+                    if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
+                }
+            } else {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
-                bf16x4 y;
+                for (int i = 0; i < 4; ++i) {
+                    const int c = n0 + 64 * wn + 16 * i + 4 * (lane / 16);
+                    bf16x4 y;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) y[r] = (__bf16)acc[i][j][r];
-                if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
+                    for (int r = 0; r < 4; ++r) y[r] = (__bf16)acc[i][j][r];
+                    if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
+                }
             }
         }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        done = 0;
+        item += gridDim.x;
+        if (!moe_tile_of(p, item, tile, col_tile)) return;
     }
 }
 
@@ -281,7 +315,7 @@ template <bool GATE>
 __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p) {
     __shared__ float a[kPlainK][kTile + 1], g[kPlainK][kPlainCols + 1], u[GATE ? kPlainK : 1][kPlainCols + 1];
     int tile, col_tile;
-    if (!moe_tile_of(p, tile, col_tile)) return;
+    if (!moe_tile_of(p, blockIdx.x, tile, col_tile)) return;
     const int expert = p.tile_expert[tile];
     const int tid = threadIdx.x, tc = tid % kPlainCols, tr = tid / kPlainCols, n0 = col_tile * kPlainCols;
     const float* const x = static_cast<const float*>(p.x);
@@ -388,8 +422,10 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
     if (dtype == TAH_DT_BF16) {
         const void* f = gate ? reinterpret_cast<const void*>(&moe_tile_kernel<true>) : reinterpret_cast<const void*>(&moe_tile_kernel<false>);
         if (hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, kStages * kStageBytes) != hipSuccess) return TAH_E_LAUNCH;
-        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), grid, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
-        else hipLaunchKernelGGL((moe_tile_kernel<false>), grid, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
+        // (walking pays where a tile is few stages, behind an expert's hidden size; the long tiles of gate|up lose a little by it)
+        const dim3 walk((unsigned)(gate || groups < kTileWalkers ? groups : kTileWalkers));
+        if (gate) hipLaunchKernelGGL((moe_tile_kernel<true>), walk, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
+        else hipLaunchKernelGGL((moe_tile_kernel<false>), walk, dim3(kTileWaves * kWave), kStages * kStageBytes, st, p);
     } else {
         if (gate) hipLaunchKernelGGL((moe_plain_kernel<true>), grid, dim3(kMoeThreads), 0, st, p);
         else hipLaunchKernelGGL((moe_plain_kernel<false>), grid, dim3(kMoeThreads), 0, st, p);
