@@ -39,7 +39,7 @@
 extern "C" {
 #endif
 
-#define TAH_DUO_ABI_VERSION 8
+#define TAH_DUO_ABI_VERSION 9
 
 enum {
     TAH_OK = 0,
@@ -460,7 +460,10 @@ int tah_silu_mul_normed(const void* gate_up, void* out, int32_t rows, int32_t in
  * vary from run to run) and are rounded to bf16 where the eager modules round. */
 enum { TAH_LINEAR_PLAIN = 0, TAH_LINEAR_GATE_UP = 1 };
 enum { TAH_ACT_NONE = 0, TAH_ACT_RELU = 1, TAH_ACT_GELU = 2,        /* GELU: x Phi(x), nn.GELU's default */
-       TAH_ACT_GELU_TANH = 3 };                                     /* its tanh form */
+       TAH_ACT_GELU_TANH = 3,                                       /* its tanh form */
+       TAH_ACT_XIELU = 4,         /* x > 0: c0 x^2 + x / 2, else c1 (exp(x) - 1 - x) + x / 2, c0 = act_c[0], c1 = act_c[1] */
+       TAH_ACT_CLAMPED_GATE = 5 };/* TAH_LINEAR_GATE_UP only, in silu's place: with limit c0, g = min(gate, c0) and
+                                   * u = clamp(up, -c0, c0), g sigmoid(c1 g) (u + 1) */
 enum { TAH_NORM_NONE = 0, TAH_NORM_RMS = 1, TAH_NORM_LAYER = 2 };
 
 /* w bf16 [n, k] row-major (nn.Linear weight), or [2 n, k] = [gate; up] stacked for TAH_LINEAR_GATE_UP; k % 32 == 0,
@@ -490,7 +493,8 @@ typedef struct tah_linear_rows_args {
     float norm_eps;
     const void* bias;         /* TAH_LINEAR_PLAIN: bf16 [n] added to the product (after its rounding to bf16, before the
                                * residual), or NULL */
-    int32_t activation;       /* TAH_LINEAR_PLAIN: TAH_ACT_* applied last (an MLP's first layer) */
+    int32_t activation;       /* TAH_LINEAR_PLAIN: TAH_ACT_* applied last (an MLP's first layer); TAH_LINEAR_GATE_UP:
+                               * TAH_ACT_NONE (silu) or TAH_ACT_CLAMPED_GATE */
     const float* ln_colsum;   /* TAH_NORM_LAYER: float32 [n], sum over k of the bf16 weight row as packed; else ignored */
     /* Several products of these sizes in one launch (per-head products of latent attention, the experts of a mixture):
      * product i (i < batch; 0 or 1: one product) uses operands and results i * stride elements further on (strides
@@ -501,6 +505,7 @@ typedef struct tah_linear_rows_args {
     int64_t w_batch_stride, x_batch_stride, out_batch_stride, out_packed_batch_stride;
     const int32_t* batch_select; /* int32 [n_select], or NULL: only products whose index is listed run */
     int32_t n_select;
+    float act_c[2];           /* constants of the activation */
 } tah_linear_rows_args;
 int tah_linear_rows(const tah_linear_rows_args* args, tah_stream_t stream);
 

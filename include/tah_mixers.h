@@ -1,6 +1,6 @@
 /* tah_mixers.h -- C ABI of the layer mechanisms of decoder models that are described layer by layer: residual rows
- * with a norm on the sublayer's output, gated delta-rule recurrence, sliding-window latent attention, mixture of
- * experts.  Same conventions as tah_duo.h (device pointers, nothing allocated, nothing synchronised, 0 or TAH_E_*),
+ * with norms around the sublayers, short convolutions of a sublayer's input, gated delta-rule recurrence, sliding-window
+ * attention on latents or on keys and values, mixture of experts.  Same conventions as tah_duo.h (device pointers, nothing allocated, nothing synchronised, 0 or TAH_E_*),
  * exported by the same library.  Sizes and constants are arguments; nothing here belongs to one model.
  *
  * Element type.  `dtype` says what activations, weights and cached rows are: TAH_DT_BF16 or TAH_DT_F32.  The residual
@@ -24,9 +24,15 @@ extern "C" {
 
 enum { TAH_DT_BF16 = 0, TAH_DT_F32 = 1 };
 
+typedef struct tah_portions {
+    const int32_t *cu, *slot, *pos0; /* [nseq + 1], [nseq], [nseq] */
+    const int32_t* row_seq;          /* [rows] */
+    int32_t nseq, rows;
+} tah_portions;
+
 /* ---- residual rows ------------------------------------------------------------------------------------------- */
 
-/* x = embed[tok], in float32, in the element type and (rows <= 32) in the rows form of tah_linear_rows; and the rows'
+/* x = scale * embed[tok], in float32, in the element type and (rows <= 32) in the rows form of tah_linear_rows; and the rows'
  * slots and positions for a decode step: row r owns slot slot_base + r, finished rows get -1. */
 typedef struct tah_embed_rows_args {
     const int64_t* tok;       /* [rows], clamped into the vocabulary */
@@ -39,13 +45,22 @@ typedef struct tah_embed_rows_args {
     int32_t *slot, *q_pos;    /* [rows] */
     uint8_t* active;          /* [rows] */
     int32_t rows, vocab, cols, dtype, slot_base;
+    float scale;
 } tah_embed_rows_args;
 int tah_embed_rows(const tah_embed_rows_args* args, tah_stream_t stream);
 
 /* x += coef * y / sqrt(mean(y^2) + eps): the norm of a sublayer's output, its weight and any layer scale in `coef`, and
  * the residual sum, all in float32.  y = y_scale[r] * y[r] + sum_j weight[r][j] * experts[index[r][j] * index_scale +
- * r * index_row] (either part may be absent).  Optionally, from the new x: its row in the element type and in rows form, and the model's output norm
- * final_coef * x / sqrt(mean(x^2) + eps) as the operand of the output head. */
+ * r * index_row] (either part may be absent; without both, x stays as it is).  Optionally, from the new x: its row in the
+ * element type and in rows form, and a norm of it, n = next_coef * x / sqrt(mean(x^2) + eps), as the next sublayer's (or
+ * the output head's) operand.
+ *
+ * Groups.  Both norms divide every group of columns by its own root mean square: group g is columns
+ * [g * group_cols, (g + 1) * group_cols), width / groups of them true ones and the rest zero.  With one group group_cols
+ * is not looked at.
+ *
+ * Input convolution (single tokens).  With `conv` the operand is h + sum_j conv[j] * h_(t - taps + 1 + j), h the normed row
+ * rounded to the element type, its last inputs in conv_state (as tah_conv_rows leaves them), where h is entered. */
 typedef struct tah_residual_norm_args {
     const void* y;            /* [rows, y_row_stride], or NULL */
     const float* y_scale;     /* [rows], or NULL: 1 */
@@ -53,7 +68,7 @@ typedef struct tah_residual_norm_args {
     const int32_t* index;     /* [rows, top] */
     const float* weight;      /* [rows, top] */
     const float* coef;        /* [cols] */
-    const float* final_coef;  /* [cols], or NULL */
+    const float* next_coef;   /* [cols], or NULL */
     float* x;                 /* [rows, cols], updated in place */
     void* xe;                 /* element type [rows, cols], or NULL */
     void* x_packed;           /* bf16 rows form, or NULL */
@@ -62,13 +77,26 @@ typedef struct tah_residual_norm_args {
     int64_t y_row_stride, experts_row_stride;
     int32_t rows, width, cols, top, index_scale, index_row, dtype;
     float eps;
+    int32_t groups, group_cols;
+    const float* conv;        /* [taps, cols], or NULL */
+    void* conv_state;         /* element type [nslots, taps, cols] */
+    const int32_t *slot, *pos; /* [rows], with conv */
+    int32_t taps, nslots;
 } tah_residual_norm_args;
 int tah_residual_norm(const tah_residual_norm_args* args, tah_stream_t stream);
 
-/* out[r][c] = gelu(in[r][c]) (tanh form) or silu(in[r][c]) * in[r][cols + c], c < cols. */
-enum { TAH_ROWS_GELU_TANH = 0, TAH_ROWS_SILU_MUL = 1 };
+/* out[r][c] = f(in[r][c]), or for the gates f(in[r][c], in[r][cols + c]), c < cols: gelu (tanh form); silu(g) u; xielu,
+ * c0 x^2 + x / 2 above zero and c1 (exp(x) - 1 - x) + x / 2 below; the clamped gate g sigmoid(c1 g) (u + 1) with g =
+ * min(g, c0), u = clamp(u, -c0, c0). */
+enum { TAH_ROWS_GELU_TANH = 0, TAH_ROWS_SILU_MUL = 1, TAH_ROWS_XIELU = 2, TAH_ROWS_CLAMPED_GATE = 3 };
 int tah_activate_rows(const void* in, int64_t in_row_stride, void* out, int64_t out_row_stride, int32_t rows, int32_t cols,
-                      int32_t kind, int32_t dtype, tah_stream_t stream);
+                      int32_t kind, float c0, float c1, int32_t dtype, tah_stream_t stream);
+
+/* Portions' rows h [rows, cols] -> h + causal convolution of h over time, per channel: out[t] = h[t] + sum_j conv[j] *
+ * h[t - taps + 1 + j], zeros before a sequence's start.  conv_state element type [nslots, taps, cols]: the last taps - 1
+ * inputs of a slot's sequence, token p at p % taps, read for a portion's first rows and brought up to its last ones. */
+int tah_conv_rows(const void* h, const float* conv, void* conv_state, const tah_portions* p, void* out, int32_t cols, int32_t taps,
+                  int32_t nslots, int32_t dtype, tah_stream_t stream);
 
 /* ---- gated delta rule ---------------------------------------------------------------------------------------- *
  * Per head, with state S [dim, vdim] in float32:  S = g S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q, where
@@ -100,11 +128,6 @@ int tah_delta_step(const tah_delta_layer* layer, const int32_t* slot, const int3
  * tah_delta_scan: the recurrence, o float32 [T, heads, vdim], and the new states; workspace as large as
  * tah_delta_scan_workspace says (0: none), which depends on the sizes and counts alone.
  * tah_delta_finish: norm and gate, out element type [T, out_row_stride]. */
-typedef struct tah_portions {
-    const int32_t *cu, *slot, *pos0; /* [nseq + 1], [nseq], [nseq] */
-    const int32_t* row_seq;          /* [rows] */
-    int32_t nseq, rows;
-} tah_portions;
 int tah_delta_prepare(const tah_delta_layer* layer, const tah_portions* p, float* q, float* k, float* v, float* log_decay,
                       float* beta, tah_stream_t stream);
 int tah_delta_scan(const tah_delta_layer* layer, const tah_portions* p, const float* q, const float* k, const float* v,
@@ -166,11 +189,59 @@ int tah_latent_decode(const tah_latent_layer* layer, const int32_t* slot, const 
                       int64_t q_latent_head_stride, const void* q, int64_t q_row_stride, void* out_packed, void* out_rows,
                       void* workspace, size_t workspace_bytes, tah_stream_t stream);
 
+/* ---- attention in a sliding window with kept first tokens ---------------------------------------------------------- *
+ * Position i sees j <= i with i - j < window or j < keep_first.  Query head h reads key/value head h / (heads / kv_heads).
+ * What a token caches per key/value head is one row of `row` elements in which the values are columns [0, value_dim) and
+ * the keys [row - key_dim, row); the two may overlap, so that keys which are also the values are kept once.  The
+ * last rot_pad columns of a key (and of a query, key_dim elements) hold the rotated part, entries 2 i and 2 i + 1 a pair,
+ * rot_dim of them and zeros behind; a new row brings the pairs unrotated at column rot_source.  A slot's cache is
+ * keep_first rows for the first tokens and a ring: token p at row p (p < keep_first), else keep_first + (p - keep_first)
+ * % ring. */
+typedef struct tah_window_layer {
+    void* cache;              /* element type [nslots, kv_heads, keep_first + ring, row] */
+    int32_t heads, kv_heads, row, key_dim, value_dim, rot_dim, rot_pad, rot_source;
+    int32_t keep_first, ring, window, nslots, dtype;
+    float scale;
+} tah_window_layer;
+/* Rows of a step: projections with a query head's key_dim columns at q_col + h * key_dim, a key/value head's row at
+ * k_col + g * row, and (g_col >= 0) a gate per head: head h's result is multiplied by sigmoid of column g_col + h. */
+typedef struct tah_window_rows {
+    void* proj;
+    int64_t proj_row_stride;
+    const float *cos, *sin;   /* float32 [table_rows, rot_dim / 2] */
+    const int32_t* pos;       /* [rows] */
+    const int32_t* slot;      /* [rows], or NULL */
+    int32_t q_col, k_col, g_col, rows, table_rows;
+} tah_window_rows;
+/* Rotates queries and keys in place; with `slot` the rows also go into their slots' caches. */
+int tah_window_prep(const tah_window_layer* layer, const tah_window_rows* rows, tah_stream_t stream);
+/* Attention of portions on prepared rows, which are the portions' own keys, and on the cache for the positions before
+ * them.  out element type [rows, out_row_stride]: head h at column h * value_dim. */
+int tah_window_attend(const tah_window_layer* layer, const tah_portions* p, const tah_window_rows* rows, void* out, int64_t out_row_stride,
+                      tah_stream_t stream);
+/* The portions' prepared rows into the cache (behind tah_window_attend, which reads what they replace). */
+int tah_window_append(const tah_window_layer* layer, const tah_portions* p, const tah_window_rows* rows, tah_stream_t stream);
+/* Single tokens: rotation, cache entry and attention.  out element type [rows, out_row_stride] and / or out_packed, the
+ * rows form [32 * heads * value_dim] (rows <= 32).  workspace: tah_window_decode_workspace bytes. */
+size_t tah_window_decode_workspace(const tah_window_layer* layer, int32_t rows);
+int tah_window_decode(const tah_window_layer* layer, const tah_window_rows* rows, void* out, int64_t out_row_stride, void* out_packed,
+                      void* workspace, size_t workspace_bytes, tah_stream_t stream);
+
 /* ---- mixture of experts -------------------------------------------------------------------------------------- *
- * tah_moe_route: logits x . router in float32, the `top` largest (the lower index among equals), softmax over them;
- * shared_gate = sigmoid(x . gate_w) when gate_w is given.  x float32 [rows, cols]; router, gate_w element type. */
-int tah_moe_route(const float* x, const void* router, const void* gate_w, int32_t rows, int32_t cols, int32_t experts,
-                  int32_t top, int32_t* index, float* weight, float* shared_gate, int32_t dtype, tah_stream_t stream);
+ * tah_moe_route: logits x . router in float32; scores are the logits (TAH_MOE_SOFTMAX) or their sigmoids (TAH_MOE_SIGMOID).
+ * The experts form `groups` equal groups of neighbours (1: none); with keep < groups only the `keep` groups with the
+ * largest sum of their two largest scores are open.  index: the `top` largest scores of the open experts (the lower index
+ * among equals); weight: softmax over the chosen logits, or the chosen scores.  shared_gate = sigmoid(x . gate_w) when
+ * gate_w is given.  x [rows, cols] float32, or (x_elem) of the element type; router, gate_w element type. */
+enum { TAH_MOE_SOFTMAX = 0, TAH_MOE_SIGMOID = 1 };
+typedef struct tah_moe_route_args {
+    const void *x, *router, *gate_w;
+    int32_t* index;           /* [rows, top] */
+    float* weight;            /* [rows, top] */
+    float* shared_gate;       /* [rows], or NULL */
+    int32_t rows, cols, experts, top, groups, keep, score, x_elem, dtype;
+} tah_moe_route_args;
+int tah_moe_route(const tah_moe_route_args* args, tah_stream_t stream);
 /* Rows sorted by expert, every expert's rows padded to whole tiles of TAH_MOE_TILE: source row of every place (-1:
  * padding), the expert of every tile (-1 past the last) and behind them the number of tiles used, and the place of
  * every (row, choice).  source holds tah_moe_places(rows, top, experts) places, tile_expert a tile for each TAH_MOE_TILE
@@ -180,10 +251,11 @@ int32_t tah_moe_places(int32_t rows, int32_t top, int32_t experts);
 int tah_moe_plan(const int32_t* index, int32_t rows, int32_t top, int32_t experts, int32_t* source, int32_t* tile_expert,
                  int32_t* place, tah_stream_t stream);
 /* Product of the sorted rows with their experts' weights.  TAH_LINEAR_GATE_UP: w [experts, 2 n, k] (gate rows, then up
- * rows), x row source[place] (`tiles` without the entry behind them), out = silu(gate) * up [places, n]; TAH_LINEAR_PLAIN: w [experts, n, k], x row `place`. */
+ * rows), x row source[place] (`tiles` without the entry behind them), out = silu(gate) * up [places, n], or with TAH_ACT_CLAMPED_GATE the
+ * clamped gate with constants c0, c1; TAH_LINEAR_PLAIN: w [experts, n, k], x row `place`. */
 int tah_moe_linear(const void* x, int64_t x_row_stride, const void* w, const int32_t* source, const int32_t* tile_expert,
-                   int32_t tiles, int32_t n, int32_t k, int32_t kind, void* out, int64_t out_row_stride, int32_t dtype,
-                   tah_stream_t stream);
+                   int32_t tiles, int32_t n, int32_t k, int32_t kind, int32_t activation, float c0, float c1, void* out,
+                   int64_t out_row_stride, int32_t dtype, tah_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import ctypes as C
 
-ABI_VERSION = 8
+ABI_VERSION = 9
 
 c_void_p, c_int32, c_int64, c_float = C.c_void_p, C.c_int32, C.c_int64, C.c_float
 
@@ -120,7 +120,7 @@ class LinearRowsArgs(C.Structure):
         ("bias", c_void_p), ("activation", c_int32), ("ln_colsum", c_void_p),
         ("batch", c_int32), ("out_packed_col_step", c_int32),
         ("w_batch_stride", c_int64), ("x_batch_stride", c_int64), ("out_batch_stride", c_int64), ("out_packed_batch_stride", c_int64),
-        ("batch_select", c_void_p), ("n_select", c_int32),
+        ("batch_select", c_void_p), ("n_select", c_int32), ("act_c", c_float * 2),
     ]
 
 
@@ -255,7 +255,7 @@ class EmbedRowsArgs(C.Structure):
     _fields_ = [
         ("tok", c_void_p), ("pos", c_void_p), ("finished", c_void_p), ("embed", c_void_p), ("x", c_void_p), ("xe", c_void_p),
         ("x_packed", c_void_p), ("slot", c_void_p), ("q_pos", c_void_p), ("active", c_void_p),
-        ("rows", c_int32), ("vocab", c_int32), ("cols", c_int32), ("dtype", c_int32), ("slot_base", c_int32),
+        ("rows", c_int32), ("vocab", c_int32), ("cols", c_int32), ("dtype", c_int32), ("slot_base", c_int32), ("scale", c_float),
     ]
 
 
@@ -264,10 +264,11 @@ class ResidualNormArgs(C.Structure):
 
     _fields_ = [
         ("y", c_void_p), ("y_scale", c_void_p), ("experts", c_void_p), ("index", c_void_p), ("weight", c_void_p), ("coef", c_void_p),
-        ("final_coef", c_void_p), ("x", c_void_p), ("xe", c_void_p), ("x_packed", c_void_p), ("normed", c_void_p),
+        ("next_coef", c_void_p), ("x", c_void_p), ("xe", c_void_p), ("x_packed", c_void_p), ("normed", c_void_p),
         ("normed_packed", c_void_p), ("y_row_stride", c_int64), ("experts_row_stride", c_int64),
         ("rows", c_int32), ("width", c_int32), ("cols", c_int32), ("top", c_int32), ("index_scale", c_int32), ("index_row", c_int32), ("dtype", c_int32),
-        ("eps", c_float),
+        ("eps", c_float), ("groups", c_int32), ("group_cols", c_int32), ("conv", c_void_p), ("conv_state", c_void_p), ("slot", c_void_p),
+        ("pos", c_void_p), ("taps", c_int32), ("nslots", c_int32),
     ]
 
 
@@ -309,6 +310,27 @@ class LatentPrepArgs(C.Structure):
     ]
 
 
+class WindowLayer(C.Structure):
+    """``tah_window_layer``"""
+
+    _fields_ = [("cache", c_void_p)] + [(n, c_int32) for n in ("heads", "kv_heads", "row", "key_dim", "value_dim", "rot_dim", "rot_pad",
+                                                              "rot_source", "keep_first", "ring", "window", "nslots", "dtype")] + [("scale", c_float)]
+
+
+class WindowRows(C.Structure):
+    """``tah_window_rows``"""
+
+    _fields_ = [("proj", c_void_p), ("proj_row_stride", c_int64), ("cos", c_void_p), ("sin", c_void_p), ("pos", c_void_p), ("slot", c_void_p),
+                ("q_col", c_int32), ("k_col", c_int32), ("g_col", c_int32), ("rows", c_int32), ("table_rows", c_int32)]
+
+
+class MoeRouteArgs(C.Structure):
+    """``tah_moe_route_args``"""
+
+    _fields_ = [(n, c_void_p) for n in ("x", "router", "gate_w", "index", "weight", "shared_gate")] + \
+               [(n, c_int32) for n in ("rows", "cols", "experts", "top", "groups", "keep", "score", "x_elem", "dtype")]
+
+
 PROTOTYPES = {
     "tah_duo_abi_version": (C.c_int, []),
     "tah_duo_error_string": (C.c_char_p, [C.c_int]),
@@ -346,7 +368,8 @@ PROTOTYPES = {
     # include/tah_mixers.h
     "tah_embed_rows": (C.c_int, [C.POINTER(EmbedRowsArgs), c_void_p]),
     "tah_residual_norm": (C.c_int, [C.POINTER(ResidualNormArgs), c_void_p]),
-    "tah_activate_rows": (C.c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int32, c_int32, c_int32, c_int32, c_void_p]),
+    "tah_activate_rows": (C.c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int32, c_int32, c_int32, c_float, c_float, c_int32, c_void_p]),
+    "tah_conv_rows": (C.c_int, [c_void_p, c_void_p, c_void_p, C.POINTER(Portions), c_void_p, c_int32, c_int32, c_int32, c_int32, c_void_p]),
     "tah_delta_step": (C.c_int, [C.POINTER(DeltaLayer), c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int32, c_void_p]),
     "tah_delta_prepare": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 6),
     "tah_delta_scan": (C.c_int, [C.POINTER(DeltaLayer), C.POINTER(Portions)] + [c_void_p] * 7 + [C.c_size_t, c_void_p]),
@@ -359,12 +382,16 @@ PROTOTYPES = {
     "tah_latent_decode_workspace": (C.c_size_t, [C.POINTER(LatentLayer), c_int32]),
     "tah_latent_decode": (C.c_int, [C.POINTER(LatentLayer), c_void_p, c_void_p, c_int32, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
                                     c_void_p, c_void_p, C.c_size_t, c_void_p]),
-    "tah_moe_route": (C.c_int, [c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_int32, c_int32, c_void_p, c_void_p, c_void_p, c_int32,
-                                c_void_p]),
+    "tah_window_prep": (C.c_int, [C.POINTER(WindowLayer), C.POINTER(WindowRows), c_void_p]),
+    "tah_window_attend": (C.c_int, [C.POINTER(WindowLayer), C.POINTER(Portions), C.POINTER(WindowRows), c_void_p, c_int64, c_void_p]),
+    "tah_window_append": (C.c_int, [C.POINTER(WindowLayer), C.POINTER(Portions), C.POINTER(WindowRows), c_void_p]),
+    "tah_window_decode_workspace": (C.c_size_t, [C.POINTER(WindowLayer), c_int32]),
+    "tah_window_decode": (C.c_int, [C.POINTER(WindowLayer), C.POINTER(WindowRows), c_void_p, c_int64, c_void_p, c_void_p, C.c_size_t, c_void_p]),
+    "tah_moe_route": (C.c_int, [C.POINTER(MoeRouteArgs), c_void_p]),
     "tah_moe_places": (c_int32, [c_int32, c_int32, c_int32]),
     "tah_moe_plan": (C.c_int, [c_void_p, c_int32, c_int32, c_int32, c_void_p, c_void_p, c_void_p, c_void_p]),
-    "tah_moe_linear": (C.c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_int32, c_int32, c_void_p, c_int64,
-                                 c_int32, c_void_p]),
+    "tah_moe_linear": (C.c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int32, c_int32, c_int32, c_int32, c_int32, c_float, c_float,
+                                 c_void_p, c_int64, c_int32, c_void_p]),
 }
 
 

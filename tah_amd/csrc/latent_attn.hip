@@ -208,23 +208,6 @@ __global__ __launch_bounds__(kLatThreads) void attend_rows_kernel(const AttendRo
 
 // ---- bf16 on the matrix cores ------------------------------------------------------------------------------------
 constexpr int kTileKeys = 64;
-constexpr float kNoScore = -1e30f;  // below every score, and finite: differences of it are numbers
-
-__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-
-__device__ __forceinline__ bf16x8 join8(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
-
-__device__ __forceinline__ bf16x4 to_bf16x4(const float (&w)[4]) { return __builtin_convertvector((f32x4{w[0], w[1], w[2], w[3]}), bf16x4); }
-
-// x over the four lane groups that share l % 16
-__device__ __forceinline__ float groups_max(float x) {
-    x = fmaxf(x, __shfl_xor(x, 16));
-    return fmaxf(x, __shfl_xor(x, 32));
-}
-__device__ __forceinline__ float groups_sum(float x) {
-    x += __shfl_xor(x, 16);
-    return x + __shfl_xor(x, 32);
-}
 
 struct AttendTile {
     const __bf16 *q, *k, *v, *ctx;  // q: head base [dim_pad | rot_pad]; ctx: rotated key part of context row 0

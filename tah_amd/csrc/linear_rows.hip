@@ -29,8 +29,7 @@
 // tried: the fence writes back and invalidates the whole L2 of the XCD.
 #include <hip/hip_runtime.h>
 
-#include "duo_device.h"
-#include "tah_duo.h"
+#include "mixer_device.h"
 
 namespace tah {
 namespace {
@@ -64,9 +63,8 @@ struct LinParams {
     int32_t yp_col_step;    // columns a product's packed result is moved by (results side by side in one rows form)
     const int32_t* select;  // run only products whose index is listed here, or null
     int32_t n_select;
+    float c0, c1;           // constants of the activation
 };
-
-__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
 // 16-byte unit of the packed rows form that holds row r, columns k ... k + 7 (k % 8 == 0)
 __device__ __host__ __forceinline__ int64_t packed_rows_unit(int r, int k) {
@@ -316,7 +314,7 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
             for (int i = 0; i < 8; ++i) {
                 // the projections' own rounding to bf16, the activation's, the product's (Qwen3MLP.forward)
                 const float g = (float)(__bf16)(sg[i] * rin), u = (float)(__bf16)(su[i] * rin);
-                out[i] = (__bf16)((float)(__bf16)silu_f(g) * u);
+                out[i] = p.act == TAH_ACT_CLAMPED_GATE ? (__bf16)clamped_gate(g, u, p.c0, p.c1) : (__bf16)((float)(__bf16)silu_f(g) * u);
             }
         } else {
 #pragma unroll
@@ -344,6 +342,9 @@ __global__ __launch_bounds__(kLinThreads) void linear_rows_kernel(const LinParam
                     const float v = (float)out[i];
                     out[i] = (__bf16)(0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v))));
                 }
+            } else if (p.act == TAH_ACT_XIELU) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) out[i] = (__bf16)xielu((float)out[i], p.c0, p.c1);
             }
         }
         if (p.y) *reinterpret_cast<bf16x8*>(p.y + batch * p.y_bs + (int64_t)row * p.y_rs + n0) = out;
@@ -450,10 +451,11 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
     const bool g24 = gate_up && a->n % kGroup24 == 0;
     if (!g24 && a->n % kTileCols != 0) return TAH_E_SHAPE;
     if (a->activation != TAH_ACT_NONE && a->activation != TAH_ACT_RELU && a->activation != TAH_ACT_GELU &&
-        a->activation != TAH_ACT_GELU_TANH)
+        a->activation != TAH_ACT_GELU_TANH && a->activation != TAH_ACT_XIELU && a->activation != TAH_ACT_CLAMPED_GATE)
         return TAH_E_SHAPE;
+    if (!gate_up && a->activation == TAH_ACT_CLAMPED_GATE) return TAH_E_SHAPE;
     if (a->input_norm != TAH_NORM_NONE && a->input_norm != TAH_NORM_RMS && a->input_norm != TAH_NORM_LAYER) return TAH_E_SHAPE;
-    if (gate_up && (a->residual || a->bias || a->activation != TAH_ACT_NONE || a->input_norm == TAH_NORM_LAYER)) return TAH_E_SHAPE;
+    if (gate_up && (a->residual || a->bias || (a->activation != TAH_ACT_NONE && a->activation != TAH_ACT_CLAMPED_GATE) || a->input_norm == TAH_NORM_LAYER)) return TAH_E_SHAPE;
     if (a->input_norm == TAH_NORM_LAYER && !a->ln_colsum && a->n > 0 && a->k > 0) return TAH_E_NULL;
     const int batch = a->batch > 1 ? a->batch : 1;
     if (a->batch < 0 || a->batch > 65535 || a->n_select < 0) return TAH_E_SHAPE;
@@ -475,6 +477,7 @@ extern "C" int tah_linear_rows(const tah_linear_rows_args* a, tah_stream_t strea
     p.res = static_cast<const __bf16*>(a->residual);
     p.bias = static_cast<const __bf16*>(a->bias);
     p.act = a->activation;
+    p.c0 = a->act_c[0]; p.c1 = a->act_c[1];
     p.colsum = a->input_norm == TAH_NORM_LAYER ? a->ln_colsum : nullptr;
     p.y = static_cast<__bf16*>(a->out);
     p.yp = static_cast<bf16x8*>(a->out_packed);

@@ -1,4 +1,4 @@
-// Device-side helpers of the layer mechanisms in row_norm.hip, delta_rule.hip, latent_attn.hip and moe.hip.
+// Device-side helpers of the layer mechanisms in row_norm.hip, delta_rule.hip, latent_attn.hip, window_attn.hip and moe.hip.
 #pragma once
 #include "duo_device.h"
 #include "tah_mixers.h"
@@ -67,6 +67,36 @@ __device__ __forceinline__ float silu_exact(float x) { return x / (1.0f + expf(-
 __device__ __forceinline__ float softplus_exact(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float gelu_tanh_exact(float x) {
     return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+}
+
+// x > 0: a x^2 + x / 2, else b (exp(x) - 1 - x) + x / 2
+__device__ __forceinline__ float xielu(float x, float a, float b) { return (x > 0.f ? a * x * x : b * (expm1f(x) - x)) + 0.5f * x; }
+// gate cut off above the limit, up on both sides of it: g sigmoid(slope g) (u + 1)
+__device__ __forceinline__ float clamped_gate(float g, float u, float limit, float slope) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + fast_exp2(-slope * kLog2e * g)) * (u + 1.0f);
+}
+__device__ __forceinline__ float clamped_gate_exact(float g, float u, float limit, float slope) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
+}
+
+// ---- attention on the matrix cores ----
+constexpr float kNoScore = -1e30f;  // below every score, and finite: differences of it are numbers
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ bf16x8 join8(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
+__device__ __forceinline__ bf16x4 to_bf16x4(const float (&w)[4]) { return __builtin_convertvector((f32x4{w[0], w[1], w[2], w[3]}), bf16x4); }
+// x over the four lane groups that share l % 16
+__device__ __forceinline__ float groups_max(float x) {
+    x = fmaxf(x, __shfl_xor(x, 16));
+    return fmaxf(x, __shfl_xor(x, 32));
+}
+__device__ __forceinline__ float groups_sum(float x) {
+    x += __shfl_xor(x, 16);
+    return x + __shfl_xor(x, 32);
 }
 
 inline bool aligned_16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }

@@ -2,8 +2,8 @@
 // weights.  (A decode step of at most 32 rows does not sort: its experts run as batched tah_linear_rows calls, every
 // expert that some row chose over all rows.)
 //
-//  * moe_route_kernel: router logits in float32 from the float32 rows, the largest ones and their softmax; RB rows per
-//    workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
+//  * moe_route_kernel: router logits in float32, their scores, the open groups of experts, the largest ones and their
+//    weights; RB rows per workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
 //  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
 //  * moe_tile_kernel: bf16 tiles of 128 places x 256 weight rows on the matrix cores, both operands staged through LDS
 //    by asynchronous copies, two stages ahead; gate and up rows of the same columns share a wave, which applies the gate.
@@ -18,23 +18,27 @@ namespace {
 constexpr int kMoeThreads = 256;
 constexpr int kMaxExperts = 1024;
 constexpr int kMaxTop = 64;
+constexpr int kGroupsPerLane = 4;  // groups of experts: at most 256
 constexpr int kTile = TAH_MOE_TILE;
 
-__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-
 // LDS: rows [RB][cols] float32, logits [RB][experts + 1]
-template <class E, int RB, int EB, int kThreads>
-__global__ __launch_bounds__(kThreads) void moe_route_kernel(const float* x, const E* router, const E* gate_w, int rows, int cols, int experts,
-                                                                int top, int32_t* index, float* weight, float* shared_gate) {
+template <class X, class E, int RB, int EB, int kThreads>
+__global__ __launch_bounds__(kThreads) void moe_route_kernel(const tah_moe_route_args p) {
     HIP_DYNAMIC_SHARED(float, sm)
+    const X* const x = static_cast<const X*>(p.x);
+    const E* const router = static_cast<const E*>(p.router);
+    const E* const gate_w = static_cast<const E*>(p.gate_w);
+    const int rows = p.rows, cols = p.cols, experts = p.experts, top = p.top;
     float* const xs = sm;
     float* const z = sm + RB * cols;
     constexpr int kWaves = kThreads / kWave;
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, row0 = blockIdx.x * RB;
     const int zs = experts + 1, total = experts + (gate_w ? 1 : 0);
-    for (int i = 4 * tid; i < RB * cols; i += 4 * kThreads) {
+    for (int i = 8 * tid; i < RB * cols; i += 8 * kThreads) {
         const int r = row0 + i / cols;
-        *reinterpret_cast<f32x4*>(xs + i) = r < rows ? *reinterpret_cast<const f32x4*>(x + (int64_t)r * cols + i % cols) : f32x4{0.f, 0.f, 0.f, 0.f};
+        float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        if (r < rows) load8(x + (int64_t)r * cols + i % cols, v);
+        store8(xs + i, v);
     }
     __syncthreads();
     for (int e0 = EB * wave; e0 < total; e0 += EB * kWaves) {
@@ -74,8 +78,50 @@ __global__ __launch_bounds__(kThreads) void moe_route_kernel(const float* x, con
         const int row = row0 + r;
         if (row >= rows) break;
         float* const zr = z + r * zs;
-        if (gate_w && lane == 0) shared_gate[row] = sigmoid_exact(zr[experts]);
-        // the largest logits one after another, the lower index among equals; a chosen one leaves the race
+        if (gate_w && lane == 0) p.shared_gate[row] = sigmoid_exact(zr[experts]);
+        if (p.score == TAH_MOE_SIGMOID) {
+            for (int e = lane; e < experts; e += kWave) zr[e] = sigmoid_exact(zr[e]);
+            TAH_WAVE_LDS_SYNC();
+        }
+        if (p.keep < p.groups) {
+            // a lane's groups: the sum of their two largest scores; then the best groups one after another, and the others'
+            // experts leave the race
+            const int size = experts / p.groups;
+            float gs[kGroupsPerLane];
+#pragma unroll
+            for (int u = 0; u < kGroupsPerLane; ++u) {
+                const int gr = lane + kWave * u;
+                float a = kNegInf, b = kNegInf;
+                for (int i = 0; gr < p.groups && i < size; ++i) {
+                    const float v = zr[gr * size + i];
+                    b = fmaxf(b, fminf(a, v));
+                    a = fmaxf(a, v);
+                }
+                gs[u] = gr < p.groups ? (size > 1 ? a + b : a) : kNegInf;
+            }
+            uint32_t open = 0;  // bit u: group lane + 64 u is open
+            for (int j = 0; j < p.keep; ++j) {
+                float bv = kNegInf;
+                int bi = 0x7fffffff;
+#pragma unroll
+                for (int u = 0; u < kGroupsPerLane; ++u)
+                    if (!(open >> u & 1) && gs[u] > bv) { bv = gs[u]; bi = lane + kWave * u; }
+#pragma unroll
+                for (int m = 32; m >= 1; m >>= 1) {
+                    const float ov = __shfl_xor(bv, m);
+                    const int oi = __shfl_xor(bi, m);
+                    if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+                }
+                if (bi % kWave == lane && bi < p.groups) open |= 1u << (bi / kWave);
+            }
+#pragma unroll
+            for (int u = 0; u < kGroupsPerLane; ++u) {
+                const int gr = lane + kWave * u;
+                for (int i = 0; gr < p.groups && !(open >> u & 1) && i < size; ++i) zr[gr * size + i] = kNegInf;
+            }
+            TAH_WAVE_LDS_SYNC();
+        }
+        // the largest scores one after another, the lower index among equals; a chosen one leaves the race
         float mine = kNegInf, first = 0.f;
         int my_index = 0;
         for (int j = 0; j < top; ++j) {
@@ -97,11 +143,11 @@ __global__ __launch_bounds__(kThreads) void moe_route_kernel(const float* x, con
             if (lane == 0) zr[bi] = kNegInf;
             TAH_WAVE_LDS_SYNC();
         }
-        const float p = lane < top ? expf(mine - first) : 0.f;
-        const float sum = wave_sum(p);
+        const float w = lane < top ? expf(mine - first) : 0.f;
+        const float sum = wave_sum(w);
         if (lane < top) {
-            index[(int64_t)row * top + lane] = my_index;
-            weight[(int64_t)row * top + lane] = p / sum;
+            p.index[(int64_t)row * top + lane] = my_index;
+            p.weight[(int64_t)row * top + lane] = p.score == TAH_MOE_SIGMOID ? mine : w / sum;
         }
     }
 }
@@ -145,7 +191,8 @@ struct MoeGemm {
     const int32_t *source, *tile_expert;
     void* out;
     int64_t x_rs, out_rs;
-    int32_t n, k, tiles, col_tiles;
+    int32_t n, k, tiles, col_tiles, act;
+    float c0, c1;
 };
 
 // Which tile of places and which tile of columns a workgroup takes.  Workgroups go to the XCDs round robin; an XCD gets a
@@ -283,7 +330,9 @@ __global__ __launch_bounds__(kTileWaves * kWave) void moe_tile_kernel(const MoeG
                     const int c = n0 + 32 * wn + 16 * i + 4 * (lane / 16);
                     bf16x4 y;
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) y[r] = (__bf16)((acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
+                    for (int r = 0; r < 4; ++r)
+                        y[r] = (__bf16)(p.act == TAH_ACT_CLAMPED_GATE ? clamped_gate(acc[i][j][r], acc[2 + i][j][r], p.c0, p.c1)
+                                                                      : (acc[i][j][r] / (1.0f + fast_exp2(-acc[i][j][r] * kLog2e))) * acc[2 + i][j][r]);
                     if (c < p.n) *reinterpret_cast<bf16x4*>(row + c) = y;
                 }
             } else {
@@ -350,21 +399,16 @@ __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p)
     if (n0 + tc >= p.n) return;
 #pragma unroll
     for (int i = 0; i < 16; ++i)
-        static_cast<float*>(p.out)[((int64_t)tile * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = GATE ? silu_exact(sg[i]) * su[i] : sg[i];
+        static_cast<float*>(p.out)[((int64_t)tile * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = !GATE ? sg[i] : (p.act == TAH_ACT_CLAMPED_GATE ? clamped_gate_exact(sg[i], su[i], p.c0, p.c1) : silu_exact(sg[i]) * su[i]);
 }
 
-template <class E>
-void launch_route(const float* x, const void* router, const void* gate_w, int rows, int cols, int experts, int top, int32_t* index, float* weight,
-                  float* shared_gate, hipStream_t st) {
-    const E* const rt = static_cast<const E*>(router);
-    const E* const gw = static_cast<const E*>(gate_w);
-    const auto lds = [&](int rb) { return (size_t)rb * (cols + experts + 1) * sizeof(float); };
-    if (rows > 256 && lds(4) <= 65536)  // many rows: four share a pass over the router's weights
-        hipLaunchKernelGGL((moe_route_kernel<E, 4, 4, 256>), dim3((rows + 3) / 4), dim3(256), lds(4), st, x, rt, gw, rows, cols, experts, top, index,
-                           weight, shared_gate);
+template <class X, class E>
+void launch_route(const tah_moe_route_args& a, hipStream_t st) {
+    const auto lds = [&](int rb) { return (size_t)rb * (a.cols + a.experts + 1) * sizeof(float); };
+    if (a.rows > 256 && lds(4) <= 65536)  // many rows: four share a pass over the router's weights
+        hipLaunchKernelGGL((moe_route_kernel<X, E, 4, 4, 256>), dim3((a.rows + 3) / 4), dim3(256), lds(4), st, a);
     else  // few rows: what counts is how much of the router's weights one row has in flight
-        hipLaunchKernelGGL((moe_route_kernel<E, 1, 2, 1024>), dim3(rows), dim3(1024), lds(1), st, x, rt, gw, rows, cols, experts, top, index, weight,
-                           shared_gate);
+        hipLaunchKernelGGL((moe_route_kernel<X, E, 1, 2, 1024>), dim3(a.rows), dim3(1024), lds(1), st, a);
 }
 
 int tile_capacity(int64_t pairs, int experts) { return (int)(pairs / kTile + (experts < pairs ? experts : pairs)); }
@@ -372,19 +416,23 @@ int tile_capacity(int64_t pairs, int experts) { return (int)(pairs / kTile + (ex
 }  // namespace
 }  // namespace tah
 
-extern "C" int tah_moe_route(const float* x, const void* router, const void* gate_w, int32_t rows, int32_t cols, int32_t experts, int32_t top,
-                             int32_t* index, float* weight, float* shared_gate, int32_t dtype, tah_stream_t stream) {
+extern "C" int tah_moe_route(const tah_moe_route_args* a, tah_stream_t stream) {
     using namespace tah;
-    if (rows < 0 || cols <= 0 || cols % 8 != 0 || experts <= 0 || experts > kMaxExperts || top <= 0 || top > kMaxTop || top > experts ||
-        (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
+    if (!a) return TAH_E_NULL;
+    if (a->rows < 0 || a->cols <= 0 || a->cols % 8 != 0 || a->experts <= 0 || a->experts > kMaxExperts || a->top <= 0 || a->top > kMaxTop ||
+        a->top > a->experts || (a->dtype != TAH_DT_BF16 && a->dtype != TAH_DT_F32) || (a->score != TAH_MOE_SOFTMAX && a->score != TAH_MOE_SIGMOID))
         return TAH_E_SHAPE;
-    if ((size_t)(cols + experts + 1) * sizeof(float) > 65536) return TAH_E_SHAPE;
-    if (rows == 0) return TAH_OK;
-    if (!x || !router || !index || !weight || (gate_w && !shared_gate)) return TAH_E_NULL;
-    if (!aligned_16(x) || !aligned_16(router) || !aligned_16(gate_w)) return TAH_E_ALIGN;
+    if (a->groups <= 0 || a->groups > kWave * kGroupsPerLane || a->experts % a->groups != 0 || a->keep <= 0 || a->keep > a->groups ||
+        a->top > a->experts / a->groups * a->keep)
+        return TAH_E_SHAPE;
+    if ((size_t)(a->cols + a->experts + 1) * sizeof(float) > 65536) return TAH_E_SHAPE;
+    if (a->rows == 0) return TAH_OK;
+    if (!a->x || !a->router || !a->index || !a->weight || (a->gate_w && !a->shared_gate)) return TAH_E_NULL;
+    if (!aligned_16(a->x) || !aligned_16(a->router) || !aligned_16(a->gate_w)) return TAH_E_ALIGN;
     hipStream_t st = static_cast<hipStream_t>(stream);
-    if (dtype == TAH_DT_BF16) launch_route<__bf16>(x, router, gate_w, rows, cols, experts, top, index, weight, shared_gate, st);
-    else launch_route<float>(x, router, gate_w, rows, cols, experts, top, index, weight, shared_gate, st);
+    if (a->dtype == TAH_DT_F32) launch_route<float, float>(*a, st);
+    else if (a->x_elem) launch_route<__bf16, __bf16>(*a, st);
+    else launch_route<float, __bf16>(*a, st);
     return launch_status();
 }
 
@@ -404,17 +452,18 @@ extern "C" int tah_moe_plan(const int32_t* index, int32_t rows, int32_t top, int
 }
 
 extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const int32_t* source, const int32_t* tile_expert, int32_t tiles, int32_t n,
-                              int32_t k, int32_t kind, void* out, int64_t out_rs, int32_t dtype, tah_stream_t stream) {
+                              int32_t k, int32_t kind, int32_t activation, float c0, float c1, void* out, int64_t out_rs, int32_t dtype,
+                              tah_stream_t stream) {
     using namespace tah;
     if (tiles < 0 || tiles > 65535 || n <= 0 || k <= 0 || n % 4 != 0 || k % 32 != 0 || x_rs < k || out_rs < n || x_rs % 8 != 0 || out_rs % 4 != 0 ||
-        (kind != TAH_LINEAR_PLAIN && kind != TAH_LINEAR_GATE_UP) || (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
+        (kind != TAH_LINEAR_PLAIN && kind != TAH_LINEAR_GATE_UP) || (activation != TAH_ACT_NONE && activation != TAH_ACT_CLAMPED_GATE) || (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
         return TAH_E_SHAPE;
     if (tiles == 0) return TAH_OK;
     if (!x || !w || !tile_expert || !out || (kind == TAH_LINEAR_GATE_UP && !source)) return TAH_E_NULL;
     if (!aligned_16(x) || !aligned_16(w) || !aligned_16(out)) return TAH_E_ALIGN;
     const bool gate = kind == TAH_LINEAR_GATE_UP;
     const int cols = dtype == TAH_DT_F32 ? kPlainCols : (gate ? kTileW / 2 : kTileW);
-    const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k, tiles, (n + cols - 1) / cols};
+    const MoeGemm p{x, w, source, tile_expert, out, x_rs, out_rs, n, k, tiles, (n + cols - 1) / cols, activation, c0, c1};
     const int64_t groups = (int64_t)((tiles + 7) / 8) * 8 * p.col_tiles;  // whole rounds over the XCDs
     if (groups > 0x7fffffff) return TAH_E_SHAPE;
     const dim3 grid((unsigned)groups);

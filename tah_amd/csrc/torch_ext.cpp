@@ -66,6 +66,7 @@ void load_library(const std::string& path, bool allow_host) {
     bind(g.embed_rows, "tah_embed_rows");
     bind(g.residual_norm, "tah_residual_norm");
     bind(g.activate_rows, "tah_activate_rows");
+    bind(g.conv_rows, "tah_conv_rows");
     bind(g.delta_step, "tah_delta_step");
     bind(g.delta_prepare, "tah_delta_prepare");
     bind(g.delta_scan, "tah_delta_scan");
@@ -76,6 +77,11 @@ void load_library(const std::string& path, bool allow_host) {
     bind(g.latent_attend, "tah_latent_attend");
     bind(g.latent_decode_workspace, "tah_latent_decode_workspace");
     bind(g.latent_decode, "tah_latent_decode");
+    bind(g.window_prep, "tah_window_prep");
+    bind(g.window_attend, "tah_window_attend");
+    bind(g.window_append, "tah_window_append");
+    bind(g.window_decode_workspace, "tah_window_decode_workspace");
+    bind(g.window_decode, "tah_window_decode");
     bind(g.moe_route, "tah_moe_route");
     bind(g.moe_places, "tah_moe_places");
     bind(g.moe_plan, "tah_moe_plan");
@@ -917,7 +923,7 @@ optional<Tensor> linear_rows(const Tensor& w_packed, const Tensor& x_packed, int
                              const optional<Tensor>& residual, const optional<Tensor>& out, const optional<Tensor>& out_packed,
                              bool want_out, int64_t input_norm, double norm_eps, const optional<Tensor>& bias, int64_t activation,
                              const optional<Tensor>& ln_colsum, int64_t batch, bool shared_rows, int64_t packed_col_step,
-                             const optional<Tensor>& select) {
+                             const optional<Tensor>& select, double act_c0, double act_c1) {
     need_lib();
     Dev d; d.see(w_packed); d.see(x_packed); d.see(residual); d.see(out); d.see(out_packed); d.see(bias); d.see(ln_colsum); d.see(select);
     if (ln_colsum.has_value())
@@ -959,6 +965,7 @@ optional<Tensor> linear_rows(const Tensor& w_packed, const Tensor& x_packed, int
     a.input_norm = (int32_t)input_norm; a.norm_eps = (float)norm_eps;
     a.bias = bias.has_value() ? bias->data_ptr() : nullptr; a.activation = (int32_t)activation;
     a.ln_colsum = ln_colsum.has_value() ? static_cast<const float*>(ln_colsum->data_ptr()) : nullptr;
+    a.act_c[0] = (float)act_c0; a.act_c[1] = (float)act_c1;
     a.batch = (int32_t)batch; a.out_packed_col_step = (int32_t)packed_col_step;
     a.w_batch_stride = wn; a.x_batch_stride = shared_rows ? 0 : 32 * k; a.out_batch_stride = rows * n;
     a.out_packed_batch_stride = packed_col_step ? 0 : 32 * n;

@@ -64,6 +64,7 @@ struct Api {
     Entry<decltype(&tah_embed_rows)> embed_rows;
     Entry<decltype(&tah_residual_norm)> residual_norm;
     Entry<decltype(&tah_activate_rows)> activate_rows;
+    Entry<decltype(&tah_conv_rows)> conv_rows;
     Entry<decltype(&tah_delta_step)> delta_step;
     Entry<decltype(&tah_delta_prepare)> delta_prepare;
     Entry<decltype(&tah_delta_scan)> delta_scan;
@@ -74,6 +75,11 @@ struct Api {
     Entry<decltype(&tah_latent_attend)> latent_attend;
     Entry<decltype(&tah_latent_decode_workspace)> latent_decode_workspace;
     Entry<decltype(&tah_latent_decode)> latent_decode;
+    Entry<decltype(&tah_window_prep)> window_prep;
+    Entry<decltype(&tah_window_attend)> window_attend;
+    Entry<decltype(&tah_window_append)> window_append;
+    Entry<decltype(&tah_window_decode_workspace)> window_decode_workspace;
+    Entry<decltype(&tah_window_decode)> window_decode;
     Entry<decltype(&tah_moe_route)> moe_route;
     Entry<decltype(&tah_moe_places)> moe_places;
     Entry<decltype(&tah_moe_plan)> moe_plan;

@@ -28,9 +28,22 @@ template <class T> T* at_(const Tensor& t) { return static_cast<T*>(mptr(t)); }
 template <class T> T* at_(const optional<Tensor>& t) { return t.has_value() ? static_cast<T*>(mptr(*t)) : nullptr; }
 void* any(const optional<Tensor>& t) { return t.has_value() ? mptr(*t) : nullptr; }
 
+// A batch of portions: what tah_portions points at.
+struct Portions {
+    Tensor cu, slot, pos0, row_seq;
+    Portions(Tensor cu_, Tensor slot_, Tensor pos0_, Tensor row_seq_) : cu(cu_), slot(slot_), pos0(pos0_), row_seq(row_seq_) {
+        flat(cu, at::kInt, slot.numel() + 1, "Portions: cu"); flat(slot, at::kInt, -1, "Portions: slot");
+        flat(pos0, at::kInt, slot.numel(), "Portions: pos0"); flat(row_seq, at::kInt, -1, "Portions: row_seq");
+    }
+    tah_portions c(Dev& d) const {
+        d.see(cu); d.see(slot); d.see(pos0); d.see(row_seq);
+        return {at_<int32_t>(cu), at_<int32_t>(slot), at_<int32_t>(pos0), at_<int32_t>(row_seq), (int32_t)slot.numel(), (int32_t)row_seq.numel()};
+    }
+};
+
 void embed_rows(const Tensor& tok, const Tensor& embed, const Tensor& x, const optional<Tensor>& xe, const optional<Tensor>& x_packed,
                 const optional<Tensor>& pos, const optional<Tensor>& finished, const optional<Tensor>& slot, const optional<Tensor>& q_pos,
-                const optional<Tensor>& active, int64_t slot_base) {
+                const optional<Tensor>& active, int64_t slot_base, double scale) {
     need_lib();
     Dev d; d.see(tok); d.see(embed); d.see(x); d.see(xe); d.see(x_packed); d.see(pos); d.see(finished); d.see(slot); d.see(q_pos); d.see(active);
     const int64_t rows = tok.numel(), cols = embed.size(1);
@@ -46,24 +59,43 @@ void embed_rows(const Tensor& tok, const Tensor& embed, const Tensor& x, const o
     a.tok = at_<int64_t>(tok); a.pos = at_<int32_t>(pos); a.finished = at_<uint8_t>(finished); a.embed = ptr(embed); a.x = at_<float>(x);
     a.xe = any(xe); a.x_packed = any(x_packed); a.slot = at_<int32_t>(slot); a.q_pos = at_<int32_t>(q_pos); a.active = at_<uint8_t>(active);
     a.rows = (int32_t)rows; a.vocab = (int32_t)embed.size(0); a.cols = (int32_t)cols; a.slot_base = (int32_t)slot_base;
+    a.scale = (float)scale;
     check_rc(g.embed_rows(&a, d.stream()), "tah_embed_rows");
 }
 
-void residual_norm(const Tensor& x, const Tensor& coef, int64_t width, double eps, const optional<Tensor>& y, const optional<Tensor>& y_scale,
+// A short causal convolution of a sublayer's input: its taps [taps, cols] and the slots' last inputs [slots, taps, cols].
+struct InputConv {
+    Tensor w, state;
+    InputConv(Tensor w_, Tensor state_) : w(w_), state(state_) {
+        TORCH_CHECK(w.dim() == 2 && state.dim() == 3 && state.size(1) == w.size(0) && state.size(2) == w.size(1),
+                    "InputConv: w [taps, cols], state [slots, taps, cols]");
+        flat(w, at::kFloat, -1, "InputConv: w");
+        dtype_of(state, "InputConv: state");
+        TORCH_CHECK(state.is_contiguous(), "InputConv: state must be contiguous");
+    }
+};
+
+void residual_norm(const Tensor& x, const optional<Tensor>& coef, int64_t width, double eps, const optional<Tensor>& y, const optional<Tensor>& y_scale,
                    const optional<Tensor>& experts, const optional<Tensor>& index, const optional<Tensor>& weight, const optional<Tensor>& xe,
-                   const optional<Tensor>& x_packed, const optional<Tensor>& final_coef, const optional<Tensor>& normed,
-                   const optional<Tensor>& normed_packed, int64_t index_scale, int64_t index_row) {
+                   const optional<Tensor>& x_packed, const optional<Tensor>& next_coef, const optional<Tensor>& normed,
+                   const optional<Tensor>& normed_packed, int64_t index_scale, int64_t index_row, int64_t groups, int64_t group_cols,
+                   const InputConv* conv, const optional<Tensor>& slot, const optional<Tensor>& pos) {
     need_lib();
     Dev d; d.see(x); d.see(coef); d.see(y); d.see(y_scale); d.see(experts); d.see(index); d.see(weight); d.see(xe); d.see(x_packed);
-    d.see(final_coef); d.see(normed); d.see(normed_packed);
+    d.see(next_coef); d.see(normed); d.see(normed_packed); d.see(slot); d.see(pos);
     TORCH_CHECK(x.dim() == 2, "residual_norm: x must be [rows, cols]");
-    TORCH_CHECK(y.has_value() || experts.has_value(), "residual_norm: nothing to add");
     const int64_t rows = x.size(0), cols = x.size(1);
-    const at::ScalarType ty = y.has_value() ? y->scalar_type() : experts->scalar_type();
+    // (the element type is that of whatever is given in it)
+    const optional<Tensor>* const elems[] = {&y, &experts, &xe, &normed, &x_packed, &normed_packed};
+    const Tensor* elem = nullptr;
+    for (const auto* t : elems)
+        if (!elem && t->has_value()) elem = &**t;
+    TORCH_CHECK(elem, "residual_norm: nothing to add and nothing to write");
+    const at::ScalarType ty = elem->scalar_type();
     tah_residual_norm_args a{};
-    a.dtype = dtype_of(y.has_value() ? *y : *experts, "residual_norm: y");
+    a.dtype = dtype_of(*elem, "residual_norm: y");
     flat(x, at::kFloat, rows * cols, "residual_norm: x");
-    flat(coef, at::kFloat, cols, "residual_norm: coef"); flat(final_coef, at::kFloat, cols, "residual_norm: final_coef");
+    flat(coef, at::kFloat, cols, "residual_norm: coef"); flat(next_coef, at::kFloat, cols, "residual_norm: next_coef");
     flat(xe, ty, rows * cols, "residual_norm: xe"); flat(normed, ty, rows * cols, "residual_norm: normed");
     flat(x_packed, at::kBFloat16, 32 * cols, "residual_norm: x_packed"); flat(normed_packed, at::kBFloat16, 32 * cols, "residual_norm: normed_packed");
     flat(y_scale, at::kFloat, rows, "residual_norm: y_scale");
@@ -76,37 +108,44 @@ void residual_norm(const Tensor& x, const Tensor& coef, int64_t width, double ep
         a.index_scale = (int32_t)index_scale; a.index_row = (int32_t)index_row;
         a.index = at_<int32_t>(*index); a.weight = at_<float>(*weight);
     }
-    a.y_scale = at_<float>(y_scale); a.coef = at_<float>(coef); a.final_coef = at_<float>(final_coef); a.x = at_<float>(x);
+    a.y_scale = at_<float>(y_scale); a.coef = at_<float>(coef); a.next_coef = at_<float>(next_coef); a.x = at_<float>(x);
     a.xe = any(xe); a.x_packed = any(x_packed); a.normed = any(normed); a.normed_packed = any(normed_packed);
     a.rows = (int32_t)rows; a.width = (int32_t)width; a.cols = (int32_t)cols; a.eps = (float)eps;
+    a.groups = (int32_t)groups; a.group_cols = (int32_t)group_cols;
+    if (conv) {
+        d.see(conv->w); d.see(conv->state);
+        TORCH_CHECK(slot.has_value() && pos.has_value() && conv->w.size(1) == cols && conv->state.scalar_type() == ty,
+                    "residual_norm: the convolution needs slot, pos and rows of its own width and type");
+        flat(slot, at::kInt, rows, "residual_norm: slot"); flat(pos, at::kInt, rows, "residual_norm: pos");
+        a.conv = at_<float>(conv->w); a.conv_state = mptr(conv->state); a.slot = at_<int32_t>(slot); a.pos = at_<int32_t>(pos);
+        a.taps = (int32_t)conv->w.size(0); a.nslots = (int32_t)conv->state.size(0);
+    }
     check_rc(g.residual_norm(&a, d.stream()), "tah_residual_norm");
 }
 
-Tensor activate_rows(const Tensor& in, int64_t kind, const optional<Tensor>& out_) {
+Tensor activate_rows(const Tensor& in, int64_t kind, const optional<Tensor>& out_, double c0, double c1) {
     need_lib();
     Dev d; d.see(in); d.see(out_);
     TORCH_CHECK(in.dim() == 2 && (in.numel() == 0 || in.stride(1) == 1), "activate_rows: a matrix with contiguous rows expected");
-    const int64_t rows = in.size(0), cols = kind == TAH_ROWS_SILU_MUL ? in.size(1) / 2 : in.size(1);
+    const int64_t rows = in.size(0), cols = kind == TAH_ROWS_SILU_MUL || kind == TAH_ROWS_CLAMPED_GATE ? in.size(1) / 2 : in.size(1);
     Tensor out = out_.has_value() ? *out_ : at::empty({rows, cols}, in.options());
     const int64_t rs = matrix(out, in.scalar_type(), rows, cols, "activate_rows: out");
-    check_rc(g.activate_rows(ptr(in), rows > 1 ? in.stride(0) : in.size(1), mptr(out), rs, (int32_t)rows, (int32_t)cols, (int32_t)kind,
+    check_rc(g.activate_rows(ptr(in), rows > 1 ? in.stride(0) : in.size(1), mptr(out), rs, (int32_t)rows, (int32_t)cols, (int32_t)kind, (float)c0, (float)c1,
                              dtype_of(in, "activate_rows: in"), d.stream()),
              "tah_activate_rows");
     return out;
 }
 
-// A batch of portions: what tah_portions points at.
-struct Portions {
-    Tensor cu, slot, pos0, row_seq;
-    Portions(Tensor cu_, Tensor slot_, Tensor pos0_, Tensor row_seq_) : cu(cu_), slot(slot_), pos0(pos0_), row_seq(row_seq_) {
-        flat(cu, at::kInt, slot.numel() + 1, "Portions: cu"); flat(slot, at::kInt, -1, "Portions: slot");
-        flat(pos0, at::kInt, slot.numel(), "Portions: pos0"); flat(row_seq, at::kInt, -1, "Portions: row_seq");
-    }
-    tah_portions c(Dev& d) const {
-        d.see(cu); d.see(slot); d.see(pos0); d.see(row_seq);
-        return {at_<int32_t>(cu), at_<int32_t>(slot), at_<int32_t>(pos0), at_<int32_t>(row_seq), (int32_t)slot.numel(), (int32_t)row_seq.numel()};
-    }
-};
+void conv_rows(const Tensor& h, const InputConv& conv, const Portions& p, const Tensor& out) {
+    need_lib();
+    Dev d; d.see(h); d.see(out); d.see(conv.w); d.see(conv.state);
+    const tah_portions P = p.c(d);
+    const int64_t cols = conv.w.size(1);
+    flat(h, conv.state.scalar_type(), P.rows * cols, "conv_rows: h"); flat(out, conv.state.scalar_type(), P.rows * cols, "conv_rows: out");
+    check_rc(g.conv_rows(ptr(h), at_<float>(conv.w), mptr(conv.state), &P, mptr(out), (int32_t)cols, (int32_t)conv.w.size(0), (int32_t)conv.state.size(0),
+                         dtype_of(h, "conv_rows: h"), d.stream()),
+             "tah_conv_rows");
+}
 
 // One gated delta-rule layer: its constants, small weights and state.
 struct DeltaLayer {
@@ -273,19 +312,78 @@ struct LatentLayer {
     }
 };
 
+// One layer of attention in a window with kept first tokens, on a cache of rows [slots, kv_heads, keep + ring, row].
+struct WindowLayer {
+    Tensor cache, cos, sin;
+    tah_window_layer L{};
+    int64_t q_col, k_col, g_col;
+    WindowLayer(Tensor cache_, Tensor cos_, Tensor sin_, int64_t heads, int64_t key_dim, int64_t value_dim, int64_t rot_dim, int64_t rot_pad,
+                int64_t rot_source, int64_t keep_first, int64_t window, double scale, int64_t q_col_, int64_t k_col_, int64_t g_col_)
+        : cache(cache_), cos(cos_), sin(sin_), q_col(q_col_), k_col(k_col_), g_col(g_col_) {
+        TORCH_CHECK(cache.dim() == 4 && cache.is_contiguous() && keep_first >= 0 && cache.size(2) > keep_first,
+                    "WindowLayer: cache [slots, kv_heads, keep_first + ring, row]");
+        TORCH_CHECK(cos.dim() == 2 && cos.size(1) == rot_dim / 2, "WindowLayer: cos / sin must be [positions, rot_dim / 2]");
+        flat(cos, at::kFloat, -1, "WindowLayer: cos"); flat(sin, at::kFloat, cos.numel(), "WindowLayer: sin");
+        L.dtype = dtype_of(cache, "WindowLayer: cache");
+        L.cache = mptr(cache);
+        L.heads = (int32_t)heads; L.kv_heads = (int32_t)cache.size(1); L.row = (int32_t)cache.size(3); L.key_dim = (int32_t)key_dim;
+        L.value_dim = (int32_t)value_dim; L.rot_dim = (int32_t)rot_dim; L.rot_pad = (int32_t)rot_pad; L.rot_source = (int32_t)rot_source;
+        L.keep_first = (int32_t)keep_first; L.ring = (int32_t)(cache.size(2) - keep_first); L.window = (int32_t)window; L.nslots = (int32_t)cache.size(0);
+        L.scale = (float)scale;
+    }
+    tah_window_rows rows(Dev& d, const Tensor& proj, const Tensor& pos, const optional<Tensor>& slot) const {
+        d.see(cache); d.see(cos); d.see(sin); d.see(proj); d.see(pos); d.see(slot);
+        const int64_t n = pos.numel();
+        int64_t need = std::max(q_col + (int64_t)L.heads * L.key_dim, k_col + (int64_t)L.kv_heads * L.row);
+        if (g_col >= 0) need = std::max(need, g_col + L.heads);
+        flat(pos, at::kInt, n, "WindowLayer: pos"); flat(slot, at::kInt, n, "WindowLayer: slot");
+        tah_window_rows r{};
+        r.proj_row_stride = matrix(proj, elem_type(L.dtype), n, need, "WindowLayer: proj");
+        r.proj = mptr(proj); r.cos = at_<float>(cos); r.sin = at_<float>(sin); r.pos = at_<int32_t>(pos); r.slot = at_<int32_t>(slot);
+        r.q_col = (int32_t)q_col; r.k_col = (int32_t)k_col; r.g_col = (int32_t)g_col; r.rows = (int32_t)n; r.table_rows = (int32_t)cos.size(0);
+        return r;
+    }
+    int64_t width() const { return (int64_t)L.heads * L.value_dim; }
+    // rotation, attention and cache of a batch of portions -> out [rows, >= heads * value_dim]; proj is rotated in place
+    void portions(const Tensor& proj, const Portions& p, const Tensor& pos, const Tensor& out) const {
+        need_lib();
+        Dev d; d.see(out);
+        const tah_window_rows r = rows(d, proj, pos, c10::nullopt);
+        const tah_portions P = p.c(d);
+        const int64_t rs = matrix(out, elem_type(L.dtype), r.rows, width(), "WindowLayer.portions: out");
+        check_rc(g.window_prep(&L, &r, d.stream()), "tah_window_prep");
+        check_rc(g.window_attend(&L, &P, &r, mptr(out), rs, d.stream()), "tah_window_attend");
+        check_rc(g.window_append(&L, &P, &r, d.stream()), "tah_window_append");
+    }
+    int64_t decode_workspace(int64_t n) const { need_lib(); return (int64_t)g.window_decode_workspace(&L, (int32_t)n); }
+    void decode(const Tensor& proj, const Tensor& slot, const Tensor& pos, const optional<Tensor>& out, const optional<Tensor>& out_packed,
+                const optional<Tensor>& workspace) const {
+        need_lib();
+        Dev d; d.see(out); d.see(out_packed); d.see(workspace);
+        const tah_window_rows r = rows(d, proj, pos, slot);
+        const int64_t rs = out.has_value() ? matrix(*out, elem_type(L.dtype), r.rows, width(), "WindowLayer.decode: out") : 0;
+        flat(out_packed, at::kBFloat16, 32 * width(), "WindowLayer.decode: out_packed");
+        flat(workspace, at::kByte, -1, "WindowLayer.decode: workspace");
+        check_rc(g.window_decode(&L, &r, any(out), rs, any(out_packed), any(workspace), workspace.has_value() ? (size_t)workspace->numel() : 0, d.stream()),
+                 "tah_window_decode");
+    }
+};
+
 void moe_route(const Tensor& x, const Tensor& router, const optional<Tensor>& gate_w, const Tensor& index, const Tensor& weight,
-               const optional<Tensor>& shared_gate) {
+               const optional<Tensor>& shared_gate, int64_t score, int64_t groups, int64_t keep) {
     need_lib();
     Dev d; d.see(x); d.see(router); d.see(gate_w); d.see(index); d.see(weight); d.see(shared_gate);
     TORCH_CHECK(x.dim() == 2 && router.dim() == 2 && router.size(1) == x.size(1) && index.dim() == 2, "moe_route: x [rows, cols], router [experts, cols]");
     const int64_t rows = x.size(0), cols = x.size(1), top = index.size(1);
-    flat(x, at::kFloat, rows * cols, "moe_route: x"); flat(router, router.scalar_type(), -1, "moe_route: router");
+    const bool x_elem = x.scalar_type() == router.scalar_type();
+    flat(x, x_elem ? router.scalar_type() : at::kFloat, rows * cols, "moe_route: x"); flat(router, router.scalar_type(), -1, "moe_route: router");
     flat(gate_w, router.scalar_type(), cols, "moe_route: gate_w"); flat(index, at::kInt, rows * top, "moe_route: index");
     flat(weight, at::kFloat, rows * top, "moe_route: weight"); flat(shared_gate, at::kFloat, rows, "moe_route: shared_gate");
     TORCH_CHECK(gate_w.has_value() == shared_gate.has_value(), "moe_route: gate_w and shared_gate come together");
-    check_rc(g.moe_route(at_<float>(x), ptr(router), any(gate_w), (int32_t)rows, (int32_t)cols, (int32_t)router.size(0), (int32_t)top, at_<int32_t>(index),
-                         at_<float>(weight), at_<float>(shared_gate), dtype_of(router, "moe_route: router"), d.stream()),
-             "tah_moe_route");
+    const tah_moe_route_args a{ptr(x), ptr(router), any(gate_w), at_<int32_t>(index), at_<float>(weight), at_<float>(shared_gate), (int32_t)rows,
+                               (int32_t)cols, (int32_t)router.size(0), (int32_t)top, (int32_t)groups, (int32_t)keep, (int32_t)score, x_elem,
+                               dtype_of(router, "moe_route: router")};
+    check_rc(g.moe_route(&a, d.stream()), "tah_moe_route");
 }
 
 // -> source [places], tile_expert [tiles and their number], place [rows, top]
@@ -303,7 +401,7 @@ std::vector<Tensor> moe_plan(const Tensor& index, int64_t experts) {
     return {source, tile, place};
 }
 
-Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& source, const Tensor& tile_expert, bool gate_up) {
+Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& source, const Tensor& tile_expert, bool gate_up, bool clamped, double c0, double c1) {
     need_lib();
     Dev d; d.see(x); d.see(w); d.see(source); d.see(tile_expert);
     TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && (!gate_up || w.size(1) % 2 == 0), "moe_linear: w must be a contiguous [experts, n, k] tensor");
@@ -312,7 +410,7 @@ Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& source, const 
     const int64_t rs = matrix(x, w.scalar_type(), gate_up ? 1 : tiles * TAH_MOE_TILE, k, "moe_linear: x");
     Tensor out = at::empty({tiles * TAH_MOE_TILE, n}, x.options());
     check_rc(g.moe_linear(ptr(x), rs, ptr(w), at_<int32_t>(source), at_<int32_t>(tile_expert), (int32_t)tiles, (int32_t)n, (int32_t)k,
-                          gate_up ? TAH_LINEAR_GATE_UP : TAH_LINEAR_PLAIN, mptr(out), n, dtype_of(w, "moe_linear: w"), d.stream()),
+                          gate_up ? TAH_LINEAR_GATE_UP : TAH_LINEAR_PLAIN, clamped ? TAH_ACT_CLAMPED_GATE : TAH_ACT_NONE, (float)c0, (float)c1, mptr(out), n, dtype_of(w, "moe_linear: w"), d.stream()),
              "tah_moe_linear");
     return out;
 }
@@ -321,7 +419,9 @@ Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& source, const 
 
 void bind_mixers(py::module_& m) {
     m.def("embed_rows", &embed_rows);
+    py::class_<InputConv>(m, "InputConv").def(py::init<Tensor, Tensor>());
     m.def("residual_norm", &residual_norm);
+    m.def("conv_rows", &conv_rows);
     m.def("activate_rows", &activate_rows);
     m.def("moe_route", &moe_route);
     m.def("moe_plan", &moe_plan);
@@ -338,6 +438,11 @@ void bind_mixers(py::module_& m) {
         .def("attend", &LatentLayer::attend)
         .def("decode_workspace", &LatentLayer::decode_workspace)
         .def("decode", &LatentLayer::decode);
+    py::class_<WindowLayer>(m, "WindowLayer")
+        .def(py::init<Tensor, Tensor, Tensor, int64_t, int64_t, int64_t, int64_t, int64_t, int64_t, int64_t, int64_t, double, int64_t, int64_t, int64_t>())
+        .def("portions", &WindowLayer::portions)
+        .def("decode_workspace", &WindowLayer::decode_workspace)
+        .def("decode", &WindowLayer::decode);
 }
 
 }  // namespace tah_ext

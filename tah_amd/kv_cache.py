@@ -212,6 +212,23 @@ class RecurrentState:
         self.conv = torch.zeros((nslots, taps, channels), dtype=dtype, device=device)
 
 
+class WindowCache:
+    """One windowed-attention layer's cache: per slot and key/value head the rows of the first ``keep`` tokens, then a ring of
+    ``ring`` rows, token p at row p (p < keep) or ``keep + (p - keep) % ring``.  ``ring`` is at least the window.  As with
+    :class:`LatentRing` positions alone decide what is read, so nothing is cleared between owners."""
+
+    def __init__(self, nslots: int, kv_heads: int, keep: int, ring: int, row: int, *, device, dtype):
+        self.rows = torch.zeros((nslots, kv_heads, keep + ring, row), dtype=dtype, device=device)
+
+
+class InputTail:
+    """What a short convolution of a sublayer's input remembers: the inputs of the last ``taps`` tokens, ``rows``
+    [slots, taps, channels], token p at ``p % taps``.  Nothing in front of position 0 is read."""
+
+    def __init__(self, nslots: int, taps: int, channels: int, *, device, dtype):
+        self.rows = torch.zeros((nslots, taps, channels), dtype=dtype, device=device)
+
+
 class SlotPool:
     """The sequence slots of an engine: which are taken, and how many tokens each has (host side)."""
 

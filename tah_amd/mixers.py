@@ -1,6 +1,6 @@
 """Layer mechanisms of decoders that are described layer by layer, each a class over the kernels of
-include/tah_mixers.h with its sizes and constants as parameters: a mixer (gated delta rule, latent attention) and a
-feed-forward (dense, mixture of experts).  ``tah_amd.stack`` puts them together.
+include/tah_mixers.h with its sizes and constants as parameters: a mixer (gated delta rule, latent attention, attention in a
+window with kept first tokens) and a feed-forward (dense, mixture of experts).  ``tah_amd.stack`` puts them together.
 
 Every mechanism runs in two forms.  ``portions(step)``: rows of several tokens per sequence (prompts, parts of prompts),
 with library GEMMs for the dense products.  ``rows(step)``: one token per sequence, at most 32 rows; in bf16 the dense
@@ -13,16 +13,47 @@ whatever a model's sizes are.
 from __future__ import annotations
 
 import dataclasses
-from typing import Dict, Optional
+import math
+from typing import Dict, Optional, Tuple
 
 import torch
 
 from . import ops
 from ._capi import TahDuoError
-from .kv_cache import LatentRing, RecurrentState
+from .kv_cache import LatentRing, RecurrentState, WindowCache
 from .ops import _call
 
-GELU_TANH, SILU_MUL = 0, 1
+
+@dataclasses.dataclass(frozen=True)
+class Activation:
+    """An element-wise function of a feed-forward's hidden rows: ``kind`` and constants for ``activate_rows``, and the keyword
+    that makes it the epilogue of ``ops.linear_rows``."""
+    kind: int
+    c: Tuple[float, float] = (0.0, 0.0)
+    rows: Dict[str, object] = dataclasses.field(default_factory=dict)
+
+    def __call__(self, h: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        return _call("activate_rows", h, self.kind, out, *self.c)
+
+
+GELU_TANH = Activation(0, rows={"gelu_tanh": True})
+SILU_MUL = Activation(1)
+
+
+def softplus(x: float) -> float:
+    return max(x, 0.0) + math.log1p(math.exp(-abs(x)))
+
+
+def xielu(p: float, q: float) -> Activation:
+    """softplus(p) x^2 + x / 2 above zero, (1/2 + softplus(q)) (exp(x) - 1 - x) + x / 2 below."""
+    c = (softplus(p), 0.5 + softplus(q))
+    return Activation(2, c, {"xielu": c})
+
+
+def clamped_gate(limit: float, slope: float = 1.702) -> Activation:
+    """g sigmoid(slope g) (u + 1) of g = min(gate, limit) and u = up cut off at both limits."""
+    c = (limit, slope)
+    return Activation(3, c, {"clamped": c})
 
 
 def pad_to(n: int, m: int = 32) -> int:
@@ -73,8 +104,9 @@ class PackedBatch:
 
 @dataclasses.dataclass
 class Step:
-    """What a forward of some rows carries through the layers.  x float32 [rows, cols] is the residual stream, xe the same
-    in the element type, xp (bf16, at most 32 rows) its rows form; the rest says whose rows they are."""
+    """What a forward of some rows carries through the layers.  x float32 [rows, cols] is the residual stream, xe what the next
+    sublayer reads, in the element type (the same rows, or with ``normed`` the norm in front of it), xp (bf16, at most 32
+    rows) its rows form; the rest says whose rows they are."""
     x: torch.Tensor
     xe: torch.Tensor
     pos: torch.Tensor                          # int32 [rows]
@@ -83,6 +115,7 @@ class Step:
     portions: object = None                    # several tokens per sequence: tah_amd._C.Portions ...
     starts: Optional[list] = None              # ... and on the host: (length, first position) per sequence
     contexts: Dict[int, tuple] = dataclasses.field(default_factory=dict)  # latent rows portions can see, per ring
+    normed: bool = False
 
     @property
     def n(self) -> int:
@@ -293,11 +326,109 @@ class LatentAttention:
             return Sublayer(m.o(out))
 
 
+# ── attention in a window with kept first tokens ─────────────────────────────────────────────────────────────────────
+@dataclasses.dataclass(frozen=True)
+class WindowSpec:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    rot_dim: int                     # the first so many dimensions of a head are rotated
+    rope_base: float
+    scale: float
+    window: Optional[int] = None     # position i sees j <= i with i - j < window (None: all) ...
+    keep_first: int = 0              # ... or j < keep_first
+    adjacent: bool = True            # rotated pairs are dimensions 2 i and 2 i + 1 (else i and i + rot_dim / 2)
+
+
+class WindowAttention:
+    """Attention with grouped query heads in a sliding window that keeps a sequence's first tokens.  Weights [out, in]: q [heads *
+    dim, width], k [kv_heads * dim, width], o [width, heads * vdim]; v [kv_heads * vdim, width], or none when the keys before
+    their rotation are the values; g [heads, width], or none: a sigmoid gate per head on its result.
+
+    What is cached of a token and key/value head is one row, values in front, keys at its end, rotated dimensions last.
+    Without v the two overlap: [rotated dimensions, unrotated | the others | rotated dimensions, rotated], the values
+    being the first two parts and the keys the last two.  Queries and the output projection follow that order, which is
+    given to the weights here."""
+
+    def __init__(self, spec: WindowSpec, w: Dict[str, torch.Tensor], cols: int):
+        s = self.spec = spec
+        H, G, D, rd = s.heads, s.kv_heads, s.dim, s.rot_dim
+        tied = "v" not in w
+        if H % G or rd > D or rd % 2 or (tied and s.vdim != D):
+            raise TahDuoError(f"attention: {H} heads on {G}, {rd} of {D} dimensions rotated, values of {s.vdim}: sizes that do not go together")
+        self.rot_pad = pad_to(rd, 8)
+        self.key_dim = pad_to(self.rot_pad + D - rd)
+        rest = self.key_dim - self.rot_pad
+        turned = list(range(rd)) if s.adjacent else [i + h * (rd // 2) for i in range(rd // 2) for h in (0, 1)]
+        others = list(range(rd, D))
+        pad = lambda idx, n: idx + [-1] * (n - len(idx))
+        key = pad(others, rest) + pad(turned, self.rot_pad)
+        if tied:
+            value = pad(turned, self.rot_pad) + pad(others, rest)
+            row, self.rot_source = value + [-1] * self.rot_pad, 0
+            kv = self._ordered(w["k"], G, D, row)
+        else:
+            value = pad(list(range(s.vdim)), pad_to(s.vdim))
+            row, self.rot_source = value + key, len(value) + rest
+            kv = torch.cat([self._ordered(w["v"], G, s.vdim, value).view(G, len(value), -1), self._ordered(w["k"], G, D, key).view(G, len(key), -1)],
+                           1).flatten(0, 1)
+        self.value_dim, self.row = len(value), len(row)
+        parts = [self._ordered(w["q"], H, D, key), kv] + ([w["g"]] if "g" in w else [])
+        self.k_col = H * self.key_dim
+        self.g_col = self.k_col + G * self.row if "g" in w else -1
+        proj = torch.cat(parts)
+        self.proj = Linear(padded(proj, pad_to(proj.shape[0]), cols))
+        self.width_o = H * self.value_dim
+        self.o = Linear(padded(self._ordered(w["o"].t().contiguous(), H, s.vdim, value).t(), cols, self.width_o))
+
+    @staticmethod
+    def _ordered(w: torch.Tensor, heads: int, size: int, order: list) -> torch.Tensor:
+        """w [heads * size, c] -> [heads * len(order), c]: a head's rows in the given order, zeros for -1."""
+        w = w.view(heads, size, -1)
+        idx = torch.tensor(order, device=w.device)
+        out = w[:, idx.clamp_min(0)]
+        out[:, idx < 0] = 0
+        return out.flatten(0, 1)
+
+    def bind(self, engine) -> "WindowAttention.Bound":
+        return WindowAttention.Bound(self, engine)
+
+    class Bound:
+        def __init__(self, m: "WindowAttention", engine):
+            s = m.spec
+            self.m = m
+            keep = min(s.keep_first, engine.max_len)
+            window = engine.max_len if s.window is None else min(s.window, engine.max_len)
+            self.cache = WindowCache(engine.B, s.kv_heads, keep, window, m.row, device=engine.device, dtype=engine.dtype)
+            self.layer = ops.lib().WindowLayer(self.cache.rows, *engine.rope(s.rope_base, s.rot_dim), s.heads, m.key_dim, m.value_dim, s.rot_dim,
+                                               m.rot_pad, m.rot_source, keep, window, s.scale, 0, m.k_col, m.g_col)
+            z = lambda n, dt=engine.dtype: torch.zeros(n, dtype=dt, device=engine.device)
+            self.workspace = z(max(int(self.layer.decode_workspace(min(engine.B, ops.LINEAR_MAX_ROWS))), 16), torch.uint8)
+            self.op = z(32 * m.width_o) if engine.packed else None
+
+        def rows(self, st: Step) -> Sublayer:
+            m = self.m
+            if st.packed:
+                _call_on(self.layer.decode, m.proj.rows(st.xp, st.n), st.slot, st.pos, None, self.op, self.workspace)
+                return Sublayer(m.o.rows(self.op, st.n))
+            out = torch.empty(st.n, m.width_o, dtype=st.xe.dtype, device=st.x.device)
+            _call_on(self.layer.decode, m.proj(st.xe), st.slot, st.pos, out, None, self.workspace)
+            return Sublayer(m.o(out))
+
+        def portions(self, st: Step) -> Sublayer:
+            m = self.m
+            out = torch.empty(st.n, m.width_o, dtype=st.xe.dtype, device=st.x.device)
+            _call_on(self.layer.portions, m.proj(st.xe), st.portions, st.pos, out)
+            return Sublayer(m.o(out))
+
+
 # ── feed-forward ─────────────────────────────────────────────────────────────────────────────────────────────────────
 class DenseMlp:
-    """down(gelu(up(x))), the tanh form of gelu.  Weights up [ff, width], down [width, ff]."""
+    """down(act(up(x))).  Weights up [ff, width], down [width, ff].  (act(0) = 0: padding stays zero.)"""
 
-    def __init__(self, w: Dict[str, torch.Tensor], cols: int):
+    def __init__(self, w: Dict[str, torch.Tensor], cols: int, act: Activation = GELU_TANH):
+        self.act = act
         ff = pad_to(w["up"].shape[0])
         self.up, self.down = Linear(padded(w["up"], ff, cols)), Linear(padded(w["down"], cols, ff))
 
@@ -312,12 +443,12 @@ class DenseMlp:
         def rows(self, st: Step) -> Sublayer:
             if not st.packed:
                 return self.portions(st)
-            self.m.up.rows(st.xp, st.n, gelu_tanh=True, out_packed=self.ap, want_out=False)
+            self.m.up.rows(st.xp, st.n, out_packed=self.ap, want_out=False, **self.m.act.rows)
             return Sublayer(self.m.down.rows(self.ap, st.n))
 
         def portions(self, st: Step) -> Sublayer:
             h = self.m.up(st.xe)
-            return Sublayer(self.m.down(_call("activate_rows", h, GELU_TANH, h)))
+            return Sublayer(self.m.down(self.m.act(h, h)))
 
 
 class GatedMlp:
@@ -335,16 +466,29 @@ class GatedMlp:
         return self.down.rows(act, n)
 
     def __call__(self, x: torch.Tensor) -> torch.Tensor:
-        return self.down(_call("activate_rows", x @ self.gate_up.t(), SILU_MUL, None))
+        return self.down(SILU_MUL(x @ self.gate_up.t()))
+
+
+@dataclasses.dataclass(frozen=True)
+class Router:
+    """How a token chooses among experts: the ``top`` largest scores, which are the logits (weights: softmax over the chosen
+    ones) or with ``sigmoid`` their sigmoids (weights: the chosen scores).  ``groups`` equal groups of neighbours: only the
+    ``keep`` groups with the largest sum of their two largest scores can be chosen from."""
+    top: int
+    sigmoid: bool = False
+    groups: int = 1
+    keep: int = 1
 
 
 class MoeMlp:
-    """Mixture of gated experts: router in float32, the ``top`` largest logits, softmax over them; optionally a shared expert
-    for every token, times sigmoid(gate . x).  Weights: router [experts, width], gate, up [experts, ff, width], down
-    [experts, width, ff]; shared: dict of a GatedMlp's weights and sg [1, width], or None."""
+    """Mixture of gated experts, the router in float32; optionally a shared expert for every token, times sigmoid(gate . x).
+    Weights: router [experts, width], gate, up [experts, ff, width], down [experts, width, ff]; shared: dict of a
+    GatedMlp's weights and sg [1, width], or None.  ``act``: the experts' gate."""
 
-    def __init__(self, top: int, w: Dict[str, torch.Tensor], shared: Optional[Dict[str, torch.Tensor]], cols: int):
-        self.top, self.experts, self.cols = top, w["router"].shape[0], cols
+    def __init__(self, router: Router, w: Dict[str, torch.Tensor], shared: Optional[Dict[str, torch.Tensor]], cols: int, act: Activation = SILU_MUL):
+        self.rule, self.act, self.top, self.experts, self.cols = router, act, router.top, w["router"].shape[0], cols
+        if self.experts % router.groups or not 0 < router.keep <= router.groups or router.top > self.experts // router.groups * router.keep:
+            raise TahDuoError(f"experts: {router.top} of {self.experts} from {router.keep} of {router.groups} groups: sizes that do not go together")
         self.router = padded(w["router"], self.experts, cols)
         E, ff = self.experts, pad_to(w["gate"].shape[1])
         self.ff = ff
@@ -375,7 +519,7 @@ class MoeMlp:
             index = torch.empty(st.n, m.top, dtype=torch.int32, device=dev)
             weight = torch.empty(st.n, m.top, dtype=torch.float32, device=dev)
             sg = torch.empty(st.n, dtype=torch.float32, device=dev) if m.shared else None
-            _call("moe_route", st.x, m.router, m.shared_gate, index, weight, sg)
+            _call("moe_route", st.xe if st.normed else st.x, m.router, m.shared_gate, index, weight, sg, int(m.rule.sigmoid), m.rule.groups, m.rule.keep)
             return index, weight, sg
 
         def rows(self, st: Step) -> Sublayer:
@@ -384,7 +528,7 @@ class MoeMlp:
                 return self.portions(st)
             index, weight, sg = self._route(st)
             # every expert that some row chose, over all rows: at this size a product costs its weights, not its rows
-            m.gate_up_rows.rows(st.xp, n, shared_rows=True, out_packed=self.ap, want_out=False, select=index)
+            m.gate_up_rows.rows(st.xp, n, shared_rows=True, out_packed=self.ap, want_out=False, select=index, **m.act.rows)
             y = m.down_rows.rows(self.ap, n, select=index)
             shared = m.shared.rows(st.xp, n, self.shared_ap) if m.shared else None
             return Sublayer(shared, sg, y.view(m.experts * n, m.cols), index, weight, index_scale=n, index_row=1)
@@ -393,8 +537,8 @@ class MoeMlp:
             m = self.m
             index, weight, sg = self._route(st)
             source, tiles, place = _call("moe_plan", index, m.experts)
-            h = _call("moe_linear", st.xe, m.gate_up, source, tiles, True)
-            y = _call("moe_linear", h, m.down, source, tiles, False)
+            h = _call("moe_linear", st.xe, m.gate_up, source, tiles, True, "clamped" in m.act.rows, *m.act.c)
+            y = _call("moe_linear", h, m.down, source, tiles, False, False, 0.0, 0.0)
             return Sublayer(m.shared(st.xe) if m.shared else None, sg, y, place, weight)
 
 

@@ -20,7 +20,7 @@ def _call(name: str, *args):
         raise _capi.TahDuoError(str(e).split("\nException raised from")[0]) from None
 
 
-lib = _lib.lib  # the extension with the library loaded (kernel objects: Portions, DeltaLayer, LatentLayer)
+lib = _lib.lib  # the extension with the library loaded (kernel objects: Portions, DeltaLayer, LatentLayer, WindowLayer)
 
 
 MAX_SCHEDULE_SEQS = 4095
@@ -250,7 +250,8 @@ def linear_rows(w_packed: torch.Tensor, x_packed: torch.Tensor, rows: int, n: in
                 out_packed: Optional[torch.Tensor] = None, want_out: bool = True, norm_eps: Optional[float] = None,
                 bias: Optional[torch.Tensor] = None, relu: bool = False, gelu: bool = False,
                 ln_colsum: Optional[torch.Tensor] = None, gelu_tanh: bool = False, batch: int = 1, shared_rows: bool = False,
-                packed_col_step: int = 0, select: Optional[torch.Tensor] = None):
+                packed_col_step: int = 0, select: Optional[torch.Tensor] = None, xielu: Optional[Tuple[float, float]] = None,
+                clamped: Optional[Tuple[float, float]] = None):
     """A linear layer of a decode step on packed operands (``tah_linear_rows``), bf16, rows <= 32.
 
     ``x @ w.T`` [rows, N], plus ``residual`` [rows, N] when given (``out=residual`` updates it in place); with
@@ -266,15 +267,19 @@ def linear_rows(w_packed: torch.Tensor, x_packed: torch.Tensor, rows: int, n: in
     ``gelu_tanh``: the tanh form of gelu.  ``batch`` products of the same sizes in one launch: ``w_packed`` holds their weights
     one after another, ``x_packed`` their rows operands (or one for all, ``shared_rows``), the results are [batch, rows, N] and
     rows forms one after another -- or, with ``packed_col_step``, side by side in one rows form, ``packed_col_step`` columns
-    apart.  ``select`` (int32): only the products whose index it lists run (the others' results keep what they held)."""
-    if relu + gelu + gelu_tanh > 1:
+    apart.  ``select`` (int32): only the products whose index it lists run (the others' results keep what they held).
+    ``xielu`` (c0, c1): ``c0 x^2 + x / 2`` above zero, ``c1 (exp(x) - 1 - x) + x / 2`` below.  ``clamped`` (limit, slope), with
+    ``gate_up``: the gate ``g sigmoid(slope g) (u + 1)`` of ``g = min(gate, limit)``, ``u`` = up cut off at both limits."""
+    if relu + gelu + gelu_tanh + (xielu is not None) + (clamped is not None) > 1:
         raise ValueError("linear_rows: one activation")
     norm = 0 if norm_eps is None else (2 if ln_colsum is not None else 1)
     if ln_colsum is not None and norm_eps is None:
         raise ValueError("linear_rows: ln_colsum needs the LayerNorm's eps")
+    act = 1 if relu else 2 if gelu else 3 if gelu_tanh else 4 if xielu else 5 if clamped else 0
+    c0, c1 = xielu or clamped or (0.0, 0.0)
     return _call("linear_rows", w_packed, x_packed, int(rows), int(n), int(k), bool(gate_up), residual, out, out_packed,
-                 bool(want_out), norm, float(norm_eps or 0.0), bias, 1 if relu else (2 if gelu else (3 if gelu_tanh else 0)), ln_colsum,
-                 int(batch), bool(shared_rows), int(packed_col_step), select)
+                 bool(want_out), norm, float(norm_eps or 0.0), bias, act, ln_colsum, int(batch), bool(shared_rows), int(packed_col_step), select,
+                 float(c0), float(c1))
 
 
 def greedy_step(logits0, logits1, hard, eos: int, tok, finished, pos, out_tokens, step_idx, out_len, n_hard, n_steps) -> None:

@@ -60,6 +60,12 @@ def _zozosun() -> None:
     register(Architecture(zozosun.NAME, zozosun.load, zozosun.engine, (torch.bfloat16, torch.float32)))
 
 
+def _zedudra() -> None:
+    from . import zedudra
+
+    register(Architecture(zedudra.NAME, zedudra.load, zedudra.engine, (torch.bfloat16, torch.float32)))
+
+
 def _qwen3() -> None:
     from .engine import EngineConfig, TaHDecodeEngine, Weights
 
@@ -69,4 +75,5 @@ def _qwen3() -> None:
 
 
 _zozosun()
+_zedudra()
 _qwen3()

@@ -1,5 +1,6 @@
 """Decode engine for decoders that are described layer by layer: a list of layers, each with a mixer and possibly a
-feed-forward of ``tah_amd.mixers``, norms on the sublayers' outputs, and a float32 residual stream.
+feed-forward of ``tah_amd.mixers``, norms on the sublayers' outputs and possibly in front of them, and a float32 residual
+stream.  Layers may share their weights; caches and states are each layer's own.
 
 :class:`StackEngine` is a :class:`tah_amd.engine.DecodeEngine`: the generation state, sampling, loop and captured step
 are the ones every model uses.  Sequences live in slots (``tah_amd.kv_cache.SlotPool``); what a slot holds -- latent
@@ -18,7 +19,7 @@ import torch
 from . import ops
 from ._capi import TahDuoError
 from .engine import DecodeEngine
-from .kv_cache import SlotPool
+from .kv_cache import InputTail, SlotPool
 from .mixers import Linear, LatentAttention, Step, Sublayer, pad_to, padded
 from .ops import _call
 
@@ -29,6 +30,45 @@ class StackLayer:
     coef1: torch.Tensor                 # float32 [cols]: the mixer's output norm and layer scale
     mlp: object = None                  # DenseMlp, MoeMlp, or None
     coef2: Optional[torch.Tensor] = None
+    pre1: Optional[torch.Tensor] = None  # float32 [cols]: norm in front of the mixer (None: it reads the residual stream) ...
+    pre2: Optional[torch.Tensor] = None  # ... and of the feed-forward
+    conv1: Optional[torch.Tensor] = None  # float32 [taps, cols], with pre1: short convolution added to the mixer's input
+
+
+@dataclasses.dataclass(frozen=True)
+class Columns:
+    """Where a row's entries lie when norms run over ``groups`` equal groups of them: every group padded to whole units of
+    eight columns, all of them to whole steps of 32."""
+    width: int
+    groups: int = 1
+
+    def __post_init__(self):
+        if self.groups < 1 or self.width % self.groups:
+            raise TahDuoError(f"a width of {self.width} does not divide into {self.groups} groups")
+
+    @property
+    def group_cols(self) -> int:
+        return pad_to(self.width // self.groups, 8) if self.groups > 1 else self.cols
+
+    @property
+    def cols(self) -> int:
+        return pad_to(self.groups * pad_to(self.width // self.groups, 8) if self.groups > 1 else self.width)
+
+    def spread(self, t: torch.Tensor, dim: int = -1) -> torch.Tensor:
+        """t with ``width`` entries along ``dim`` -> with ``groups * group_cols``, every group followed by its padding."""
+        n = self.width // self.groups
+        if self.groups == 1 or n == self.group_cols:
+            return t
+        t = t.movedim(dim, -1)
+        out = torch.zeros(*t.shape[:-1], self.groups, self.group_cols, dtype=t.dtype, device=t.device)
+        out[..., :n] = t.reshape(*t.shape[:-1], self.groups, n)
+        return out.flatten(-2).movedim(-1, dim).contiguous()
+
+    def gather(self, x: torch.Tensor) -> torch.Tensor:
+        """The entries of padded rows."""
+        if self.groups == 1:
+            return x[..., :self.width]
+        return x[..., :self.groups * self.group_cols].unflatten(-1, (self.groups, -1))[..., :self.width // self.groups].flatten(-2)
 
 
 @dataclasses.dataclass
@@ -41,6 +81,12 @@ class StackModel:
     head: Linear                        # [vocab padded, cols]
     final_coef: torch.Tensor            # float32 [cols]
     layers: List[StackLayer]
+    groups: int = 1                     # of columns that are divided by a root mean square of their own
+    embed_scale: float = 1.0
+
+    @property
+    def columns(self) -> Columns:
+        return Columns(self.width, self.groups)
 
     @property
     def cols(self) -> int:
@@ -67,6 +113,7 @@ def make_head(w: torch.Tensor, cols: int) -> Linear:
 class _Bound:
     mixer: object
     mlp: object
+    conv: object = None
 
 
 class StackEngine(DecodeEngine):
@@ -88,12 +135,18 @@ class StackEngine(DecodeEngine):
             self.bound.append(_Bound(None, None))
             self.bound[i].mixer = L.mixer.bind(self)
             self.bound[i].mlp = L.mlp.bind(self) if L.mlp is not None else None
+            if L.conv1 is not None:
+                tail = InputTail(self.B, L.conv1.shape[0], model.cols, device=dev, dtype=self.dtype)
+                self.bound[i].conv = ops.lib().InputConv(L.conv1, tail.rows)
         cols = model.cols
+        self.normed = any(L.pre1 is not None for L in model.layers)  # sublayers read norms of the residual stream
+        if any((L.pre1 is None) == self.normed or (L.mlp is not None and (L.pre2 is None) == self.normed) for L in model.layers):
+            raise TahDuoError("either every sublayer has a norm in front of it or none has")
         self.group = min(batch, ops.LINEAR_MAX_ROWS)  # rows of a single-token pass
         z = lambda *s, dt=torch.float32: torch.zeros(*s, dtype=dt, device=dev)
         i32 = lambda: z(batch, dt=torch.int32)
         self.x = z(batch, cols)
-        self.xe = z(batch, cols, dt=self.dtype) if self.packed else self.x
+        self.xe = z(batch, cols, dt=self.dtype) if self.packed or self.normed else self.x
         self.slot, self.qpos, self.act = i32(), i32(), z(batch, dt=torch.bool)
         self.xp = z(32 * cols, dt=self.dtype) if self.packed else None
         self.hp = z(32 * cols, dt=self.dtype) if self.packed else None
@@ -118,28 +171,43 @@ class StackEngine(DecodeEngine):
         return self._rope[key]
 
     # ── layers ───────────────────────────────────────────────────────────
-    def _add(self, st: Step, r: Sublayer, coef: torch.Tensor, final: Optional[torch.Tensor], h: torch.Tensor) -> None:
+    def _front(self, i: int):
+        """(norm, convolution, whether it is the output norm) between the residual stream and layer i's mixer, or behind the
+        last layer the output head."""
         m = self.cfg
-        last = final is not None
-        # (in float32 the element-type rows are the residual rows themselves)
-        _call("residual_norm", st.x, coef, m.width, m.eps, r.y, r.y_scale, r.experts, r.index, r.weight,
-              st.xe if self.packed and not last and not st.packed else None, st.xp if not last else None, final,
-              h if last and not st.packed else None, self.hp if last and st.packed else None, r.index_scale, r.index_row)
+        return (m.final_coef, None, True) if i == len(m.layers) else (m.layers[i].pre1, self.bound[i].conv, False)
+
+    def _add(self, st: Step, r: Sublayer, coef: Optional[torch.Tensor], front: tuple, h: torch.Tensor) -> None:
+        """A sublayer's result into the residual stream, and from it what the next sublayer (or the output head) reads."""
+        m, (norm, conv, last) = self.cfg, front
+        geometry = (m.groups, m.columns.group_cols)
+        args = (st.x, coef, m.width, m.eps, r.y, r.y_scale, r.experts, r.index, r.weight)
+        tail = (r.index_scale, r.index_row, *geometry)
+        if last:
+            _call("residual_norm", *args, None, None, norm, None if st.packed else h, self.hp if st.packed else None, *tail, None, None, None)
+        elif norm is None:  # (in float32 the element-type rows are the residual rows themselves)
+            _call("residual_norm", *args, st.xe if self.packed and not st.packed else None, st.xp, None, None, None, *tail, None, None, None)
+        elif conv is None or st.slot is not None:
+            _call("residual_norm", *args, None, None, norm, st.xe, st.xp, *tail, conv, st.slot if conv else None, st.pos if conv else None)
+        else:
+            n = torch.empty_like(st.xe)
+            _call("residual_norm", *args, None, None, norm, n, None, *tail, None, None, None)
+            _call("conv_rows", n, conv, st.portions, st.xe)
 
     def _layers(self, st: Step, h: torch.Tensor, trace: Optional[list] = None) -> None:
         """All layers on the step's rows; the output norm's rows go to ``h`` (or, packed, to ``self.hp``)."""
         single = st.slot is not None
-        m = self.cfg
-        for i, (L, b) in enumerate(zip(m.layers, self.bound)):
-            last = i + 1 == len(m.layers)
-            final = m.final_coef if last else None
+        st.normed = self.normed
+        if st.normed:
+            self._add(st, Sublayer(), None, self._front(0), h)
+        for i, (L, b) in enumerate(zip(self.cfg.layers, self.bound)):
             r = b.mixer.rows(st) if single else b.mixer.portions(st)
-            self._add(st, r, L.coef1, final if b.mlp is None else None, h)
+            self._add(st, r, L.coef1, self._front(i + 1) if b.mlp is None else (L.pre2, None, False), h)
             if b.mlp is not None:
                 r = b.mlp.rows(st) if single else b.mlp.portions(st)
-                self._add(st, r, L.coef2, final, h)
+                self._add(st, r, L.coef2, self._front(i + 1), h)
             if trace is not None:
-                trace.append(st.x.clone())
+                trace.append(self.cfg.columns.gather(st.x).clone())
 
     def _single(self, tok, pos, finished) -> torch.Tensor:
         """One token per slot (rows of finished slots are dropped): logits [B, vocab].  Nothing is read by the host."""
@@ -147,7 +215,8 @@ class StackEngine(DecodeEngine):
         for a in range(0, self.B, self.group):
             b = min(a + self.group, self.B)
             sl = slice(a, b)
-            _call("embed_rows", tok[sl], m.embed, self.x[sl], None, self.xp, pos[sl], finished[sl], self.slot[sl], self.qpos[sl], self.act[sl], a)
+            _call("embed_rows", tok[sl], m.embed, self.x[sl], None, None if self.normed else self.xp, pos[sl], finished[sl], self.slot[sl], self.qpos[sl],
+                  self.act[sl], a, m.embed_scale)
             st = Step(self.x[sl], self.xe[sl], self.qpos[sl], self.xp, slot=self.slot[sl])
             self._layers(st, self.h[sl])
             if self.packed:
@@ -170,8 +239,8 @@ class StackEngine(DecodeEngine):
         meta = torch.tensor(cu + list(slots) + list(starts) + seq + pos + want, dtype=torch.int32).to(dev)
         cu_d, slot_d, start_d, seq_d, pos_d, want_d = (t.contiguous() for t in meta.split([len(cu), len(lens), len(lens), N, N, len(want)]))
         x = torch.empty(N, m.cols, dtype=torch.float32, device=dev)
-        xe = torch.empty(N, m.cols, dtype=self.dtype, device=dev) if self.packed else x
-        _call("embed_rows", ids, m.embed, x, xe if self.packed else None, None, None, None, None, None, None, 0)
+        xe = torch.empty(N, m.cols, dtype=self.dtype, device=dev) if self.packed or self.normed else x
+        _call("embed_rows", ids, m.embed, x, xe if self.packed and not self.normed else None, None, None, None, None, None, None, 0, m.embed_scale)
         st = Step(x, xe, pos_d, portions=ops.lib().Portions(cu_d, slot_d, start_d, seq_d), starts=list(zip(lens, starts)))
         h = torch.empty(N, m.cols, dtype=self.dtype, device=dev)
         self._layers(st, h, trace)

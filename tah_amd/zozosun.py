@@ -14,7 +14,7 @@ from typing import Dict, List, Optional
 import torch
 
 from ._capi import TahDuoError
-from .mixers import DeltaMixer, DeltaSpec, DenseMlp, LatentAttention, LatentSpec, MoeMlp, pad_to, padded
+from .mixers import DeltaMixer, DeltaSpec, DenseMlp, LatentAttention, LatentSpec, MoeMlp, Router, pad_to, padded
 from .stack import StackEngine, StackLayer, StackModel, make_head, norm_coef
 
 NAME = "Zozosun"
@@ -64,7 +64,7 @@ def load(config: dict, tensors: Dict[str, torch.Tensor], device, dtype: torch.dt
         n, top = spec["router"]["experts"], spec["router"]["top"]
         w = {k: torch.stack([mat(f"{pre}e{e}.{k}") for e in range(n)]) for k in ("gate", "up", "down")}
         shared = {k: mat(f"{pre}shared.{k}") for k in ("gate", "up", "down", "sg")} if spec.get("shared") else None
-        return MoeMlp(top, dict(w, router=mat(pre + "router")), shared, cols)
+        return MoeMlp(Router(top), dict(w, router=mat(pre + "router")), shared, cols)
 
     layers: List[StackLayer] = []
     for i, layer in enumerate(config["layers"]):

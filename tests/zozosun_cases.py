@@ -59,7 +59,7 @@ def rows_case(dev, dtype, rows=5, width=72, cols=96, top=3, experts=4, seed=1):
     pos, fin = i32(list(range(3, 3 + rows)), dev), torch.tensor([i % 3 == 1 for i in range(rows)]).to(dev)
     x, xe, xp = z(rows, cols, dt=torch.float32), z(rows, cols), (z(32 * cols) if packed else None)
     slot, qpos, act = i32([9] * rows, dev), i32([9] * rows, dev), z(rows, dt=torch.bool)
-    _call("embed_rows", tok, embed, x, xe, xp, pos, fin, slot, qpos, act, 7)
+    _call("embed_rows", tok, embed, x, xe, xp, pos, fin, slot, qpos, act, 7, 1.0)
     assert torch.equal(x, embed[tok].float()) and torch.equal(xe, embed[tok])
     if packed:
         assert torch.equal(unpack_rows(xp.cpu(), cols)[:rows], xe.cpu())
@@ -87,7 +87,7 @@ def rows_case(dev, dtype, rows=5, width=72, cols=96, top=3, experts=4, seed=1):
         experts_on = use in ("experts", "both")
         _call("residual_norm", xd, coef.to(dev), width, eps, y.to(dev) if use != "experts" else None,
               ys.to(dev) if use in ("y_scaled", "both") else None, ex.to(dev) if experts_on else None,
-              idx.to(torch.int32).to(dev) if experts_on else None, wt.to(dev) if experts_on else None, xe, xp, fcoef.to(dev), nrm, nrmp, rows, 1)
+              idx.to(torch.int32).to(dev) if experts_on else None, wt.to(dev) if experts_on else None, xe, xp, fcoef.to(dev), nrm, nrmp, rows, 1, 1, cols, None, None, None)
         close(xd, want, torch.float32, f"residual {use}")
         assert torch.equal(xe, xd.to(dtype))
         wn = torch.zeros_like(want)
@@ -96,8 +96,8 @@ def rows_case(dev, dtype, rows=5, width=72, cols=96, top=3, experts=4, seed=1):
         if packed:
             assert torch.equal(unpack_rows(xp.cpu(), cols)[:rows], xe.cpu()) and torch.equal(unpack_rows(nrmp.cpu(), cols)[:rows], nrm.cpu())
     a = (2 * rnd(g, rows, 2 * cols)).to(dtype)
-    close(_call("activate_rows", a.to(dev), 0, None), R.gelu_tanh(a.double()), dtype, "gelu")
-    close(_call("activate_rows", a.to(dev), 1, None), R.silu(a.double()[:, :cols]) * a.double()[:, cols:], dtype, "silu * up")
+    close(_call("activate_rows", a.to(dev), 0, None, 0.0, 0.0), R.gelu_tanh(a.double()), dtype, "gelu")
+    close(_call("activate_rows", a.to(dev), 1, None, 0.0, 0.0), R.silu(a.double()[:, :cols]) * a.double()[:, cols:], dtype, "silu * up")
 
 
 def linear_batch_case(dev, rows, n, k, batch, seed=2):
@@ -313,7 +313,7 @@ def latent_case(dev, dtype, m, total, cuts, steps, capacity=None, slots=3, stand
 
 # ── mixture of experts ───────────────────────────────────────────────────────────────────────────────────────────────
 def moe_case(dev, dtype, rows, width, ff, experts, top, shared_ff, seed=5):
-    from tah_amd.mixers import MoeMlp, Step, pad_to
+    from tah_amd.mixers import MoeMlp, Router, Step, pad_to
 
     class Engine:
         packed = dtype == BF
@@ -336,7 +336,7 @@ def moe_case(dev, dtype, rows, width, ff, experts, top, shared_ff, seed=5):
         flat.update({"shared." + k: t.double() for k, t in sh.items()})
     want = R.moe_mlp(x.double(), flat, {"router": {"top": top}, "shared": sh})
     d = lambda t: {k: v.to(dev) for k, v in t.items()} if t else None
-    b = MoeMlp(top, d(w), d(sh), cols).bind(Engine)
+    b = MoeMlp(Router(top), d(w), d(sh), cols).bind(Engine)
     idx, _ = R.route(x.double(), w["router"].double(), top)
     pos = i32([0] * rows, dev)
 
