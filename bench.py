@@ -750,24 +750,46 @@ def stack_config(layers: int = 12, width: int = 2048, vocab: int = 151936):
     return {"architecture": "Zozosun", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out}
 
 
-def bench_stack(steps: int, warmup: int, layers: int = 12):
-    """Prefill and decode throughput of a Zozosun model at the layer sizes of a real one (random weights), beside the Qwen3
-    engine with as many layers of the same width and vocabulary (no token takes a second iteration there)."""
+def zedudra_config(layers: int = 12, width: int = 2048, vocab: int = 151936):
+    """A Zedudra model with the layer sizes of a few-billion-parameter model, every second feed-forward a mixture of 64
+    experts."""
+    mixer = {"heads": 16, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "rot": {"base": 1e6, "dims": 64},
+             "mask": {"size": 1024, "keep_first": 4}}
+    dense = {"kind": "dense", "ff": 6144}
+    moe = {"kind": "moe", "router": {"experts": 64, "top": 8, "groups": {"count": 8, "keep": 4}}, "expert": {"ff": 768, "limit": 7.0}}
+    return {"architecture": "Zedudra", "width": width, "vocab": vocab, "norm": {"eps": 1e-6, "groups": 8}, "canon": {"taps": 4},
+            "embedding": {"scale": width ** 0.5},
+            "layers": [{"type": "attention", "mixer": dict(mixer), "mlp": moe if i % 2 else dense} for i in range(layers)]}
+
+
+STACK_WORKLOADS = {
+    "zozosun": "gated delta rule (32 heads of 128 x 128, convolutions of 4) in three of four layers, latent attention (16 heads, 128 + 64, "
+               "rank 512, window 1024) in the fourth, feed-forward 6144 or 64 experts of 768 (8 per token) and a shared one",
+    "zedudra": "attention in a window of 1024 and 4 kept tokens (16 / 8 heads of 128, keys as values, 64 dimensions rotated), input "
+               "convolutions of 4, norms over 8 groups, feed-forward 6144 or 64 experts of 768 (8 per token from 4 of 8 groups)",
+}
+
+
+def bench_stack(steps: int, warmup: int, layers: int = 12, design: str = "zozosun"):
+    """Prefill and decode throughput of a layer-by-layer model at the layer sizes of a real one (random weights), beside the
+    Qwen3 engine with as many layers of the same width and vocabulary (no token takes a second iteration there)."""
+    import importlib
+
     import torch
 
-    from tah_amd import zozosun
     from tah_amd.engine import EngineConfig, TaHDecodeEngine, Weights
 
-    cfg = stack_config(layers)
-    model = zozosun.load(cfg, zozosun.random_tensors(cfg, "cuda", seed=1), "cuda")
+    arch = importlib.import_module(f"tah_amd.{design}")
+    cfg = {"zozosun": stack_config, "zedudra": zedudra_config}[design](layers)
+    model = arch.load(cfg, arch.random_tensors(cfg, "cuda", seed=1), "cuda")
     w = Weights.random_init(EngineConfig(layers=layers), "cuda", seed=1239)
     w.threshold = 2.0  # above every probability: one iteration per token
     g = torch.Generator().manual_seed(5)
     yield
 
     def build(kind, B, length):
-        if kind == "zozosun":
-            return zozosun.engine(model, B, length)
+        if kind == design:
+            return arch.engine(model, B, length)
         return TaHDecodeEngine(w, B, length, max_hard=512)
 
     def timed(f, n):
@@ -780,10 +802,9 @@ def bench_stack(steps: int, warmup: int, layers: int = 12):
         torch.cuda.synchronize()
         return (time.perf_counter() - t0) / n
 
-    out = {"workload": f"{layers} layers, width 2048, vocab 151936, bf16, random weights; zozosun: gated delta rule (32 heads of 128 x 128, "
-                       "convolutions of 4) in three of four layers, latent attention (16 heads, 128 + 64, rank 512, window 1024) in the fourth, "
-                       "feed-forward 6144 or 64 experts of 768 (8 per token) and a shared one; qwen3: 16 / 8 heads of 128, feed-forward 6144"}
-    for kind in ("zozosun", "qwen3"):
+    out = {"workload": f"{layers} layers, width 2048, vocab 151936, bf16, random weights; {design}: {STACK_WORKLOADS[design]}; "
+                       "qwen3: 16 / 8 heads of 128, feed-forward 6144"}
+    for kind in (design, "qwen3"):
         res = out[kind] = {}
         for B, T in STACK_SIZES["prefill"]:
             eng = build(kind, B, T)
@@ -822,9 +843,10 @@ def main() -> int:
     ap.add_argument("--spinup", type=int, default=200,
                     help="untimed launches of the headline kernel before its warm-up steps (the GPU's clock needs tens of "
                          "milliseconds of work to leave its idle state)")
-    ap.add_argument("--only", choices=["all", "fwd", "decode", "fwd_bwd", "host_layer", "context", "qk_prep", "topk_mix", "sample_rows", "e2e", "stack"], default="all",
-                    help="run only one leg (the JSON line then lacks the other legs); stack: prefill and decode of a Zozosun model "
-                         "beside the Qwen3 engine, not part of all")
+    ap.add_argument("--only", choices=["all", "fwd", "decode", "fwd_bwd", "host_layer", "context", "qk_prep", "topk_mix", "sample_rows", "e2e", "stack", "zedudra"],
+                    default="all",
+                    help="run only one leg (the JSON line then lacks the other legs); stack, zedudra: prefill and decode of a Zozosun or "
+                         "Zedudra model beside the Qwen3 engine, not part of all")
     ap.add_argument("--calib-copy", action="store_true",
                     help="profiling aid: also run one plain 256 MiB device copy (known traffic for counter scaling)")
     args = ap.parse_args()
@@ -880,8 +902,8 @@ def main() -> int:
         legs.append(("sample_rows", bench_sample_rows(args.steps, args.warmup)))
     if args.only in ("all", "e2e"):
         legs.append(("e2e_decode", bench_e2e_decode(args.e2e_tokens, temperature=args.e2e_temperature, top_k=args.e2e_top_k)))
-    if args.only == "stack":
-        legs.append(("stack", bench_stack(args.steps, args.warmup)))
+    if args.only in ("stack", "zedudra"):
+        legs.append((args.only, bench_stack(args.steps, args.warmup, design="zozosun" if args.only == "stack" else "zedudra")))
     for _, leg in legs:
         next(leg)  # runs the leg up to its `yield`: inputs built and resident
     sched = launch_order(ops, dev)

@@ -5,6 +5,8 @@
 
 namespace tah {
 
+typedef __attribute__((__vector_size__(8 * sizeof(float)))) float f32x8;
+
 // Eight elements of a row as float32.
 __device__ __forceinline__ void load8(const __bf16* p, float (&v)[8]) {
     const bf16x8 x = *reinterpret_cast<const bf16x8*>(p);
@@ -84,11 +86,39 @@ __device__ __forceinline__ float clamped_gate_exact(float g, float u, float limi
 }
 
 // ---- attention on the matrix cores ----
+// Which of a SIMD's waves is served first from here on (within the kernel)
+#ifdef TAH_CPU_EMU
+#define TAH_WAVE_PRIORITY(n)
+#else
+#define TAH_WAVE_PRIORITY(n) __builtin_amdgcn_s_setprio(n)
+#endif
 constexpr float kNoScore = -1e30f;  // below every score, and finite: differences of it are numbers
 
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 __device__ __forceinline__ bf16x8 join8(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
 __device__ __forceinline__ bf16x4 to_bf16x4(const float (&w)[4]) { return __builtin_convertvector((f32x4{w[0], w[1], w[2], w[3]}), bf16x4); }
+// Eight numbers as two bf16 terms each, the leading bits and what they leave: sixteen bits of them together.
+__device__ __forceinline__ void split_bf16x8(const float (&w)[8], bf16x8& hi, bf16x8& lo) {
+    uint32_t h[4];
+    float rest[8];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const uint32_t a = __float_as_uint(w[2 * i]), b = __float_as_uint(w[2 * i + 1]) & 0xffff0000u;
+        h[i] = (a >> 16) | b;
+        rest[2 * i] = w[2 * i] - __uint_as_float(a & 0xffff0000u);
+        rest[2 * i + 1] = w[2 * i + 1] - __uint_as_float(b);
+    }
+    __builtin_memcpy(&hi, h, 16);
+    lo = __builtin_convertvector((f32x8{rest[0], rest[1], rest[2], rest[3], rest[4], rest[5], rest[6], rest[7]}), bf16x8);
+}
+// The larger of two scores (finite or -inf), in one instruction: fmaxf has to quieten NaNs of operands it knows nothing about.
+__device__ __forceinline__ float score_max(float a, float b) {
+#ifdef TAH_CPU_EMU
+    return fmaxf(a, b);
+#else
+    return __builtin_amdgcn_fmed3f(a, b, 3.0e38f);
+#endif
+}
 // x over the four lane groups that share l % 16
 __device__ __forceinline__ float groups_max(float x) {
     x = fmaxf(x, __shfl_xor(x, 16));

@@ -35,8 +35,8 @@ __global__ __launch_bounds__(kRowThreads) void embed_rows_kernel(const tah_embed
 }
 
 // Sum of a row's values over its group, one partial sum s[u] per thread and unit, for each of the thread's units.
-// GROUPS: several groups of group_units units each; `unit_sums` is LDS of as many floats as the row has units, `red` of
-// a float per wave and (GROUPS) per group.
+// GROUPS: several groups of group_units units each, added up inside a wave where the groups divide it; else through LDS:
+// `unit_sums` of as many floats as the row has units, `group_sum` of as many as it has groups.  `red`: a float per wave.
 template <int U, bool GROUPS>
 __device__ __forceinline__ void group_sums(float (&s)[U], int units, int groups, int group_units, float* red, float* unit_sums, float* group_sum) {
     const int tid = threadIdx.x;
@@ -47,6 +47,11 @@ __device__ __forceinline__ void group_sums(float (&s)[U], int units, int groups,
         t = block_sum<kRowThreads / kWave>(t, red);
 #pragma unroll
         for (int u = 0; u < U; ++u) s[u] = t;
+    } else if (group_units <= kWave && (group_units & (group_units - 1)) == 0) {
+        for (int d = group_units / 2; d >= 1; d >>= 1) {
+#pragma unroll
+            for (int u = 0; u < U; ++u) s[u] += __shfl_xor(s[u], d);
+        }
     } else {
 #pragma unroll
         for (int u = 0; u < U; ++u)
@@ -218,6 +223,59 @@ __global__ __launch_bounds__(kWave) void conv_rows_kernel(const E* h, const floa
     }
 }
 
+// The same for up to four taps: a thread asks for all of its rows, and the inputs in front of them, before it uses the first.
+constexpr int kFewTaps = 4, kFewRows = 16;
+
+template <class E>
+__global__ __launch_bounds__(kWave) void conv_few_rows_kernel(const E* h, const float* conv, E* state, const tah_portions P, E* out, int cols, int taps,
+                                                              int nslots) {
+    int tile = blockIdx.y, b = 0, row0 = 0, row_end = 0;
+    if (!find_tile(P.cu, P.nseq, kFewRows, tile, b, row0, row_end)) return;
+    const int c = 8 * (blockIdx.x * kWave + threadIdx.x);
+    if (c >= cols) return;
+    const int first = P.cu[b], last = P.cu[b + 1], slot = P.slot[b], pos0 = P.pos0[b];
+    const bool live = slot >= 0 && slot < nslots;
+    E* const ring = state + (int64_t)(live ? slot : 0) * taps * cols + c;
+    constexpr int kFront = kFewTaps - 1;
+    E v[kFront + kFewRows][8];  // row row0 - kFront + i; rows nobody reads repeat one that is there
+    bool there[kFront];
+#pragma unroll
+    for (int i = 0; i < kFront; ++i) {
+        const int at = row0 - kFront + i, pos = pos0 + at - first;
+        there[i] = at >= first || (live && pos >= 0 && kFront - i < taps);
+        const E* const src = at >= first || !there[i] ? h + (int64_t)(at >= first ? at : row0) * cols + c : ring + (int64_t)(pos % taps) * cols;
+        __builtin_memcpy(v[i], src, sizeof(v[i]));
+    }
+#pragma unroll
+    for (int i = 0; i < kFewRows; ++i) __builtin_memcpy(v[kFront + i], h + (int64_t)(row0 + i < row_end ? row0 + i : row0) * cols + c, sizeof(v[i]));
+    float w[kFewTaps][8];  // of the input d rows back
+#pragma unroll
+    for (int d = 0; d < kFewTaps; ++d) {
+        load8(conv + (int64_t)(d < taps ? taps - 1 - d : 0) * cols + c, w[d]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) w[d][e] = d < taps ? w[d][e] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < kFewRows; ++i) {
+        float y[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) y[e] = (float)v[kFront + i][e] + w[0][e] * (float)v[kFront + i][e];
+#pragma unroll
+        for (int d = 1; d < kFewTaps; ++d) {
+            const bool on = kFront + i - d >= kFront || there[kFront + i - d < kFront ? kFront + i - d : 0];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) y[e] += on ? w[d][e] * (float)v[kFront + i - d][e] : 0.f;
+        }
+        if (row0 + i < row_end) store8(out + (int64_t)(row0 + i) * cols + c, y);
+    }
+    if (row0 != first || !live) return;
+    for (int r = last - taps + 1 > first ? last - taps + 1 : first; r < last; ++r) {
+        float x[8];
+        load8(h + (int64_t)r * cols + c, x);
+        store8(ring + (int64_t)((pos0 + r - first) % taps) * cols, x);
+    }
+}
+
 template <class E, int KIND>
 __global__ __launch_bounds__(kRowThreads) void activate_rows_kernel(const E* in, int64_t in_rs, E* out, int64_t out_rs, int cols, float c0, float c1) {
     const int row = blockIdx.y;
@@ -251,9 +309,10 @@ void launch_residual(const tah_residual_norm_args& p, hipStream_t st) {
 
 template <class E>
 void launch_conv(const void* h, const float* conv, void* state, const tah_portions& p, void* out, int cols, int taps, int nslots, hipStream_t st) {
-    const dim3 grid((cols / 8 + kWave - 1) / kWave, p.rows / kConvRows + p.nseq);
-    hipLaunchKernelGGL((conv_rows_kernel<E>), grid, dim3(kWave), 0, st, static_cast<const E*>(h), conv, static_cast<E*>(state), p, static_cast<E*>(out), cols,
-                       taps, nslots);
+    const bool few = taps <= kFewTaps;
+    const dim3 grid((cols / 8 + kWave - 1) / kWave, p.rows / (few ? kFewRows : kConvRows) + p.nseq);
+    auto* const f = few ? &conv_few_rows_kernel<E> : &conv_rows_kernel<E>;
+    hipLaunchKernelGGL(f, grid, dim3(kWave), 0, st, static_cast<const E*>(h), conv, static_cast<E*>(state), p, static_cast<E*>(out), cols, taps, nslots);
 }
 
 template <class E>
@@ -322,7 +381,7 @@ extern "C" int tah_conv_rows(const void* h, const float* conv, void* conv_state,
     using namespace tah;
     if (!p) return TAH_E_NULL;
     if (p->rows < 0 || p->nseq < 0 || cols <= 0 || cols % 8 != 0 || taps <= 0 || taps - 1 > kConvRows || nslots <= 0 || !dtype_ok(dtype) ||
-        p->rows / kConvRows + p->nseq > 65535)
+        p->rows / kFewRows + p->nseq > 65535)
         return TAH_E_SHAPE;
     if (p->rows == 0 || p->nseq == 0) return TAH_OK;
     if (!h || !conv || !conv_state || !out || !p->cu || !p->slot || !p->pos0) return TAH_E_NULL;

@@ -4,7 +4,7 @@
 // than either.  A slot keeps its first tokens and a ring as long as the window.
 //
 //  * window_prep_kernel: rotates queries and keys of a step's rows in place (and enters single tokens into the cache).
-//  * window_tile_kernel (bf16): portions.  Eight waves, 16 queries x 2 each, of all query heads of one key/value head, so that
+//  * window_tile_kernel (bf16): portions.  Four waves, 16 queries x 2 each, of all query heads of one key/value head, so that
 //    one pass over its keys (64 rows at a time, in LDS once for keys and values) serves them all; S^T = K Q^T and O^T =
 //    V^T P^T, V^T read from the row-major tile by transpose reads.  Keys before the portion come from the cache, its own
 //    from the projections; tiles outside the window and behind the kept tokens are not visited.
@@ -191,23 +191,28 @@ __global__ __launch_bounds__(kWinThreads) void window_rows_kernel(const WindowCa
 
 // ---- portions on the matrix cores --------------------------------------------------------------------------------
 constexpr int kTileKeys = 64;
-constexpr int kTileWaves = 8;
+constexpr int kTileWaves = 4;  // (two workgroups of four run better side by side than one of eight: their barriers differ)
 constexpr int kTileThreads = kTileWaves * kWave;
 constexpr int kTileQueries = 2 * kTileWaves;  // tiles of 16 queries of one head
+constexpr int kTileRows = 8 * kTileKeys / kTileThreads;  // rows of a key tile per thread, eight threads to a row
 
-// Row stride of a tile in LDS: an odd multiple of 16 elements, so that rows lie 8 banks apart in a different order of eights
+// Row stride of a tile in LDS: an odd multiple of 16 elements, so that eight rows' same sixteen elements lie in different
+// banks; the sixteen-byte units of a pair change places in every other eight rows, so that one unit of sixteen rows does too.
 __device__ __host__ __forceinline__ int tile_stride(int row) { return (row + 15) / 32 * 32 + 16; }
+__device__ __forceinline__ int tile_unit(int row, int stride, int unit) { return row * stride + 8 * (unit ^ ((row >> 3) & 1)); }
+
+constexpr float kSlack = 8.0f;  // in powers of two
 
 struct WindowTile {
     WindowCall c;
-    int32_t slots, per_xcd, chunks, heads_per_tile;  // chunks of at most 16 query heads per key/value head
+    int32_t slots, per_xcd, chunks, heads_per_tile;  // a key/value head's query heads in chunks of so many
     float scale_log2;
 };
 
 // NQ: 32-wide steps of a key (at most), NV: 16-wide tiles of a value row (at most; kExact: just so many), NU: 16-byte units of
-// a key tile per thread (at most).
+// a key tile per thread (at most; eight threads to a row).
 template <int NQ, int NV, int NU, bool kExact>
-__global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowTile p) {
+__global__ __launch_bounds__(kTileThreads) TAH_WAVES_PER_EU(NQ <= 4 ? 2 : 1, 8) void window_tile_kernel(const WindowTile p) {
     HIP_DYNAMIC_SHARED(unsigned char, tile_lds)
     const tah_window_layer& L = p.c.L;
     const tah_window_rows& R = p.c.R;
@@ -257,7 +262,11 @@ __global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowT
     const int keep = L.keep_first, kept = keep < j_lo ? keep : j_lo;  // kept tokens in front of the window's keys
     const RingView view(keep, L.ring, j_lo);
     f32x4 acc[NV][2];
-    float m[2] = {kNoScore, kNoScore}, l[2] = {0.f, 0.f};
+    f32x4 l[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+    float m[2] = {kNoScore, kNoScore};
+    bf16x8 ones;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ones[i] = (__bf16)1.0f;
 #pragma unroll
     for (int i = 0; i < NV; ++i)
 #pragma unroll
@@ -266,15 +275,12 @@ __global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowT
     const __bf16* const mine = proj + R.k_col + g * L.row;
     const __bf16* const cache = static_cast<const __bf16*>(L.cache) +
                                 ((int64_t)(slot < 0 || slot >= L.nslots ? 0 : slot) * L.kv_heads + g) * (keep + L.ring) * L.row;
-    int ukey[NU], ux[NU], udst[NU];
-    bf16x8 f[NU];
-#pragma unroll
-    for (int i = 0; i < NU; ++i) {
-        const int u = tid + kTileThreads * i;
-        ukey[i] = u < kTileKeys * units ? u / units : -1;
-        ux[i] = 8 * (u % units);
-        udst[i] = (u / units) * ks + ux[i];
-    }
+    // operand addresses: of K, row 16 x + c, unit koff / 8 + 4 s + gq; of V^T, rows 16 x + 4 gq + c / 4, elements 16 i + 4 (c % 4)
+    // (koff % 16 == 0: a unit's partner is not in another pair)
+    const int k_at = c * ks + koff + 8 * (gq ^ (c >> 3)), v_at = (4 * gq + c / 4) * ks + 8 * ((c % 4 / 2) ^ (gq >> 1)) + 4 * (c % 2);
+    const int fkey = tid / 8, fu = tid % 8;  // this thread's rows fkey + kTileKeys / kTileRows * r, and units fu, fu + 8, ... of them
+    constexpr int kRowStep = kTileKeys / kTileRows;
+    bf16x8 f[kTileRows][NU];
     // Tiles of keys: those of the kept tokens, [0, kept), then the window's, [j_lo, j_hi], at multiples of 64 positions.  A
     // place outside these repeats the nearest key inside (its score is masked).
     const int kept_tiles = (kept + kTileKeys - 1) / kTileKeys, t_lo = j_lo / kTileKeys, t_hi = j_hi / kTileKeys;
@@ -283,17 +289,21 @@ __global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowT
     auto fetch = [&](int it) __attribute__((always_inline)) {
         const int j0 = first_key(it), lo = it < kept_tiles ? 0 : j_lo, hi = it < kept_tiles ? kept - 1 : j_hi;
 #pragma unroll
-        for (int i = 0; i < NU; ++i) {
-            int j = j0 + ukey[i];
+        for (int r = 0; r < kTileRows; ++r) {
+            int j = j0 + fkey + kRowStep * r;
             j = j < lo ? lo : (j > hi ? hi : j);
-            const __bf16* const src = j >= pos0 ? mine + (int64_t)(j - shift) * R.proj_row_stride : cache + (int64_t)view.row(j) * L.row;
-            if (ukey[i] >= 0) f[i] = *reinterpret_cast<const bf16x8*>(src + ux[i]);
+            const __bf16* const src = (j >= pos0 ? mine + (int64_t)(j - shift) * R.proj_row_stride : cache + (int64_t)view.row(j) * L.row) + 8 * fu;
+#pragma unroll
+            for (int i = 0; i < NU; ++i)
+                if (fu + 8 * i < units) f[r][i] = *reinterpret_cast<const bf16x8*>(src + 64 * i);
         }
     };
     auto store = [&](int at) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < NU; ++i)
-            if (ukey[i] >= 0) *reinterpret_cast<bf16x8*>(kt + at + udst[i]) = f[i];
+        for (int r = 0; r < kTileRows; ++r)
+#pragma unroll
+            for (int i = 0; i < NU; ++i)
+                if (fu + 8 * i < units) *reinterpret_cast<bf16x8*>(kt + at + tile_unit(fkey + kRowStep * r, ks, fu + 8 * i)) = f[r][i];
     };
     fetch(0);
     store(0);
@@ -309,64 +319,72 @@ __global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowT
         if (any) {
             f32x4 sc[4][2];
 #pragma unroll
-            for (int x = 0; x < 4; ++x) {
+            for (int x = 0; x < 4; ++x)
 #pragma unroll
                 for (int t = 0; t < 2; ++t) sc[x][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+            TAH_WAVE_PRIORITY(1);  // (a wave in a run of products goes before one in its softmax: the two then alternate)
 #pragma unroll
-                for (int s = 0; s < NQ; ++s)
-                    if (kExact || s < nq) {
-                        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + now + (16 * x + c) * ks + koff + 32 * s + 8 * gq);
+            for (int s = 0; s < NQ; ++s) {
+                if (kExact || s < nq) {
+#pragma unroll
+                    for (int x = 0; x < 4; ++x) {
+                        const bf16x8 a = *reinterpret_cast<const bf16x8*>(kt + now + k_at + 16 * x * ks + 32 * s);
 #pragma unroll
                         for (int t = 0; t < 2; ++t) sc[x][t] = mfma16(a, q[t][s], sc[x][t]);
                     }
+                }
             }
+            TAH_WAVE_PRIORITY(0);
             bf16x8 ph[2][2], pl[2][2];  // [pair of key tiles][query tile]
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
                 if (!all) {
                     // kept tokens' tiles end at `kept` (what follows comes again with the window's tiles)
-                    const int lo = own[t] - L.window, hi = window_tile ? own[t] : kept - 1, from = window_tile ? keep : kept;
-                    const int start = window_tile ? j_lo : 0;
+                    // (as distances from this lane's first key)
+                    const int base = j0 + 4 * gq, lo = own[t] - L.window - base, hi = (window_tile ? own[t] : kept - 1) - base;
+                    const int from = (window_tile ? keep : kept) - base, start = (window_tile ? j_lo : 0) - base;
 #pragma unroll
                     for (int x = 0; x < 4; ++x)
 #pragma unroll
                         for (int r = 0; r < 4; ++r) {
-                            const int j = j0 + 16 * x + 4 * gq + r;
-                            if (j > hi || (j <= lo && j >= from) || j < start) sc[x][t][r] = kNegInf;
+                            const int j = 16 * x + r;
+                            const bool off = (j > hi) | ((j <= lo) & (j >= from)) | (j < start);
+                            sc[x][t][r] = off ? kNegInf : sc[x][t][r];
                         }
                 }
                 // (maximum before the scale, which is positive; scale and difference are one multiply-add)
-                float mx = fmaxf(fmaxf(sc[0][t][0], sc[0][t][1]), fmaxf(sc[0][t][2], sc[0][t][3]));
+                float mx = score_max(sc[0][t][0], sc[0][t][1]);
 #pragma unroll
-                for (int x = 1; x < 4; ++x) mx = fmaxf(mx, fmaxf(fmaxf(sc[x][t][0], sc[x][t][1]), fmaxf(sc[x][t][2], sc[x][t][3])));
+                for (int e = 2; e < 16; ++e) mx = score_max(mx, sc[e / 4][t][e % 4]);
+                // The weights are taken against a running reference, not the maximum itself: it moves only when a score of the wave
+                // passes it by kSlack, so that most tiles leave the sums alone; weights stay below 2^kSlack.
                 mx = fmaxf(m[t], groups_max(mx) * p.scale_log2);
-                const float a = fast_exp2(m[t] - mx);
-                m[t] = mx;
-                float sum = 0.f;
-#pragma unroll
-                for (int x = 0; x < 4; ++x) {
-                    float w[4];
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        w[r] = fast_exp2(__builtin_fmaf(sc[x][t][r], p.scale_log2, -mx));
-                        sum += w[r];
-                    }
-                    const bf16x4 hi = to_bf16x4(w);
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) w[r] -= (float)hi[r];
-                    const bf16x4 lo = to_bf16x4(w);
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        ph[x / 2][t][4 * (x % 2) + r] = hi[r];
-                        pl[x / 2][t][4 * (x % 2) + r] = lo[r];
-                    }
-                }
-                l[t] = l[t] * a + sum;
-                if (__ballot(a != 1.0f) != 0) {
+                if (__ballot(mx > m[t] + kSlack) != 0) {
+                    const float a = fast_exp2(m[t] - mx);
+                    m[t] = mx;
 #pragma unroll
                     for (int i = 0; i < NV; ++i)
 #pragma unroll
                         for (int r = 0; r < 4; ++r) acc[i][t][r] *= a;
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) l[t][r] *= a;
+                }
+#pragma unroll
+                for (int x = 0; x < 2; ++x) {
+                    float w[8];
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) w[e] = fast_exp2(__builtin_fmaf(sc[2 * x + e / 4][t][e % 4], p.scale_log2, -m[t]));
+                    split_bf16x8(w, ph[x][t], pl[x][t]);
+                }
+            }
+            TAH_WAVE_PRIORITY(1);
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                // the weights' sums, all keys of the tile at once, in every row of the result
+#pragma unroll
+                for (int x = 0; x < 2; ++x) {
+                    l[t] = mfma16(ones, ph[x][t], l[t]);
+                    l[t] = mfma16(ones, pl[x][t], l[t]);
                 }
             }
 #pragma unroll
@@ -374,22 +392,22 @@ __global__ __launch_bounds__(kTileThreads) void window_tile_kernel(const WindowT
                 if (kExact || i < nv) {
 #pragma unroll
                     for (int x = 0; x < 2; ++x) {
-                        const __bf16* at = kt + now + (32 * x + 4 * gq + c / 4) * ks + 16 * i + 4 * (c % 4);
+                        const __bf16* at = kt + now + v_at + 32 * x * ks + 16 * i;
                         const bf16x8 a = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
                                                lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * ks)));
 #pragma unroll
-                        for (int t = 0; t < 2; ++t) {
-                            acc[i][t] = mfma16(a, ph[x][t], acc[i][t]);
-                            acc[i][t] = mfma16(a, pl[x][t], acc[i][t]);
-                        }
+                        for (int t = 0; t < 2; ++t) acc[i][t] = mfma16(a, ph[x][t], acc[i][t]);
+#pragma unroll
+                        for (int t = 0; t < 2; ++t) acc[i][t] = mfma16(a, pl[x][t], acc[i][t]);
                     }
                 }
+            TAH_WAVE_PRIORITY(0);
         }
         if (more) store(buffer - now);
     }
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
-        float inv = 1.0f / groups_sum(l[t]);
+        float inv = 1.0f / l[t][0];
         if (on[t]) {
             if (R.g_col >= 0) inv *= sigmoid_exact((float)proj[(int64_t)qrow[t] * R.proj_row_stride + R.g_col + head[t]]);
             __bf16* const out = static_cast<__bf16*>(p.c.out) + (int64_t)qrow[t] * p.c.out_rs + (int64_t)head[t] * L.value_dim + 4 * gq;
@@ -418,8 +436,8 @@ struct WindowDecode {
     float scale_log2;
 };
 
-// grid (splits, kv_heads * chunks of 16 query heads, rows).  NQ, NV as above; NU: 16-byte units of 32 rows per lane (at most);
-// W: waves.  LDS: W tiles of 32 rows (later the waves' results), 16 queries, a rotated key.
+// grid (splits, kv_heads * chunks of 16 query heads, rows).  NQ, NV as above; NU: 16-byte units of a row per lane (at most; eight
+// lanes to a row, four rows a lane); W: waves.  LDS: W tiles of 32 rows (later the waves' results), 16 queries, a rotated key.
 template <int NQ, int NV, int NU, int W, bool kExact>
 __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDecode p) {
     HIP_DYNAMIC_SHARED(unsigned char, dec_lds)
@@ -449,25 +467,23 @@ __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDe
     const int kept = L.keep_first < lo ? L.keep_first : lo, nk = live ? kept + pos - lo + 1 : 0;  // kept first tokens, then the window
     const int begin = blockIdx.x * p.keys_per_split;
     const int end = begin + p.keys_per_split < nk ? begin + p.keys_per_split : nk;
-    int ukey[NU], ux[NU];
-    bf16x8 f[NU];
+    const int fkey = lane / 8, fu = lane % 8;  // this lane's rows fkey + 8 r, and units fu, fu + 8, ... of them
+    bf16x8 fa[4][NU], fb[4][NU];
+    auto fetch = [&](int x0, bf16x8 (&f)[4][NU]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < NU; ++i) {
-        const int u = lane + kWave * i;
-        ukey[i] = u < kDecKeys * units ? u / units : -1;
-        ux[i] = 8 * (u % units);
-    }
-    auto fetch = [&](int x0) __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < NU; ++i) {
-            int x = x0 + ukey[i];
+        for (int r = 0; r < 4; ++r) {
+            int x = x0 + fkey + 8 * r;
             x = x < nk ? x : nk - 1;
-            const __bf16* const src = x == nk - 1 ? fresh : cache + (int64_t)view.row(x < kept ? x : lo + x - kept) * L.row;
-            if (ukey[i] >= 0) f[i] = *reinterpret_cast<const bf16x8*>(src + ux[i]);
+            const __bf16* const src = (x == nk - 1 ? fresh : cache + view.row(x < kept ? x : lo + x - kept) * L.row) + 8 * fu;
+#pragma unroll
+            for (int i = 0; i < NU; ++i)
+                if (fu + 8 * i < units) f[r][i] = *reinterpret_cast<const bf16x8*>(src + 64 * i);
         }
     };
+    constexpr int kPass = W * kDecKeys, kAhead = NQ <= 4 ? 2 : 1;  // passes whose rows are under way at a time
     int x0 = begin + wave * kDecKeys;
-    if (x0 < end) fetch(x0);
+    if (x0 < end) fetch(x0, fa);
+    if (kAhead > 1 && x0 + kPass < end) fetch(x0 + kPass, fb);
     // queries (heads past the last one repeat it; nobody reads them) and the new key's rotated part
     const int half = L.rot_dim / 2, tpos = pos < R.table_rows ? pos : R.table_rows - 1, rot0 = L.key_dim - L.rot_pad;
     const float* const co = R.cos + (int64_t)tpos * half;
@@ -500,19 +516,23 @@ __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDe
 #pragma unroll
     for (int i = 0; i < NV; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = kNoScore, l = 0.f;
-    for (; x0 < end; x0 += W * kDecKeys) {
+    auto step = [&](bf16x8 (&f)[4][NU]) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < NU; ++i)
-            if (ukey[i] >= 0) {
-                const int x = x0 + ukey[i];
-                if (x >= nk - 1) {  // the new token: its rotated part, and its place in the cache
-                    if (ux[i] >= L.row - L.rot_pad) f[i] = *reinterpret_cast<const bf16x8*>(kr + ux[i] - (L.row - L.rot_pad));
-                    if (x == nk - 1 && chunk == 0) *reinterpret_cast<bf16x8*>(cache + (int64_t)view.row(pos) * L.row + ux[i]) = f[i];
+        for (int r = 0; r < 4; ++r) {
+            const int key = fkey + 8 * r, x = x0 + key;
+#pragma unroll
+            for (int i = 0; i < NU; ++i)
+                if (fu + 8 * i < units) {
+                    const int at = 8 * (fu + 8 * i);
+                    if (x >= nk - 1) {  // the new token: its rotated part, and its place in the cache
+                        if (at >= L.row - L.rot_pad) f[r][i] = *reinterpret_cast<const bf16x8*>(kr + at - (L.row - L.rot_pad));
+                        if (x == nk - 1 && chunk == 0) *reinterpret_cast<bf16x8*>(cache + view.row(pos) * L.row + at) = f[r][i];
+                    }
+                    *reinterpret_cast<bf16x8*>(kt + tile_unit(key, ks, fu + 8 * i)) = f[r][i];
                 }
-                *reinterpret_cast<bf16x8*>(kt + ukey[i] * ks + ux[i]) = f[i];
-            }
+        }
         TAH_WAVE_LDS_SYNC();
-        if (x0 + W * kDecKeys < end) fetch(x0 + W * kDecKeys);
+        if (x0 + kAhead * kPass < end) fetch(x0 + kAhead * kPass, f);
         // register r of sc[x], lane (c, gq): key 16 x + 4 gq + r, head c
         f32x4 sc[2];
 #pragma unroll
@@ -521,7 +541,7 @@ __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDe
 #pragma unroll
             for (int s = 0; s < NQ; ++s)
                 if (kExact || s < nq)
-                    sc[x] = mfma16(*reinterpret_cast<const bf16x8*>(kt + (16 * x + c) * ks + koff + 32 * s + 8 * gq), q[s], sc[x]);
+                    sc[x] = mfma16(*reinterpret_cast<const bf16x8*>(kt + tile_unit(16 * x + c, ks, koff / 8 + 4 * s + gq)), q[s], sc[x]);
         }
         float mw = kNoScore;
 #pragma unroll
@@ -535,19 +555,17 @@ __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDe
         m = mn;
         l *= a;
         bf16x8 ph, pl;
+        float w[8];
 #pragma unroll
-        for (int x = 0; x < 2; ++x)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const float w = fast_exp2(sc[x][r] - mn);
-                l += w;
-                ph[4 * x + r] = (__bf16)w;
-                pl[4 * x + r] = (__bf16)(w - (float)ph[4 * x + r]);
-            }
+        for (int e = 0; e < 8; ++e) {
+            w[e] = fast_exp2(sc[e / 4][e % 4] - mn);
+            l += w[e];
+        }
+        split_bf16x8(w, ph, pl);
 #pragma unroll
         for (int i = 0; i < NV; ++i)
             if (kExact || i < nv) {
-                const __bf16* const at = kt + (4 * gq + c / 4) * ks + 16 * i + 4 * (c % 4);
+                const __bf16* const at = kt + tile_unit(4 * gq + c / 4, ks, 2 * i + c % 4 / 2) + 4 * (c % 2);
                 const bf16x8 v = join8(lds_read_tr16(reinterpret_cast<const unsigned char*>(at)),
                                        lds_read_tr16(reinterpret_cast<const unsigned char*>(at + 16 * ks)));
 #pragma unroll
@@ -556,6 +574,11 @@ __global__ __launch_bounds__(W * kWave) void window_decode_kernel(const WindowDe
                 acc[i] = mfma16(v, pl, acc[i]);
             }
         TAH_WAVE_LDS_SYNC();  // the tile is read before it is written again
+        x0 += kPass;
+    };
+    while (x0 < end) {
+        step(fa);
+        if (kAhead > 1 && x0 < end) step(fb);
     }
     // the waves' results meet in LDS: [wave][head][value_dim + 4] over the tiles
     l = groups_sum(l);
@@ -646,9 +669,9 @@ int check_layer(const tah_window_layer* L) {
     if (!L) return TAH_E_NULL;
     if (L->heads <= 0 || L->kv_heads <= 0 || L->heads % L->kv_heads != 0 || L->heads > 65535 || L->key_dim <= 0 || L->key_dim % 32 != 0 ||
         L->value_dim <= 0 || L->value_dim % 32 != 0 || L->row % 8 != 0 || L->row < L->key_dim || L->row < L->value_dim ||
-        L->row > L->key_dim + L->value_dim || L->rot_dim < 0 || L->rot_dim % 2 != 0 || L->rot_pad % 8 != 0 || L->rot_pad < L->rot_dim ||
+        L->row > L->key_dim + L->value_dim || (L->row - L->key_dim) % 16 != 0 || L->rot_dim < 0 || L->rot_dim % 2 != 0 || L->rot_pad % 16 != 0 || L->rot_pad < L->rot_dim ||
         L->rot_pad > L->key_dim || L->rot_source < 0 || L->rot_source % 8 != 0 || L->rot_source + L->rot_pad > L->row || L->keep_first < 0 ||
-        L->ring <= 0 || L->window <= 0 || L->window > L->ring || L->nslots <= 0 || (L->dtype != TAH_DT_BF16 && L->dtype != TAH_DT_F32))
+        L->ring <= 0 || (int64_t)(L->keep_first + (int64_t)L->ring) * L->row >= (1 << 30) || L->window <= 0 || L->window > L->ring || L->nslots <= 0 || (L->dtype != TAH_DT_BF16 && L->dtype != TAH_DT_F32))
         return TAH_E_SHAPE;
     if (L->key_dim > 8192 || L->value_dim > kWinThreads * kRowValues) return TAH_E_SHAPE;
     if (!L->cache) return TAH_E_NULL;
@@ -693,8 +716,8 @@ int launch_tile(WindowTile t, hipStream_t st) {
     const void* const f = reinterpret_cast<const void*>(&window_tile_kernel<NQ, NV, NU, kExact>);
     if (lds > 65536 && hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return TAH_E_LAUNCH;
     const int per = t.c.L.heads / t.c.L.kv_heads;
-    t.heads_per_tile = per < 16 ? per : 16;
-    t.chunks = (per + 15) / 16;
+    t.chunks = (per + kTileQueries - 1) / kTileQueries;
+    t.heads_per_tile = (per + t.chunks - 1) / t.chunks;
     t.slots = t.c.P.rows / (16 * (kTileQueries / t.heads_per_tile)) + t.c.P.nseq;
     const int64_t items = (int64_t)t.slots * t.c.L.kv_heads * t.chunks;
     if (items > (1 << 28)) return TAH_E_SHAPE;
@@ -705,7 +728,7 @@ int launch_tile(WindowTile t, hipStream_t st) {
 
 // how a decode call splits its keys: enough workgroups for the chip, and work for every wave of one
 constexpr int kDecodeGroups = 256;
-int decode_waves(int row) { return row <= 272 ? 8 : 4; }
+int decode_waves(int row) { return row <= 256 ? 8 : 4; }
 void decode_split(const tah_window_layer& L, int rows, int& splits, int& keys_per_split) {
     const int pass = kDecKeys * decode_waves(L.row), keys = L.keep_first + L.window;
     const int most = (keys + pass - 1) / pass, groups = rows * L.kv_heads * ((L.heads / L.kv_heads + 15) / 16);
@@ -755,7 +778,7 @@ extern "C" int tah_window_attend(const tah_window_layer* L, const tah_portions* 
         WindowTile t{};
         t.c = c;
         t.scale_log2 = L->scale * kLog2e;
-        // (units per thread: row / 64, rounded up; rows are at most key_dim + value_dim)
+        // (units per thread: row / 64, rounded up; rows are at most key_dim + value_dim elements)
         if (L->key_dim == 128 && L->value_dim == 128 && L->row <= 192) return launch_tile<4, 8, 3, true>(t, st);
         if (L->key_dim <= 64 && L->value_dim <= 64) return launch_tile<2, 4, 2, false>(t, st);
         if (L->key_dim <= 128 && L->value_dim <= 128) return launch_tile<4, 8, 4, false>(t, st);
@@ -818,12 +841,12 @@ extern "C" int tah_window_decode(const tah_window_layer* L, const tah_window_row
             return TAH_E_WORKSPACE;
         d.part = static_cast<float*>(workspace);
     }
-    // (units per lane: row / 16, rounded up)
+    // (units per lane and row: row / 64, rounded up)
     int rc;
-    if (L->key_dim == 128 && L->value_dim == 128 && L->row <= 192) rc = launch_decode<4, 8, 12, 8, true>(d, st);
-    else if (L->key_dim <= 64 && L->value_dim <= 64) rc = launch_decode<2, 4, 8, 8, false>(d, st);
-    else if (L->row <= 272) rc = launch_decode<8, 16, 17, 8, false>(d, st);
-    else rc = launch_decode<8, 16, 32, 4, false>(d, st);
+    if (L->key_dim == 128 && L->value_dim == 128 && L->row <= 192) rc = launch_decode<4, 8, 3, 8, true>(d, st);
+    else if (L->key_dim <= 64 && L->value_dim <= 64) rc = launch_decode<2, 4, 2, 8, false>(d, st);
+    else if (L->row <= 256) rc = launch_decode<8, 16, 4, 8, false>(d, st);
+    else rc = launch_decode<8, 16, 8, 4, false>(d, st);
     if (rc != TAH_OK || d.splits == 1) return rc;
     hipLaunchKernelGGL(window_merge_kernel, dim3(L->heads, R->rows), dim3(kWave), 0, st, d);
     return launch_status();

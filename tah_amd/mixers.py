@@ -357,7 +357,7 @@ class WindowAttention:
         tied = "v" not in w
         if H % G or rd > D or rd % 2 or (tied and s.vdim != D):
             raise TahDuoError(f"attention: {H} heads on {G}, {rd} of {D} dimensions rotated, values of {s.vdim}: sizes that do not go together")
-        self.rot_pad = pad_to(rd, 8)
+        self.rot_pad = pad_to(rd, 16)
         self.key_dim = pad_to(self.rot_pad + D - rd)
         rest = self.key_dim - self.rot_pad
         turned = list(range(rd)) if s.adjacent else [i + h * (rd // 2) for i in range(rd // 2) for h in (0, 1)]
