@@ -34,11 +34,10 @@ def add_conv(h, w):
     """h [T, channels] plus a causal convolution of it; w [channels, taps], last column for the current token."""
     T, taps = h.shape[0], w.shape[1]
     y = h.clone()
-    for t in range(T):
-        for j in range(taps):
-            s = t - (taps - 1 - j)
-            if s >= 0:
-                y[t] += w[:, j] * h[s]
+    for j in range(taps):
+        back = taps - 1 - j
+        if back < T:
+            y[back:] += w[:, j] * h[:T - back]
     return y
 
 
@@ -56,15 +55,15 @@ def rotate_pairs(x, pos, base, dims):
 
 
 def visible(i, j, size, keep):
-    return j <= i and (i - j < size or j < keep)
+    return (j <= i) & ((i - j < size) | (j < keep))
 
 
-def attention(q, k, v, m, pos0=0):
+def attention(q, k, v, m):
     """q [T, heads, dim], k [T, kv_heads, dim], v [T, kv_heads, vdim] (unrotated) -> [T, heads, vdim]."""
     T, H, per = q.shape[0], q.shape[1], q.shape[1] // k.shape[1]
-    pos = torch.arange(pos0, pos0 + T)
+    pos = torch.arange(T)
     qr, kr = (rotate_pairs(x, pos, m["rot"]["base"], m["rot"]["dims"]) for x in (q, k))
-    seen = torch.tensor([[visible(i, j, m["mask"]["size"], m["mask"]["keep_first"]) for j in range(T)] for i in range(T)])
+    seen = visible(pos[:, None], pos[None], m["mask"]["size"], m["mask"]["keep_first"])
     out = torch.zeros(T, H, v.shape[-1], dtype=q.dtype)
     for h in range(H):
         s = (qr[:, h] @ kr[:, h // per].t()) * m["scale"]
@@ -100,24 +99,24 @@ def expert(h, w, limit):
 def route(h, w_router, top, groups):
     """Chosen experts and their weights per token: sigmoid scores, the best groups by their two largest, the largest
     in those."""
-    idx, wt = [], []
-    for z in h @ w_router.t():
-        s = sigmoid(z)
-        n, size = groups["count"], s.numel() // groups["count"]
-        best = sorted(range(n), key=lambda g: -float(s[g * size:(g + 1) * size].sort(descending=True).values[:2].sum()))
+    scores = sigmoid(h @ w_router.t())
+    idx = []
+    for s in scores.tolist():
+        n, size = groups["count"], len(s) // groups["count"]
+        best = sorted(range(n), key=lambda g: -sum(sorted(s[g * size:(g + 1) * size])[-2:]))
         allowed = [e for g in best[:groups["keep"]] for e in range(g * size, (g + 1) * size)]
-        chosen = sorted(allowed, key=lambda e: -float(s[e]))[:top]
-        idx.append(chosen)
-        wt.append(torch.stack([s[e] for e in chosen]))
-    return torch.tensor(idx), torch.stack(wt)
+        idx.append(sorted(allowed, key=lambda e: -s[e])[:top])
+    idx = torch.tensor(idx)
+    return idx, scores.gather(1, idx)
 
 
 def moe_mlp(h, w, spec):
     idx, p = route(h, w["router"], spec["router"]["top"], spec["router"]["groups"])
     out = torch.zeros_like(h)
-    for t in range(h.shape[0]):
-        for e, pe in zip(idx[t].tolist(), p[t]):
-            out[t] += pe * expert(h[t], part(w, f"e{e}."), spec["expert"]["limit"])
+    for e in range(spec["router"]["experts"]):
+        y = expert(h, part(w, f"e{e}."), spec["expert"]["limit"])
+        for c in range(idx.shape[1]):
+            out += torch.where(idx[:, c:c + 1] == e, p[:, c:c + 1] * y, torch.zeros_like(y))
     return out
 
 

@@ -25,7 +25,7 @@ def build(san: str = "") -> str:
     name = {"": "libtah_duo_emu.so", "address": "libtah_duo_emu_asan.so", "thread": "libtah_duo_emu_tsan.so"}[san]
     out = os.path.join(CSRC, "emu", name)
     srcs = [os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith((".hip", ".h"))]
-    srcs += [os.path.join(CSRC, "emu", "hip", "hip_runtime.h"), os.path.join(ROOT, "include", "tah_duo.h")]
+    srcs += [os.path.join(CSRC, "emu", "hip", "hip_runtime.h")] + [os.path.join(ROOT, "include", f) for f in ("tah_duo.h", "tah_mixers.h")]
     if os.path.exists(out) and all(os.path.getmtime(out) >= os.path.getmtime(s) for s in srcs):
         return out
     cmd = ["make", "-s", "-C", CSRC, "emu", f"EMU_OUT=emu/{name}"]

@@ -1,5 +1,5 @@
-"""The Zozosun decoder through its engine (tah_amd.stack) against the plain oracle: prompts, portions, decoding, batches, slots
-used again, generation through the shared loop, loading through the registry, the trace runner."""
+"""Decoders through the layer-by-layer engine (tah_amd.stack) against their plain oracles: prompts, portions, decoding, batches,
+slots used again, generation through the shared loop, loading through the registry, the trace runner."""
 import io
 import json
 import os
@@ -7,15 +7,14 @@ import os
 import pytest
 import torch
 
-from oracle import zozosun_ref as R
 from tests import emu_util
-from tests import zozosun_cases as Z
+from tests import stack_cases as Z
 
 BF = torch.bfloat16
 needs_clang = pytest.mark.skipif(not emu_util.have_host_clang(), reason="host clang++ not available")
 BOTH = pytest.mark.parametrize("dtype", ["f32", "bf16"])
-MODELS = pytest.mark.parametrize("which", ["odd", "even"])
-CONFIGS = {"odd": Z.ODD, "even": Z.EVEN}
+CONFIGS = Z.CONFIGS
+MODELS = pytest.mark.parametrize("which", sorted(CONFIGS))
 
 
 def setup(which, dtype, dev, batch, max_len):
@@ -30,11 +29,11 @@ def setup(which, dtype, dev, batch, max_len):
 def test_faults_would_show(which):
     """Window edges, and a state lost half-way, are far outside the float32 tolerance with these weights."""
     cfg = CONFIGS[which]
-    Z.wrong_oracles_differ(cfg, Z.tensors_for(cfg), Z.tokens_of(cfg, 160, 1))
+    Z.wrong_oracles_differ(cfg, Z.tensors_for(cfg), Z.tokens_of(cfg, 100, 1))
 
 
 def test_checkpoint_reader_and_registry(tmp_path):
-    from tah_amd import TahDuoError, checkpoint, registry, zozosun
+    from tah_amd import TahDuoError, checkpoint, registry
     t = {"a": torch.randn(3, 5).to(BF), "b.c": torch.arange(7, dtype=torch.int32), "odd": torch.tensor([1, 2, 3], dtype=torch.uint8),
          "f": torch.randn(2, 2), "empty": torch.zeros(0, 4)}
     checkpoint.write_safetensors(str(tmp_path / "model.safetensors"), t)
@@ -46,15 +45,44 @@ def test_checkpoint_reader_and_registry(tmp_path):
         f.truncate(os.path.getsize(tmp_path / "model.safetensors") - 3)
     with pytest.raises(TahDuoError):
         checkpoint.read_tensors(str(tmp_path))
-    assert {"Zozosun", "Qwen3ForCausalLM"} <= set(registry.architectures())
+    assert {"Zedudra", "Zozosun", "Qwen3ForCausalLM"} <= set(registry.architectures())
     assert registry.of_config({"architecture": "Zozosun"}).name == "Zozosun"
     assert registry.of_config({"architectures": ["Qwen3ForCausalLM"]}).name == "Qwen3ForCausalLM"
     with pytest.raises(TahDuoError):
         registry.of_config({"architecture": "nothing"})
-    assert set(zozosun.shapes(Z.EVEN)) == set(Z.tensors_for(Z.EVEN))
-    bad = dict(Z.ODD, layers=[dict(Z.ODD["layers"][0], type="other")])
-    with pytest.raises(TahDuoError):
-        zozosun.shapes(bad)
+    for cfg in CONFIGS.values():
+        assert registry.of_config(cfg).load is Z.design(cfg).load
+        with pytest.raises(TahDuoError):
+            Z.design(cfg).shapes(dict(cfg, layers=[dict(cfg["layers"][0], type="other")]))
+
+
+def test_shared_weights_and_sizes_that_do_not_go_together():
+    """Layers on another layer's weights bring no tensors, and are the same layer; sizes are checked where weights are read."""
+    import copy
+
+    from tah_amd import TahDuoError, zedudra
+    cfg = CONFIGS["zedudra odd"]
+    t = Z.tensors_for(cfg)
+    assert {n.split(".")[0] for n in t if n[0] == "l"} == {"l0", "l1", "l3"}
+    m = Z.load(cfg, t, torch.float32, "cpu")
+    assert m.layers[2] is m.layers[0] and m.layers[4] is m.layers[1] and m.layers[3] is not m.layers[1]
+
+    def broken(f):
+        c = copy.deepcopy(cfg)
+        f(c)
+        with pytest.raises(TahDuoError):
+            Z.load(c, t, torch.float32, "cpu")
+    broken(lambda c: c["canon"].update(taps=4))
+    broken(lambda c: c["norm"].update(groups=5))
+    broken(lambda c: c["layers"][0]["mixer"].update(vdim=8))
+    broken(lambda c: c["layers"][0]["mlp"].update(kind="other"))
+    broken(lambda c: c["layers"][0]["mlp"]["router"]["groups"].update(count=4))
+    broken(lambda c: c["layers"][2].update(weights_of=2))
+    broken(lambda c: c["layers"][2].update(weights_of=9))
+    chain = copy.deepcopy(cfg)
+    chain["layers"].append(dict(chain["layers"][4], weights_of=4))
+    assert zedudra.shapes(chain) == zedudra.shapes(cfg)
+    assert len({id(l) for l in Z.load(chain, t, torch.float32, "cpu").layers}) == 3
 
 
 def test_slot_pool():
@@ -105,9 +133,13 @@ def sequence_case(which, dtype, dev, n, all_cuts, max_len=None):
 
 @needs_clang
 @BOTH
-def test_portions_and_decoding_on_cpu_shim(dtype):
+@pytest.mark.parametrize("which", ["zozosun odd", "zedudra odd"])
+def test_portions_and_decoding_on_cpu_shim(which, dtype):
     with emu_util.emulated():
-        sequence_case("odd", dtype, "cpu", 13, [(7, 2, 2)])
+        if which.startswith("zozosun"):
+            sequence_case(which, dtype, "cpu", 13, [(7, 2, 2)])
+        else:
+            sequence_case(which, dtype, "cpu", 7, [(4, 2)])
 
 
 # ── GPU ──────────────────────────────────────────────────────────────────────────────────────────────────────────────
@@ -129,39 +161,40 @@ def test_long_decoding_gpu(which, dtype):
 
 
 @pytest.mark.gpu
+@MODELS
 @BOTH
-def test_batches_of_unequal_requests_and_slots_used_again_gpu(dtype):
+def test_batches_of_unequal_requests_and_slots_used_again_gpu(which, dtype):
     """Requests of different lengths start, continue in portions or single tokens, and end at different times, all in the same
     calls; each position's logits are those of the request alone.  Slots change owners on the way."""
-    for which in ("odd", "even"):
-        cfg, t, eng, check = setup(which, dtype, "cuda", 3, 120)
-        reqs = [Z.tokens_of(cfg, n, 10 + i) for i, n in enumerate((90, 9, 41, 1, 60, 25, 2))]
-        waiting, live, step = list(range(len(reqs))), {}, 0
-        while waiting or live:
-            while waiting and len(live) < 3:
-                live[waiting.pop(0)] = [eng.alloc(), 0]
-            entries, places = [], []
-            for j, r in enumerate(sorted(live)):
-                s, at = live[r]
-                n = min((1, 7, 2, 1, 23, 1, 3, 16)[(step + 3 * j) % 8], len(reqs[r]) - at)
-                entries.append((s, reqs[r][at:at + n]))
-                places.append((r, at, n))
-            lg = eng.extend(entries)
-            k = 0
-            for r, at, n in places:
-                check(lg[k:k + n], reqs[r], range(at, at + n), f"{which} request {r} at {at}")
-                k += n
-                live[r][1] += n
-                if live[r][1] == len(reqs[r]):
-                    eng.release(live.pop(r)[0])
-            step += 1
+    cfg, t, eng, check = setup(which, dtype, "cuda", 3, 120)
+    reqs = [Z.tokens_of(cfg, n, 10 + i) for i, n in enumerate((90, 9, 41, 1, 60, 25, 2))]
+    waiting, live, step = list(range(len(reqs))), {}, 0
+    while waiting or live:
+        while waiting and len(live) < 3:
+            live[waiting.pop(0)] = [eng.alloc(), 0]
+        entries, places = [], []
+        for j, r in enumerate(sorted(live)):
+            s, at = live[r]
+            n = min((1, 7, 2, 1, 23, 1, 3, 16)[(step + 3 * j) % 8], len(reqs[r]) - at)
+            entries.append((s, reqs[r][at:at + n]))
+            places.append((r, at, n))
+        lg = eng.extend(entries)
+        k = 0
+        for r, at, n in places:
+            check(lg[k:k + n], reqs[r], range(at, at + n), f"{which} request {r} at {at}")
+            k += n
+            live[r][1] += n
+            if live[r][1] == len(reqs[r]):
+                eng.release(live.pop(r)[0])
+        step += 1
 
 
 @pytest.mark.gpu
 @BOTH
-def test_wanted_rows_and_refusals_gpu(dtype):
+@pytest.mark.parametrize("which", ["zozosun odd", "zedudra odd"])
+def test_wanted_rows_and_refusals_gpu(which, dtype):
     from tah_amd import TahDuoError
-    cfg, t, eng, check = setup("odd", dtype, "cuda", 2, 20)
+    cfg, t, eng, check = setup(which, dtype, "cuda", 2, 20)
     a, b = eng.alloc(), eng.alloc()
     ta, tb = Z.tokens_of(cfg, 12, 5), Z.tokens_of(cfg, 9, 6)
     lg = eng.extend([(a, ta), (b, tb)], want=[[11, 2], []])
@@ -179,7 +212,7 @@ def oracle_greedy(cfg, t, prompt, n, eos=-1):
     """Greedy tokens and the smallest gap between the two largest logits on the way."""
     seq, gap = list(prompt), float("inf")
     for _ in range(n):
-        z = R.forward(cfg, t, seq)[-1]
+        z = Z.oracle(cfg).forward(cfg, t, seq)[-1]
         top = z.topk(2).values
         gap = min(gap, float((top[0] - top[1]) / z.pow(2).mean().sqrt()))
         seq.append(int(z.argmax()))
@@ -255,10 +288,11 @@ def test_captured_generation_equals_eager_steps_gpu(which):
 
 @pytest.mark.gpu
 @BOTH
-def test_trace_runner_gpu(dtype, tmp_path):
+@pytest.mark.parametrize("which", ["zozosun odd", "zedudra odd", "zedudra even"])
+def test_trace_runner_gpu(which, dtype, tmp_path):
     """A checkpoint folder through the command's main: portions, single tokens, requests that end, wanted rows."""
     from tah_amd import checkpoint, trace
-    cfg = Z.ODD if dtype == "f32" else Z.without_close_calls(Z.ODD)
+    cfg = CONFIGS[which] if dtype == "f32" else Z.without_close_calls(CONFIGS[which])
     t = Z.tensors_for(cfg, sharp=3.0 if dtype == "f32" else 1.0)
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     checkpoint.write_safetensors(str(tmp_path / "model.safetensors"), t)
