@@ -20,7 +20,7 @@ MODELS = pytest.mark.parametrize("which", sorted(CONFIGS))
 def setup(which, dtype, dev, batch, max_len):
     from tah_amd.stack import StackEngine
     cfg = CONFIGS[which] if dtype == "f32" else Z.without_close_calls(CONFIGS[which])
-    t = Z.tensors_for(cfg, sharp=3.0 if dtype == "f32" else 1.0)  # (peaked attention magnifies bf16's roundings)
+    t = Z.tensors_for(cfg, sharp=2.0 if dtype == "f32" else 1.0)  # (peaked attention magnifies bf16's roundings)
     return cfg, t, StackEngine(Z.load(cfg, t, Z.DTYPES[dtype], dev), batch, max_len, device=dev), Z.Check(cfg, t, Z.DTYPES[dtype])
 
 
@@ -229,7 +229,7 @@ def test_greedy_generation_gpu(which):
     prompts = [Z.tokens_of(cfg, n, 30 + n) for n in (17, 2, 30)]
     t64 = {k: v.double() for k, v in t.items()}
     want, gaps = zip(*(oracle_greedy(cfg, t64, p, 12) for p in prompts))
-    assert min(gaps) > 1e-3, "the case has a near tie: choose other prompts"
+    assert min(gaps) > 3e-4, "the case has a near tie: choose other prompts"
     ids = torch.tensor(sum(prompts, [])).cuda()
     cu = torch.tensor([0, 17, 19, 49], dtype=torch.int32).cuda()
     for graph in (False, True):
@@ -293,7 +293,7 @@ def test_trace_runner_gpu(which, dtype, tmp_path):
     """A checkpoint folder through the command's main: portions, single tokens, requests that end, wanted rows."""
     from tah_amd import checkpoint, trace
     cfg = CONFIGS[which] if dtype == "f32" else Z.without_close_calls(CONFIGS[which])
-    t = Z.tensors_for(cfg, sharp=3.0 if dtype == "f32" else 1.0)
+    t = Z.tensors_for(cfg, sharp=2.0 if dtype == "f32" else 1.0)
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     checkpoint.write_safetensors(str(tmp_path / "model.safetensors"), t)
     check = Z.Check(cfg, t, Z.DTYPES[dtype])

@@ -47,6 +47,13 @@ def looking_queries(k, heads, m, dtype):
     return q.to(dtype)
 
 
+def attention_on_rounded(q, k, v, m, dtype):
+    """The oracle's attention with queries and keys rounded to the element type after their rotation, as they are cached."""
+    pos = torch.arange(q.shape[0])
+    qr, kr = (R.rotate_pairs(x, pos, m["rot"]["base"], m["rot"]["dims"]).to(dtype).double() for x in (q, k))
+    return R.attention(qr, kr, v, dict(m, rot=dict(m["rot"], dims=0)))
+
+
 def window_case(dev, dtype, m, total, cuts, steps, stand_out=True, gate=True, own_values=0, adjacent=True, max_len=None, slots=3, seed=6):
     """One sequence next to a shorter one, portions of the given sizes, then single tokens next to a dropped row; twice, the
     second time on the slots and rings of the first.  The layer's input rows hold queries, keys (values) and gates side by
@@ -89,7 +96,7 @@ def window_case(dev, dtype, m, total, cuts, steps, stand_out=True, gate=True, ow
             v = pick("v", G).double() if own_values else k
             if not adjacent:
                 q, k = half_split(q, rd), half_split(k, rd)
-            o = R.attention(q, k, v, m)
+            o = attention_on_rounded(q, k, v, m, dtype)
             sg = R.sigmoid(pick("g", H).double()) if gate else torch.ones(n + steps, H, 1, dtype=torch.float64)
             xs.append(x)
             want.append((o * sg.view(n + steps, H, 1)).reshape(n + steps, H * V))
@@ -114,8 +121,7 @@ def window_case(dev, dtype, m, total, cuts, steps, stand_out=True, gate=True, ow
             for b in range(2):
                 got[b].append(y[b:b + 1])
         for b in range(2):
-            # (scores of 9 and more: in bf16 the roundings of queries and keys move the weights by a few per cent)
-            close(torch.cat(got[b])[:, :H * V], want[b], dtype, f"window attention, sequence {b}, run {rerun}", tol=0.1 if dtype == BF else None)
+            close(torch.cat(got[b])[:, :H * V], want[b], dtype, f"window attention, sequence {b}, run {rerun}")
     assert bool((layer.cache.rows[1] == 50.0).all())  # a slot nobody owned
     if stand_out and adjacent and total + steps >= W + K + 6:  # the edges are in the numbers: one position more or less shows
         q, k, v, sg = seen[0]
@@ -134,7 +140,7 @@ def group_norm_case(dev, dtype, rows, width, groups, top=2, experts=3, seed=7):
     from tah_amd.ops import _call
     from tah_amd.stack import Columns
     g, at, eps = torch.Generator().manual_seed(seed), Columns(width, groups), 0.03
-    cols, scale = at.cols, torch.exp(torch.arange(groups) * 0.7).repeat_interleave(width // groups)  # groups of unlike sizes
+    cols, scale = at.cols, torch.exp(torch.arange(groups) % 5 * 0.7).repeat_interleave(width // groups)  # groups of unlike sizes
     up = lambda t: torch.nn.functional.pad(at.spread(t), (0, cols - at.spread(t).shape[-1]))
     assert torch.equal(at.gather(up(torch.arange(width)[None])), torch.arange(width)[None])
     x, y, ex = rnd(g, rows, width) * scale, (rnd(g, rows, width) * scale).to(dtype), rnd(g, experts * rows, width).to(dtype)
@@ -237,7 +243,7 @@ def activation_case(dev, dtype, rows=5, n=48, k=64, seed=9):
         close(act(z.to(dev)), R.clamped_gate(z.double()[:, :n], z.double()[:, n:], limit), dtype, "clamped gate")
         if dtype == BF:
             w, x = (2 * rnd(g, 2 * n, k) * k ** -0.5).to(BF), rnd(g, rows, k).to(BF)
-            z = x.double() @ w.double().t()
+            z = (x.double() @ w.double().t()).to(BF).double()   # (rounded where the product ends)
             y = ops.linear_rows(ops.linear_pack_weight(w.to(dev), gate_up=True), ops.linear_pack_rows(x.to(dev)), rows, n, k, gate_up=True, **act.rows)
             close(y, R.clamped_gate(z[:, :n], z[:, n:], limit), BF, "product, clamped gate")
 
@@ -256,7 +262,7 @@ def moe_case(dev, dtype, rows, width, ff, experts, top, groups, keep, limit, see
     spec = {"router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}}, "expert": {"limit": limit}}
     want = R.moe_mlp(x.double(), flat, spec)
     idx, p = R.route(x.double(), flat["router"], top, spec["router"]["groups"])
-    if keep < groups and rows >= 20:  # the groups matter: without them some token chooses otherwise
+    if keep < groups < experts and rows >= 20:  # the groups matter: without them some token chooses otherwise
         free, _ = R.route(x.double(), flat["router"], top, {"count": 1, "keep": 1})
         assert bool((free.sort(1).values != idx.sort(1).values).any())
     b = MoeMlp(Router(top, True, groups, keep), {k: t.to(dev) for k, t in w.items()}, None, cols, clamped_gate(limit)).bind(Host(dev, dtype, 1, 1))
@@ -303,7 +309,7 @@ ODD = config(44, 61, 4, 3, 2.5, [
     0,
     (window_of(4, 2, 12, 2, 1, 2, 30.0, 0.7), dense_of(52)),
     1,
-], eps=3e-3)
+], eps=0.1)
 # multiples of the matrix steps, more query heads than one tile takes, heads wider than 128
 EVEN = config(96, 128, 3, 4, 9.0, [
     (window_of(8, 4, 32, 16, 9, 4, 10000.0, 0.3), dense_of(160)),
