@@ -1,7 +1,8 @@
 /* tah_mixers.h -- C ABI of the layer mechanisms of decoder models that are described layer by layer: residual rows
  * with norms around the sublayers, short convolutions of a sublayer's input, gated delta-rule recurrence, sliding-window
- * attention on latents or on keys and values, mixture of experts.  Same conventions as tah_duo.h (device pointers, nothing allocated, nothing synchronised, 0 or TAH_E_*),
- * exported by the same library.  Sizes and constants are arguments; nothing here belongs to one model.
+ * attention on latents or on keys and values, mixture of experts.  Same conventions as tah_duo.h (device pointers, nothing
+ * allocated, nothing synchronised, 0 or TAH_E_*), exported by the same library.  Sizes and constants are arguments; nothing
+ * here belongs to one model.
  *
  * Element type.  `dtype` says what activations, weights and cached rows are: TAH_DT_BF16 or TAH_DT_F32.  The residual
  * rows, norms, attention scores and weights, router logits and recurrent state are float32 with either.

@@ -3,7 +3,8 @@
 // expert that some row chose over all rows.)
 //
 //  * moe_route_kernel: router logits in float32, their scores, the open groups of experts, the largest ones and their
-//    weights; RB rows per workgroup share the router's weights, and a wave takes EB experts at a time so that they share the rows' reads.
+//    weights; RB rows per workgroup share the router's weights, and a wave takes EB experts at a time so that they share
+//    the rows' reads.
 //  * moe_plan_kernel: counting sort of the (row, choice) pairs by expert, each expert's rows padded to whole tiles.
 //  * moe_tile_kernel: bf16 tiles of 128 places x 256 weight rows on the matrix cores, both operands staged through LDS
 //    by asynchronous copies, two stages ahead; gate and up rows of the same columns share a wave, which applies the gate.
@@ -399,7 +400,8 @@ __global__ __launch_bounds__(kMoeThreads) void moe_plain_kernel(const MoeGemm p)
     if (n0 + tc >= p.n) return;
 #pragma unroll
     for (int i = 0; i < 16; ++i)
-        static_cast<float*>(p.out)[((int64_t)tile * kTile + tr + 8 * i) * p.out_rs + n0 + tc] = !GATE ? sg[i] : (p.act == TAH_ACT_CLAMPED_GATE ? clamped_gate_exact(sg[i], su[i], p.c0, p.c1) : silu_exact(sg[i]) * su[i]);
+        static_cast<float*>(p.out)[((int64_t)tile * kTile + tr + 8 * i) * p.out_rs + n0 + tc] =
+            !GATE ? sg[i] : (p.act == TAH_ACT_CLAMPED_GATE ? clamped_gate_exact(sg[i], su[i], p.c0, p.c1) : silu_exact(sg[i]) * su[i]);
 }
 
 template <class X, class E>
@@ -456,7 +458,8 @@ extern "C" int tah_moe_linear(const void* x, int64_t x_rs, const void* w, const 
                               tah_stream_t stream) {
     using namespace tah;
     if (tiles < 0 || tiles > 65535 || n <= 0 || k <= 0 || n % 4 != 0 || k % 32 != 0 || x_rs < k || out_rs < n || x_rs % 8 != 0 || out_rs % 4 != 0 ||
-        (kind != TAH_LINEAR_PLAIN && kind != TAH_LINEAR_GATE_UP) || (activation != TAH_ACT_NONE && activation != TAH_ACT_CLAMPED_GATE) || (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
+        (kind != TAH_LINEAR_PLAIN && kind != TAH_LINEAR_GATE_UP) || (activation != TAH_ACT_NONE && activation != TAH_ACT_CLAMPED_GATE) ||
+        (dtype != TAH_DT_BF16 && dtype != TAH_DT_F32))
         return TAH_E_SHAPE;
     if (tiles == 0) return TAH_OK;
     if (!x || !w || !tile_expert || !out || (kind == TAH_LINEAR_GATE_UP && !source)) return TAH_E_NULL;

@@ -1,6 +1,7 @@
 // Residual rows of a layer-by-layer decoder, gfx950: token rows into the residual stream, the norm of a sublayer's
-// output with its residual sum and the norm and short convolution in front of the next one, and element-wise activations.  HBM-bound; one workgroup per row, eight columns per
-// thread and pass, everything between load and store in float32.
+// output with its residual sum and the norm and short convolution in front of the next one, and element-wise
+// activations.  HBM-bound; one workgroup per row, eight columns per thread and pass, everything between load and store in
+// float32.
 #include <hip/hip_runtime.h>
 
 #include "mixer_device.h"

@@ -669,9 +669,10 @@ int check_layer(const tah_window_layer* L) {
     if (!L) return TAH_E_NULL;
     if (L->heads <= 0 || L->kv_heads <= 0 || L->heads % L->kv_heads != 0 || L->heads > 65535 || L->key_dim <= 0 || L->key_dim % 32 != 0 ||
         L->value_dim <= 0 || L->value_dim % 32 != 0 || L->row % 8 != 0 || L->row < L->key_dim || L->row < L->value_dim ||
-        L->row > L->key_dim + L->value_dim || (L->row - L->key_dim) % 16 != 0 || L->rot_dim < 0 || L->rot_dim % 2 != 0 || L->rot_pad % 16 != 0 || L->rot_pad < L->rot_dim ||
-        L->rot_pad > L->key_dim || L->rot_source < 0 || L->rot_source % 8 != 0 || L->rot_source + L->rot_pad > L->row || L->keep_first < 0 ||
-        L->ring <= 0 || (int64_t)(L->keep_first + (int64_t)L->ring) * L->row >= (1 << 30) || L->window <= 0 || L->window > L->ring || L->nslots <= 0 || (L->dtype != TAH_DT_BF16 && L->dtype != TAH_DT_F32))
+        L->row > L->key_dim + L->value_dim || (L->row - L->key_dim) % 16 != 0 || L->rot_dim < 0 || L->rot_dim % 2 != 0 ||
+        L->rot_pad % 16 != 0 || L->rot_pad < L->rot_dim || L->rot_pad > L->key_dim || L->rot_source < 0 || L->rot_source % 8 != 0 || L->rot_source + L->rot_pad > L->row || L->keep_first < 0 ||
+        L->ring <= 0 || (int64_t)(L->keep_first + (int64_t)L->ring) * L->row >= (1 << 30) || L->window <= 0 || L->window > L->ring ||
+        L->nslots <= 0 || (L->dtype != TAH_DT_BF16 && L->dtype != TAH_DT_F32))
         return TAH_E_SHAPE;
     if (L->key_dim > 8192 || L->value_dim > kWinThreads * kRowValues) return TAH_E_SHAPE;
     if (!L->cache) return TAH_E_NULL;
