@@ -42,10 +42,10 @@ MOE_SMALL = [(5, 40, 12, 4, 2, 9), (3, 32, 32, 3, 1, 0)]
 MOE_GPU = MOE_SMALL + [(32, 96, 48, 16, 4, 64), (200, 160, 96, 8, 8, 32), (700, 256, 192, 64, 6, 128), (31, 512, 100, 7, 3, 0), (300, 72, 40, 5, 5, 17)]
 # (sizes, prompt, portions, decoded tokens, further arguments): windows inside, at and across the 64-key tiles and the 32-key
 # passes, kept tokens that fill tiles of their own, more query heads than a tile or a pass takes, heads of up to 256
-WINDOW_SMALL = [(D.window_of(2, 1, 12, 6, 4, 2), 11, (2, 7, 2), 4, {}), (D.window_of(3, 3, 32, 32, 6, 3), 13, (13,), 3, {}),
+WINDOW_SMALL = [(D.window_of(2, 1, 12, 6, 4, 2), 11, (2, 7, 2), 4, {}), (D.window_of(2, 2, 32, 32, 6, 3), 13, (13,), 2, {}),
                 (D.window_of(2, 1, 16, 8, 5, 1), 7, (5, 2), 3, dict(own_values=20, adjacent=False, gate=False))]
 WINDOW_GPU = WINDOW_SMALL + [
-    (D.window_of(16, 8, 128, 64, 64, 4), 200, (64, 2, 63, 71), 70, {}), (D.window_of(8, 2, 128, 32, 33, 3), 150, (150,), 40, {}),
+    (D.window_of(16, 8, 128, 64, 64, 4), 200, (64, 2, 63, 71), 70, {}), (D.window_of(10, 2, 128, 48, 33, 3), 150, (150,), 40, {}),
     (D.window_of(20, 1, 64, 32, 65, 1), 140, (1 + 62, 2, 75), 66, {}), (D.window_of(5, 5, 24, 24, 128, 7), 260, (130, 130), 9, {}),
     (D.window_of(33, 1, 96, 2, 31, 5), 90, (33, 57), 34, {}), (D.window_of(4, 2, 160, 40, 40, 70), 180, (90, 90), 45, {}),
     (D.window_of(6, 2, 256, 256, 100, 130), 310, (200, 2, 108), 12, {}), (D.window_of(2, 2, 300, 20, 9, 2), 40, (40,), 12, {}),
